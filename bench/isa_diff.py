@@ -33,7 +33,8 @@ def kernels(asm: str) -> dict[str, list[str]]:
 
 def compile_asm(src: Path, workdir: Path) -> str:
     workdir.mkdir(parents=True, exist_ok=True)
-    subprocess.run([HIPCC, "--offload-arch=gfx950", "-O3", "-std=c++17", "-c", str(src), "-o", "x.o",
+    subprocess.run([HIPCC, "--offload-arch=gfx950", "-O3", "-std=c++17",
+           "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-c", str(src), "-o", "x.o",
                     "-save-temps=obj"], cwd=workdir, check=True, capture_output=True, timeout=1800)
     (s,) = workdir.glob(f"{src.stem}-hip-amdgcn-amd-amdhsa-gfx950.s")
     return s.read_text()

@@ -102,6 +102,20 @@ _SIGS = {
                                                                    _c_void_p], _c_int),
     "kgs_paged_decode_rope_bf16": ([_c_void_p, _c_int] + [_c_void_p] * 11 + [_c_int] * 7 +
                                    [_c_long, ctypes.c_float, _c_int, _c_int, _c_void_p], _c_int),
+    # hyper-connections, latent attention, delta rule (hyper.hip, latent.hip, delta.hip, activation.hip)
+    "kgs_hyper_step": ([_c_void_p] * 7 + [_c_int] * 3 + [_c_long] * 2 + [ctypes.c_float, _c_int, _c_void_p], _c_int),
+    "kgs_hyper_embed": ([_c_void_p] * 7 + [_c_int] * 3 + [_c_long] * 2 + [ctypes.c_float, _c_int, _c_void_p], _c_int),
+    "kgs_act_mul": ([_c_void_p] * 2 + [_c_int] * 2 + [_c_long] * 2 + [_c_int] * 2 + [_c_void_p], _c_int),
+    "kgs_softcap": ([_c_void_p] * 2 + [_c_int] * 2 + [_c_long, ctypes.c_float, _c_int, _c_void_p], _c_int),
+    "kgs_latent_norm": ([_c_void_p, _c_long] + [_c_int] * 6 + [_c_void_p] * 5 + [_c_int, ctypes.c_float, _c_int,
+                                                                                _c_void_p], _c_int),
+    "kgs_head_proj": ([_c_void_p] * 6 + [_c_long] * 5 + [_c_int] * 5 + [_c_void_p], _c_int),
+    "kgs_latent_attn": ([_c_void_p] * 10 + [_c_int] * 8 + [ctypes.c_float, _c_void_p], _c_int),
+    "kgs_latent_attn_simple": ([_c_void_p] * 6 + [_c_int] * 4 + [ctypes.c_float, _c_int, _c_void_p], _c_int),
+    "kgs_attn_fwd_ragged_bf16": ([_c_void_p] * 5 + [_c_int] * 3 + [_c_long] * 4 + [ctypes.c_float, _c_void_p, _c_long,
+                                                                                  _c_void_p], _c_int),
+    "kgs_delta_forward": ([ctypes.POINTER(_c_void_p), ctypes.POINTER(_c_long), _c_void_p], _c_int),
+    "kgs_delta_out": ([_c_void_p] * 4 + [_c_int] * 3 + [_c_long] * 2 + [ctypes.c_float, _c_int, _c_void_p], _c_int),
     # peer-to-peer all-reduce (native/kernels/allreduce_p2p.hip)
     "kgs_ar_signal_bytes": ([], _c_int),
     "kgs_ar_max_blocks": ([], _c_int),

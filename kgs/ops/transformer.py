@@ -226,6 +226,26 @@ def attention_chunk(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, heads: in
     return out
 
 
+def attention_ragged(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, items: torch.Tensor, heads: int,
+                     head_dim: int, scale: float, out: torch.Tensor, gate: torch.Tensor | None = None) -> torch.Tensor:
+    """Causal flash attention of ragged prompt portions in one launch (head_dim 64
+    or 128, as many key heads as query heads). ``items`` int32 ``[n, 4]``: a block
+    of up to 128 query rows each -- its first row in ``q`` / ``out``, the row of
+    its sequence's key 0 in ``k`` / ``v``, the first row's position, the rows.
+    ``gate [rows, >= heads]``: head outputs times its sigmoid."""
+    for t, n in ((q, "q"), (k, "k"), (v, "v"), (out, "out")):
+        _need(t, n)
+    if items.dtype != torch.int32 or items.dim() != 2 or items.shape[1] != 4 or not items.is_contiguous():
+        raise ValueError("items must be contiguous int32 [n, 4]")
+    rc = _lib.lib().kgs_attn_fwd_ragged_bf16(q.data_ptr(), k.data_ptr(), v.data_ptr(), out.data_ptr(),
+                                             items.data_ptr(), items.shape[0], heads, head_dim, q.stride(0),
+                                             k.stride(0), v.stride(0), out.stride(0), float(scale),
+                                             0 if gate is None else gate.data_ptr(),
+                                             0 if gate is None else gate.stride(0), _lib.stream_handle(q.device))
+    _lib.check(rc, "attention_ragged")
+    return out
+
+
 def ref_attention_chunk(q, k, v, heads, kv_heads, head_dim=128, scale=None):
     """fp32 reference of :func:`attention_chunk` (bottom-right causal)."""
     S, Sk = q.shape[0], k.shape[0]

@@ -23,9 +23,10 @@ import numpy as np
 import torch
 
 from kgs.models.llama import LlamaConfig
+from kgs.models.registry import of_config
 from kgs.ops.decode import PAGE, PagedKVCache
 
-from .model import ServingModel, gate_up_panel_widths
+from .model import gate_up_panel_widths
 from .trace import TRACE
 
 
@@ -81,6 +82,7 @@ class EngineConfig:
     w4x_panels: bool = True           # tile-panel copies of the split-K decode projections (qkv, o, down)
     gate_up_panels: bool = True       # SwiGLU tile-panel copies of gate|up for the unsplit decode routes
     overlap: bool = True              # plan/launch step t+1 before step t's tokens are read back (LLMEngine.step)
+    dtype: str = "bfloat16"           # "float32": everything in 32-bit (models whose serving class has it)
     seed: int = 0
 
 
@@ -92,22 +94,20 @@ def _bucket(n: int, cap: int) -> int:
 
 
 class LLMEngine:
-    def __init__(self, model_cfg: LlamaConfig, cfg: EngineConfig | None = None, device="cuda", backend: str = "kgs"):
+    def __init__(self, model_cfg, cfg: EngineConfig | None = None, device="cuda", backend: str = "kgs"):
         from kgs._native import _serve
 
         self.cfg = cfg = cfg or EngineConfig()
         self.device = torch.device(device)
         self.backend = backend
+        self.serving_class = of_config(model_cfg).serving_class()
         num_pages = cfg.num_pages or self._pages_from_memory(model_cfg)
-        self.model = ServingModel(model_cfg, device=device, backend=backend, seed=cfg.seed, num_pages=num_pages,
-                                  max_model_len=cfg.max_model_len, fused_max_batch=cfg.fused_max_batch,
-                                  decode_weights=cfg.decode_weights, kv_cache_dtype=cfg.kv_cache_dtype,
-                                  packed_decode=cfg.packed_decode, prefill_weights=cfg.prefill_weights,
-                                  fuse_splitk=cfg.fuse_splitk, w4x_panels=cfg.w4x_panels,
-                                  gate_up_panels=cfg.gate_up_panels)
+        self.model = self.serving_class.for_engine(model_cfg, cfg, device, backend, num_pages)
         sc = _serve.SchedulerConfig()
         sc.num_pages, sc.page_size, sc.max_batch = num_pages, PAGE, cfg.max_batch
-        sc.max_prefill_tokens, sc.max_model_len, sc.pad_multiple = cfg.max_prefill_tokens, cfg.max_model_len, 128
+        sc.max_prefill_tokens, sc.max_model_len = cfg.max_prefill_tokens, cfg.max_model_len
+        sc.pad_multiple = self.model.pad_multiple
+        sc.state_slots = cfg.max_batch if self.model.has_state else 0
         sc.chunk_tokens = cfg.chunked_prefill
         sc.prefix_caching = cfg.prefix_caching
         self.sched = _serve.Scheduler(sc)
@@ -145,10 +145,16 @@ class LLMEngine:
         self._pinned = None  # two host buffers the in-flight tokens are copied into, alternately
         self._flip = 0
 
-    def _pages_from_memory(self, mc: LlamaConfig) -> int:
+    def _pages_from_memory(self, mc) -> int:
         if self.device.type != "cuda":
             return 256
         free, _ = torch.cuda.mem_get_info(self.device)
+        if not isinstance(mc, LlamaConfig):
+            m = self.serving_class.memory(mc, self.cfg.dtype, self.cfg.max_batch)
+            avail = max(0, (free - m["weights"] - m["state"] - (8 << 30)) * self.cfg.kv_fraction)
+            # more pages than every running sequence can fill are of no use
+            most = self.cfg.max_batch * math.ceil(self.cfg.max_model_len / PAGE) + 1
+            return int(min(most, max(64, avail // m["page"])))
         h, i, kvd = mc.hidden, mc.intermediate, mc.kv_heads * mc.head_dim
         per_layer = h * (h + 2 * kvd) + h * h + 2 * h * i + i * h
         weights = 2 * (mc.layers * per_layer + 2 * mc.vocab * h)
@@ -431,6 +437,56 @@ class LLMEngine:
             self.step()
         return [self.requests.pop(r) for r in rids]
 
+    # ---------------------------------------------------------------- feeding
+    def open_feed(self) -> int:
+        """Admit a request whose tokens the caller supplies step by step
+        (:meth:`feed`): trace replay, scoring of given text. It holds cache pages for
+        its tokens and a state slot until :meth:`close_feed`."""
+        if not self.model.ragged:
+            raise ValueError("this model's steps take whole prompts; only ragged models can be fed")
+        rid = next(self._ids)
+        if not self.sched.open(rid):
+            raise RuntimeError(f"no room for another request (max_batch {self.cfg.max_batch})")
+        return rid
+
+    def close_feed(self, rid: int) -> None:
+        if not self.sched.abort(rid):
+            raise KeyError(f"request {rid} is not open")
+        self.sched.release(rid)
+
+    def feed(self, entries: list[tuple[int, list, list]]) -> torch.Tensor:
+        """Run ONE step on exactly the given tokens: ``entries`` are (request, its
+        next tokens, the places among them whose logits are wanted). Portions of
+        prompts and single tokens run as one batch, steps of single tokens only as
+        a decode step (replayed from its hipGraph). Returns the logits at the wanted
+        places, in order, ``[wanted, vocab]``."""
+        if not entries:
+            return torch.empty((0, self.vocab), device=self.device)
+        for rid, toks, want in entries:
+            if any(not 0 <= w < len(toks) for w in want):
+                raise ValueError(f"request {rid}: wanted places {want} outside its {len(toks)} tokens")
+        plan = self.sched.feed([e[0] for e in entries], [np.asarray(e[1], dtype=np.int32) for e in entries])
+        if plan.kind == 0:
+            raise RuntimeError(f"step of {[(e[0], len(e[1])) for e in entries]} tokens does not fit "
+                               f"({self.sched.num_free_pages} free pages) or names a request that is not open")
+        if self.validate:
+            self._check_plan(plan)
+        first = {int(r): int(plan.seq_starts[j]) if j < plan.n_prefill else
+                 len(plan.tokens) - len(plan.seq_ids) + j for j, r in enumerate(plan.seq_ids)}
+        rows = np.array([first[e[0]] + w for e in entries for w in e[2]], dtype=np.int64)
+        nstep = self.stats["mixed_steps"] + self.stats["decode_steps"]
+        TRACE.mark(f"feed step {nstep} kind={plan.kind} seqs={len(plan.seq_ids)} rows={len(plan.tokens)} begin")
+        if plan.kind == 2:
+            self.stats["decode_steps"] += 1
+            self.stats["decode_tokens"] += len(plan.seq_ids)
+            logits = self._run_decode(plan).index_select(0, self._dev(rows, torch.int64))
+            if self.use_graphs:  # the graph's staging buffers are free again before the next step fills them
+                torch.cuda.current_stream(self.device).synchronize()
+            return logits
+        self.stats["mixed_steps"] += 1
+        self.stats["prefill_tokens"] += int(plan.seq_lens.sum())
+        return self.model.run_plan(plan, logit_rows=rows)
+
     # -------------------------------------------------------------- checks
     def _check_plan(self, plan) -> None:
         """Every index a step's kernels turn into an address, checked on the host
@@ -462,8 +518,12 @@ class LLMEngine:
                 sl = np.asarray(plan.slots)
                 if np.any((sl >= 0) & (sl // PAGE != last)):
                     bad.append("decode slot not in the last page of its context")
-        if plan.kind == 3 and plan.n_prefill:
+        if plan.kind in (1, 3) and plan.n_prefill:
             rng("pf_block_tables", plan.pf_block_tables, 0, npg)
+        if self.model.has_state:
+            rng("state_slots", plan.state_slots, 1, self.sched.num_state_slots + 1)
+            if len(plan.state_slots) != len(plan.seq_ids):
+                bad.append(f"{len(plan.state_slots)} state slots for {len(plan.seq_ids)} sequences")
         if bad:
             raise RuntimeError(f"scheduler plan (kind {plan.kind}, {len(plan.seq_ids)} seqs) failed its checks: "
                                + "; ".join(bad))
@@ -476,12 +536,16 @@ class LLMEngine:
         return t.to(dtype)
 
     def _run_prefill(self, plan, tokens: torch.Tensor | None = None) -> torch.Tensor:
+        if self.model.ragged:
+            return self.model.run_plan(plan, tokens)
         return self.model.prefill(tokens if tokens is not None else self._dev(plan.tokens),
                                   self._dev(plan.positions), self._dev(plan.slots),
                                   plan.seq_starts.tolist(), plan.seq_lens.tolist(), plan.padded_lens.tolist())
 
     def _run_mixed(self, plan, tokens: torch.Tensor | None = None) -> torch.Tensor:
         """``tokens``: the input tokens on the device (overlapped steps), else the plan's."""
+        if self.model.ragged:
+            return self.model.run_plan(plan, tokens)
         npf = plan.n_prefill
         pf_bt = self._dev(plan.pf_block_tables) if npf else None
         chunks = [(int(plan.seq_starts[j]), int(plan.seq_lens[j]), int(plan.padded_lens[j]), int(plan.ctx_starts[j]),
@@ -496,9 +560,10 @@ class LLMEngine:
         """``tokens``: the input tokens on the device (overlapped steps), else the plan's."""
         b = len(plan.seq_ids)
         if not self.use_graphs:
+            extra = (self._dev(plan.state_slots),) if self.model.has_state else ()
             return self.model.decode(tokens if tokens is not None else self._dev(plan.tokens),
                                      self._dev(plan.positions), self._dev(plan.slots),
-                                     self._dev(plan.block_tables), self._dev(plan.ctx_lens))
+                                     self._dev(plan.block_tables), self._dev(plan.ctx_lens), *extra)
         bb = _bucket(b, self.cfg.max_batch)
         wb = _bucket(plan.max_pages, math.ceil(self.cfg.max_model_len / PAGE))
         g = self._graphs.get((bb, wb)) or self._capture(bb, wb)
@@ -517,6 +582,9 @@ class LLMEngine:
         hn["ctx"][:b] = plan.ctx_lens
         hn["bt"][:] = 0
         hn["bt"][:b, :plan.max_pages] = plan.block_tables
+        if self.model.has_state:
+            hn["state"][:] = 0
+            hn["state"][:b] = plan.state_slots
         for k in host:
             io[k].copy_(host[k], non_blocking=True)
         if tokens is not None:
@@ -532,10 +600,14 @@ class LLMEngine:
 
         host = {"tokens": pinned(bb), "positions": pinned(bb), "slots": pinned(bb), "ctx": pinned(bb),
                 "bt": pinned((bb, wb))}
+        if self.model.has_state:  # padded rows: the null slot 0
+            host["state"] = pinned(bb)
         host["slots"][:] = -1
         host["ctx"][:] = 1
         io = {k: v.to(self.device) for k, v in host.items()}
-        run = lambda: self.model.decode(io["tokens"], io["positions"], io["slots"], io["bt"], io["ctx"])  # noqa: E731
+        extra = (io["state"],) if self.model.has_state else ()
+        run = lambda: self.model.decode(io["tokens"], io["positions"], io["slots"], io["bt"], io["ctx"],  # noqa: E731
+                                        *extra)
         s = torch.cuda.Stream(self.device)
         s.wait_stream(torch.cuda.current_stream(self.device))
         with torch.cuda.stream(s):

@@ -55,6 +55,20 @@ def gate_up_panel_widths(n: int, k: int) -> set:
 
 
 class ServingModel:
+    ragged = False      # prompt steps come padded, portions are multiples of pad_multiple
+    pad_multiple = 128  # the flash-attention prefill kernel's q-block
+    has_state = False   # no per-sequence recurrent state
+
+    @classmethod
+    def for_engine(cls, cfg: LlamaConfig, ec, device, backend: str, num_pages: int) -> "ServingModel":
+        if ec.dtype != "bfloat16":
+            raise ValueError(f"the Llama serving model runs in bfloat16, not {ec.dtype}")
+        return cls(cfg, device=device, backend=backend, seed=ec.seed, num_pages=num_pages,
+                   max_model_len=ec.max_model_len, fused_max_batch=ec.fused_max_batch,
+                   decode_weights=ec.decode_weights, kv_cache_dtype=ec.kv_cache_dtype,
+                   packed_decode=ec.packed_decode, prefill_weights=ec.prefill_weights,
+                   fuse_splitk=ec.fuse_splitk, w4x_panels=ec.w4x_panels, gate_up_panels=ec.gate_up_panels)
+
     def __init__(self, cfg: LlamaConfig, device="cuda", backend: str = "kgs", seed: int = 0,
                  num_pages: int = 1024, max_model_len: int = 8192, fused_max_batch: int = 48,
                  decode_weights: str = "bf16", kv_cache_dtype: str = "bf16", packed_decode: bool = True,

@@ -61,6 +61,10 @@ HIPCC = str(ROCM / "bin" / "hipcc")
 MANIFEST = "build_manifest.json"
 CXX = os.environ.get("CXX", "g++")
 
+# packed fp32 VALU instructions stay out of all device code (hipcc's host pass
+# reports that it does not know the feature; harmless)
+NO_PACKED_F32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
+
 HIP_FLAGS = [
     f"--offload-arch={ARCH}",
     "-O3",
@@ -70,6 +74,7 @@ HIP_FLAGS = [
     "-Wno-unused-function",
     "-Wno-unused-variable",
     "-munsafe-fp-atomics",
+    *NO_PACKED_F32,
 ]
 
 
@@ -162,7 +167,7 @@ def targets(out: Path | None = None) -> list[Target]:
             odir / "kgs-gpuprobe",
             [NATIVE / "probe" / "gpuprobe.hip"],
             HIPCC,
-            flags=[f"--offload-arch={ARCH}", "-O2", "-std=c++17", "-Wall"],
+            flags=[f"--offload-arch={ARCH}", "-O2", "-std=c++17", "-Wall", *NO_PACKED_F32],
             link_flags=[f"-L{odir}", "-lkgs_kernels", "-Wl,-rpath,$ORIGIN", "-pthread"],
             shared=False,
         ),
@@ -171,7 +176,7 @@ def targets(out: Path | None = None) -> list[Target]:
             odir / "kgs-graph-memset-repro",
             [NATIVE / "probe" / "graph_memset_repro.hip"],
             HIPCC,
-            flags=[f"--offload-arch={ARCH}", "-O2", "-std=c++17", "-Wall"],
+            flags=[f"--offload-arch={ARCH}", "-O2", "-std=c++17", "-Wall", *NO_PACKED_F32],
             link_flags=[],
             shared=False,
         ),
@@ -232,7 +237,7 @@ def targets(out: Path | None = None) -> list[Target]:
             odir / "kgs-rccl-bench",
             [rdir / "rccl_bench.cpp"],
             HIPCC,
-            flags=[f"--offload-arch={ARCH}", "-O2", "-std=c++17", f"-I{ROCM / 'include'}"],
+            flags=[f"--offload-arch={ARCH}", "-O2", "-std=c++17", f"-I{ROCM / 'include'}", *NO_PACKED_F32],
             link_flags=[f"-L{ROCM / 'lib'}", "-lrccl", f"-Wl,-rpath,{ROCM / 'lib'}"],
             shared=False,
             optional=True,

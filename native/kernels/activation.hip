@@ -1,0 +1,85 @@
+// Elementwise steps around the projections, for any width and for bf16 or fp32
+// activations: the gated feed-forward product act(gate) * up from one fused
+// gate|up row, and the tanh soft cap of the logits.
+#include "kgs_common.h"
+
+namespace kgs {
+namespace act {
+
+enum { ACT_SILU = 0, ACT_GELU_TANH = 1 };
+
+template <int ACT>
+__device__ __forceinline__ float f(float z) {
+  if constexpr (ACT == ACT_SILU) return z / (1.0f + expf(-z));
+  return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+}
+
+template <int ACT>
+__global__ __launch_bounds__(256) void mul_f32(const float* gu, float* o, int n, long ldi, long ldo) {
+  const long r = blockIdx.y;
+  const int c = blockIdx.x * 256 + threadIdx.x;
+  if (c < n) o[r * ldo + c] = f<ACT>(gu[r * ldi + c]) * gu[r * ldi + n + c];
+}
+
+// 8 columns per thread (n % 8 == 0, 16-B rows)
+template <int ACT>
+__global__ __launch_bounds__(256) void mul_bf16(const unsigned short* gu, unsigned short* o, int n, long ldi, long ldo) {
+  const long r = blockIdx.y;
+  const int c = (blockIdx.x * 256 + threadIdx.x) * 8;
+  if (c >= n) return;
+  const bf16x8 g = *(const bf16x8*)(gu + r * ldi + c), u = *(const bf16x8*)(gu + r * ldi + n + c);
+  float v[8];
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    const float z = bf2f((unsigned short)g[i]);
+    v[i] = (ACT == ACT_GELU_TANH ? gelu_tanh(z) : f<ACT>(z)) * bf2f((unsigned short)u[i]);
+  }
+  *(bf16x8*)(o + r * ldo + c) = pack_bf16x8(v, 0);
+}
+
+// logits [rows, ld] -> fp32 [rows, n]: cap * tanh(x / cap), or x with cap 0
+template <typename T>
+__global__ __launch_bounds__(256) void softcap(const T* x, float* o, int n, long ld, float cap) {
+  const long r = blockIdx.y;
+  const int c = blockIdx.x * 256 + threadIdx.x;
+  if (c >= n) return;
+  float v;
+  if constexpr (sizeof(T) == 2) v = bf2f(x[r * ld + c]);
+  else v = x[r * ld + c];
+  o[r * n + c] = cap > 0.f ? cap * tanhf(v / cap) : v;
+}
+
+}  // namespace act
+}  // namespace kgs
+
+KGS_EXPORT int kgs_act_mul(const void* gu, void* o, int rows, int n, long ldi, long ldo, int act, int f32,
+                           hipStream_t s) {
+  using namespace kgs::act;
+  if (rows <= 0 || rows > 65535 * 16 || n <= 0 || ldi < 2l * n || ldo < n) return KGS_ERR_SHAPE;
+  if (act != ACT_SILU && act != ACT_GELU_TANH) return KGS_ERR_ARG;
+  if (!f32 && (n % 8 || ldi % 8 || ldo % 8 || (((uintptr_t)gu | (uintptr_t)o) & 15))) return KGS_ERR_ALIGN;
+  const long per = 65535;
+  for (long r0 = 0; r0 < rows; r0 += per) {
+    const unsigned nr = (unsigned)(rows - r0 < per ? rows - r0 : per);
+    if (f32) {
+      auto k = act == ACT_SILU ? mul_f32<ACT_SILU> : mul_f32<ACT_GELU_TANH>;
+      hipLaunchKernelGGL(k, dim3((n + 255) / 256, nr), dim3(256), 0, s, (const float*)gu + r0 * ldi,
+                         (float*)o + r0 * ldo, n, ldi, ldo);
+    } else {
+      auto k = act == ACT_SILU ? mul_bf16<ACT_SILU> : mul_bf16<ACT_GELU_TANH>;
+      hipLaunchKernelGGL(k, dim3((n / 8 + 255) / 256, nr), dim3(256), 0, s, (const unsigned short*)gu + r0 * ldi,
+                         (unsigned short*)o + r0 * ldo, n, ldi, ldo);
+    }
+  }
+  return (int)hipGetLastError();
+}
+
+KGS_EXPORT int kgs_softcap(const void* x, void* o, int rows, int n, long ld, float cap, int f32, hipStream_t s) {
+  using namespace kgs::act;
+  if (rows <= 0 || rows > 65535 || n <= 0 || ld < n) return KGS_ERR_SHAPE;
+  const dim3 grid((n + 255) / 256, rows);
+  if (f32) hipLaunchKernelGGL(softcap<float>, grid, dim3(256), 0, s, (const float*)x, (float*)o, n, ld, cap);
+  else hipLaunchKernelGGL(softcap<unsigned short>, grid, dim3(256), 0, s, (const unsigned short*)x, (float*)o, n, ld,
+                          cap);
+  return (int)hipGetLastError();
+}

@@ -1,6 +1,8 @@
 // Flash-attention forward for gfx950 (bf16 in/out, fp32 softmax/accumulate),
 // head_dim 128, causal or full, GQA -- the prefill attention of the Llama
-// stand-in (kgs/models/llama.py). Q, K and V are read in place from the fused
+// stand-in (kgs/models/llama.py); and its ragged form (head_dim 64 or 128, prompt
+// portions of any length at any position, an optional per-head output gate) for
+// latent attention over expanded keys and values. Q, K and V are read in place from the fused
 // QKV projection output ([tokens, (H + 2 HKV) * 128], any row stride) and O is
 // written as [tokens, H * 128], the layout the O projection consumes: no
 // transposes around the kernel.
@@ -33,12 +35,9 @@ namespace kgs {
 namespace attn {
 
 typedef float f32x16 __attribute__((ext_vector_type(16)));
-typedef short bf16x4s __attribute__((ext_vector_type(4)));
 
-constexpr int HD = 128;
 constexpr int QB = 128;  // query rows per workgroup (4 waves x 32)
 constexpr int KB = 64;   // keys per tile
-constexpr int TILE_BYTES = KB * HD * 2;  // 16 KB
 constexpr float NEG = -1.0e30f;
 constexpr float RESCALE = 8.0f;  // deferred-max threshold, log2 units: P <= 256
 
@@ -53,52 +52,82 @@ struct Args {
   int causal;
   int Sk;    // keys per sequence (= S, or S + qoff for a chunk over a cached context)
   int qoff;  // position of query row 0 among the keys: causal row i sees keys <= qoff + i
+  // ragged form: one int4 per (sequence, q-block) -- first query row, first key
+  // row of the sequence, position of the first query row, valid query rows
+  const int4* items;
+  const unsigned short* gate;  // or null: [rows, ldg], head h's output times sigmoid(gate[row][h])
+  long ldg;
 };
 
-__device__ __forceinline__ int swz(int r) { return ((r & 3) << 2) | ((r >> 2) & 3); }
-__device__ __forceinline__ int off(int r, int c) { return 256 * r + 16 * (c ^ swz(r)); }
-
-__device__ __forceinline__ bf16x8 tr_frag(const char* lo, const char* hi) {
-  const bf16x4s a = __builtin_amdgcn_ds_read_tr16_b64_v4i16((KGS_LDS bf16x4s*)lo);
-  const bf16x4s b = __builtin_amdgcn_ds_read_tr16_b64_v4i16((KGS_LDS bf16x4s*)hi);
-  return __builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7);
+// XOR image of a row's 16-B chunks (HD / 8 of them)
+template <int HD>
+__device__ __forceinline__ int swz(int r) {
+  if constexpr (HD == 128) return ((r & 3) << 2) | ((r >> 2) & 3);
+  return ((r & 2) << 1) | ((r >> 2) & 3);
 }
+template <int HD>
+__device__ __forceinline__ int off(int r, int c) { return 2 * HD * r + 16 * (c ^ swz<HD>(r)); }
 
 __device__ __forceinline__ bf16x8 pack8(const f32x16& s, int base) { return pack_bf16x8(s, base); }
 
+// RAGGED: any number of query rows per sequence at any position (Args::items),
+// rows and keys past a block's end clamped on load and dropped on store; always
+// causal. Otherwise B equal sequences of S rows, a multiple of QB.
+template <int HD, bool RAGGED>
 __global__ __launch_bounds__(256, 2) __attribute__((amdgpu_waves_per_eu(2, 2))) void fwd(Args a) {
+  constexpr int TILE_BYTES = KB * HD * 2;  // 16 KB at 128
+  constexpr int ND = HD / 32, NK = HD / 16;
   __shared__ __attribute__((aligned(16))) char smem[2][2][TILE_BYTES];  // [buf][K, V]
 
   const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int l32 = lane & 31, hh = lane >> 5;
-  const int nqb = a.S / QB;
-  const int nwg = gridDim.x;
-  // XCD-aware order: 8 consecutive dispatch slots of one XCD take 4 heads of
-  // one KV group; work ids stay heaviest-first in dispatch time.
-  int lid = blockIdx.x;
-  if ((nwg & 31) == 0) {
-    const int t = lid >> 3, x = lid & 7;
-    lid = ((t >> 2) << 5) | (x << 2) | (t & 3);
-  }
-  const int per = a.B * a.H;
-  const int qi = lid / per, rem = lid - qi * per;
-  const int qb = a.causal ? nqb - 1 - qi : qi;
-  const int b = rem / a.H, h = rem - b * a.H;
-  const int kvh = h / (a.H / a.HKV);
+  int h, kvh, q0, qw, qrow, qoff, nval = QB;
+  long tok0, ktok0;
+  bool causal = true;
+  if constexpr (RAGGED) {
+    const int item = blockIdx.x / a.H;
+    h = kvh = blockIdx.x - item * a.H;
+    const int4 it = a.items[item];
+    tok0 = it.x;
+    ktok0 = it.y;
+    qoff = it.z;
+    nval = it.w;
+    q0 = 0;
+    qw = 32 * w;
+    qrow = qw + l32;
+  } else {
+    const int nqb = a.S / QB;
+    const int nwg = gridDim.x;
+    // XCD-aware order: 8 consecutive dispatch slots of one XCD take 4 heads of
+    // one KV group; work ids stay heaviest-first in dispatch time.
+    int lid = blockIdx.x;
+    if ((nwg & 31) == 0) {
+      const int t = lid >> 3, x = lid & 7;
+      lid = ((t >> 2) << 5) | (x << 2) | (t & 3);
+    }
+    const int per = a.B * a.H;
+    const int qi = lid / per, rem = lid - qi * per;
+    const int qb = a.causal ? nqb - 1 - qi : qi;
+    const int b = rem / a.H;
+    h = rem - b * a.H;
+    kvh = h / (a.H / a.HKV);
 
-  const int q0 = qb * QB;
-  const int qw = q0 + 32 * w;       // this wave's first query row
-  const int qrow = qw + l32;        // this lane's query row
-  const long tok0 = (long)b * a.S;     // first query token of the sequence
-  const long ktok0 = (long)b * a.Sk;   // its first key token
-  const int qoff = a.qoff;
+    q0 = qb * QB;
+    qw = q0 + 32 * w;       // this wave's first query row
+    qrow = qw + l32;        // this lane's query row
+    tok0 = (long)b * a.S;     // first query token of the sequence
+    ktok0 = (long)b * a.Sk;   // its first key token
+    qoff = a.qoff;
+    causal = a.causal != 0;
+  }
+  const int lrow = RAGGED ? min(qrow, nval - 1) : qrow;  // the row this lane loads
 
   // Q fragments (B operand of S^T = K.Q^T): lane holds Q[qrow][16ks + 8hh .. +7]
-  bf16x8 qf[8];
+  bf16x8 qf[NK];
   {
-    const bf16x8* qp = (const bf16x8*)(a.q + (tok0 + qrow) * a.ldq + (long)h * HD + 8 * hh);
+    const bf16x8* qp = (const bf16x8*)(a.q + (tok0 + lrow) * a.ldq + (long)h * HD + 8 * hh);
 #pragma unroll
-    for (int ks = 0; ks < 8; ++ks) qf[ks] = qp[2 * ks];
+    for (int ks = 0; ks < NK; ++ks) qf[ks] = qp[2 * ks];
   }
 
   const unsigned short* kbase = a.k + ktok0 * a.ldk + (long)kvh * HD;
@@ -109,25 +138,26 @@ __global__ __launch_bounds__(256, 2) __attribute__((amdgpu_waves_per_eu(2, 2))) 
   // at slot (r, c') of the XOR image, so it fetches column c = c' ^ swz(r).
   auto dma_tiles = [&](int jn, int sb) {
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int ch = 4 * w + i;
-      const int r = 4 * ch + (lane >> 4), c = (lane & 15) ^ swz(r);
-      const long row = (long)jn * KB + r;
+    for (int i = 0; i < ND; ++i) {
+      const int ch = ND * w + i;
+      const int r = (512 / HD) * ch + lane / (HD / 8), c = (lane & (HD / 8 - 1)) ^ swz<HD>(r);
+      long row = (long)jn * KB + r;
+      if constexpr (RAGGED) row = min(row, (long)(qoff + nval - 1));
       glds16(kbase + row * a.ldk + 8 * c, smem[sb][0] + 1024 * ch);
       glds16(vbase + row * a.ldv + 8 * c, smem[sb][1] + 1024 * ch);
     }
   };
 
-  const int ntile = a.causal ? (qoff + q0 + QB) / KB : a.Sk / KB;
+  const int ntile = RAGGED ? (qoff + nval - 1) / KB + 1 : causal ? (qoff + q0 + QB) / KB : a.Sk / KB;
   dma_tiles(0, 0);
   // Q fragments and tile 0 complete before the loop (a vmcnt the waitcnt pass
   // sees, so it does not carry the Q loads into the loop header)
   __builtin_amdgcn_s_waitcnt(0x0f70);  // vmcnt(0)
   __syncthreads();
 
-  f32x16 o[4];
+  f32x16 o[ND];
 #pragma unroll
-  for (int d = 0; d < 4; ++d) o[d] = f32x16{};
+  for (int d = 0; d < ND; ++d) o[d] = f32x16{};
   float m = NEG, l = 0.f;
   const float sl2 = a.sl2;
 
@@ -139,28 +169,28 @@ __global__ __launch_bounds__(256, 2) __attribute__((amdgpu_waves_per_eu(2, 2))) 
     // the other buffer was released by the previous tile's barrier
     if (j + 1 < ntile) dma_tiles(j + 1, buf ^ 1);
     const int kv0 = j * KB;
-    if (!a.causal || kv0 <= qoff + qw + 31) {
+    if (!causal || kv0 <= qoff + qw + 31) {
       const char* Ks = smem[buf][0];
       const char* Vs = smem[buf][1];
       // all 16 K fragments of the tile are read up front (the registers the
       // LDS-DMA staging freed), so the QK^T MFMAs never wait on one LDS read
-      bf16x8 kf[2][8];
+      bf16x8 kf[2][NK];
 #pragma unroll
       for (int t = 0; t < 2; ++t)
 #pragma unroll
-        for (int ks = 0; ks < 8; ++ks) kf[t][ks] = *(const bf16x8*)(Ks + off(32 * t + l32, 2 * ks + hh));
+        for (int ks = 0; ks < NK; ++ks) kf[t][ks] = *(const bf16x8*)(Ks + off<HD>(32 * t + l32, 2 * ks + hh));
       __builtin_amdgcn_sched_barrier(0);  // keep the reads ahead (the scheduler sinks them otherwise)
       f32x16 s[2];
 #pragma unroll
       for (int t = 0; t < 2; ++t) {
         s[t] = f32x16{};
 #pragma unroll
-        for (int ks = 0; ks < 8; ++ks) s[t] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf[t][ks], qf[ks], s[t], 0, 0, 0);
+        for (int ks = 0; ks < NK; ++ks) s[t] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf[t][ks], qf[ks], s[t], 0, 0, 0);
       }
       // the first half of the tile's V fragments is read now, so its LDS
       // latency hides under the softmax below (all 16 would spill at 2 waves
       // per SIMD); the second half is read under the first half's P.V MFMAs
-      bf16x8 vfr[4][2][2];
+      bf16x8 vfr[ND][2][2];
       auto read_v = [&](int d) {
         const int c0 = 4 * d + 2 * (g & 1) + (tp >> 1);
 #pragma unroll
@@ -168,13 +198,13 @@ __global__ __launch_bounds__(256, 2) __attribute__((amdgpu_waves_per_eu(2, 2))) 
 #pragma unroll
           for (int sp = 0; sp < 2; ++sp) {
             const int kvb = 32 * t + 16 * sp + 4 * hh + tq;
-            vfr[d][t][sp] = tr_frag(Vs + off(kvb, c0) + 8 * (tp & 1), Vs + off(kvb + 8, c0) + 8 * (tp & 1));
+            vfr[d][t][sp] = tr_frag(Vs + off<HD>(kvb, c0) + 8 * (tp & 1), Vs + off<HD>(kvb + 8, c0) + 8 * (tp & 1));
           }
       };
       read_v(0);
       read_v(1);
       __builtin_amdgcn_sched_barrier(0);
-      if (a.causal && kv0 + KB - 1 > qoff + qw) {
+      if (causal && kv0 + KB - 1 > qoff + qw) {
 #pragma unroll
         for (int t = 0; t < 2; ++t)
 #pragma unroll
@@ -201,7 +231,7 @@ __global__ __launch_bounds__(256, 2) __attribute__((amdgpu_waves_per_eu(2, 2))) 
         m = mn;
         l *= alpha;
 #pragma unroll
-        for (int d = 0; d < 4; ++d) o[d] *= alpha;
+        for (int d = 0; d < ND; ++d) o[d] *= alpha;
       }
       const float msl = m * sl2;
 #pragma unroll
@@ -218,10 +248,12 @@ __global__ __launch_bounds__(256, 2) __attribute__((amdgpu_waves_per_eu(2, 2))) 
         pf[t][0] = pack8(s[t], 0);
         pf[t][1] = pack8(s[t], 8);
       }
-      read_v(2);
-      read_v(3);
+      if constexpr (ND == 4) {
+        read_v(2);
+        read_v(3);
+      }
 #pragma unroll
-      for (int d = 0; d < 4; ++d)
+      for (int d = 0; d < ND; ++d)
 #pragma unroll
         for (int t = 0; t < 2; ++t)
 #pragma unroll
@@ -233,10 +265,14 @@ __global__ __launch_bounds__(256, 2) __attribute__((amdgpu_waves_per_eu(2, 2))) 
   }
 
   l = xor32_sum(l);
-  const float inv = 1.0f / l;
+  float inv = 1.0f / l;
+  if constexpr (RAGGED) {
+    if (qrow >= nval) return;
+    if (a.gate) inv /= 1.0f + __expf(-bf2f(a.gate[(tok0 + qrow) * a.ldg + h]));
+  }
   unsigned short* op = a.o + (tok0 + qrow) * a.ldo + (long)h * HD;
 #pragma unroll
-  for (int d = 0; d < 4; ++d)
+  for (int d = 0; d < ND; ++d)
 #pragma unroll
     for (int r4 = 0; r4 < 4; ++r4) {
       const int dcol = 32 * d + 8 * r4 + 4 * hh;
@@ -261,6 +297,7 @@ KGS_EXPORT int kgs_attn_fwd_bf16_ex(const void* q, const void* k, const void* v,
                                    int HKV, int hd, long ldq, long ldk, long ldv, long ldo, float scale, int causal,
                                    hipStream_t s) {
   using namespace kgs::attn;
+  constexpr int HD = 128;
   if (B <= 0 || S <= 0 || H <= 0 || HKV <= 0 || H % HKV) return KGS_ERR_SHAPE;
   if (hd != HD || S % QB || Sk < S || (Sk - S) % KB) return KGS_ERR_SHAPE;
   if (ldq < (long)H * HD || ldk < (long)HKV * HD || ldv < (long)HKV * HD || ldo < (long)H * HD) return KGS_ERR_SHAPE;
@@ -269,8 +306,9 @@ KGS_EXPORT int kgs_attn_fwd_bf16_ex(const void* q, const void* k, const void* v,
   const long nwg = (long)B * H * (S / QB);
   if (nwg > 0x7fffffff) return KGS_ERR_SHAPE;
   Args a{(const unsigned short*)q, (const unsigned short*)k, (const unsigned short*)v, (unsigned short*)o,
-         ldq, ldk, ldv, ldo, B, S, H, HKV, scale * 1.4426950408889634f, causal ? 1 : 0, Sk, Sk - S};
-  hipLaunchKernelGGL(fwd, dim3((unsigned)nwg), dim3(256), 0, s, a);
+         ldq, ldk, ldv, ldo, B, S, H, HKV, scale * 1.4426950408889634f, causal ? 1 : 0, Sk, Sk - S,
+         nullptr, nullptr, 0};
+  hipLaunchKernelGGL((fwd<HD, false>), dim3((unsigned)nwg), dim3(256), 0, s, a);
   return (int)hipGetLastError();
 }
 
@@ -278,4 +316,28 @@ KGS_EXPORT int kgs_attn_fwd_bf16(const void* q, const void* k, const void* v, vo
                                 int hd, long ldq, long ldk, long ldv, long ldo, float scale, int causal,
                                 hipStream_t s) {
   return kgs_attn_fwd_bf16_ex(q, k, v, o, B, S, S, H, HKV, hd, ldq, ldk, ldv, ldo, scale, causal, s);
+}
+
+// Causal attention of ragged sequences, head_dim 64 or 128, as many key heads as
+// query heads. items: nitems int4 (first query row, first key row of its
+// sequence, position of that query row, rows <= 128), any order (heaviest first
+// keeps the tail short). Every row index an item names must lie in q / o, every
+// key row first_key + position in k / v.
+KGS_EXPORT int kgs_attn_fwd_ragged_bf16(const void* q, const void* k, const void* v, void* o, const void* items,
+                                       int nitems, int H, int hd, long ldq, long ldk, long ldv, long ldo, float scale,
+                                       const void* gate, long ldg, hipStream_t s) {
+  using namespace kgs::attn;
+  if (nitems <= 0 || H <= 0 || (hd != 64 && hd != 128)) return KGS_ERR_SHAPE;
+  const long w = (long)H * hd;
+  if (ldq < w || ldk < w || ldv < w || ldo < w || (gate && ldg < H)) return KGS_ERR_SHAPE;
+  const uintptr_t al = (uintptr_t)q | (uintptr_t)k | (uintptr_t)v | (uintptr_t)o | (uintptr_t)items;
+  if ((al & 15) || (ldq | ldk | ldv | ldo) & 7) return KGS_ERR_ALIGN;
+  if ((long)nitems * H > 0x7fffffff) return KGS_ERR_SHAPE;
+  Args a{(const unsigned short*)q, (const unsigned short*)k, (const unsigned short*)v, (unsigned short*)o,
+         ldq, ldk, ldv, ldo, 0, 0, H, H, scale * 1.4426950408889634f, 1, 0, 0,
+         (const int4*)items, (const unsigned short*)gate, ldg};
+  const dim3 grid((unsigned)(nitems * H));
+  if (hd == 128) hipLaunchKernelGGL((fwd<128, true>), grid, dim3(256), 0, s, a);
+  else hipLaunchKernelGGL((fwd<64, true>), grid, dim3(256), 0, s, a);
+  return (int)hipGetLastError();
 }

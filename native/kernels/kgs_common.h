@@ -118,6 +118,15 @@ __device__ __forceinline__ void glds16(const void* gsrc, void* lds_base) {
   __builtin_amdgcn_global_load_lds((KGS_GLB void*)gsrc, (KGS_LDS void*)lds_base, 16, 0, 0);
 }
 
+// Transposed LDS read: each 16-lane group reads a 4 x 16 block of 16-bit elements
+// (lane 4q + p: row q, columns 4p .. 4p+3) and lane i gets column i's 4 rows;
+// two such reads are one 8-element MFMA fragment.
+__device__ __forceinline__ bf16x8 tr_frag(const char* lo, const char* hi) {
+  const bf16x4 a = __builtin_amdgcn_ds_read_tr16_b64_v4i16((KGS_LDS bf16x4*)lo);
+  const bf16x4 b = __builtin_amdgcn_ds_read_tr16_b64_v4i16((KGS_LDS bf16x4*)hi);
+  return __builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7);
+}
+
 // Bijective XCD-aware remap of a 1-D grid: blocks that the dispatcher deals to
 // the same XCD (bid % 8 equal) get a contiguous range of logical ids, so
 // neighbouring output tiles share that XCD's L2 (guide T1).

@@ -1,0 +1,515 @@
+// Latent attention: a token's keys and values of every head are linear maps of
+// one small vector c (the latent), and only c is cached, in pages
+// [page][32 tokens][RP] (RP: the latent size padded to a kernel size, pad zero).
+//
+// The absorbed form needs no expanded keys or values: with
+//   qlat_h = W_uk,h^T q_h        score_j = (qlat_h . c_j) * scale
+//   olat_h = sum_j p_j c_j       o_h     = W_uv,h olat_h
+// attention is multi-query over c itself, every head (and every query token of a
+// prompt portion) a row over the same keys. Kernels:
+//   * latent_norm   the RMS norms of both latents of a token's fused input
+//                   projection; c goes straight into its cache slot;
+//   * head_proj     the per-head products (W_uk^T q, W_uv olat), the latter with
+//                   the per-head sigmoid output gate in its store;
+//   * attn          rows x pages on v_mfma_f32_16x16x32_bf16, split over the
+//                   context, + merge;
+//   * attn_simple   the same on the VALU for any RP and for fp32 caches.
+#include "kgs_common.h"
+
+namespace kgs {
+namespace latent {
+
+constexpr int PAGE = 32;
+constexpr float NEG = -1.0e30f;
+constexpr float RESCALE = 8.0f;  // deferred-max threshold, log2 units
+
+template <typename T>
+__device__ __forceinline__ float ld(const T* p) {
+  if constexpr (sizeof(T) == 2) return bf2f(*(const unsigned short*)p);
+  else return *p;
+}
+template <typename T>
+__device__ __forceinline__ void st(T* p, float v) {
+  if constexpr (sizeof(T) == 2) *(unsigned short*)p = f2bf(v);
+  else *p = v;
+}
+
+__device__ __forceinline__ float wave_sum(float v) {
+#pragma unroll
+  for (int m = 8; m >= 1; m >>= 1) v += __shfl_xor(v, m, 64);
+  return xor32_sum(xor16_sum(v));
+}
+__device__ __forceinline__ float wave_max(float v) {
+#pragma unroll
+  for (int m = 8; m >= 1; m >>= 1) v = fmaxf(v, __shfl_xor(v, m, 64));
+  return xor32_max(xor16_max(v));
+}
+__device__ __forceinline__ float sigmoid(float x) { return 1.0f / (1.0f + expf(-x)); }
+
+// ---------------------------------------------------------------- latent_norm
+struct NormArgs {
+  const void* z;  // [T, ldz] fused input projection
+  long ldz;
+  int oq, nq, qp;  // query latent: first column, size, padded size of cq
+  int oc, nc, rp;  // key/value latent (nc 0: the layer has none of its own)
+  const float *wq, *wc;
+  void* cq;              // [T, qp]
+  void* cache;           // this layer's pages
+  const int* slots;      // [T], -1: not cached
+  float eps;
+};
+
+// one workgroup per token: wave 0 the query latent, wave 1 the cached one
+template <typename T>
+__global__ __launch_bounds__(128) void norm(NormArgs a) {
+  const int lane = threadIdx.x & 63;
+  const long t = blockIdx.x;
+  const bool second = threadIdx.x >= 64;
+  const int n = second ? a.nc : a.nq, np = second ? a.rp : a.qp;
+  if (n == 0) return;
+  const int slot = second ? a.slots[t] : 0;
+  if (slot < 0) return;
+  const T* z = (const T*)a.z + t * a.ldz + (second ? a.oc : a.oq);
+  const float* w = second ? a.wc : a.wq;
+  T* out = second ? (T*)a.cache + (long)slot * a.rp : (T*)a.cq + t * a.qp;
+  float ss = 0.f;
+  for (int i = lane; i < n; i += 64) {
+    const float v = ld(z + i);
+    ss += v * v;
+  }
+  const float r = 1.0f / sqrtf(wave_sum(ss) / n + a.eps);
+  for (int i = lane; i < np; i += 64) st(out + i, i < n ? ld(z + i) * r * w[i] : 0.f);
+}
+
+// ------------------------------------------------------------------ head_proj
+struct ProjArgs {
+  const void* a;     // input row of token i, head h: a + in_row(i) * lda + h * ha
+  const void* w;     // [H][N][K]
+  void* out;         // out + out_row(i) * ldo + h * ho
+  const int *idx_in, *idx_out;  // token i's row, or null (i)
+  const void* gate;  // [rows, ldg] per output row, head h at column h; or null
+  long lda, ha, ldo, ho, ldg;
+  int Nt, H, N, K;
+};
+
+// D^T[n][token] = W[n][k] a^T[k][token]; wave: 16 outputs x 16 TT tokens of one head
+template <int TT>
+__global__ __launch_bounds__(256) void head_proj(ProjArgs p) {
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
+  const int l16 = lane & 15, g = lane >> 4;
+  const int nt = blockIdx.x * 4 + w, h = blockIdx.z, t0 = blockIdx.y * 16 * TT;
+  if (nt * 16 >= p.N) return;
+  const unsigned short* wp = (const unsigned short*)p.w + ((long)h * p.N + nt * 16 + l16) * p.K + 8 * g;
+  const unsigned short* ap[TT];
+#pragma unroll
+  for (int i = 0; i < TT; ++i) {
+    int t = t0 + 16 * i + l16;
+    t = t < p.Nt ? t : p.Nt - 1;
+    const long r = p.idx_in ? p.idx_in[t] : t;
+    ap[i] = (const unsigned short*)p.a + r * p.lda + h * p.ha + 8 * g;
+  }
+  f32x4 acc[TT];
+#pragma unroll
+  for (int i = 0; i < TT; ++i) acc[i] = f32x4{};
+#pragma unroll 4
+  for (int k = 0; k < p.K; k += 32) {
+    const bf16x8 wf = *(const bf16x8*)(wp + k);
+#pragma unroll
+    for (int i = 0; i < TT; ++i)
+      acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, *(const bf16x8*)(ap[i] + k), acc[i], 0, 0, 0);
+  }
+#pragma unroll
+  for (int i = 0; i < TT; ++i) {
+    const int t = t0 + 16 * i + l16;
+    if (t >= p.Nt) continue;
+    const long r = p.idx_out ? p.idx_out[t] : t;
+    const float s = p.gate ? sigmoid(bf2f(((const unsigned short*)p.gate)[r * p.ldg + h])) : 1.0f;
+    uint2 o;
+    o.x = pack_bf16x2(acc[i][0] * s, acc[i][1] * s);
+    o.y = pack_bf16x2(acc[i][2] * s, acc[i][3] * s);
+    *(uint2*)((unsigned short*)p.out + r * p.ldo + h * p.ho + nt * 16 + 4 * g) = o;
+  }
+}
+
+__global__ __launch_bounds__(256) void head_proj_f32(ProjArgs p) {
+  const int i = blockIdx.x, h = blockIdx.y;
+  const long ri = p.idx_in ? p.idx_in[i] : i, ro = p.idx_out ? p.idx_out[i] : i;
+  const float* a = (const float*)p.a + ri * p.lda + h * p.ha;
+  float* o = (float*)p.out + ro * p.ldo + h * p.ho;
+  const float s = p.gate ? sigmoid(((const float*)p.gate)[ro * p.ldg + h]) : 1.0f;
+  for (int n = threadIdx.x; n < p.N; n += 256) {
+    const float* w = (const float*)p.w + ((long)h * p.N + n) * p.K;
+    float acc = 0.f;
+    for (int k = 0; k < p.K; ++k) acc = __builtin_fmaf(a[k], w[k], acc);
+    o[n] = acc * s;
+  }
+}
+
+// ----------------------------------------------------------------------- attn
+// Query tokens of the call are numbered 0 .. Nt - 1; sequence b holds tokens
+// q0[b] .. q0[b] + n[b] - 1 at positions pos0[b] .. , its pages in bt[b].
+struct Args {
+  const void* q;      // [Nt * H, RP]
+  const void* cache;  // [pages][32][RP]
+  void* o;            // [Nt * H, RP]
+  float* part_o;      // [nsplit][Nt * H][RP]
+  float* part_ml;     // [nsplit][Nt * H][2]
+  const int *q0, *n, *pos0, *bt;
+  const int* items;   // (sequence, tile) pairs, or null: blockIdx.x = b * tiles + tile
+  const int *tok_seq, *tok_pos;  // attn_simple
+  int H, W, tiles, nsplit, Nt, RP;
+  float scale, sl2;  // sl2 = scale * log2(e)
+};
+
+template <int RT>
+struct Geo {
+  static constexpr int RP = 32 * RT, CH = 4 * RT, PITCH = 64 * RT, PAGEB = PAGE * PITCH;
+  static constexpr int LOW = CH & -CH, P = LOW > 16 ? 16 : LOW;
+  // XOR of a row's 16-B chunk index: rows that share banks land on other chunks
+  __device__ static __forceinline__ int swz(int r) {
+    if constexpr (P == 16) return ((r & 3) << 2) | ((r >> 1) & 2) | ((r >> 3) & 1);
+    else if constexpr (P == 8) return (r >> 1) & 7;
+    else return (r >> 2) & 3;
+  }
+  __device__ static __forceinline__ int off(int r, int c) { return PITCH * r + 16 * (c ^ swz(r)); }
+};
+
+// Workgroup: 16 rows per wave of one sequence's (token, head) rows, head fastest,
+// over the pages of one context split. S^T = C Q^T, so a lane owns row
+// (lane & 15) and keys 16 t + 4 (lane >> 4) + r of a page; the same registers
+// are the B operand of O^T = C^T P^T, whose A operand is the page read
+// transposed (ds_read_b64_tr_b16) in that key order.
+template <int RT>
+__global__ __launch_bounds__(512) void attn(Args a) {
+  using G = Geo<RT>;
+  extern __shared__ __attribute__((aligned(16))) char smem[];  // two pages
+  const int lane = threadIdx.x & 63, nw = blockDim.x >> 6;
+  const int w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int l16 = lane & 15, g = lane >> 4, tq = (lane >> 2) & 3, tp = lane & 3;
+  int b, tile;
+  if (a.items) {
+    b = a.items[2 * blockIdx.x];
+    tile = a.items[2 * blockIdx.x + 1];
+  } else {
+    b = blockIdx.x / a.tiles;
+    tile = blockIdx.x - b * a.tiles;
+  }
+  const int rows = a.n[b] * a.H, pos0 = a.pos0[b];
+  const long base = (long)a.q0[b] * a.H;  // row 0 of the sequence
+  const int r0 = tile * 16 * nw;          // the workgroup's rows
+  if (r0 >= rows) return;
+  const int last = min(r0 + 16 * nw, rows) - 1;
+  const int myrow = r0 + 16 * w + l16;
+  const int row = min(myrow, last);
+  const int pos = pos0 + row / a.H;
+  const int wmax = pos0 + min(r0 + 16 * w + 15, last) / a.H;  // this wave's last position
+  const int npages = (pos0 + last / a.H) / PAGE + 1;
+  const int pps = (npages + a.nsplit - 1) / a.nsplit;
+  const int p0 = blockIdx.y * pps, p1 = min(p0 + pps, npages);
+  const int* bt = a.bt + (long)b * a.W;
+  const unsigned short* cache = (const unsigned short*)a.cache;
+  const long nrows = (long)a.Nt * a.H;
+
+  if (p0 >= p1) {  // an empty split: only reachable with nsplit > 1
+    if (myrow <= last && g == 0) {
+      float* ml = a.part_ml + 2 * (blockIdx.y * nrows + base + myrow);
+      ml[0] = NEG;
+      ml[1] = 0.f;
+    }
+    return;
+  }
+
+  auto dma = [&](int page, int buf) {
+    const unsigned short* src = cache + (long)page * PAGE * G::RP;
+    for (int i = w; i < 2 * RT; i += nw) {
+      const int L = 64 * i + lane, r = L / G::CH, c = (L % G::CH) ^ G::swz(r);
+      glds16(src + r * G::RP + 8 * c, smem + buf * G::PAGEB + 1024 * i);
+    }
+  };
+
+  bf16x8 qf[RT];
+  {
+    const bf16x8* qp = (const bf16x8*)((const unsigned short*)a.q + (base + row) * G::RP + 8 * g);
+#pragma unroll
+    for (int k = 0; k < RT; ++k) qf[k] = qp[4 * k];
+  }
+  dma(bt[p0], 0);
+  __builtin_amdgcn_s_waitcnt(0x0f70);  // vmcnt(0)
+  __syncthreads();
+
+  f32x4 acc[2 * RT];
+#pragma unroll
+  for (int i = 0; i < 2 * RT; ++i) acc[i] = f32x4{};
+  float m = NEG, l = 0.f;
+  const float sl2 = a.sl2;
+
+  for (int p = p0; p < p1; ++p) {
+    const int buf = (p - p0) & 1;
+    if (p + 1 < p1) dma(bt[p + 1], buf ^ 1);  // that buffer was released by the last barrier
+    const char* C = smem + buf * G::PAGEB;
+    if (p * PAGE <= wmax) {
+      f32x4 s[2];
+#pragma unroll
+      for (int t = 0; t < 2; ++t) {
+        s[t] = f32x4{};
+#pragma unroll
+        for (int k = 0; k < RT; ++k)
+          s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(C + G::off(16 * t + l16, 4 * k + g)), qf[k],
+                                                         s[t], 0, 0, 0);
+      }
+      float mx = m;
+#pragma unroll
+      for (int t = 0; t < 2; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          if (p * PAGE + 16 * t + 4 * g + r > pos) s[t][r] = NEG;
+          mx = fmaxf(mx, s[t][r]);
+        }
+      mx = xor32_max(xor16_max(mx));
+      const bool grow = (mx - m) * sl2 > RESCALE;
+      if (__any(grow)) {
+        const float mn = grow ? mx : m;
+        const float alpha = __builtin_amdgcn_exp2f((m - mn) * sl2);
+        m = mn;
+        l *= alpha;
+#pragma unroll
+        for (int i = 0; i < 2 * RT; ++i) acc[i] *= alpha;
+      }
+      const float msl = m * sl2;
+      float pr[8];
+#pragma unroll
+      for (int t = 0; t < 2; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const float e = s[t][r] == NEG ? 0.f : __builtin_amdgcn_exp2f(__builtin_fmaf(s[t][r], sl2, -msl));
+          pr[4 * t + r] = e;
+          l += e;
+        }
+      const bf16x8 pf = pack_bf16x8(pr, 0);
+#pragma unroll
+      for (int i = 0; i < 2 * RT; ++i) {
+        const int c0 = 2 * i + (tp >> 1), k0 = 4 * g + tq;
+        const bf16x8 vf = tr_frag(C + G::off(k0, c0) + 8 * (tp & 1), C + G::off(16 + k0, c0) + 8 * (tp & 1));
+        acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf, acc[i], 0, 0, 0);
+      }
+    }
+    __builtin_amdgcn_s_waitcnt(0x0f70);  // vmcnt(0): the next page has landed
+    __syncthreads();
+  }
+  l = xor32_sum(xor16_sum(l));
+  if (myrow > last) return;
+  if (a.nsplit == 1) {
+    const float inv = 1.0f / l;
+    unsigned short* op = (unsigned short*)a.o + (base + myrow) * G::RP + 4 * g;
+#pragma unroll
+    for (int i = 0; i < 2 * RT; ++i) {
+      uint2 v;
+      v.x = pack_bf16x2(acc[i][0] * inv, acc[i][1] * inv);
+      v.y = pack_bf16x2(acc[i][2] * inv, acc[i][3] * inv);
+      *(uint2*)(op + 16 * i) = v;
+    }
+  } else {
+    const long pr = blockIdx.y * nrows + base + myrow;
+    float* po = a.part_o + pr * G::RP + 4 * g;
+#pragma unroll
+    for (int i = 0; i < 2 * RT; ++i) *(f32x4*)(po + 16 * i) = acc[i];
+    if (g == 0) {
+      a.part_ml[2 * pr] = m;
+      a.part_ml[2 * pr + 1] = l;
+    }
+  }
+}
+
+// one wave per row: o = sum_s 2^((m_s - m) sl2) acc_s / sum_s 2^(..) l_s
+__global__ __launch_bounds__(256) void merge(Args a) {
+  const int lane = threadIdx.x & 63;
+  const long nrows = (long)a.Nt * a.H, row = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (row >= nrows) return;
+  float m = NEG;
+  for (int s = 0; s < a.nsplit; ++s) {
+    const float* ml = a.part_ml + 2 * (s * nrows + row);
+    if (ml[1] > 0.f) m = fmaxf(m, ml[0]);
+  }
+  float l = 0.f;
+  for (int s = 0; s < a.nsplit; ++s) {
+    const float* ml = a.part_ml + 2 * (s * nrows + row);
+    if (ml[1] > 0.f) l += ml[1] * __builtin_amdgcn_exp2f((ml[0] - m) * a.sl2);
+  }
+  const float inv = 1.0f / l;
+  for (int c = 4 * lane; c < a.RP; c += 256) {
+    f32x4 v = f32x4{};
+    for (int s = 0; s < a.nsplit; ++s) {
+      const long pr = s * nrows + row;
+      if (a.part_ml[2 * pr + 1] > 0.f)
+        v += *(const f32x4*)(a.part_o + pr * a.RP + c) * (__builtin_amdgcn_exp2f((a.part_ml[2 * pr] - m) * a.sl2) * inv);
+    }
+    uint2 o;
+    o.x = pack_bf16x2(v[0], v[1]);
+    o.y = pack_bf16x2(v[2], v[3]);
+    *(uint2*)((unsigned short*)a.o + row * a.RP + c) = o;
+  }
+}
+
+// ---------------------------------------------------------------- attn_simple
+constexpr int SIMPLE_MAX = 2048;  // largest RP
+
+template <typename T>
+__global__ __launch_bounds__(256) void attn_simple(Args a) {
+  __shared__ float qs[SIMPLE_MAX];
+  __shared__ float ps[256];
+  __shared__ float red[4];
+  const int tid = threadIdx.x, RP = a.RP;
+  const long row = blockIdx.x;
+  const int tok = (int)(row / a.H), pos = a.tok_pos[tok];
+  const int* bt = a.bt + (long)a.tok_seq[tok] * a.W;
+  const T* cache = (const T*)a.cache;
+  for (int i = tid; i < RP; i += 256) qs[i] = ld((const T*)a.q + row * RP + i);
+  float acc[SIMPLE_MAX / 256];
+#pragma unroll
+  for (int i = 0; i < SIMPLE_MAX / 256; ++i) acc[i] = 0.f;
+  float m = NEG, l = 0.f;
+  __syncthreads();
+  for (int k0 = 0; k0 <= pos; k0 += 256) {
+    const int key = k0 + tid;
+    float s = NEG;
+    if (key <= pos) {
+      const T* c = cache + ((long)bt[key / PAGE] * PAGE + key % PAGE) * RP;
+      s = 0.f;
+      for (int i = 0; i < RP; ++i) s = __builtin_fmaf(qs[i], ld(c + i), s);
+      s *= a.scale;
+    }
+    float mx = wave_max(s);
+    if ((tid & 63) == 0) red[tid >> 6] = mx;
+    __syncthreads();
+    mx = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
+    mx = fmaxf(mx, m);
+    const float e = key <= pos ? expf(s - mx) : 0.f;
+    ps[tid] = e;
+    const float alpha = expf(m - mx);
+    m = mx;
+    const float sum = wave_sum(e);
+    __syncthreads();
+    if ((tid & 63) == 0) red[tid >> 6] = sum;
+    __syncthreads();
+    l = l * alpha + (red[0] + red[1] + red[2] + red[3]);
+    const int nk = min(256, pos + 1 - k0);
+#pragma unroll
+    for (int i = 0; i < SIMPLE_MAX / 256; ++i) {
+      const int col = tid + 256 * i;
+      if (col < RP) {
+        float v = acc[i] * alpha;
+        for (int j = 0; j < nk; ++j) {
+          const int kj = k0 + j;
+          v = __builtin_fmaf(ps[j], ld(cache + ((long)bt[kj / PAGE] * PAGE + kj % PAGE) * RP + col), v);
+        }
+        acc[i] = v;
+      }
+    }
+    __syncthreads();
+  }
+  const float inv = 1.0f / l;
+#pragma unroll
+  for (int i = 0; i < SIMPLE_MAX / 256; ++i) {
+    const int col = tid + 256 * i;
+    if (col < RP) st((T*)a.o + row * RP + col, acc[i] * inv);
+  }
+}
+
+template <int RT>
+static hipError_t launch_attn(const Args& a, int ntiles, int nw, hipStream_t s) {
+  const size_t lds = 2 * Geo<RT>::PAGEB;
+  if (lds > 48 * 1024) {
+    const hipError_t e =
+        hipFuncSetAttribute((const void*)attn<RT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    if (e != hipSuccess) return e;
+  }
+  hipLaunchKernelGGL(attn<RT>, dim3(ntiles, a.nsplit), dim3(64 * nw), lds, s, a);
+  return hipGetLastError();
+}
+
+}  // namespace latent
+}  // namespace kgs
+
+KGS_EXPORT int kgs_latent_norm(const void* z, long ldz, int oq, int nq, int qp, int oc, int nc, int rp,
+                               const void* wq, const void* wc, void* cq, void* cache, const void* slots, int T,
+                               float eps, int f32, hipStream_t s) {
+  using namespace kgs::latent;
+  if (T <= 0 || nq <= 0 || qp < nq || nc < 0 || (nc && rp < nc) || oq < 0 || oc < 0 || ldz < oq + nq ||
+      (nc && ldz < oc + nc))
+    return KGS_ERR_SHAPE;
+  NormArgs a{z, ldz, oq, nq, qp, oc, nc, rp, (const float*)wq, (const float*)wc, cq, cache, (const int*)slots, eps};
+  if (f32) hipLaunchKernelGGL(norm<float>, dim3(T), dim3(128), 0, s, a);
+  else hipLaunchKernelGGL(norm<unsigned short>, dim3(T), dim3(128), 0, s, a);
+  return (int)hipGetLastError();
+}
+
+// out[out_row(i)][h][n] = (sum_k a[in_row(i)][h][k] w[h][n][k]) * sigmoid(gate[out_row(i)][h])
+KGS_EXPORT int kgs_head_proj(const void* a, const void* w, void* out, const void* idx_in, const void* idx_out,
+                             const void* gate, long lda, long ha, long ldo, long ho, long ldg, int Nt, int H, int N,
+                             int K, int f32, hipStream_t s) {
+  using namespace kgs::latent;
+  if (Nt <= 0 || H <= 0 || N <= 0 || K <= 0 || ha < K || ho < N || lda < (H - 1) * ha + K || ldo < (H - 1) * ho + N ||
+      H > 65535)
+    return KGS_ERR_SHAPE;
+  ProjArgs p{a, w, out, (const int*)idx_in, (const int*)idx_out, gate, lda, ha, ldo, ho, ldg, Nt, H, N, K};
+  if (f32) {
+    hipLaunchKernelGGL(head_proj_f32, dim3(Nt, H), dim3(256), 0, s, p);
+    return (int)hipGetLastError();
+  }
+  if (N % 16 || K % 32) return KGS_ERR_SHAPE;
+  if ((((uintptr_t)a | (uintptr_t)w | (uintptr_t)out) & 15) || (lda | ha) % 8 || (ldo | ho) % 4) return KGS_ERR_ALIGN;
+  const int gx = (N / 16 + 3) / 4;
+  if (Nt <= 16) hipLaunchKernelGGL(head_proj<1>, dim3(gx, 1, H), dim3(256), 0, s, p);
+  else if (Nt <= 32) hipLaunchKernelGGL(head_proj<2>, dim3(gx, 1, H), dim3(256), 0, s, p);
+  else if ((Nt + 63) / 64 > 65535) return KGS_ERR_SHAPE;
+  else hipLaunchKernelGGL(head_proj<4>, dim3(gx, (Nt + 63) / 64, H), dim3(256), 0, s, p);
+  return (int)hipGetLastError();
+}
+
+// MFMA form: RP one of 32 x {1, 2, 3, 4, 6, 8, 12, 16}, bf16. ntiles workgroups
+// per split (items: ntiles (sequence, tile) pairs; null: B x tiles). A tile is
+// 16 nw rows.
+KGS_EXPORT int kgs_latent_attn(const void* q, const void* cache, void* o, void* part_o, void* part_ml, const void* q0,
+                               const void* n, const void* pos0, const void* bt, const void* items, int ntiles,
+                               int tiles, int nw, int nsplit, int H, int W, int Nt, int RP, float scale,
+                               hipStream_t s) {
+  using namespace kgs::latent;
+  if (ntiles <= 0 || H <= 0 || W <= 0 || Nt <= 0 || nw < 1 || nw > 8 || nsplit < 1 || nsplit > 1024 ||
+      (!items && tiles <= 0))
+    return KGS_ERR_SHAPE;
+  if (nsplit > 1 && (!part_o || !part_ml)) return KGS_ERR_ARG;
+  if (((uintptr_t)q | (uintptr_t)cache | (uintptr_t)o | (uintptr_t)part_o) & 15) return KGS_ERR_ALIGN;
+  Args a{q, cache, o, (float*)part_o, (float*)part_ml, (const int*)q0, (const int*)n, (const int*)pos0,
+         (const int*)bt, (const int*)items, nullptr, nullptr, H, W, tiles, nsplit, Nt, RP, scale,
+         scale * 1.4426950408889634f};
+  hipError_t e;
+  switch (RP) {
+    case 32: e = launch_attn<1>(a, ntiles, nw, s); break;
+    case 64: e = launch_attn<2>(a, ntiles, nw, s); break;
+    case 96: e = launch_attn<3>(a, ntiles, nw, s); break;
+    case 128: e = launch_attn<4>(a, ntiles, nw, s); break;
+    case 192: e = launch_attn<6>(a, ntiles, nw, s); break;
+    case 256: e = launch_attn<8>(a, ntiles, nw, s); break;
+    case 384: e = launch_attn<12>(a, ntiles, nw, s); break;
+    case 512: e = launch_attn<16>(a, ntiles, nw, s); break;
+    default: return KGS_ERR_SHAPE;
+  }
+  if (e == hipSuccess && nsplit > 1) {
+    hipLaunchKernelGGL(merge, dim3(((long)Nt * H + 3) / 4), dim3(256), 0, s, a);
+    e = hipGetLastError();
+  }
+  return (int)e;
+}
+
+KGS_EXPORT int kgs_latent_attn_simple(const void* q, const void* cache, void* o, const void* tok_seq,
+                                      const void* tok_pos, const void* bt, int H, int W, int Nt, int RP, float scale,
+                                      int f32, hipStream_t s) {
+  using namespace kgs::latent;
+  if (H <= 0 || W <= 0 || Nt <= 0 || RP <= 0 || RP > SIMPLE_MAX) return KGS_ERR_SHAPE;
+  Args a{q, cache, o, nullptr, nullptr, nullptr, nullptr, nullptr, (const int*)bt, nullptr, (const int*)tok_seq,
+         (const int*)tok_pos, H, W, 0, 1, Nt, RP, scale, 0.f};
+  const dim3 grid((unsigned)((long)Nt * H));
+  if (f32) hipLaunchKernelGGL(attn_simple<float>, grid, dim3(256), 0, s, a);
+  else hipLaunchKernelGGL(attn_simple<unsigned short>, grid, dim3(256), 0, s, a);
+  return (int)hipGetLastError();
+}

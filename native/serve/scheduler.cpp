@@ -148,6 +148,9 @@ Scheduler::Scheduler(const SchedulerConfig& cfg) : cfg_(cfg), alloc_(cfg.num_pag
   const int pad = std::max(1, cfg_.pad_multiple);
   cfg_.pad_multiple = pad;
   cfg_.max_prefill_tokens = std::max(cfg_.max_prefill_tokens, (cfg_.max_model_len + pad - 1) / pad * pad);
+  for (int i = cfg_.state_slots; i >= 1; --i) free_slots_.push_back(i);
+  // cached pages hold no recurrent state: a sequence with one starts at its first token
+  if (cfg_.state_slots > 0) cfg_.prefix_caching = false;
   // prefix caching skips cached leading pages with a chunk over the cached
   // context: it runs on mixed steps
   if (cfg_.prefix_caching && cfg_.chunk_tokens <= 0) cfg_.chunk_tokens = cfg_.max_prefill_tokens;
@@ -174,9 +177,105 @@ bool Scheduler::add(int64_t id, const std::vector<int32_t>& prompt, int max_new_
 void Scheduler::free_pages(Sequence& s) {
   for (int p : s.pages) alloc_.free(p);
   s.pages.clear();
+  if (s.slot > 0) free_slots_.push_back(s.slot);
+  s.slot = 0;
   s.cached = 0;
   s.hashed = 0;
   s.tail_hash = 0;
+}
+
+void Scheduler::take_slot(Sequence& s) {
+  if (cfg_.state_slots <= 0) return;
+  s.slot = free_slots_.back();
+  free_slots_.pop_back();
+}
+
+void Scheduler::fill_tables(const std::vector<int64_t>& ids, std::vector<int32_t>& bt, int& max_pages) const {
+  max_pages = 0;
+  for (int64_t id : ids) max_pages = std::max(max_pages, (int)seqs_.at(id).pages.size());
+  bt.assign(ids.size() * (size_t)max_pages, 0);
+  for (size_t i = 0; i < ids.size(); ++i) {
+    const Sequence& s = seqs_.at(ids[i]);
+    std::copy(s.pages.begin(), s.pages.end(), bt.begin() + i * max_pages);
+  }
+}
+
+void Scheduler::fill_slots(StepPlan& plan) const {
+  if (cfg_.state_slots <= 0) return;
+  for (int64_t id : plan.seq_ids) plan.state_slots.push_back(seqs_.at(id).slot);
+}
+
+bool Scheduler::open(int64_t id) {
+  if (seqs_.count(id) || !have_slot() || (int)running_.size() + fed_ >= cfg_.max_batch) return false;
+  Sequence s;
+  s.id = id;
+  s.fed = true;
+  s.max_new = cfg_.max_model_len;
+  s.state = SeqState::kRunning;
+  s.arrival = next_arrival_++;
+  take_slot(s);
+  seqs_.emplace(id, std::move(s));
+  fed_++;
+  return true;
+}
+
+StepPlan Scheduler::feed(const std::vector<int64_t>& ids, const std::vector<std::vector<int32_t>>& tokens) {
+  StepPlan plan;
+  const int ps = cfg_.page_size;
+  if (ids.size() != tokens.size() || ids.empty()) return plan;
+  int need = 0;
+  for (size_t i = 0; i < ids.size(); ++i) {
+    auto it = seqs_.find(ids[i]);
+    if (it == seqs_.end() || !it->second.fed || it->second.state != SeqState::kRunning) return plan;
+    if (std::count(ids.begin(), ids.end(), ids[i]) != 1) return plan;
+    const Sequence& s = it->second;
+    const size_t total = s.tokens.size() + tokens[i].size();
+    if (tokens[i].empty() || total > (size_t)cfg_.max_model_len) return plan;
+    need += pages_for((int)total) - (int)s.pages.size();
+  }
+  if (need > alloc_.num_free()) return plan;
+  for (size_t i = 0; i < ids.size(); ++i) {
+    Sequence& s = seqs_.at(ids[i]);
+    s.tokens.insert(s.tokens.end(), tokens[i].begin(), tokens[i].end());
+    while ((int)s.pages.size() < pages_for((int)s.tokens.size())) s.pages.push_back(alloc_.alloc());
+  }
+  std::vector<int64_t> pf, dec;
+  for (size_t i = 0; i < ids.size(); ++i)
+    (tokens[i].size() > 1 || seqs_.at(ids[i]).cached == 0 ? pf : dec).push_back(ids[i]);
+  for (int64_t id : pf) {
+    Sequence& s = seqs_.at(id);
+    const int n = (int)s.tokens.size() - s.cached;
+    const int padded = (n + cfg_.pad_multiple - 1) / cfg_.pad_multiple * cfg_.pad_multiple;
+    plan.seq_ids.push_back(id);
+    plan.seq_starts.push_back((int)plan.tokens.size());
+    plan.seq_lens.push_back(n);
+    plan.padded_lens.push_back(padded);
+    plan.ctx_starts.push_back(s.cached);
+    plan.last_chunk.push_back(1);
+    for (int t = 0; t < padded; ++t) {
+      const int pos = s.cached + t;
+      plan.tokens.push_back(t < n ? s.tokens[pos] : 0);
+      plan.positions.push_back(pos);
+      plan.slots.push_back(t < n ? s.pages[pos / ps] * ps + pos % ps : -1);
+    }
+    s.cached += n;
+  }
+  plan.n_prefill = (int)pf.size();
+  fill_tables(pf, plan.pf_block_tables, plan.pf_max_pages);
+  fill_tables(dec, plan.block_tables, plan.max_pages);
+  for (int64_t id : dec) {
+    Sequence& s = seqs_.at(id);
+    const int pos = s.cached;
+    plan.seq_ids.push_back(id);
+    plan.tokens.push_back(s.tokens.back());
+    plan.positions.push_back(pos);
+    plan.slots.push_back(s.pages[pos / ps] * ps + pos % ps);
+    plan.ctx_lens.push_back(pos + 1);
+    s.cached = pos + 1;
+  }
+  fill_slots(plan);
+  plan.kind = pf.empty() ? 2 : 3;
+  return plan;
 }
 
 bool Scheduler::abort(int64_t id) {
@@ -189,6 +288,7 @@ bool Scheduler::abort(int64_t id) {
     running_.erase(std::remove(running_.begin(), running_.end(), id), running_.end());
     free_pages(s);
   }
+  if (s.fed) fed_--;
   s.state = SeqState::kFinished;
   return true;
 }
@@ -207,7 +307,7 @@ bool Scheduler::try_prefill(StepPlan& plan) {
   // keep ~1% of the cache free after admission so running sequences can grow
   const int watermark = std::max(1, (cfg_.num_pages - 1) / 100);
   int budget = cfg_.max_prefill_tokens;
-  while (!waiting_.empty() && (int)running_.size() < cfg_.max_batch) {
+  while (!waiting_.empty() && (int)running_.size() + fed_ < cfg_.max_batch && have_slot()) {
     Sequence& s = seqs_.at(waiting_.front());
     const int len = (int)s.tokens.size();
     const int padded = (len + pad - 1) / pad * pad;
@@ -222,6 +322,9 @@ bool Scheduler::try_prefill(StepPlan& plan) {
     plan.seq_starts.push_back(start);
     plan.seq_lens.push_back(len);
     plan.padded_lens.push_back(padded);
+    plan.ctx_starts.push_back(0);
+    plan.last_chunk.push_back(1);
+    take_slot(s);
     for (int t = 0; t < padded; ++t) {
       const bool real = t < len;
       plan.tokens.push_back(real ? s.tokens[t] : 0);
@@ -234,6 +337,9 @@ bool Scheduler::try_prefill(StepPlan& plan) {
     running_.push_back(s.id);
   }
   if (plan.seq_ids.empty()) return false;
+  plan.n_prefill = (int)plan.seq_ids.size();
+  fill_tables(plan.seq_ids, plan.pf_block_tables, plan.pf_max_pages);
+  fill_slots(plan);
   plan.kind = 1;
   return true;
 }
@@ -262,10 +368,7 @@ void Scheduler::build_decode(StepPlan& plan) {
   }
   if (running_.empty()) return;
   plan.kind = 2;
-  int maxp = 0;
-  for (int64_t id : running_) maxp = std::max(maxp, (int)seqs_.at(id).pages.size());
-  plan.max_pages = maxp;
-  plan.block_tables.assign(running_.size() * (size_t)maxp, 0);
+  fill_tables(running_, plan.block_tables, plan.max_pages);
   for (size_t i = 0; i < running_.size(); ++i) {
     Sequence& s = seqs_.at(running_[i]);
     const int pos = s.cached;
@@ -274,9 +377,9 @@ void Scheduler::build_decode(StepPlan& plan) {
     plan.positions.push_back(pos);
     plan.slots.push_back(s.pages[pos / ps] * ps + pos % ps);
     plan.ctx_lens.push_back(pos + 1);
-    std::copy(s.pages.begin(), s.pages.end(), plan.block_tables.begin() + i * maxp);
     s.cached = pos + 1;
   }
+  fill_slots(plan);
 }
 
 StepPlan Scheduler::schedule_mixed() {
@@ -352,9 +455,10 @@ StepPlan Scheduler::schedule_mixed() {
       if (budget < pad) break;
       if (!decode_ready(s) && s.cached < (int)s.tokens.size()) add_chunk(s);
     }
-    while (!waiting_.empty() && budget >= pad && (int)running_.size() < cfg_.max_batch) {
+    while (!waiting_.empty() && budget >= pad && (int)running_.size() + fed_ < cfg_.max_batch && have_slot()) {
       Sequence& s = seqs_.at(waiting_.front());
       if (!add_chunk(s)) break;
+      take_slot(s);
       waiting_.pop_front();
       s.state = SeqState::kRunning;
       s.arrival = next_arrival_++;
@@ -370,20 +474,8 @@ StepPlan Scheduler::schedule_mixed() {
   }
   plan.n_prefill = (int)pf.size();
   // 3) decode rows after the chunks
-  if (!pf.empty()) {
-    int maxp = 0;
-    for (int64_t id : pf) maxp = std::max(maxp, (int)seqs_.at(id).pages.size());
-    plan.pf_max_pages = maxp;
-    plan.pf_block_tables.assign(pf.size() * (size_t)maxp, 0);
-    for (size_t i = 0; i < pf.size(); ++i) {
-      const Sequence& s = seqs_.at(pf[i]);
-      std::copy(s.pages.begin(), s.pages.end(), plan.pf_block_tables.begin() + i * maxp);
-    }
-  }
-  int maxp = 0;
-  for (int64_t id : dec) maxp = std::max(maxp, (int)seqs_.at(id).pages.size());
-  plan.max_pages = maxp;
-  plan.block_tables.assign(dec.size() * (size_t)maxp, 0);
+  fill_tables(pf, plan.pf_block_tables, plan.pf_max_pages);
+  fill_tables(dec, plan.block_tables, plan.max_pages);
   for (size_t i = 0; i < dec.size(); ++i) {
     Sequence& s = seqs_.at(dec[i]);
     const int pos = s.cached;
@@ -392,12 +484,12 @@ StepPlan Scheduler::schedule_mixed() {
     plan.positions.push_back(pos);
     plan.slots.push_back(s.pages[pos / ps] * ps + pos % ps);
     plan.ctx_lens.push_back(pos + 1);
-    std::copy(s.pages.begin(), s.pages.end(), plan.block_tables.begin() + i * maxp);
     s.cached = pos + 1;
     // a page filled by generated tokens is cacheable too (multi-turn chat:
     // the next turn's prompt starts with this one's prompt + answer)
     if (cfg_.prefix_caching && s.cached % ps == 0) register_full_pages(s);
   }
+  fill_slots(plan);
   // no chunk this step: a plain decode plan (the engine replays its hipGraph)
   plan.kind = plan.seq_ids.empty() ? 0 : pf.empty() ? 2 : 3;
   return plan;
@@ -488,6 +580,17 @@ std::string Scheduler::check_invariants() const {
     owned += owners[p] > 0;
   }
   if (owned + alloc_.num_free() != cfg_.num_pages - 1) err << "page leak: owned " << owned << " free " << alloc_.num_free() << "; ";
+  if (cfg_.state_slots > 0) {
+    std::vector<int> held(cfg_.state_slots + 1, 0);
+    for (int f : free_slots_) held[f]++;
+    for (const auto& kv : seqs_) {
+      const Sequence& s = kv.second;
+      if ((s.state == SeqState::kRunning) != (s.slot > 0)) err << "seq " << s.id << " state slot " << s.slot << "; ";
+      if (s.slot > 0) held[s.slot]++;
+    }
+    for (int i = 1; i <= cfg_.state_slots; ++i)
+      if (held[i] != 1) err << "state slot " << i << " held " << held[i] << " times; ";
+  }
   if ((int)running_.size() > cfg_.max_batch) err << "running over max_batch; ";
   for (int64_t id : running_)
     if (seqs_.at(id).state != SeqState::kRunning) err << "running list has non-running " << id << "; ";

@@ -77,6 +77,8 @@ struct Sequence {
   int cached = 0;               // tokens whose k/v are in the cache
   SeqState state = SeqState::kWaiting;
   int preemptions = 0;
+  int slot = 0;                 // recurrent-state slot (0: none; slot 0 is the null slot)
+  bool fed = false;             // opened with open(): its tokens come from feed()
   int hashed = 0;               // leading pages registered in the prefix cache
   uint64_t tail_hash = 0;       // chained hash of those pages
 };
@@ -92,7 +94,7 @@ struct StepPlan {
   std::vector<int32_t> ctx_lens;
   int max_pages = 0;
   std::vector<int64_t> preempted;
-  // mixed: seq_ids[0 .. n_prefill) are prefill chunks (rows first, with
+  // prefill and mixed: seq_ids[0 .. n_prefill) are prefill chunks (rows first, with
   // seq_starts / seq_lens / padded_lens), the rest decode rows (block_tables /
   // ctx_lens); ctx_starts = tokens cached before the chunk, last_chunk = the
   // chunk completes the prompt (its last row is sampled), pf_block_tables
@@ -102,6 +104,8 @@ struct StepPlan {
   std::vector<uint8_t> last_chunk;
   std::vector<int32_t> pf_block_tables;
   int pf_max_pages = 0;
+  // recurrent-state slot of every sequence of seq_ids (SchedulerConfig::state_slots > 0)
+  std::vector<int32_t> state_slots;
 };
 
 struct SchedulerConfig {
@@ -112,6 +116,8 @@ struct SchedulerConfig {
   int max_model_len = 8192;
   int pad_multiple = 128;
   int chunk_tokens = 0;           // > 0: mixed steps of at most this many rows (chunked prefill)
+  int state_slots = 0;            // > 0: models with per-sequence recurrent state -- slots 1 .. state_slots
+                                  // (0 is the null slot of padded decode rows), one per running sequence
   bool prefix_caching = false;    // share full prompt pages across sequences (implies chunked prefill)
 };
 
@@ -141,6 +147,16 @@ class Scheduler {
   static constexpr int32_t kPendingToken = -1;
   std::vector<int64_t> update_pending(const std::vector<int64_t>& ids);
   int fill_pending(const std::vector<int64_t>& ids, const std::vector<int32_t>& toks);
+  // Sequences fed by the caller (trace replay, scoring of given tokens): open()
+  // admits one with no tokens, feed() appends tokens to any number of open
+  // sequences and returns ONE mixed plan that runs exactly those tokens -- a
+  // portion of several tokens, or a sequence's first, as a prefill row block;
+  // single later tokens as decode rows. abort() gives pages and slot back. fed
+  // sequences are left alone by schedule(). feed() returns an idle plan (kind 0)
+  // and changes nothing when an id is unknown or repeated, a portion is empty
+  // or too long, or the pages or slots do not suffice.
+  bool open(int64_t id);
+  StepPlan feed(const std::vector<int64_t>& ids, const std::vector<std::vector<int32_t>>& tokens);
   const Sequence* get(int64_t id) const;
   void release(int64_t id);  // drop a finished sequence's record
   int num_waiting() const { return (int)waiting_.size(); }
@@ -159,12 +175,18 @@ class Scheduler {
   bool decode_ready(const Sequence& s) const { return s.cached == (int)s.tokens.size() - 1; }
   void preempt(Sequence& s, StepPlan& plan);
   void free_pages(Sequence& s);
+  bool have_slot() const { return cfg_.state_slots <= 0 || !free_slots_.empty(); }
+  void take_slot(Sequence& s);
+  void fill_tables(const std::vector<int64_t>& ids, std::vector<int32_t>& bt, int& max_pages) const;
+  void fill_slots(StepPlan& plan) const;
 
   SchedulerConfig cfg_;
   BlockAllocator alloc_;
   std::unordered_map<int64_t, Sequence> seqs_;
   std::deque<int64_t> waiting_;
   std::vector<int64_t> running_;  // admission order
+  std::vector<int32_t> free_slots_;  // LIFO
+  int fed_ = 0;                      // open fed sequences
   int64_t next_arrival_ = 0;
   int64_t prefix_hits_ = 0;
   int match_prefix(Sequence& s);     // acquire cached leading pages; returns tokens matched

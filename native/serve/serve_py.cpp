@@ -38,6 +38,7 @@ PYBIND11_MODULE(_serve, m) {
       .def_readwrite("max_model_len", &SchedulerConfig::max_model_len)
       .def_readwrite("pad_multiple", &SchedulerConfig::pad_multiple)
       .def_readwrite("chunk_tokens", &SchedulerConfig::chunk_tokens)
+      .def_readwrite("state_slots", &SchedulerConfig::state_slots)
       .def_readwrite("prefix_caching", &SchedulerConfig::prefix_caching);
 
   py::class_<StepPlan>(m, "StepPlan")
@@ -62,6 +63,7 @@ PYBIND11_MODULE(_serve, m) {
       .def_readonly("pf_max_pages", &StepPlan::pf_max_pages)
       .def_property_readonly("ctx_starts", [](const StepPlan& p) { return arr(p.ctx_starts); })
       .def_property_readonly("last_chunk", [](const StepPlan& p) { return arr(p.last_chunk); })
+      .def_property_readonly("state_slots", [](const StepPlan& p) { return arr(p.state_slots); })
       .def_property_readonly("pf_block_tables", [](const StepPlan& p) {
         auto a = arr(p.pf_block_tables);
         if (p.pf_max_pages > 0) a.resize({(py::ssize_t)p.n_prefill, (py::ssize_t)p.pf_max_pages});
@@ -72,6 +74,8 @@ PYBIND11_MODULE(_serve, m) {
       .def(py::init<const SchedulerConfig&>(), py::arg("config"))
       .def("add", &Scheduler::add, py::arg("id"), py::arg("prompt"), py::arg("max_new_tokens"))
       .def("abort", &Scheduler::abort)
+      .def("open", &Scheduler::open, py::arg("id"))
+      .def("feed", &Scheduler::feed, py::arg("ids"), py::arg("tokens"))
       .def("schedule", &Scheduler::schedule)
       .def(
           "update",
@@ -125,11 +129,13 @@ PYBIND11_MODULE(_serve, m) {
              d["cached"] = q->cached;
              d["pages"] = q->pages.size();
              d["preemptions"] = q->preemptions;
+             d["slot"] = q->slot;
              return d;
            })
       .def("release", &Scheduler::release)
       .def_property_readonly("num_waiting", &Scheduler::num_waiting)
       .def_property_readonly("num_running", &Scheduler::num_running)
+      .def_property_readonly("num_state_slots", [](const Scheduler& s) { return s.config().state_slots; })
       .def_property_readonly("num_free_pages", &Scheduler::num_free_pages)
       .def_property_readonly("prefix_hit_tokens", &Scheduler::prefix_hit_tokens)
       .def_property_readonly("num_cached_pages", &Scheduler::num_cached_pages)

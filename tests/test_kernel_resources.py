@@ -21,7 +21,8 @@ pytestmark = [pytest.mark.skipif(not Path(HIPCC).exists() and shutil.which("hipc
 
 def _compile(src: str, odir: Path, save_temps: bool = False, subdir: str = "kernels") -> tuple[dict, str]:
     """Resource remarks per kernel (and, with save_temps, the device assembly)."""
-    cmd = [HIPCC if Path(HIPCC).exists() else "hipcc", "--offload-arch=gfx950", "-O3", "-std=c++17", "-c",
+    cmd = [HIPCC if Path(HIPCC).exists() else "hipcc", "--offload-arch=gfx950", "-O3", "-std=c++17",
+           "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-c",
            "-I", str(ROOT / "native" / "kernels"),
            str(ROOT / "native" / subdir / src), "-o", str(odir / (src + ".o")),
            "-Rpass-analysis=kernel-resource-usage"]
