@@ -59,5 +59,8 @@ def to_spec(cfg) -> dict:
 
 
 def from_spec(d: dict):
+    """Inverse of :func:`to_spec`; plain fields are a Llama configuration's."""
+    if "architecture" not in d:
+        d = {"architecture": "Llama", "spec": d}
     cls = ARCHITECTURES[d["architecture"]].config_class()
     return cls.from_spec(d["spec"]) if hasattr(cls, "from_spec") else cls(**d["spec"])

@@ -374,7 +374,11 @@ def main(argv=None) -> int:
     ap.add_argument("--host", default="0.0.0.0")
     ap.add_argument("--port", type=int, default=8000)
     ap.add_argument("--model-name", default="meta-llama/Meta-Llama-3-8B")
-    ap.add_argument("--layers", type=int, default=32)
+    ap.add_argument("--model", default=None,
+                    help="model folder (config.json + model.safetensors; architectures: kgs.models.registry); "
+                         "default: Llama-3-8B with random weights")
+    ap.add_argument("--dtype", choices=("bfloat16", "float32"), default="bfloat16")
+    ap.add_argument("--layers", type=int, default=32, help="of the default model")
     ap.add_argument("--max-batch", type=int, default=256)
     ap.add_argument("--max-model-len", type=int, default=8192)
     ap.add_argument("--tokenizer", default=None, help="local HF tokenizer.json (default: byte-level)")
@@ -401,20 +405,19 @@ def main(argv=None) -> int:
     import uvicorn
 
     from kgs.models.llama import LlamaConfig
+    from kgs.models.registry import load_config, to_spec
 
     from .engine import EngineConfig, LLMEngine
 
-    mc = LlamaConfig.llama3_8b(layers=a.layers)
+    mc = load_config(a.model) if a.model else LlamaConfig.llama3_8b(layers=a.layers)
     ec = EngineConfig(max_batch=a.max_batch, max_model_len=a.max_model_len, cuda_graphs=not a.no_graphs,
                       chunked_prefill=a.chunked_prefill, prefix_caching=a.prefix_caching,
                       kv_cache_dtype=a.kv_cache_dtype, decode_weights=a.decode_weights,
-                      prefill_weights=a.prefill_weights, overlap=a.overlap)
+                      prefill_weights=a.prefill_weights, overlap=a.overlap, dtype=a.dtype)
     if a.data_parallel > 1 or a.engine_process:
-        import dataclasses
-
         from .dp import DPEngineLoop
 
-        runner = DPEngineLoop(max(1, a.data_parallel), dataclasses.asdict(mc), ec, device=a.device,
+        runner = DPEngineLoop(max(1, a.data_parallel), to_spec(mc), ec, device=a.device,
                               backend=a.backend, warmup_widths=[8, 32])
     else:
         eng = LLMEngine(mc, ec, device=a.device, backend=a.backend)

@@ -36,12 +36,21 @@ def _graph_widths(a):
     return widths or None
 
 
-def run_engine(a) -> dict:
+def _model_config(model: str, layers: int | None):
+    """A named Llama, or the model in a folder (config.json + model.safetensors)."""
+    if os.path.isdir(model):
+        from kgs.models.registry import load_config
+
+        return load_config(model)
     from kgs.models.llama import LlamaConfig
 
+    return LlamaConfig.named(model, layers)
+
+
+def run_engine(a) -> dict:
     from .engine import EngineConfig, LLMEngine, SamplingParams
 
-    mc = LlamaConfig.named(a.model, a.layers)
+    mc = _model_config(a.model, a.layers)
     ec = EngineConfig(max_batch=a.max_batch, max_model_len=a.max_model_len, cuda_graphs=not a.no_graphs,
                       max_prefill_tokens=a.max_prefill_tokens, fused_max_batch=a.fused_max_batch,
                       decode_weights=a.decode_weights, kv_cache_dtype=a.kv_cache_dtype,
@@ -91,7 +100,7 @@ def run_engine(a) -> dict:
         "fused_max_batch": a.fused_max_batch, "decode_weights": a.decode_weights,
         "kv_cache_dtype": a.kv_cache_dtype, "prefill_weights": a.prefill_weights,
         "fuse_splitk": not a.no_fuse_splitk, "w4x_panels": not a.no_w4x_panels,
-        "gate_up_panels": eng.model.gate_up_panels is not None, "overlap": eng.overlap,
+        "gate_up_panels": getattr(eng.model, "gate_up_panels", None) is not None, "overlap": eng.overlap,
         "nt_weights": NT_WEIGHTS,
         "chunked_prefill": a.chunked_prefill,
         "prefix_caching": a.prefix_caching, "shared_prefix": a.shared_prefix,
@@ -117,11 +126,9 @@ def run_online(a, mc=None, device="cuda", backend="kgs") -> dict:
     (t_done - t_first) / (tokens - 1)), ITL (every gap between two tokens of a
     request) and end-to-end latency, p50/p99 -- the metrics of vLLM's
     benchmark_serving, without the HTTP hop."""
-    from kgs.models.llama import LlamaConfig
-
     from .engine import EngineConfig, LLMEngine, SamplingParams
 
-    mc = mc or LlamaConfig.named(getattr(a, "model", "llama3-8b"), a.layers)
+    mc = mc or _model_config(getattr(a, "model", "llama3-8b"), a.layers)
     ec = EngineConfig(max_batch=a.max_batch, max_model_len=a.max_model_len, cuda_graphs=not a.no_graphs,
                       max_prefill_tokens=a.max_prefill_tokens, fused_max_batch=a.fused_max_batch,
                       decode_weights=a.decode_weights, kv_cache_dtype=a.kv_cache_dtype,
@@ -222,7 +229,8 @@ def main(argv=None) -> int:
     ap.add_argument("--max-batch", type=int, default=256)
     ap.add_argument("--max-model-len", type=int, default=4096)
     ap.add_argument("--max-prefill-tokens", type=int, default=16384)
-    ap.add_argument("--model", choices=("llama3-8b", "llama3-70b"), default="llama3-8b")
+    ap.add_argument("--model", default="llama3-8b",
+                    help="llama3-8b, llama3-70b (random weights) or a model folder (config.json + model.safetensors)")
     ap.add_argument("--layers", type=int, default=None, help="default: the model's (32 / 80)")
     ap.add_argument("--no-packed-decode", action="store_true",
                     help="one weight copy: decode on hipBLASLt / split-K (needed for llama3-70b on one GPU)")
@@ -257,6 +265,8 @@ def main(argv=None) -> int:
     ap.add_argument("--hf", action="store_true", help="also run the HF transformers baseline")
     ap.add_argument("--hf-only", action="store_true")
     a = ap.parse_args(argv)
+    if a.model not in ("llama3-8b", "llama3-70b") and not os.path.isdir(a.model):
+        ap.error(f"--model {a.model}: neither a known name nor a folder")
     if a.layers is None:
         a.layers = 80 if a.model == "llama3-70b" else 32
     if a.model == "llama3-70b" and not a.no_packed_decode and a.decode_weights == "bf16":

@@ -35,7 +35,7 @@ def _worker(index: int, spec: dict, inq, outq) -> None:
 
 
 def _serve_replica(index: int, spec: dict, inq, outq) -> None:
-    from kgs.models.llama import LlamaConfig
+    from kgs.models.registry import from_spec
 
     from .engine import LLMEngine
 
@@ -44,7 +44,7 @@ def _serve_replica(index: int, spec: dict, inq, outq) -> None:
         import torch
 
         torch.cuda.set_device(index)
-    eng = LLMEngine(LlamaConfig(**spec["model"]), spec["engine"], device=device, backend=spec["backend"])
+    eng = LLMEngine(from_spec(spec["model"]), spec["engine"], device=device, backend=spec["backend"])
     if spec.get("warmup_widths"):
         eng.warmup(widths=spec["warmup_widths"])
     outq.put(("ready", index, None))
