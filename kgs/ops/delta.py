@@ -7,12 +7,15 @@ from __future__ import annotations
 import ctypes
 from dataclasses import dataclass
 
+import numpy as np
 import torch
 
 from . import _lib
 from .hyper import _act, _f32
 
 MAX_DIM = 256
+CHUNK = 16       # tokens per chunk of the chunked form (delta.hip CH)
+CHUNK_MIN = 16   # portions from here on go by chunks, shorter ones step token by token
 
 
 @dataclass
@@ -53,12 +56,37 @@ class DeltaState:
 @dataclass
 class RaggedSeqs:
     """Sequences of a call (int32, device): each row's sequence, and per sequence
-    its first row, rows, first position and state slot."""
+    its first row, rows, first position and state slot. ``chunks`` / ``cseqs`` (see
+    :func:`chunk_plan`): the sequences that go by chunks; ``step_rows`` /
+    ``step_seqs``: rows and numbers of the others, None when that is all of them."""
     row_seq: torch.Tensor
     row0: torch.Tensor
     n: torch.Tensor
     pos0: torch.Tensor
     slot: torch.Tensor
+    chunks: torch.Tensor | None = None
+    cseqs: torch.Tensor | None = None
+    step_rows: torch.Tensor | None = None
+    step_seqs: torch.Tensor | None = None
+
+
+def chunk_plan(row0, n) -> dict:
+    """Host arrays of a batch's split: ``chunks [c, 4]`` (first row, rows, sequence,
+    0), ``cseqs [s, 4]`` (sequence, first chunk, chunks, first row; longest first),
+    ``step_rows``, ``step_seqs``. Empty when every sequence steps."""
+    row0, n = np.asarray(row0), np.asarray(n)
+    big = np.flatnonzero(n >= CHUNK_MIN)
+    if not len(big):
+        return {}
+    nc = -(-n[big] // CHUNK)
+    first = np.cumsum(nc) - nc
+    seq = np.repeat(big, nc)
+    at = (np.arange(nc.sum()) - np.repeat(first, nc)) * CHUNK
+    chunks = np.stack([row0[seq] + at, np.minimum(CHUNK, n[seq] - at), seq, np.zeros_like(seq)], 1)
+    cseqs = np.stack([big, first, nc, row0[big]], 1)[np.argsort(-nc, kind="stable")]
+    small = np.flatnonzero(n < CHUNK_MIN)
+    rows = np.concatenate([np.arange(row0[s], row0[s] + n[s]) for s in small]) if len(small) else np.zeros(0, np.int64)
+    return {"chunks": chunks, "cseqs": cseqs, "step_rows": rows, "step_seqs": small}
 
 
 def delta_forward(z: torch.Tensor, offs: tuple[int, int, int, int], a2: torch.Tensor, cw: torch.Tensor,
@@ -77,15 +105,24 @@ def delta_forward(z: torch.Tensor, offs: tuple[int, int, int, int], a2: torch.Te
     def f32(*shape):
         return torch.empty(shape, dtype=torch.float32, device=dev)
 
-    q, k, v, lg = f32(T, G, sh.kp), f32(T, G, sh.kp), f32(T, H, V), f32(T, H, sh.kp)
-    beta, qk, o = f32(T, H), f32(T, G), f32(T, H, V)
-    ptrs = (ctypes.c_void_p * 19)(
+    o = f32(T, H, V)
+    nc = 0 if seqs.chunks is None else seqs.chunks.shape[0]
+    nstep = (T, B) if not nc else (seqs.step_rows.shape[0], seqs.step_seqs.shape[0])
+    # indexed by row: only stepped rows' parts are touched
+    prep = [f32(T, G, sh.kp), f32(T, G, sh.kp), f32(T, H, V), f32(T, H, sh.kp), f32(T, H), f32(T, G)] if nstep[0] else []
+    work = [f32(nc, H, CHUNK, sh.kp), f32(nc, H, CHUNK, sh.kp), f32(nc, H, sh.kp, CHUNK), f32(nc, H, sh.kp),
+            f32(nc, H, CHUNK, V), f32(nc, H, CHUNK, CHUNK)] if nc else []
+    ptr = lambda ts, n: [t.data_ptr() for t in ts] if ts else [0] * n  # noqa: E731
+    opt = lambda t: 0 if t is None or not nc else t.data_ptr()  # noqa: E731
+    ptrs = (ctypes.c_void_p * 29)(
         z.data_ptr(), a2.data_ptr(), _f32(cw, (sh.taps, sh.channels), "cw"), _f32(a_log, (H,), "a_log"),
         _f32(dt_bias, (H * K,), "dt_bias"), seqs.row_seq.data_ptr(), seqs.row0.data_ptr(), seqs.n.data_ptr(),
-        seqs.pos0.data_ptr(), seqs.slot.data_ptr(), q.data_ptr(), k.data_ptr(), v.data_ptr(), lg.data_ptr(),
-        beta.data_ptr(), qk.data_ptr(), o.data_ptr(), state.S.data_ptr(), state.conv.data_ptr())
-    dims = (ctypes.c_long * 15)(z.stride(0), a2.stride(0), *offs, sh.taps, G, H, K, V, sh.kp, B, T,
-                                int(z.dtype == torch.float32))
+        seqs.pos0.data_ptr(), seqs.slot.data_ptr(), *ptr(prep, 6), o.data_ptr(), state.S.data_ptr(),
+        state.conv.data_ptr(), opt(seqs.step_rows), opt(seqs.step_seqs), opt(seqs.chunks), opt(seqs.cseqs), *ptr(work, 6))
+    pairs = not (K % 2 or V % 2 or z.stride(0) % 2 or a2.stride(0) % 2 or any(x % 2 for x in offs[:3]) or
+                 z.data_ptr() % 4 or a2.data_ptr() % 4)
+    dims = (ctypes.c_long * 20)(z.stride(0), a2.stride(0), *offs, sh.taps, G, H, K, V, sh.kp, B, T,
+                                int(z.dtype == torch.float32), *nstep, nc, seqs.cseqs.shape[0] if nc else 0, int(pairs))
     _lib.check(_lib.lib().kgs_delta_forward(ptrs, dims, _lib.stream_handle(dev)), f"delta_forward[{T}x{H}x{K}x{V}]")
     return o
 

@@ -25,7 +25,7 @@ import torch
 from kgs.models.ruruzen import DeltaSpec, LatentSpec, RuruzenConfig
 from kgs.ops.activation import act_mul, softcap
 from kgs.ops.decode import PAGE
-from kgs.ops.delta import DeltaShape, DeltaState, RaggedSeqs, delta_forward, delta_out
+from kgs.ops.delta import DeltaShape, DeltaState, RaggedSeqs, chunk_plan, delta_forward, delta_out
 from kgs.ops.hyper import MAX_STREAMS, hyper_embed, hyper_step
 from kgs.ops.latent import (KERNEL_SIZES, LatentCache, LatentRows, head_proj, latent_attention, latent_norm,
                             padded_latent, split_count, waves_for)
@@ -35,6 +35,7 @@ from kgs.ops.transformer import attention_ragged
 from .trace import TRACE as T
 
 DTYPES = {"bfloat16": torch.bfloat16, "float32": torch.float32}
+EXPAND_MIN = 16  # shorter portions are not worth the expansion's launches
 QBLOCK = 128  # query rows of one attention_ragged item
 
 
@@ -113,11 +114,13 @@ class Geometry:
     rp: int
     hd: int                    # head size of the expanded form, 0: absorbed only
 
-    def expand(self, n: int) -> bool:
-        """Whether a portion of ``n`` tokens runs on expanded keys and values: per
-        context token and head the expansion costs ``4 rp hd`` flops and saves
-        ``4 (rp - hd)`` per query token."""
-        return self.hd > 0 and n * (self.rp - self.hd) > self.rp * self.hd
+    def expand(self, n: int, pos0: int) -> bool:
+        """Whether a portion of ``n`` tokens after ``pos0`` runs on expanded keys and
+        values. Per head that expands every context token (``4 rp hd`` flops each)
+        where the absorbed form maps every query token (as many), and pays ``4 hd``
+        per (query, key) pair where the absorbed form pays ``4 rp``."""
+        pairs = n * (pos0 + 0.5 * n)
+        return self.hd > 0 and n >= EXPAND_MIN and pos0 * self.rp * self.hd < (self.rp - self.hd) * pairs
 
 
 # -------------------------------------------------------------------- sublayers
@@ -135,13 +138,15 @@ class _Weights:
 
     def stack(self, names, cols: int) -> tuple[torch.Tensor, list[int]]:
         """Several projections of one input as one matrix, each from a multiple of
-        64 rows on; returns it and the first rows."""
+        64 rows on (a large one ends on whole GEMM tiles); returns it and the first rows."""
         parts, offs, n = [], [], 0
         for name in names:
             p = self.mat(name, pad64(self.w[name].shape[0]), cols)
             offs.append(n)
             n += p.shape[0]
             parts.append(p)
+        if n > 1024 and n % 256:  # whole 256-wide GEMM tiles
+            parts.append(torch.zeros((256 - n % 256, cols), dtype=self.dtype, device=self.device))
         return torch.cat(parts).contiguous(), offs
 
 
@@ -371,6 +376,7 @@ class HybridModel:
         row_seq = np.repeat(order, n[order])
         pos = pos0[row_seq] + np.arange(len(tokens)) - row0[row_seq]
         refs = [pk.add(a) for a in (tokens, slots, row_seq, row0, n, pos0, slot, bt, logit_rows)]
+        split = {k: pk.add(v) for k, v in chunk_plan(row0, n).items()} if self.has_state else {}
         host = {g: self._host_plan(pk, g, row0, n, pos0, bt, row_seq, pos, refs) for g in self.geometries}
         get = pk.send()
         d = [get(r) for r in refs]
@@ -384,13 +390,13 @@ class HybridModel:
             expanded = None if e is None else Expanded(get(e[0]), get(e[1]).long())
             plans[g] = LatentPlan(absorbed, expanded)
         return Batch(dev_tokens.to(torch.int32).contiguous() if dev_tokens is not None else d[0], d[1],
-                     RaggedSeqs(d[2], d[3], d[4], d[5], d[6]), plans, d[8].long())
+                     RaggedSeqs(d[2], d[3], d[4], d[5], d[6], **{k: get(r) for k, r in split.items()}), plans, d[8].long())
 
     @staticmethod
     def _host_plan(pk: HostPack, g: Geometry, row0, n, pos0, bt, row_seq, pos, refs):
         """Splits the sequences between the absorbed and the expanded form and lays
         out both launches; returns references into ``pk``."""
-        big = np.array([g.expand(int(x)) for x in n], bool)
+        big = np.array([g.expand(int(x), int(p)) for x, p in zip(n, pos0)], bool)
         absorbed = expanded = None
         sel = np.flatnonzero(~big)
         if len(sel):

@@ -8,13 +8,24 @@
 // zeros whatever the slot holds, so freeing a slot needs no clear. One token per
 // sequence (decode) is the n = 1 case of the same kernels.
 //
+// Short sequences (decode) step token by token:
 //   prep   the short causal convolutions + silu of q, k, v (tail of the previous
 //          portion from the pool), unit norms, log decays, step sizes;
-//   scan   the recurrence and the convolution tails' update;
-//   out    per-head RMS norm and output gate.
+//   scan   the recurrence.
+// Longer ones go by chunks of C = 16 tokens. With b_i the log decays summed from
+// the chunk's start, S_0 the state before it and every exponent taken as a
+// difference b_i - b_j <= 0 (any decay is safe):
+//   A_ij = sum_c k_ic k_jc e^(b_ic - b_jc), P_ij the same with q_i   (j <= i)
+//   T = (I + diag(beta) tril(A, -1))^-1 diag(beta)
+//   U = T V - (T K~) S_0        K~_i = k_i e^(b_i)
+//   O = Q~ S_0 + P U            Q~_i = q_i e^(b_i)
+//   S = diag(e^(b_C)) S_0 + K^^T U   K^_j = k_j e^(b_C - b_j)
+//   chunk_prep  everything that does not need S_0, one workgroup per (chunk, head);
+//   chunk_scan  the three products with the state per chunk, on fp32 MFMAs.
+// tails updates the convolution tails, out applies the per-head norm and gate.
 //
-// Everything from prep on is fp32. K is padded to KP, a multiple of 32, in q, k,
-// log g and the state (pads are zero and stay zero). The state is stored
+// Everything after the convolutions is fp32. K is padded to KP, a multiple of 32,
+// in q, k, log g and the state (pads are zero and stay zero). The state is stored
 // transposed, [slot][head][V][KP].
 #include "kgs_common.h"
 
@@ -36,7 +47,6 @@ __device__ __forceinline__ float wave_sum(float v) {
   for (int m = 8; m >= 1; m >>= 1) v += __shfl_xor(v, m, 64);
   return xor32_sum(xor16_sum(v));
 }
-__device__ __forceinline__ float sigmoid(float x) { return 1.0f / (1.0f + expf(-x)); }
 
 struct Args {
   // inputs of prep
@@ -60,83 +70,152 @@ struct Args {
   // pools of this layer
   float* S;     // [slots][H][V][KP]
   float* conv;  // [slots][taps - 1][C]
+  // the call's two ways: stepped sequences (rows / seqs: their rows and numbers, or
+  // null when all are) and chunked ones
+  const int *rows, *seqs;
+  int nrows, nseqs;
+  const int4* chunks;  // (first row, rows, sequence, -)
+  const int4* cseqs;   // (sequence, first chunk, chunks, first row)
+  int nchunks, ncseqs;
+  float *cW, *cQ, *cK, *cE, *cU, *cP;  // per (chunk, head): [16][KP] x 2, [KP][16], [KP], [16][V], [16][16]
 };
 
-// ----------------------------------------------------------------------- prep
-// channel c (0 .. C-1) of row t after the convolution and silu
-template <typename T>
-__device__ __forceinline__ float conv_silu(const Args& a, long t, int c, int col, int r0, int p0, long slot) {
-  float s = 0.f;
-  for (int j = 0; j < a.taps; ++j) {
-    const long src = t - (a.taps - 1) + j;
-    float x;
-    if (src >= r0) x = ld((const T*)a.z + src * a.ldz + col);
-    else x = p0 > 0 ? a.conv[(slot * (a.taps - 1) + (src - r0 + a.taps - 1)) * a.C + c] : 0.f;
-    s = __builtin_fmaf(a.cw[(long)j * a.C + c], x, s);
+// fp32 activations take the precise functions, bf16 ones the hardware's
+constexpr float LOG2E = 1.4426950408889634f;
+template <bool FAST>
+__device__ __forceinline__ float sigm(float x) {
+  if constexpr (FAST) return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-LOG2E * x));
+  return 1.0f / (1.0f + expf(-x));
+}
+// log(1 + e^x); the fast form takes log1p(e) as log(u) e / (u - 1), u = 1 + e, whose
+// rounding errors cancel (D. Goldberg, "What Every Computer Scientist Should Know
+// About Floating-Point Arithmetic")
+template <bool FAST>
+__device__ __forceinline__ float softplus(float x) {
+  if constexpr (FAST) {
+    const float e = __builtin_amdgcn_exp2f(-LOG2E * fabsf(x)), u = 1.0f + e;
+    const float l = u == 1.0f ? e : 0.6931471805599453f * __builtin_amdgcn_logf(u) * e * __builtin_amdgcn_rcpf(u - 1.0f);
+    return fmaxf(x, 0.f) + l;
   }
-  return s / (1.0f + expf(-s));
+  return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x)));
 }
 
-// one workgroup per (row, q/k head) with the value heads that read it
-template <typename T>
-__global__ __launch_bounds__(256) void prep(Args a) {
-  extern __shared__ float buf[];  // [2][KP]
-  __shared__ float red[3][4];
-  const int tid = threadIdx.x;
-  const long t = blockIdx.x;
-  const int gh = blockIdx.y, K = a.K, KP = a.KP, V = a.V, rep = a.H / a.G;
-  const int b = a.row_seq[t];
-  const int r0 = a.row0[b], p0 = a.pos0[b];
-  const long slot = a.slot[b];
-  float sq = 0.f, sk = 0.f, sqk = 0.f;
-  for (int i = tid; i < KP; i += 256) {
-    float q = 0.f, k = 0.f;
+// N consecutive channels (1, or 2 on an even boundary)
+template <typename T, int N>
+__device__ __forceinline__ void ldn(const T* p, float (&v)[N]) {
+  if constexpr (N == 2 && sizeof(T) == 2) {
+    const unsigned u = *(const unsigned*)p;
+    v[0] = bf2f((unsigned short)(u & 0xffff));
+    v[1] = bf2f((unsigned short)(u >> 16));
+  } else {
+#pragma unroll
+    for (int i = 0; i < N; ++i) v[i] = ld(p + i);
+  }
+}
+
+// channels c .. c + N - 1 (column col of z) of row t after the convolution and silu
+template <typename T, int N>
+__device__ __forceinline__ void conv_silu(const Args& a, long t, int c, int col, int r0, int p0, long slot,
+                                          float (&y)[N]) {
+  float s[N] = {};
+#pragma unroll 4
+  for (int j = 0; j < a.taps; ++j) {
+    const long src = t - (a.taps - 1) + j;
+    float x[N] = {};
+    if (src >= r0) ldn((const T*)a.z + src * a.ldz + col, x);
+    else if (p0 > 0) ldn(a.conv + (slot * (a.taps - 1) + (src - r0 + a.taps - 1)) * a.C + c, x);
+#pragma unroll
+    for (int i = 0; i < N; ++i) s[i] = __builtin_fmaf(a.cw[(long)j * a.C + c + i], x[i], s[i]);
+  }
+#pragma unroll
+  for (int i = 0; i < N; ++i) y[i] = s[i] * sigm<sizeof(T) == 2>(s[i]);
+}
+
+// Where a token's prepared values go: global rows or a chunk's LDS
+struct Dst {
+  float *q, *k, *qk;         // [KP], [KP], one value (or null)
+  float *v, *lg, *beta;      // of value head h: v + (h - h0) * V, lg + (h - h0) * KP, beta + (h - h0)
+};
+
+// One wave: a token's q / k head gh and the value heads h0 .. h0 + nh - 1 that read it
+template <typename T, int N>
+__device__ __forceinline__ void prep_token(const Args& a, long t, int gh, int h0, int nh, int r0, int p0, long slot,
+                                           const Dst& d) {
+  constexpr bool FAST = sizeof(T) == 2;
+  constexpr int E = 256 / (64 * N);
+  const int lane = threadIdx.x & 63, K = a.K, KP = a.KP, V = a.V;
+  float q[E][N], k[E][N], sq = 0.f, sk = 0.f, sqk = 0.f;
+#pragma unroll
+  for (int e = 0; e < E; ++e) {
+    const int i = N * (lane + 64 * e);
+#pragma unroll
+    for (int x = 0; x < N; ++x) q[e][x] = k[e][x] = 0.f;
     if (i < K) {
       const int c = gh * K + i;
-      q = conv_silu<T>(a, t, c, a.oq + c, r0, p0, slot);
-      k = conv_silu<T>(a, t, a.G * K + c, a.ok + c, r0, p0, slot);
+      conv_silu<T, N>(a, t, c, a.oq + c, r0, p0, slot, q[e]);
+      conv_silu<T, N>(a, t, a.G * K + c, a.ok + c, r0, p0, slot, k[e]);
+#pragma unroll
+      for (int x = 0; x < N; ++x) {
+        sq = __builtin_fmaf(q[e][x], q[e][x], sq);
+        sk = __builtin_fmaf(k[e][x], k[e][x], sk);
+        sqk = __builtin_fmaf(q[e][x], k[e][x], sqk);
+      }
     }
-    buf[i] = q;
-    buf[KP + i] = k;
-    sq += q * q;
-    sk += k * k;
-    sqk += q * k;
   }
   sq = wave_sum(sq);
   sk = wave_sum(sk);
-  sqk = wave_sum(sqk);
-  if ((tid & 63) == 0) {
-    red[0][tid >> 6] = sq;
-    red[1][tid >> 6] = sk;
-    red[2][tid >> 6] = sqk;
-  }
-  __syncthreads();
-  sq = red[0][0] + red[0][1] + red[0][2] + red[0][3];
-  sk = red[1][0] + red[1][1] + red[1][2] + red[1][3];
-  sqk = red[2][0] + red[2][1] + red[2][2] + red[2][3];
   const float rq = 1.0f / sqrtf(sq + 1e-6f) / sqrtf((float)K), rk = 1.0f / sqrtf(sk + 1e-6f);
-  for (int i = tid; i < KP; i += 256) {
-    a.q[(t * a.G + gh) * KP + i] = buf[i] * rq;
-    a.k[(t * a.G + gh) * KP + i] = buf[KP + i] * rk;
+  if (d.qk) {
+    sqk = wave_sum(sqk);
+    if (lane == 0) *d.qk = sqk * rq * rk;
   }
-  if (tid == 0) a.qk[t * a.G + gh] = sqk * rq * rk;
-  for (int i = tid; i < rep * V; i += 256) {
-    const int c = gh * rep * V + i;
-    a.v[t * a.H * V + c] = conv_silu<T>(a, t, 2 * a.G * K + c, a.ov + c, r0, p0, slot);
-  }
-  for (int i = tid; i < rep * KP; i += 256) {
-    const int h = gh * rep + i / KP, c = i % KP;
-    float lg = 0.f;
-    if (c < K) {
-      const float x = ld((const T*)a.a2 + t * a.lda + h * K + c) + a.dt_bias[h * K + c];
-      lg = -expf(a.A_log[h]) * (fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))));
+#pragma unroll
+  for (int e = 0; e < E; ++e) {
+    const int i = N * (lane + 64 * e);
+    if (i < KP) {
+#pragma unroll
+      for (int x = 0; x < N; ++x) {
+        d.q[i + x] = q[e][x] * rq;
+        d.k[i + x] = k[e][x] * rk;
+      }
     }
-    a.lg[(t * a.H + h) * KP + c] = lg;
   }
-  for (int i = tid; i < rep; i += 256) {
-    const int h = gh * rep + i;
-    a.beta[t * a.H + h] = sigmoid(ld((const T*)a.z + t * a.ldz + a.ob + h));
+  for (int h = h0; h < h0 + nh; ++h) {
+    for (int i = N * lane; i < V; i += 64 * N) {
+      float v[N];
+      const int c = h * V + i;
+      conv_silu<T, N>(a, t, 2 * a.G * K + c, a.ov + c, r0, p0, slot, v);
+#pragma unroll
+      for (int x = 0; x < N; ++x) d.v[(h - h0) * V + i + x] = v[x];
+    }
+    const float A = -expf(a.A_log[h]);
+    for (int i = N * lane; i < KP; i += 64 * N) {
+      float x[N] = {};
+      if (i < K) {
+        ldn((const T*)a.a2 + t * a.lda + h * K + i, x);
+#pragma unroll
+        for (int j = 0; j < N; ++j) x[j] = A * softplus<FAST>(x[j] + a.dt_bias[h * K + i + j]);
+      }
+#pragma unroll
+      for (int j = 0; j < N; ++j) d.lg[(h - h0) * KP + i + j] = x[j];
+    }
   }
+  if (lane < nh) d.beta[lane] = sigm<FAST>(ld((const T*)a.z + t * a.ldz + a.ob + h0 + lane));
+  for (int i = lane + 64; i < nh; i += 64) d.beta[i] = sigm<FAST>(ld((const T*)a.z + t * a.ldz + a.ob + h0 + i));
+}
+
+// ----------------------------------------------------------------------- prep
+// one wave per (row of a stepped sequence, q / k head)
+template <typename T, int N>
+__global__ __launch_bounds__(256) void prep(Args a) {
+  const long unit = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (unit >= (long)a.nrows * a.G) return;
+  const int gh = (int)(unit % a.G), rep = a.H / a.G;
+  const long t = a.rows ? a.rows[unit / a.G] : unit / a.G;
+  const int b = a.row_seq[t];
+  prep_token<T, N>(a, t, gh, gh * rep, rep, a.row0[b], a.pos0[b], a.slot[b],
+                   Dst{a.q + (t * a.G + gh) * a.KP, a.k + (t * a.G + gh) * a.KP, a.qk + t * a.G + gh,
+                       a.v + (t * a.H + gh * rep) * a.V, a.lg + (t * a.H + gh * rep) * a.KP, a.beta + t * a.H + gh * rep});
 }
 
 // ----------------------------------------------------------------------- scan
@@ -147,35 +226,17 @@ __device__ __forceinline__ float xor8_sum(float x) {  // row_ror:8 within 16 lan
   return x + __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x128, 0xf, 0xf, false));
 }
 
-// The convolution tails after the call: the last taps - 1 inputs of the sequence.
-template <typename T>
-__device__ __forceinline__ void conv_tail(const Args& a, int b, int part, int parts) {
-  const int r0 = a.row0[b], n = a.n[b], p0 = a.pos0[b], m = a.taps - 1;
-  const long slot = a.slot[b];
-  for (int c = part * 256 + threadIdx.x; c < a.C; c += parts * 256) {
-    const int GK = a.G * a.K;
-    const int col = c < GK ? a.oq + c : c < 2 * GK ? a.ok + c - GK : a.ov + c - 2 * GK;
-    for (int j = 0; j < m; ++j) {  // ascending: reads are ahead of the writes
-      const int src = n + j;       // index in (old tail, this portion)
-      float x;
-      if (src < m) x = p0 > 0 ? a.conv[(slot * m + src) * a.C + c] : 0.f;
-      else x = ld((const T*)a.z + (long)(r0 + src - m) * a.ldz + col);
-      a.conv[(slot * m + j) * a.C + c] = x;
-    }
-  }
-}
-
 // A wave owns 8 columns of one head's state: lane (rg = lane >> 3, col = lane & 7)
 // holds rows 32 i + 4 rg + j of its column, so the two dot products of a token
 // (with k and with q, the latter completed by (q . k) u) are one 3-step exchange.
-template <typename T, int NI>
+template <int NI>
 __global__ __launch_bounds__(256) void scan(Args a) {
   constexpr int KP = 32 * NI;
   __shared__ __attribute__((aligned(16))) float sq[TB][KP], sk[TB][KP], sg[TB][KP];
   __shared__ float sv[TB][COLS], sb[TB], sqk[TB];
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
   const int rg = lane >> 3;
-  const int b = blockIdx.z, h = blockIdx.y, c0 = blockIdx.x * COLS;
+  const int b = a.seqs ? a.seqs[blockIdx.z] : blockIdx.z, h = blockIdx.y, c0 = blockIdx.x * COLS;
   const int col = c0 + 8 * w + (lane & 7), V = a.V, H = a.H, G = a.G;
   const int gh = h / (H / G);
   const int r0 = a.row0[b], n = a.n[b];
@@ -234,8 +295,248 @@ __global__ __launch_bounds__(256) void scan(Args a) {
 #pragma unroll
     for (int i = 0; i < NI; ++i) *(f32x4*)(Sp + 32 * i) = S[i];
   }
-  conv_tail<T>(a, b, h * gridDim.x + blockIdx.x, H * gridDim.x);
 }
+
+// --------------------------------------------------------------------- chunks
+constexpr int CH = 16;  // tokens per chunk
+
+__host__ __device__ __forceinline__ int chunk_ld(int n) { return n + 4; }  // LDS row pitch
+
+// one workgroup per (chunk, head)
+template <typename T, int N>
+__global__ __launch_bounds__(256, 4) void chunk_prep(Args a) {
+  extern __shared__ __attribute__((aligned(16))) float sm[];
+  __shared__ __attribute__((aligned(16))) float sA[CH][CH + 4], sT[CH][CH + 4], sbeta[CH];
+  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+  const int KP = a.KP, V = a.V, H = a.H, ldk = chunk_ld(KP), ldv = chunk_ld(V);
+  float *sq = sm, *sk = sq + CH * ldk, *sb = sk + CH * ldk, *sv = sb + CH * ldk;
+  const int h = blockIdx.x % H;
+  const long ck = blockIdx.x / H;
+  const int4 it = a.chunks[ck];  // first row, rows, sequence
+  const int b = it.z, n = it.y, gh = h / (H / a.G);
+  for (int i = w; i < CH; i += 4) {
+    if (i < n) {
+      prep_token<T, N>(a, it.x + i, gh, h, 1, a.row0[b], a.pos0[b], a.slot[b],
+                       Dst{sq + i * ldk, sk + i * ldk, nullptr, sv + i * ldv, sb + i * ldk, sbeta + i});
+    } else {  // past the end: no write, no decay
+      for (int c = lane; c < KP; c += 64) sq[i * ldk + c] = sk[i * ldk + c] = sb[i * ldk + c] = 0.f;
+      for (int c = lane; c < V; c += 64) sv[i * ldv + c] = 0.f;
+      if (lane == 0) sbeta[i] = 0.f;
+    }
+  }
+  __syncthreads();
+  for (int c = tid; c < KP; c += 256) {  // b, in log2 units
+    float s = 0.f;
+#pragma unroll
+    for (int i = 0; i < CH; ++i) {
+      s += sb[i * ldk + c];
+      sb[i * ldk + c] = s * LOG2E;
+    }
+  }
+  __syncthreads();
+  const long base = ck * H + h;
+  float* P = a.cP + base * CH * CH;
+  if (tid < 240) {  // pair (i, j), j < i, each over half of the channels
+    const int p = tid >> 1, half = tid & 1;
+    int i = (int)((1.0f + sqrtf(1.0f + 8.0f * p)) * 0.5f);
+    while (i * (i - 1) / 2 > p) --i;
+    while ((i + 1) * i / 2 <= p) ++i;
+    const int j = p - i * (i - 1) / 2;
+    float sa = 0.f, sp = 0.f;
+    for (int c = half * (KP / 2); c < (half + 1) * (KP / 2); c += 4) {
+      const f32x4 ki = *(const f32x4*)(sk + i * ldk + c), qi = *(const f32x4*)(sq + i * ldk + c);
+      const f32x4 bi = *(const f32x4*)(sb + i * ldk + c), kj = *(const f32x4*)(sk + j * ldk + c);
+      const f32x4 bj = *(const f32x4*)(sb + j * ldk + c);
+#pragma unroll
+      for (int x = 0; x < 4; ++x) {
+        const float y = kj[x] * __builtin_amdgcn_exp2f(bi[x] - bj[x]);
+        sa = __builtin_fmaf(ki[x], y, sa);
+        sp = __builtin_fmaf(qi[x], y, sp);
+      }
+    }
+    sa += __shfl_xor(sa, 1, 64);
+    sp += __shfl_xor(sp, 1, 64);
+    if (half == 0) {
+      sA[i][j] = sa;
+      P[i * CH + j] = sp;
+      P[j * CH + i] = 0.f;
+    }
+  } else {
+    const int i = tid - 240;
+    float sp = 0.f;
+    for (int c = 0; c < KP; c += 4) {
+      const f32x4 ki = *(const f32x4*)(sk + i * ldk + c), qi = *(const f32x4*)(sq + i * ldk + c);
+#pragma unroll
+      for (int x = 0; x < 4; ++x) sp = __builtin_fmaf(qi[x], ki[x], sp);
+    }
+    P[i * CH + i] = sp;
+  }
+  __syncthreads();
+  if (tid < CH) {  // column tid of T by forward substitution
+    float t[CH];
+#pragma unroll
+    for (int i = 0; i < CH; ++i) {
+      asm volatile("" ::: "memory");
+      float s = 0.f;
+#pragma unroll
+      for (int m = 0; m < i; ++m) s = __builtin_fmaf(sA[i][m], t[m], s);
+      t[i] = i < tid ? 0.f : i == tid ? sbeta[i] : -sbeta[i] * s;
+      sT[i][tid] = t[i];
+    }
+  }
+  __syncthreads();
+  // T K~, Q~, K^^T and e^(b_C) per key channel, T V per value channel
+  for (int c = tid; c < KP + V; c += 256) {
+    float x[CH];
+    if (c < KP) {
+      float* Q = a.cQ + base * CH * KP + c;
+      float* Kt = a.cK + (base * KP + c) * CH;
+      const float bc = sb[(CH - 1) * ldk + c];
+#pragma unroll
+      for (int i = 0; i < CH; ++i) {
+        const float bi = sb[i * ldk + c], k = sk[i * ldk + c], e = __builtin_amdgcn_exp2f(bi);
+        x[i] = k * e;
+        Q[i * KP] = sq[i * ldk + c] * e;
+      }
+#pragma unroll
+      for (int i = 0; i < CH; i += 4) {
+        f32x4 v;
+#pragma unroll
+        for (int y = 0; y < 4; ++y)
+          v[y] = sk[(i + y) * ldk + c] * __builtin_amdgcn_exp2f(bc - sb[(i + y) * ldk + c]);
+        *(f32x4*)(Kt + i) = v;
+      }
+      a.cE[base * KP + c] = __builtin_amdgcn_exp2f(bc);
+    } else {
+#pragma unroll
+      for (int i = 0; i < CH; ++i) x[i] = sv[i * ldv + c - KP];
+    }
+    float* o = c < KP ? a.cW + base * CH * KP + c : a.cU + base * CH * V + c - KP;
+    const int ldo = c < KP ? KP : V;
+#pragma unroll
+    for (int i = 0; i < CH; ++i) {
+      asm volatile("" ::: "memory");  // T's rows are read here, not all kept in registers
+      float s = 0.f;
+#pragma unroll
+      for (int j = 0; j <= i; j += 4) {
+        const f32x4 t = *(const f32x4*)&sT[i][j];  // zero above the diagonal
+#pragma unroll
+        for (int y = 0; y < 4; ++y) s = __builtin_fmaf(t[y], x[j + y], s);
+      }
+      o[i * ldo] = s;
+    }
+  }
+}
+
+// One workgroup per (sequence, head, 16 state columns); wave w holds the state's
+// 16-row tiles w, w + 4, ... as MFMA accumulators: lane (g = lane >> 4, n = lane & 15)
+// has rows 4 g + r of a tile for column n. Register r of an accumulator is at the
+// same time the B operand of a v_mfma_f32_16x16x4_f32 whose four contraction
+// indices are 4 g + r, so state and U feed the products without moving; the A
+// operands are read as float4s in that order. The waves' partial products over
+// their rows meet in LDS, one barrier per chunk.
+template <int MT>
+__global__ __launch_bounds__(256) void chunk_scan(Args a) {
+  __shared__ f32x4 part[2][2][4][64];  // [buffer][U | O][wave][lane]
+  const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int l16 = lane & 15, g = lane >> 4;
+  const int KP = a.KP, V = a.V, H = a.H, nslab = (V + 15) / 16, ntile = KP / 16;
+  const int lid = xcd_remap(blockIdx.x, gridDim.x);  // a head's slabs share an XCD's L2
+  const int slab = lid % nslab, h = lid / nslab % H;
+  const int4 sq = a.cseqs[lid / nslab / H];  // sequence, first chunk, chunks, first row
+  const int b = sq.x, n = a.n[b], col = slab * 16 + l16;
+  const bool live = col < V;
+  float* Sp = a.S + (((long)a.slot[b] * H + h) * V + (live ? col : 0)) * KP + 4 * g;
+  f32x4 S[MT];
+#pragma unroll
+  for (int m = 0; m < MT; ++m) {
+    const int tile = w + 4 * m;
+    S[m] = tile < ntile && a.pos0[b] > 0 && live ? *(const f32x4*)(Sp + 16 * tile) : f32x4{};
+  }
+  struct Frag {
+    f32x4 W[MT], Q[MT], K[MT], E[MT], U, P;
+  };
+  auto fetch = [&](int c, Frag& f) {
+    const long base = (long)(sq.y + c) * H + h;
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+      const int tile = w + 4 * m;
+      if (tile < ntile) {
+        f.W[m] = *(const f32x4*)(a.cW + (base * CH + l16) * KP + 16 * tile + 4 * g);
+        f.Q[m] = *(const f32x4*)(a.cQ + (base * CH + l16) * KP + 16 * tile + 4 * g);
+        f.K[m] = *(const f32x4*)(a.cK + (base * KP + 16 * tile + l16) * CH + 4 * g);
+        f.E[m] = *(const f32x4*)(a.cE + base * KP + 16 * tile + 4 * g);
+      } else {
+        f.W[m] = f.Q[m] = f.K[m] = f.E[m] = f32x4{};
+      }
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) f.U[r] = live ? a.cU[(base * CH + 4 * g + r) * V + col] : 0.f;
+    f.P = *(const f32x4*)(a.cP + (base * CH + l16) * CH + 4 * g);
+  };
+  Frag f;
+  fetch(0, f);
+  for (int c = 0; c < sq.z; ++c) {
+    Frag nx;
+    if (c + 1 < sq.z) fetch(c + 1, nx);
+    f32x4 pu = f32x4{}, po = f32x4{};
+#pragma unroll
+    for (int m = 0; m < MT; ++m)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        pu = __builtin_amdgcn_mfma_f32_16x16x4f32(f.W[m][r], S[m][r], pu, 0, 0, 0);
+        po = __builtin_amdgcn_mfma_f32_16x16x4f32(f.Q[m][r], S[m][r], po, 0, 0, 0);
+      }
+    const int buf = c & 1;
+    part[buf][0][w][lane] = pu;
+    part[buf][1][w][lane] = po;
+    __syncthreads();
+    const f32x4 U = f.U - (part[buf][0][0][lane] + part[buf][0][1][lane] + part[buf][0][2][lane] + part[buf][0][3][lane]);
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+      S[m] *= f.E[m];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) S[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.K[m][r], U[r], S[m], 0, 0, 0);
+    }
+    if (w == (c & 3)) {
+      f32x4 O = part[buf][1][0][lane] + part[buf][1][1][lane] + part[buf][1][2][lane] + part[buf][1][3][lane];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) O = __builtin_amdgcn_mfma_f32_16x16x4f32(f.P[r], U[r], O, 0, 0, 0);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int t = CH * c + 4 * g + r;
+        if (t < n && live) a.o[((long)(sq.w + t) * H + h) * V + col] = O[r];
+      }
+    }
+    f = nx;
+  }
+  if (live) {
+#pragma unroll
+    for (int m = 0; m < MT; ++m)
+      if (w + 4 * m < ntile) *(f32x4*)(Sp + 16 * (w + 4 * m)) = S[m];
+  }
+}
+
+// ---------------------------------------------------------------------- tails
+// The convolution tails after the call: the last taps - 1 inputs of the sequence.
+template <typename T>
+__global__ __launch_bounds__(256) void tails(Args a) {
+  const int b = blockIdx.y;
+  const int r0 = a.row0[b], n = a.n[b], p0 = a.pos0[b], m = a.taps - 1;
+  const long slot = a.slot[b];
+  for (int c = blockIdx.x * 256 + threadIdx.x; c < a.C; c += gridDim.x * 256) {
+    const int GK = a.G * a.K;
+    const int col = c < GK ? a.oq + c : c < 2 * GK ? a.ok + c - GK : a.ov + c - 2 * GK;
+    for (int j = 0; j < m; ++j) {  // ascending: reads are ahead of the writes
+      const int src = n + j;       // index in (old tail, this portion)
+      float x;
+      if (src < m) x = p0 > 0 ? a.conv[(slot * m + src) * a.C + c] : 0.f;
+      else x = ld((const T*)a.z + (long)(r0 + src - m) * a.ldz + col);
+      a.conv[(slot * m + j) * a.C + c] = x;
+    }
+  }
+}
+
 
 // ------------------------------------------------------------------------ out
 struct OutArgs {
@@ -248,50 +549,80 @@ struct OutArgs {
   float eps;
 };
 
+// one wave per (row, head)
 template <typename T>
 __global__ __launch_bounds__(256) void out(OutArgs a) {
-  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
+  constexpr bool FAST = sizeof(T) == 2;
+  const int lane = threadIdx.x & 63, V = a.V;
   const long t = blockIdx.x;
-  const T* gate = (const T*)a.gate + t * a.ldg;
+  const int h = blockIdx.y * 4 + (threadIdx.x >> 6);
   T* y = (T*)a.y + t * a.ldy;
-  for (int h = w; h < a.H; h += 4) {
-    const float* o = a.o + (t * a.H + h) * a.V;
-    float ss = 0.f;
-    for (int i = lane; i < a.V; i += 64) ss += o[i] * o[i];
-    const float r = 1.0f / sqrtf(wave_sum(ss) / a.V + a.eps);
-    for (int i = lane; i < a.V; i += 64) st(y + h * a.V + i, o[i] * r * a.w[i] * sigmoid(ld(gate + h * a.V + i)));
+  if (blockIdx.y == 0)
+    for (int i = a.H * V + threadIdx.x; i < a.ldy; i += 256) st(y + i, 0.f);
+  if (h >= a.H) return;
+  const T* gate = (const T*)a.gate + t * a.ldg + h * V;
+  const float* o = a.o + (t * a.H + h) * V;
+  y += h * V;
+  if (V == 128) {
+    const float2 x = *(const float2*)(o + 2 * lane);
+    float gt[2];
+    ldn<T, 2>(gate + 2 * lane, gt);
+    const float2 w = *(const float2*)(a.w + 2 * lane);
+    const float r = 1.0f / sqrtf(wave_sum(x.x * x.x + x.y * x.y) / V + a.eps);
+    const float y0 = x.x * r * w.x * sigm<FAST>(gt[0]), y1 = x.y * r * w.y * sigm<FAST>(gt[1]);
+    if constexpr (FAST) *(unsigned*)(y + 2 * lane) = pack_bf16x2(y0, y1);
+    else *(float2*)(y + 2 * lane) = make_float2(y0, y1);
+    return;
   }
-  for (int i = a.H * a.V + threadIdx.x; i < a.ldy; i += 256) st(y + i, 0.f);
+  float ss = 0.f;
+  for (int i = lane; i < V; i += 64) ss += o[i] * o[i];
+  const float r = 1.0f / sqrtf(wave_sum(ss) / V + a.eps);
+  for (int i = lane; i < V; i += 64) st(y + i, o[i] * r * a.w[i] * sigm<FAST>(ld(gate + i)));
 }
 
-template <typename T>
-static hipError_t run_prep(const Args& a, hipStream_t s) {
-  hipLaunchKernelGGL(prep<T>, dim3(a.T, a.G), dim3(256), 2 * a.KP * sizeof(float), s, a);
-  return hipGetLastError();
-}
-
-template <typename T>
-static hipError_t run_scan(const Args& a, hipStream_t s) {
-  const dim3 grid((a.V + COLS - 1) / COLS, a.H, a.B);
-  switch (a.KP / 32) {
-    case 1: hipLaunchKernelGGL((scan<T, 1>), grid, dim3(256), 0, s, a); break;
-    case 2: hipLaunchKernelGGL((scan<T, 2>), grid, dim3(256), 0, s, a); break;
-    case 3: hipLaunchKernelGGL((scan<T, 3>), grid, dim3(256), 0, s, a); break;
-    case 4: hipLaunchKernelGGL((scan<T, 4>), grid, dim3(256), 0, s, a); break;
-    case 5: hipLaunchKernelGGL((scan<T, 5>), grid, dim3(256), 0, s, a); break;
-    case 6: hipLaunchKernelGGL((scan<T, 6>), grid, dim3(256), 0, s, a); break;
-    case 7: hipLaunchKernelGGL((scan<T, 7>), grid, dim3(256), 0, s, a); break;
-    case 8: hipLaunchKernelGGL((scan<T, 8>), grid, dim3(256), 0, s, a); break;
-    default: return hipErrorInvalidValue;
+template <typename T, int N>
+static hipError_t run(const Args& a, hipStream_t s) {
+  if (a.nrows > 0) {
+    const long units = (long)a.nrows * a.G;
+    hipLaunchKernelGGL((prep<T, N>), dim3((unsigned)((units + 3) / 4)), dim3(256), 0, s, a);
+    const dim3 grid((a.V + COLS - 1) / COLS, a.H, a.nseqs);
+    switch (a.KP / 32) {
+      case 1: hipLaunchKernelGGL(scan<1>, grid, dim3(256), 0, s, a); break;
+      case 2: hipLaunchKernelGGL(scan<2>, grid, dim3(256), 0, s, a); break;
+      case 3: hipLaunchKernelGGL(scan<3>, grid, dim3(256), 0, s, a); break;
+      case 4: hipLaunchKernelGGL(scan<4>, grid, dim3(256), 0, s, a); break;
+      case 5: hipLaunchKernelGGL(scan<5>, grid, dim3(256), 0, s, a); break;
+      case 6: hipLaunchKernelGGL(scan<6>, grid, dim3(256), 0, s, a); break;
+      case 7: hipLaunchKernelGGL(scan<7>, grid, dim3(256), 0, s, a); break;
+      default: hipLaunchKernelGGL(scan<8>, grid, dim3(256), 0, s, a); break;
+    }
   }
+  if (a.nchunks > 0) {
+    const size_t lds = sizeof(float) * CH * (3 * chunk_ld(a.KP) + chunk_ld(a.V));
+    if (lds > 48 * 1024) {
+      const hipError_t e =
+          hipFuncSetAttribute((const void*)chunk_prep<T, N>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+      if (e != hipSuccess) return e;
+    }
+    hipLaunchKernelGGL((chunk_prep<T, N>), dim3((unsigned)(a.nchunks * a.H)), dim3(256), lds, s, a);
+    const dim3 grid((unsigned)((a.V + 15) / 16 * a.H * a.ncseqs));
+    switch ((a.KP + 63) / 64) {
+      case 1: hipLaunchKernelGGL(chunk_scan<1>, grid, dim3(256), 0, s, a); break;
+      case 2: hipLaunchKernelGGL(chunk_scan<2>, grid, dim3(256), 0, s, a); break;
+      case 3: hipLaunchKernelGGL(chunk_scan<3>, grid, dim3(256), 0, s, a); break;
+      default: hipLaunchKernelGGL(chunk_scan<4>, grid, dim3(256), 0, s, a); break;
+    }
+  }
+  if (a.taps > 1) hipLaunchKernelGGL(tails<T>, dim3((a.C + 255) / 256, a.B), dim3(256), 0, s, a);
   return hipGetLastError();
 }
 
 }  // namespace delta
 }  // namespace kgs
 
-// ptrs: z a2 cw A_log dt_bias row_seq row0 n pos0 slot q k v lg beta qk o S conv (19 device pointers)
-// dims: ldz lda oq ok ov ob taps G H K V KP B T f32 (15 values)
+// ptrs (29 device pointers): z a2 cw A_log dt_bias row_seq row0 n pos0 slot q k v lg beta qk o S conv
+//   rows seqs chunks cseqs cW cQ cK cE cU cP
+// dims (20): ldz lda oq ok ov ob taps G H K V KP B T f32 nrows nseqs nchunks ncseqs, even (channel pairs aligned)
 KGS_EXPORT int kgs_delta_forward(const void* const* ptrs, const long* dims, hipStream_t s) {
   using namespace kgs::delta;
   Args a{};
@@ -314,6 +645,16 @@ KGS_EXPORT int kgs_delta_forward(const void* const* ptrs, const long* dims, hipS
   a.o = (float*)ptrs[16];
   a.S = (float*)ptrs[17];
   a.conv = (float*)ptrs[18];
+  a.rows = (const int*)ptrs[19];
+  a.seqs = (const int*)ptrs[20];
+  a.chunks = (const int4*)ptrs[21];
+  a.cseqs = (const int4*)ptrs[22];
+  a.cW = (float*)ptrs[23];
+  a.cQ = (float*)ptrs[24];
+  a.cK = (float*)ptrs[25];
+  a.cE = (float*)ptrs[26];
+  a.cU = (float*)ptrs[27];
+  a.cP = (float*)ptrs[28];
   a.ldz = dims[0];
   a.lda = dims[1];
   a.oq = (int)dims[2];
@@ -328,7 +669,11 @@ KGS_EXPORT int kgs_delta_forward(const void* const* ptrs, const long* dims, hipS
   a.KP = (int)dims[11];
   a.B = (int)dims[12];
   a.T = (int)dims[13];
-  const bool f32 = dims[14] != 0;
+  const bool f32 = dims[14] != 0, pairs = dims[19] != 0;
+  a.nrows = (int)dims[15];
+  a.nseqs = (int)dims[16];
+  a.nchunks = (int)dims[17];
+  a.ncseqs = (int)dims[18];
   a.C = 2 * a.G * a.K + a.H * a.V;
   if (a.taps < 1 || a.G < 1 || a.H < 1 || a.H % a.G || a.K < 1 || a.V < 1 || a.B < 1 || a.T < 1 || a.KP % 32 ||
       a.KP < a.K || a.KP > 256 || a.G > 65535 || a.H > 65535 || a.B > 65535)
@@ -336,8 +681,15 @@ KGS_EXPORT int kgs_delta_forward(const void* const* ptrs, const long* dims, hipS
   if (a.ldz < a.oq + a.G * a.K || a.ldz < a.ok + a.G * a.K || a.ldz < a.ov + a.H * a.V || a.ldz < a.ob + a.H ||
       a.lda < (long)a.H * a.K)
     return KGS_ERR_SHAPE;
-  hipError_t e = f32 ? run_prep<float>(a, s) : run_prep<unsigned short>(a, s);
-  if (e == hipSuccess) e = f32 ? run_scan<float>(a, s) : run_scan<unsigned short>(a, s);
+  if (a.nrows < 0 || a.nseqs < 0 || a.nchunks < 0 || a.ncseqs < 0 || a.nseqs > 65535 || a.V > 1024 ||
+      (a.nrows > 0) != (a.nseqs > 0) || (a.nchunks > 0) != (a.ncseqs > 0) || (long)a.nchunks * a.H > 0x7fffffff)
+    return KGS_ERR_SHAPE;
+  if (a.nchunks > 0 && (!a.chunks || !a.cseqs || !a.cW || !a.cQ || !a.cK || !a.cE || !a.cU || !a.cP)) return KGS_ERR_ARG;
+  if (pairs && (a.K % 2 || a.V % 2 || (a.ldz | a.lda | a.oq | a.ok | a.ov) % 2 || ((uintptr_t)a.z | (uintptr_t)a.a2) & 3))
+    return KGS_ERR_ALIGN;
+  hipError_t e;
+  if (f32) e = pairs ? run<float, 2>(a, s) : run<float, 1>(a, s);
+  else e = pairs ? run<unsigned short, 2>(a, s) : run<unsigned short, 1>(a, s);
   return (int)e;
 }
 
@@ -346,7 +698,10 @@ KGS_EXPORT int kgs_delta_out(const void* o, const void* w, const void* gate, voi
   using namespace kgs::delta;
   if (T <= 0 || H <= 0 || V <= 0 || ldg < (long)H * V || ldy < (long)H * V) return KGS_ERR_SHAPE;
   OutArgs a{(const float*)o, (const float*)w, gate, y, ldg, ldy, H, V, eps};
-  if (f32) hipLaunchKernelGGL(out<float>, dim3(T), dim3(256), 0, s, a);
-  else hipLaunchKernelGGL(out<unsigned short>, dim3(T), dim3(256), 0, s, a);
+  if (V == 128 && (ldg % 2 || ldy % 2 || ((uintptr_t)gate & 3) || (((uintptr_t)o | (uintptr_t)w | (uintptr_t)y) & 7)))
+    return KGS_ERR_ALIGN;
+  const dim3 grid(T, (H + 3) / 4);
+  if (f32) hipLaunchKernelGGL(out<float>, grid, dim3(256), 0, s, a);
+  else hipLaunchKernelGGL(out<unsigned short>, grid, dim3(256), 0, s, a);
   return (int)hipGetLastError();
 }

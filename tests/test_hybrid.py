@@ -173,7 +173,9 @@ def test_launch_plan_splits_portions_and_orders_rows():
     from kgs.serve.hybrid import Geometry, HostPack, HybridModel
 
     g = Geometry(heads=4, rp=256, hd=64)
-    assert g.expand(86) and not g.expand(85) and not Geometry(4, 64, 64).expand(10000) and not Geometry(4, 256, 0).expand(999)
+    # behind a long context a portion is worth expanding from rp hd / (rp - hd) = 85 tokens on, at the start from 16
+    assert g.expand(86, 10 ** 6) and not g.expand(85, 10 ** 6) and g.expand(16, 0) and not g.expand(15, 0)
+    assert not Geometry(4, 64, 64).expand(10000, 0) and not Geometry(4, 256, 0).expand(999, 0)
     n = np.array([300, 3, 130, 1])
     pos0 = np.array([0, 31, 64, 99])
     row0 = np.cumsum(n) - n
@@ -194,6 +196,18 @@ def test_launch_plan_splits_portions_and_orders_rows():
                                       [431, 300, 192, 2]]
     ends = (items[:, 2] + items[:, 3]).tolist()
     assert ends == sorted(ends, reverse=True)
+
+
+def test_delta_chunk_plan():
+    from kgs.ops.delta import chunk_plan
+
+    n = np.array([3, 40, 1, 16])
+    row0 = np.array([0, 3, 43, 44])
+    p = chunk_plan(row0, n)
+    assert p["chunks"].tolist() == [[3, 16, 1, 0], [19, 16, 1, 0], [35, 8, 1, 0], [44, 16, 3, 0]]
+    assert p["cseqs"].tolist() == [[1, 0, 3, 3], [3, 3, 1, 44]]
+    assert p["step_rows"].tolist() == [0, 1, 2, 43] and p["step_seqs"].tolist() == [0, 2]
+    assert chunk_plan(row0[:1], n[:1]) == {}
 
 
 # -------------------------------------------------------------------- oracle

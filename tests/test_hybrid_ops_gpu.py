@@ -260,7 +260,7 @@ class DeltaCase:
     def run(self, portions):
         """portions: per call a list of (first row, rows, position, slot); rows of a
         call are gathered into one batch. Returns o by row."""
-        from kgs.ops.delta import RaggedSeqs, delta_forward
+        from kgs.ops.delta import RaggedSeqs, chunk_plan, delta_forward
 
         i32 = lambda a: torch.tensor(a, dtype=torch.int32, device="cuda")  # noqa: E731
         out = torch.zeros(self.z.shape[0], self.H, self.V)
@@ -269,7 +269,8 @@ class DeltaCase:
             n = [c[1] for c in call]
             row0 = [sum(n[:i]) for i in range(len(n))]
             seqs = RaggedSeqs(i32([b for b, m in enumerate(n) for _ in range(m)]), i32(row0), i32(n),
-                              i32([c[2] for c in call]), i32([c[3] for c in call]))
+                              i32([c[2] for c in call]), i32([c[3] for c in call]),
+                              **{k: i32(v.tolist()).reshape(v.shape) for k, v in chunk_plan(row0, n).items()})
             o = delta_forward(self.z[rows].cuda(), self.offs, self.a2[rows].cuda(), self.cw.cuda(), self.a_log.cuda(),
                               self.dt_bias.cuda(), self.sh, self.state, seqs)
             out[rows] = o.cpu()
@@ -302,7 +303,7 @@ def test_delta_portions_equal_the_whole(dt, shape):
     T = 41
     c = DeltaCase(*shape, T, dtype=DT[dt])
     ref, S = c.ref(0, T)
-    for cut in ([T], [1] * T, [2, 2, 1, 3, 8, 9, 16], [17, 1, 1, 2, 20]):
+    for cut in ([T], [1] * T, [2, 2, 1, 3, 8, 9, 16], [17, 1, 1, 2, 20], [32, 9], [15, 26]):
         at, calls = 0, []
         for n in cut:
             calls.append([(at, n, at, 2)])
