@@ -74,9 +74,9 @@ def split_count(ntiles: int, max_pages: int) -> int:
     return max(1, min(2 * CUS // max(1, ntiles), (max_pages + 1) // 2, 64))
 
 
-def waves_for(rows: int) -> int:
+def waves_for(rows: int, rp: int) -> int:
     """Waves (of 16 rows) per workgroup for sequences of ``rows`` (token, head) rows."""
-    return max(1, min(MAX_WAVES, (rows + 15) // 16))
+    return max(1, min(MAX_WAVES if rp <= 256 else MAX_WAVES // 2, (rows + 15) // 16))
 
 
 def latent_norm(z: torch.Tensor, oq: int, wq: torch.Tensor, qp: int, oc: int, wc: torch.Tensor | None,

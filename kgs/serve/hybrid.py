@@ -403,7 +403,7 @@ class HybridModel:
             ns = n[sel]
             q0 = np.cumsum(ns) - ns
             rows = ns * g.heads
-            waves = waves_for(int(rows.max()))
+            waves = waves_for(int(rows.max()), g.rp)
             tiles = -(-rows // (16 * waves))
             # the tiles with the longest context first
             seq = np.repeat(np.arange(len(sel)), tiles)
@@ -450,7 +450,7 @@ class HybridModel:
         f = self._fixed_seqs(nb)
         plans = {}
         for g in self.geometries:
-            waves = waves_for(g.heads)
+            waves = waves_for(g.heads, g.rp)
             tiles = -(-g.heads // (16 * waves))
             plans[g] = LatentPlan(LatentRows(
                 nt=nb, q0=f["ar"], n=f["one"], pos0=positions, bt=block_tables, tok_seq=f["ar"], tok_pos=positions,

@@ -22,7 +22,7 @@
 //   S = diag(e^(b_C)) S_0 + K^^T U   K^_j = k_j e^(b_C - b_j)
 //   chunk_prep  everything that does not need S_0, one workgroup per (chunk, head);
 //   chunk_scan  the three products with the state per chunk, on fp32 MFMAs.
-// tails updates the convolution tails, out applies the per-head norm and gate.
+// Both scans also update the convolution tails; out applies the per-head norm and gate.
 //
 // Everything after the convolutions is fp32. K is padded to KP, a multiple of 32,
 // in q, k, log g and the state (pads are zero and stay zero). The state is stored
@@ -42,12 +42,6 @@ __device__ __forceinline__ void st(T* p, float v) {
   if constexpr (sizeof(T) == 2) *(unsigned short*)p = f2bf(v);
   else *p = v;
 }
-__device__ __forceinline__ float wave_sum(float v) {
-#pragma unroll
-  for (int m = 8; m >= 1; m >>= 1) v += __shfl_xor(v, m, 64);
-  return xor32_sum(xor16_sum(v));
-}
-
 struct Args {
   // inputs of prep
   const void* z;   // [T, ldz]: q (G K), k (G K), v (H V) channels at oq, ok, ov; step sizes (H) at ob
@@ -113,32 +107,84 @@ __device__ __forceinline__ void ldn(const T* p, float (&v)[N]) {
   }
 }
 
-// channels c .. c + N - 1 (column col of z) of row t after the convolution and silu
+// channels c .. c + N - 1 (column col of z) of row src of the sequence that starts at
+// row r0 (position p0): rows ahead of it come from the pool's tail
 template <typename T, int N>
+__device__ __forceinline__ void conv_in(const Args& a, long src, int c, int col, int r0, int p0, long slot,
+                                        float (&x)[N]) {
+#pragma unroll
+  for (int i = 0; i < N; ++i) x[i] = 0.f;
+  if (src >= r0) ldn((const T*)a.z + src * a.ldz + col, x);
+  else if (p0 > 0) ldn(a.conv + (slot * (a.taps - 1) + (src - r0 + a.taps - 1)) * a.C + c, x);
+}
+
+// ... of row t after the convolution and silu. TAPS 0: any number.
+template <typename T, int N, int TAPS>
 __device__ __forceinline__ void conv_silu(const Args& a, long t, int c, int col, int r0, int p0, long slot,
                                           float (&y)[N]) {
   float s[N] = {};
-#pragma unroll 4
-  for (int j = 0; j < a.taps; ++j) {
-    const long src = t - (a.taps - 1) + j;
-    float x[N] = {};
-    if (src >= r0) ldn((const T*)a.z + src * a.ldz + col, x);
-    else if (p0 > 0) ldn(a.conv + (slot * (a.taps - 1) + (src - r0 + a.taps - 1)) * a.C + c, x);
+  if constexpr (TAPS > 0) {
+    float x[TAPS][N];  // all loads are in flight before the first use
 #pragma unroll
-    for (int i = 0; i < N; ++i) s[i] = __builtin_fmaf(a.cw[(long)j * a.C + c + i], x[i], s[i]);
+    for (int j = 0; j < TAPS; ++j) conv_in<T, N>(a, t - (TAPS - 1) + j, c, col, r0, p0, slot, x[j]);
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+      for (int i = 0; i < N; ++i) s[i] = __builtin_fmaf(a.cw[(long)j * a.C + c + i], x[j][i], s[i]);
+  } else {
+    for (int j = 0; j < a.taps; ++j) {
+      float x[N];
+      conv_in<T, N>(a, t - (a.taps - 1) + j, c, col, r0, p0, slot, x);
+#pragma unroll
+      for (int i = 0; i < N; ++i) s[i] = __builtin_fmaf(a.cw[(long)j * a.C + c + i], x[i], s[i]);
+    }
   }
 #pragma unroll
   for (int i = 0; i < N; ++i) y[i] = s[i] * sigm<sizeof(T) == 2>(s[i]);
 }
 
-// Where a token's prepared values go: global rows or a chunk's LDS
+// Rows t0 .. t0 + 15 (n of them real) of channels c .. c + N - 1, each input row read once
+template <typename T, int N, int TAPS, class F>
+__device__ __forceinline__ void conv_rows(const Args& a, long t0, int n, int c, int col, int r0, int p0, long slot,
+                                          F store) {
+  if constexpr (TAPS > 0) {
+    float x[16 + TAPS - 1][N], w[TAPS][N];
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) ldn(a.cw + (long)j * a.C + c, w[j]);
+#pragma unroll
+    for (int j = 0; j < 16 + TAPS - 1; ++j) {
+#pragma unroll
+      for (int i = 0; i < N; ++i) x[j][i] = 0.f;
+      if (j - (TAPS - 1) < n) conv_in<T, N>(a, t0 - (TAPS - 1) + j, c, col, r0, p0, slot, x[j]);
+    }
+#pragma unroll
+    for (int t = 0; t < 16; ++t) {
+      float y[N] = {};
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+        for (int i = 0; i < N; ++i) y[i] = __builtin_fmaf(w[j][i], x[t + j][i], y[i]);
+#pragma unroll
+      for (int i = 0; i < N; ++i) y[i] = t < n ? y[i] * sigm<sizeof(T) == 2>(y[i]) : 0.f;
+      store(t, y);
+    }
+  } else {
+    for (int t = 0; t < 16; ++t) {
+      float y[N] = {};
+      if (t < n) conv_silu<T, N, 0>(a, t0 + t, c, col, r0, p0, slot, y);
+      store(t, y);
+    }
+  }
+}
+
+// Where a token's prepared values go
 struct Dst {
-  float *q, *k, *qk;         // [KP], [KP], one value (or null)
+  float *q, *k, *qk;         // [KP], [KP], one value
   float *v, *lg, *beta;      // of value head h: v + (h - h0) * V, lg + (h - h0) * KP, beta + (h - h0)
 };
 
 // One wave: a token's q / k head gh and the value heads h0 .. h0 + nh - 1 that read it
-template <typename T, int N>
+template <typename T, int N, int TAPS>
 __device__ __forceinline__ void prep_token(const Args& a, long t, int gh, int h0, int nh, int r0, int p0, long slot,
                                            const Dst& d) {
   constexpr bool FAST = sizeof(T) == 2;
@@ -152,8 +198,8 @@ __device__ __forceinline__ void prep_token(const Args& a, long t, int gh, int h0
     for (int x = 0; x < N; ++x) q[e][x] = k[e][x] = 0.f;
     if (i < K) {
       const int c = gh * K + i;
-      conv_silu<T, N>(a, t, c, a.oq + c, r0, p0, slot, q[e]);
-      conv_silu<T, N>(a, t, a.G * K + c, a.ok + c, r0, p0, slot, k[e]);
+      conv_silu<T, N, TAPS>(a, t, c, a.oq + c, r0, p0, slot, q[e]);
+      conv_silu<T, N, TAPS>(a, t, a.G * K + c, a.ok + c, r0, p0, slot, k[e]);
 #pragma unroll
       for (int x = 0; x < N; ++x) {
         sq = __builtin_fmaf(q[e][x], q[e][x], sq);
@@ -165,10 +211,8 @@ __device__ __forceinline__ void prep_token(const Args& a, long t, int gh, int h0
   sq = wave_sum(sq);
   sk = wave_sum(sk);
   const float rq = 1.0f / sqrtf(sq + 1e-6f) / sqrtf((float)K), rk = 1.0f / sqrtf(sk + 1e-6f);
-  if (d.qk) {
-    sqk = wave_sum(sqk);
-    if (lane == 0) *d.qk = sqk * rq * rk;
-  }
+  sqk = wave_sum(sqk);
+  if (lane == 0) *d.qk = sqk * rq * rk;
 #pragma unroll
   for (int e = 0; e < E; ++e) {
     const int i = N * (lane + 64 * e);
@@ -184,7 +228,7 @@ __device__ __forceinline__ void prep_token(const Args& a, long t, int gh, int h0
     for (int i = N * lane; i < V; i += 64 * N) {
       float v[N];
       const int c = h * V + i;
-      conv_silu<T, N>(a, t, 2 * a.G * K + c, a.ov + c, r0, p0, slot, v);
+      conv_silu<T, N, TAPS>(a, t, 2 * a.G * K + c, a.ov + c, r0, p0, slot, v);
 #pragma unroll
       for (int x = 0; x < N; ++x) d.v[(h - h0) * V + i + x] = v[x];
     }
@@ -206,14 +250,14 @@ __device__ __forceinline__ void prep_token(const Args& a, long t, int gh, int h0
 
 // ----------------------------------------------------------------------- prep
 // one wave per (row of a stepped sequence, q / k head)
-template <typename T, int N>
+template <typename T, int N, int TAPS>
 __global__ __launch_bounds__(256) void prep(Args a) {
   const long unit = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (unit >= (long)a.nrows * a.G) return;
   const int gh = (int)(unit % a.G), rep = a.H / a.G;
   const long t = a.rows ? a.rows[unit / a.G] : unit / a.G;
   const int b = a.row_seq[t];
-  prep_token<T, N>(a, t, gh, gh * rep, rep, a.row0[b], a.pos0[b], a.slot[b],
+  prep_token<T, N, TAPS>(a, t, gh, gh * rep, rep, a.row0[b], a.pos0[b], a.slot[b],
                    Dst{a.q + (t * a.G + gh) * a.KP, a.k + (t * a.G + gh) * a.KP, a.qk + t * a.G + gh,
                        a.v + (t * a.H + gh * rep) * a.V, a.lg + (t * a.H + gh * rep) * a.KP, a.beta + t * a.H + gh * rep});
 }
@@ -226,10 +270,31 @@ __device__ __forceinline__ float xor8_sum(float x) {  // row_ror:8 within 16 lan
   return x + __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x128, 0xf, 0xf, false));
 }
 
+// The convolution tails after the call, the last taps - 1 inputs of the sequence:
+// workgroup `part` of `parts` of it takes its share of the channels. Runs in the
+// kernel after the one that reads the old tails.
+template <typename T>
+__device__ __forceinline__ void conv_tail(const Args& a, int b, int part, int parts) {
+  const int r0 = a.row0[b], n = a.n[b], p0 = a.pos0[b], m = a.taps - 1;
+  const long slot = a.slot[b];
+  for (int c = part * 256 + threadIdx.x; c < a.C; c += parts * 256) {
+    const int GK = a.G * a.K;
+    const int col = c < GK ? a.oq + c : c < 2 * GK ? a.ok + c - GK : a.ov + c - 2 * GK;
+    for (int j = 0; j < m; ++j) {  // ascending: reads are ahead of the writes
+      const int src = n + j;       // index in (old tail, this portion)
+      float x;
+      if (src < m) x = p0 > 0 ? a.conv[(slot * m + src) * a.C + c] : 0.f;
+      else x = ld((const T*)a.z + (long)(r0 + src - m) * a.ldz + col);
+      a.conv[(slot * m + j) * a.C + c] = x;
+    }
+  }
+}
+
+
 // A wave owns 8 columns of one head's state: lane (rg = lane >> 3, col = lane & 7)
 // holds rows 32 i + 4 rg + j of its column, so the two dot products of a token
 // (with k and with q, the latter completed by (q . k) u) are one 3-step exchange.
-template <int NI>
+template <typename T, int NI>
 __global__ __launch_bounds__(256) void scan(Args a) {
   constexpr int KP = 32 * NI;
   __shared__ __attribute__((aligned(16))) float sq[TB][KP], sk[TB][KP], sg[TB][KP];
@@ -295,81 +360,159 @@ __global__ __launch_bounds__(256) void scan(Args a) {
 #pragma unroll
     for (int i = 0; i < NI; ++i) *(f32x4*)(Sp + 32 * i) = S[i];
   }
+  conv_tail<T>(a, b, h * gridDim.x + blockIdx.x, H * gridDim.x);
 }
 
 // --------------------------------------------------------------------- chunks
 constexpr int CH = 16;  // tokens per chunk
 
-__host__ __device__ __forceinline__ int chunk_ld(int n) { return n + 4; }  // LDS row pitch
+// LDS row pitch: two rows apart are 32 banks apart for n a multiple of 32
+__host__ __device__ __forceinline__ int chunk_ld(int n) { return n + 16; }
 
 // one workgroup per (chunk, head)
-template <typename T, int N>
+template <typename T, int N, int TAPS>
 __global__ __launch_bounds__(256, 4) void chunk_prep(Args a) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
-  __shared__ __attribute__((aligned(16))) float sA[CH][CH + 4], sT[CH][CH + 4], sbeta[CH];
+  __shared__ __attribute__((aligned(16))) float sA[CH][CH + 4], sT[CH][CH + 4], sbeta[CH], srq[CH], srk[CH];
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
   const int KP = a.KP, V = a.V, H = a.H, ldk = chunk_ld(KP), ldv = chunk_ld(V);
   float *sq = sm, *sk = sq + CH * ldk, *sb = sk + CH * ldk, *sv = sb + CH * ldk;
-  const int h = blockIdx.x % H;
-  const long ck = blockIdx.x / H;
+  const int ck = __builtin_amdgcn_readfirstlane(blockIdx.x / H), h = blockIdx.x - ck * H;
   const int4 it = a.chunks[ck];  // first row, rows, sequence
-  const int b = it.z, n = it.y, gh = h / (H / a.G);
-  for (int i = w; i < CH; i += 4) {
-    if (i < n) {
-      prep_token<T, N>(a, it.x + i, gh, h, 1, a.row0[b], a.pos0[b], a.slot[b],
-                       Dst{sq + i * ldk, sk + i * ldk, nullptr, sv + i * ldv, sb + i * ldk, sbeta + i});
-    } else {  // past the end: no write, no decay
-      for (int c = lane; c < KP; c += 64) sq[i * ldk + c] = sk[i * ldk + c] = sb[i * ldk + c] = 0.f;
-      for (int c = lane; c < V; c += 64) sv[i * ldv + c] = 0.f;
-      if (lane == 0) sbeta[i] = 0.f;
-    }
-  }
-  __syncthreads();
-  for (int c = tid; c < KP; c += 256) {  // b, in log2 units
-    float s = 0.f;
+  const int b = it.z, n = it.y, gh = __builtin_amdgcn_readfirstlane(h / (H / a.G));
+  const int r0 = a.row0[b], p0 = a.pos0[b], K = a.K;
+  const long slot = a.slot[b], t0 = it.x;
+  constexpr bool FAST = sizeof(T) == 2;
+  // threads by channel groups of N: q, k, v convolutions, then the decays
+  const int nk = KP / N, nv = (V + N - 1) / N;
+  for (int u = tid; u < 3 * nk + nv; u += 256) {
+    if (u < 2 * nk) {
+      const bool isk = u >= nk;
+      const int c = N * (isk ? u - nk : u);
+      float* dst = (isk ? sk : sq) + c;
+      auto put = [&](int t, const float (&y)[N]) {
 #pragma unroll
-    for (int i = 0; i < CH; ++i) {
-      s += sb[i * ldk + c];
-      sb[i * ldk + c] = s * LOG2E;
+        for (int i = 0; i < N; ++i) dst[t * ldk + i] = y[i];
+      };
+      const int ch = (isk ? a.G * K : 0) + gh * K + c, col = (isk ? a.ok : a.oq) + gh * K + c;
+      if (c < K) conv_rows<T, N, TAPS>(a, t0, n, ch, col, r0, p0, slot, put);
+      else
+        for (int t = 0; t < CH; ++t) put(t, {});
+    } else if (u < 2 * nk + nv) {
+      const int c = N * (u - 2 * nk);
+      conv_rows<T, N, TAPS>(a, t0, n, 2 * a.G * K + h * V + c, a.ov + h * V + c, r0, p0, slot,
+                            [&](int t, const float (&y)[N]) {
+#pragma unroll
+                              for (int i = 0; i < N; ++i) sv[t * ldv + c + i] = y[i];
+                            });
+    } else {
+      const int c = N * (u - 2 * nk - nv);
+      const float A = -expf(a.A_log[h]) * LOG2E;  // b: sums of log decays, in log2 units
+      float s[N] = {}, dt[N] = {};
+      if (c < K) ldn(a.dt_bias + h * K + c, dt);
+      float x[CH][N];
+#pragma unroll
+      for (int t = 0; t < CH; ++t) {
+#pragma unroll
+        for (int i = 0; i < N; ++i) x[t][i] = 0.f;
+        if (t < n && c < K) ldn((const T*)a.a2 + (t0 + t) * a.lda + h * K + c, x[t]);
+      }
+#pragma unroll
+      for (int t = 0; t < CH; ++t)
+#pragma unroll
+        for (int i = 0; i < N; ++i) {
+          if (t < n && c < K) s[i] += A * softplus<FAST>(x[t][i] + dt[i]);
+          sb[t * ldk + c + i] = s[i];
+        }
+    }
+  }
+  if (tid < CH) sbeta[tid] = tid < n ? sigm<FAST>(ld((const T*)a.z + (t0 + tid) * a.ldz + a.ob + h)) : 0.f;
+  __syncthreads();
+  for (int i = w; i < CH; i += 4) {  // unit norms, as factors
+    float ssq = 0.f, ssk = 0.f, sqk = 0.f;
+    for (int c = lane; c < KP; c += 64) {
+      const float q = sq[i * ldk + c], k = sk[i * ldk + c];
+      ssq = __builtin_fmaf(q, q, ssq);
+      ssk = __builtin_fmaf(k, k, ssk);
+      sqk = __builtin_fmaf(q, k, sqk);
+    }
+    ssq = wave_sum(ssq);
+    ssk = wave_sum(ssk);
+    sqk = wave_sum(sqk);
+    if (lane == 0) {
+      const float rq = 1.0f / sqrtf(ssq + 1e-6f) / sqrtf((float)K), rk = 1.0f / sqrtf(ssk + 1e-6f);
+      srq[i] = rq;
+      srk[i] = rk;
+      a.cP[((long)ck * H + h) * CH * CH + i * CH + i] = sqk * rq * rk;  // P's diagonal has no decay
     }
   }
   __syncthreads();
-  const long base = ck * H + h;
+  const long base = (long)ck * H + h;
   float* P = a.cP + base * CH * CH;
-  if (tid < 240) {  // pair (i, j), j < i, each over half of the channels
-    const int p = tid >> 1, half = tid & 1;
-    int i = (int)((1.0f + sqrtf(1.0f + 8.0f * p)) * 0.5f);
-    while (i * (i - 1) / 2 > p) --i;
-    while ((i + 1) * i / 2 <= p) ++i;
-    const int j = p - i * (i - 1) / 2;
-    float sa = 0.f, sp = 0.f;
-    for (int c = half * (KP / 2); c < (half + 1) * (KP / 2); c += 4) {
-      const f32x4 ki = *(const f32x4*)(sk + i * ldk + c), qi = *(const f32x4*)(sq + i * ldk + c);
-      const f32x4 bi = *(const f32x4*)(sb + i * ldk + c), kj = *(const f32x4*)(sk + j * ldk + c);
-      const f32x4 bj = *(const f32x4*)(sb + j * ldk + c);
+  // A and P in 2 x 2 tiles of (i, j): 28 tiles below the diagonal over 8 slices of the
+  // channels each, and the 8 pairs (2 x + 1, 2 x) on it over 4 slices
+  if (tid < 224) {
+    const int blk = tid >> 3, sl = tid & 7;
+    int bi = 1;
+    while ((bi + 1) * bi / 2 <= blk) ++bi;
+    const int i = 2 * bi, j = 2 * (blk - bi * (bi - 1) / 2);
+    float sa[2][2] = {}, sp[2][2] = {};
+    for (int c = 4 * sl; c < KP; c += 32) {
+      f32x4 ki[2], qi[2], xi[2], kj[2], xj[2];
 #pragma unroll
-      for (int x = 0; x < 4; ++x) {
-        const float y = kj[x] * __builtin_amdgcn_exp2f(bi[x] - bj[x]);
-        sa = __builtin_fmaf(ki[x], y, sa);
-        sp = __builtin_fmaf(qi[x], y, sp);
+      for (int y = 0; y < 2; ++y) {
+        ki[y] = *(const f32x4*)(sk + (i + y) * ldk + c);
+        qi[y] = *(const f32x4*)(sq + (i + y) * ldk + c);
+        xi[y] = *(const f32x4*)(sb + (i + y) * ldk + c);
+        kj[y] = *(const f32x4*)(sk + (j + y) * ldk + c);
+        xj[y] = *(const f32x4*)(sb + (j + y) * ldk + c);
+      }
+#pragma unroll
+      for (int y = 0; y < 2; ++y)
+#pragma unroll
+        for (int z = 0; z < 2; ++z)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            const float v = kj[z][e] * __builtin_amdgcn_exp2f(xi[y][e] - xj[z][e]);
+            sa[y][z] = __builtin_fmaf(ki[y][e], v, sa[y][z]);
+            sp[y][z] = __builtin_fmaf(qi[y][e], v, sp[y][z]);
+          }
+    }
+#pragma unroll
+    for (int y = 0; y < 2; ++y)
+#pragma unroll
+      for (int z = 0; z < 2; ++z) {
+        const float ra = sum8(sa[y][z]), rp = sum8(sp[y][z]);
+        if (sl == 2 * y + z) {
+          const float f = srk[j + z];
+          sA[i + y][j + z] = ra * srk[i + y] * f;
+          P[(i + y) * CH + j + z] = rp * srq[i + y] * f;
+          P[(j + z) * CH + i + y] = 0.f;
+        }
+      }
+  } else {
+    const int j = 2 * ((tid - 224) >> 2), i = j + 1, sl = tid & 3;
+    float sa = 0.f, sp = 0.f;
+    for (int c = 4 * sl; c < KP; c += 16) {
+      const f32x4 ki = *(const f32x4*)(sk + i * ldk + c), qi = *(const f32x4*)(sq + i * ldk + c);
+      const f32x4 xi = *(const f32x4*)(sb + i * ldk + c), kj = *(const f32x4*)(sk + j * ldk + c);
+      const f32x4 xj = *(const f32x4*)(sb + j * ldk + c);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float v = kj[e] * __builtin_amdgcn_exp2f(xi[e] - xj[e]);
+        sa = __builtin_fmaf(ki[e], v, sa);
+        sp = __builtin_fmaf(qi[e], v, sp);
       }
     }
-    sa += __shfl_xor(sa, 1, 64);
-    sp += __shfl_xor(sp, 1, 64);
-    if (half == 0) {
-      sA[i][j] = sa;
-      P[i * CH + j] = sp;
+    sa += dpp_move<0xB1>(sa);
+    sp += dpp_move<0xB1>(sp);
+    sa += dpp_move<0x4E>(sa);
+    sp += dpp_move<0x4E>(sp);
+    if (sl == 0) {
+      sA[i][j] = sa * srk[i] * srk[j];
+      P[i * CH + j] = sp * srq[i] * srk[j];
       P[j * CH + i] = 0.f;
     }
-  } else {
-    const int i = tid - 240;
-    float sp = 0.f;
-    for (int c = 0; c < KP; c += 4) {
-      const f32x4 ki = *(const f32x4*)(sk + i * ldk + c), qi = *(const f32x4*)(sq + i * ldk + c);
-#pragma unroll
-      for (int x = 0; x < 4; ++x) sp = __builtin_fmaf(qi[x], ki[x], sp);
-    }
-    P[i * CH + i] = sp;
   }
   __syncthreads();
   if (tid < CH) {  // column tid of T by forward substitution
@@ -394,16 +537,16 @@ __global__ __launch_bounds__(256, 4) void chunk_prep(Args a) {
       const float bc = sb[(CH - 1) * ldk + c];
 #pragma unroll
       for (int i = 0; i < CH; ++i) {
-        const float bi = sb[i * ldk + c], k = sk[i * ldk + c], e = __builtin_amdgcn_exp2f(bi);
+        const float bi = sb[i * ldk + c], k = sk[i * ldk + c] * srk[i], e = __builtin_amdgcn_exp2f(bi);
         x[i] = k * e;
-        Q[i * KP] = sq[i * ldk + c] * e;
+        Q[i * KP] = sq[i * ldk + c] * srq[i] * e;
       }
 #pragma unroll
       for (int i = 0; i < CH; i += 4) {
         f32x4 v;
 #pragma unroll
         for (int y = 0; y < 4; ++y)
-          v[y] = sk[(i + y) * ldk + c] * __builtin_amdgcn_exp2f(bc - sb[(i + y) * ldk + c]);
+          v[y] = sk[(i + y) * ldk + c] * srk[i + y] * __builtin_amdgcn_exp2f(bc - sb[(i + y) * ldk + c]);
         *(f32x4*)(Kt + i) = v;
       }
       a.cE[base * KP + c] = __builtin_amdgcn_exp2f(bc);
@@ -428,115 +571,161 @@ __global__ __launch_bounds__(256, 4) void chunk_prep(Args a) {
   }
 }
 
-// One workgroup per (sequence, head, 16 state columns); wave w holds the state's
+// One workgroup per (sequence, head, 16 NS state columns); wave w holds the state's
 // 16-row tiles w, w + 4, ... as MFMA accumulators: lane (g = lane >> 4, n = lane & 15)
-// has rows 4 g + r of a tile for column n. Register r of an accumulator is at the
-// same time the B operand of a v_mfma_f32_16x16x4_f32 whose four contraction
-// indices are 4 g + r, so state and U feed the products without moving; the A
-// operands are read as float4s in that order. The waves' partial products over
-// their rows meet in LDS, one barrier per chunk.
-template <int MT>
+// has rows 4 g + r of a tile for columns n, 16 + n, .... Register r of an accumulator
+// is at the same time the B operand of a v_mfma_f32_16x16x4_f32 whose four
+// contraction indices are 4 g + r, so state and U feed the products without
+// moving; the A operands are read as float4s in that order. The waves' partial
+// products over their rows meet in LDS, one barrier per chunk.
+// NS 2 reads the A operands half as often; NS 1 spreads few heads over more CUs.
+template <typename T, int MT, int NS>
 __global__ __launch_bounds__(256) void chunk_scan(Args a) {
-  __shared__ f32x4 part[2][2][4][64];  // [buffer][U | O][wave][lane]
+  __shared__ f32x4 part[2][2][NS][4][64];  // [buffer][U | O][tile][wave][lane]
   const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int l16 = lane & 15, g = lane >> 4;
-  const int KP = a.KP, V = a.V, H = a.H, nslab = (V + 15) / 16, ntile = KP / 16;
+  const int KP = a.KP, V = a.V, H = a.H, nslab = (V + 16 * NS - 1) / (16 * NS), ntile = KP / 16;
   const int lid = xcd_remap(blockIdx.x, gridDim.x);  // a head's slabs share an XCD's L2
-  const int slab = lid % nslab, h = lid / nslab % H;
-  const int4 sq = a.cseqs[lid / nslab / H];  // sequence, first chunk, chunks, first row
-  const int b = sq.x, n = a.n[b], col = slab * 16 + l16;
-  const bool live = col < V;
-  float* Sp = a.S + (((long)a.slot[b] * H + h) * V + (live ? col : 0)) * KP + 4 * g;
-  f32x4 S[MT];
+  // (divisions run on the vector unit: back to scalars, so that bases stay uniform)
+  const int sh = __builtin_amdgcn_readfirstlane(lid / nslab), slab = __builtin_amdgcn_readfirstlane(lid - sh * nslab);
+  const int si = __builtin_amdgcn_readfirstlane(sh / H), h = sh - si * H;
+  const int4 sq = a.cseqs[si];  // sequence, first chunk, chunks, first row
+  const int b = sq.x, n = a.n[b];
+  int col[NS];
+  bool live[NS];
+  f32x4 S[MT][NS];
+  float* Sh = a.S + ((long)a.slot[b] * H + h) * V * KP + 4 * g;
 #pragma unroll
-  for (int m = 0; m < MT; ++m) {
-    const int tile = w + 4 * m;
-    S[m] = tile < ntile && a.pos0[b] > 0 && live ? *(const f32x4*)(Sp + 16 * tile) : f32x4{};
-  }
-  struct Frag {
-    f32x4 W[MT], Q[MT], K[MT], E[MT], U, P;
-  };
-  auto fetch = [&](int c, Frag& f) {
-    const long base = (long)(sq.y + c) * H + h;
+  for (int s = 0; s < NS; ++s) {
+    col[s] = (slab * NS + s) * 16 + l16;
+    live[s] = col[s] < V;
+    col[s] = min(col[s], V - 1);
 #pragma unroll
     for (int m = 0; m < MT; ++m) {
       const int tile = w + 4 * m;
-      if (tile < ntile) {
-        f.W[m] = *(const f32x4*)(a.cW + (base * CH + l16) * KP + 16 * tile + 4 * g);
-        f.Q[m] = *(const f32x4*)(a.cQ + (base * CH + l16) * KP + 16 * tile + 4 * g);
-        f.K[m] = *(const f32x4*)(a.cK + (base * KP + 16 * tile + l16) * CH + 4 * g);
-        f.E[m] = *(const f32x4*)(a.cE + base * KP + 16 * tile + 4 * g);
-      } else {
-        f.W[m] = f.Q[m] = f.K[m] = f.E[m] = f32x4{};
-      }
+      S[m][s] = tile < ntile && a.pos0[b] > 0 ? *(const f32x4*)(Sh + (long)col[s] * KP + 16 * tile) : f32x4{};
     }
-#pragma unroll
-    for (int r = 0; r < 4; ++r) f.U[r] = live ? a.cU[(base * CH + 4 * g + r) * V + col] : 0.f;
-    f.P = *(const f32x4*)(a.cP + (base * CH + l16) * CH + 4 * g);
+  }
+  struct Frag {
+    f32x4 W[MT], Q[MT], K[MT], E[MT], U[NS], P;
   };
-  Frag f;
-  fetch(0, f);
-  for (int c = 0; c < sq.z; ++c) {
-    Frag nx;
-    if (c + 1 < sq.z) fetch(c + 1, nx);
-    f32x4 pu = f32x4{}, po = f32x4{};
+  // Loads without conditions (a wave's rows past the last tile repeat it, columns
+  // past V the last one), so that the number in flight is known at every wait;
+  // a uniform base and 32-bit lane offsets.
+  unsigned lw[MT], lk[MT], le[MT], lu[NS];
 #pragma unroll
-    for (int m = 0; m < MT; ++m)
+  for (int m = 0; m < MT; ++m) {
+    const int tile = min(w + 4 * m, ntile - 1);
+    lw[m] = l16 * KP + 16 * tile + 4 * g;
+    lk[m] = (16 * tile + l16) * CH + 4 * g;
+    le[m] = 16 * tile + 4 * g;
+  }
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        pu = __builtin_amdgcn_mfma_f32_16x16x4f32(f.W[m][r], S[m][r], pu, 0, 0, 0);
-        po = __builtin_amdgcn_mfma_f32_16x16x4f32(f.Q[m][r], S[m][r], po, 0, 0, 0);
-      }
-    const int buf = c & 1;
-    part[buf][0][w][lane] = pu;
-    part[buf][1][w][lane] = po;
-    __syncthreads();
-    const f32x4 U = f.U - (part[buf][0][0][lane] + part[buf][0][1][lane] + part[buf][0][2][lane] + part[buf][0][3][lane]);
+  for (int s = 0; s < NS; ++s) lu[s] = 4 * g * V + col[s];
+  const unsigned lp = l16 * CH + 4 * g;
+  auto fetch = [&](int c, Frag& f) {
+    const long base = (long)(sq.y + c) * H + h;
+    const float *W = a.cW + base * CH * KP, *Q = a.cQ + base * CH * KP, *K = a.cK + base * CH * KP;
+    const float *E = a.cE + base * KP, *U = a.cU + base * CH * V, *P = a.cP + base * CH * CH;
 #pragma unroll
     for (int m = 0; m < MT; ++m) {
-      S[m] *= f.E[m];
-#pragma unroll
-      for (int r = 0; r < 4; ++r) S[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.K[m][r], U[r], S[m], 0, 0, 0);
+      f.W[m] = *(const f32x4*)(W + lw[m]);
+      f.Q[m] = *(const f32x4*)(Q + lw[m]);
+      f.K[m] = *(const f32x4*)(K + lk[m]);
+      f.E[m] = *(const f32x4*)(E + le[m]);
     }
-    if (w == (c & 3)) {
-      f32x4 O = part[buf][1][0][lane] + part[buf][1][1][lane] + part[buf][1][2][lane] + part[buf][1][3][lane];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) O = __builtin_amdgcn_mfma_f32_16x16x4f32(f.P[r], U[r], O, 0, 0, 0);
+    for (int s = 0; s < NS; ++s)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int t = CH * c + 4 * g + r;
-        if (t < n && live) a.o[((long)(sq.w + t) * H + h) * V + col] = O[r];
-      }
-    }
-    f = nx;
-  }
-  if (live) {
+      for (int r = 0; r < 4; ++r) f.U[s][r] = (U + (unsigned)(r * V))[lu[s]];
+    f.P = *(const f32x4*)(P + lp);
+    __builtin_amdgcn_sched_barrier(0);  // chunks are loaded in order: their waits are counted in it
+  };
+  // a ring of RING chunks' operands in registers: loads run RING - 1 chunks ahead
+  constexpr int RING = MT == 1 || (MT == 2 && NS == 1) ? 4 : MT == 2 ? 3 : 2;
+  auto step = [&](int c, Frag& f) __attribute__((always_inline)) {
+    f32x4 pu[NS], po[NS];
+#pragma unroll
+    for (int s = 0; s < NS; ++s) pu[s] = po[s] = f32x4{};
 #pragma unroll
     for (int m = 0; m < MT; ++m)
-      if (w + 4 * m < ntile) *(f32x4*)(Sp + 16 * (w + 4 * m)) = S[m];
-  }
-}
-
-// ---------------------------------------------------------------------- tails
-// The convolution tails after the call: the last taps - 1 inputs of the sequence.
-template <typename T>
-__global__ __launch_bounds__(256) void tails(Args a) {
-  const int b = blockIdx.y;
-  const int r0 = a.row0[b], n = a.n[b], p0 = a.pos0[b], m = a.taps - 1;
-  const long slot = a.slot[b];
-  for (int c = blockIdx.x * 256 + threadIdx.x; c < a.C; c += gridDim.x * 256) {
-    const int GK = a.G * a.K;
-    const int col = c < GK ? a.oq + c : c < 2 * GK ? a.ok + c - GK : a.ov + c - 2 * GK;
-    for (int j = 0; j < m; ++j) {  // ascending: reads are ahead of the writes
-      const int src = n + j;       // index in (old tail, this portion)
-      float x;
-      if (src < m) x = p0 > 0 ? a.conv[(slot * m + src) * a.C + c] : 0.f;
-      else x = ld((const T*)a.z + (long)(r0 + src - m) * a.ldz + col);
-      a.conv[(slot * m + j) * a.C + c] = x;
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+#pragma unroll
+        for (int s = 0; s < NS; ++s) {
+          pu[s] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.W[m][r], S[m][s][r], pu[s], 0, 0, 0);
+          po[s] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.Q[m][r], S[m][s][r], po[s], 0, 0, 0);
+        }
+    const int buf = c & 1;
+#pragma unroll
+    for (int s = 0; s < NS; ++s) {
+      part[buf][0][s][w][lane] = pu[s];
+      part[buf][1][s][w][lane] = po[s];
     }
+    __syncthreads();
+    f32x4 U[NS];
+#pragma unroll
+    for (int s = 0; s < NS; ++s)
+      U[s] = f.U[s] - (part[buf][0][s][0][lane] + part[buf][0][s][1][lane] + part[buf][0][s][2][lane] +
+                       part[buf][0][s][3][lane]);
+#pragma unroll
+    for (int m = 0; m < MT; ++m)
+#pragma unroll
+      for (int s = 0; s < NS; ++s) S[m][s] *= f.E[m];
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+#pragma unroll
+      for (int m = 0; m < MT; ++m)
+#pragma unroll
+        for (int s = 0; s < NS; ++s)
+          S[m][s] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.K[m][r], U[s][r], S[m][s], 0, 0, 0);
+#pragma unroll
+    for (int m = 0; m < MT; ++m)
+      if (w + 4 * m >= ntile) {  // no such rows
+#pragma unroll
+        for (int s = 0; s < NS; ++s) S[m][s] = f32x4{};
+      }
+#pragma unroll
+    for (int s = 0; s < NS; ++s)
+      if (w == ((c + 2 * s) & 3)) {
+        f32x4 O = part[buf][1][s][0][lane] + part[buf][1][s][1][lane] + part[buf][1][s][2][lane] +
+                  part[buf][1][s][3][lane];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) O = __builtin_amdgcn_mfma_f32_16x16x4f32(f.P[r], U[s][r], O, 0, 0, 0);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int t = CH * c + 4 * g + r;
+          if (t < n && live[s]) a.o[((long)(sq.w + t) * H + h) * V + col[s]] = O[r];
+        }
+      }
+    fetch(min(c + RING, sq.z - 1), f);
+  };
+  Frag f0, f1, f2, f3;
+  fetch(0, f0);
+  fetch(min(1, sq.z - 1), f1);
+  if constexpr (RING > 2) fetch(min(2, sq.z - 1), f2);
+  if constexpr (RING > 3) fetch(min(3, sq.z - 1), f3);
+  int c = 0;
+  for (; c + RING <= sq.z; c += RING) {
+    step(c, f0);
+    step(c + 1, f1);
+    if constexpr (RING > 2) step(c + 2, f2);
+    if constexpr (RING > 3) step(c + 3, f3);
   }
+  if (c < sq.z) step(c, f0);
+  if constexpr (RING > 2)
+    if (c + 1 < sq.z) step(c + 1, f1);
+  if constexpr (RING > 3)
+    if (c + 2 < sq.z) step(c + 2, f2);
+#pragma unroll
+  for (int s = 0; s < NS; ++s)
+    if (live[s]) {
+#pragma unroll
+      for (int m = 0; m < MT; ++m)
+        if (w + 4 * m < ntile) *(f32x4*)(Sh + (long)col[s] * KP + 16 * (w + 4 * m)) = S[m][s];
+    }
+  conv_tail<T>(a, b, h * nslab + slab, H * nslab);
 }
-
 
 // ------------------------------------------------------------------------ out
 struct OutArgs {
@@ -580,41 +769,53 @@ __global__ __launch_bounds__(256) void out(OutArgs a) {
   for (int i = lane; i < V; i += 64) st(y + i, o[i] * r * a.w[i] * sigm<FAST>(ld(gate + i)));
 }
 
-template <typename T, int N>
+template <typename T, int NS>
+static void run_chunk_scan(const Args& a, hipStream_t s) {
+  const dim3 grid((unsigned)((a.V + 16 * NS - 1) / (16 * NS) * a.H * a.ncseqs));
+  switch ((a.KP + 63) / 64) {
+    case 1: hipLaunchKernelGGL((chunk_scan<T, 1, NS>), grid, dim3(256), 0, s, a); break;
+    case 2: hipLaunchKernelGGL((chunk_scan<T, 2, NS>), grid, dim3(256), 0, s, a); break;
+    case 3: hipLaunchKernelGGL((chunk_scan<T, 3, NS>), grid, dim3(256), 0, s, a); break;
+    default: hipLaunchKernelGGL((chunk_scan<T, 4, NS>), grid, dim3(256), 0, s, a); break;
+  }
+}
+
+template <typename T, int N, int TAPS>
 static hipError_t run(const Args& a, hipStream_t s) {
   if (a.nrows > 0) {
     const long units = (long)a.nrows * a.G;
-    hipLaunchKernelGGL((prep<T, N>), dim3((unsigned)((units + 3) / 4)), dim3(256), 0, s, a);
+    hipLaunchKernelGGL((prep<T, N, TAPS>), dim3((unsigned)((units + 3) / 4)), dim3(256), 0, s, a);
     const dim3 grid((a.V + COLS - 1) / COLS, a.H, a.nseqs);
     switch (a.KP / 32) {
-      case 1: hipLaunchKernelGGL(scan<1>, grid, dim3(256), 0, s, a); break;
-      case 2: hipLaunchKernelGGL(scan<2>, grid, dim3(256), 0, s, a); break;
-      case 3: hipLaunchKernelGGL(scan<3>, grid, dim3(256), 0, s, a); break;
-      case 4: hipLaunchKernelGGL(scan<4>, grid, dim3(256), 0, s, a); break;
-      case 5: hipLaunchKernelGGL(scan<5>, grid, dim3(256), 0, s, a); break;
-      case 6: hipLaunchKernelGGL(scan<6>, grid, dim3(256), 0, s, a); break;
-      case 7: hipLaunchKernelGGL(scan<7>, grid, dim3(256), 0, s, a); break;
-      default: hipLaunchKernelGGL(scan<8>, grid, dim3(256), 0, s, a); break;
+      case 1: hipLaunchKernelGGL((scan<T, 1>), grid, dim3(256), 0, s, a); break;
+      case 2: hipLaunchKernelGGL((scan<T, 2>), grid, dim3(256), 0, s, a); break;
+      case 3: hipLaunchKernelGGL((scan<T, 3>), grid, dim3(256), 0, s, a); break;
+      case 4: hipLaunchKernelGGL((scan<T, 4>), grid, dim3(256), 0, s, a); break;
+      case 5: hipLaunchKernelGGL((scan<T, 5>), grid, dim3(256), 0, s, a); break;
+      case 6: hipLaunchKernelGGL((scan<T, 6>), grid, dim3(256), 0, s, a); break;
+      case 7: hipLaunchKernelGGL((scan<T, 7>), grid, dim3(256), 0, s, a); break;
+      default: hipLaunchKernelGGL((scan<T, 8>), grid, dim3(256), 0, s, a); break;
     }
   }
   if (a.nchunks > 0) {
     const size_t lds = sizeof(float) * CH * (3 * chunk_ld(a.KP) + chunk_ld(a.V));
     if (lds > 48 * 1024) {
       const hipError_t e =
-          hipFuncSetAttribute((const void*)chunk_prep<T, N>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+          hipFuncSetAttribute((const void*)chunk_prep<T, N, TAPS>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
       if (e != hipSuccess) return e;
     }
-    hipLaunchKernelGGL((chunk_prep<T, N>), dim3((unsigned)(a.nchunks * a.H)), dim3(256), lds, s, a);
-    const dim3 grid((unsigned)((a.V + 15) / 16 * a.H * a.ncseqs));
-    switch ((a.KP + 63) / 64) {
-      case 1: hipLaunchKernelGGL(chunk_scan<1>, grid, dim3(256), 0, s, a); break;
-      case 2: hipLaunchKernelGGL(chunk_scan<2>, grid, dim3(256), 0, s, a); break;
-      case 3: hipLaunchKernelGGL(chunk_scan<3>, grid, dim3(256), 0, s, a); break;
-      default: hipLaunchKernelGGL(chunk_scan<4>, grid, dim3(256), 0, s, a); break;
-    }
+    hipLaunchKernelGGL((chunk_prep<T, N, TAPS>), dim3((unsigned)(a.nchunks * a.H)), dim3(256), lds, s, a);
+    const long wide = (long)((a.V + 31) / 32) * a.H * a.ncseqs;
+    if (a.V > 16 && wide >= 256) run_chunk_scan<T, 2>(a, s);
+    else run_chunk_scan<T, 1>(a, s);
   }
-  if (a.taps > 1) hipLaunchKernelGGL(tails<T>, dim3((a.C + 255) / 256, a.B), dim3(256), 0, s, a);
   return hipGetLastError();
+}
+
+template <typename T>
+static hipError_t run(const Args& a, bool pairs, hipStream_t s) {
+  if (pairs) return a.taps == 4 ? run<T, 2, 4>(a, s) : run<T, 2, 0>(a, s);
+  return run<T, 1, 0>(a, s);
 }
 
 }  // namespace delta
@@ -687,10 +888,7 @@ KGS_EXPORT int kgs_delta_forward(const void* const* ptrs, const long* dims, hipS
   if (a.nchunks > 0 && (!a.chunks || !a.cseqs || !a.cW || !a.cQ || !a.cK || !a.cE || !a.cU || !a.cP)) return KGS_ERR_ARG;
   if (pairs && (a.K % 2 || a.V % 2 || (a.ldz | a.lda | a.oq | a.ok | a.ov) % 2 || ((uintptr_t)a.z | (uintptr_t)a.a2) & 3))
     return KGS_ERR_ALIGN;
-  hipError_t e;
-  if (f32) e = pairs ? run<float, 2>(a, s) : run<float, 1>(a, s);
-  else e = pairs ? run<unsigned short, 2>(a, s) : run<unsigned short, 1>(a, s);
-  return (int)e;
+  return (int)(f32 ? run<float>(a, pairs, s) : run<unsigned short>(a, pairs, s));
 }
 
 KGS_EXPORT int kgs_delta_out(const void* o, const void* w, const void* gate, void* y, int T, int H, int V, long ldg,

@@ -75,12 +75,6 @@ __device__ __forceinline__ void st4(T* p, float4 v) {
   }
 }
 
-__device__ __forceinline__ float wave_sum(float v) {
-#pragma unroll
-  for (int m = 8; m >= 1; m >>= 1) v += __shfl_xor(v, m, 64);
-  return xor32_sum(xor16_sum(v));
-}
-
 // sum over the workgroup, the same value in every thread; red: NT / 64 floats
 __device__ __forceinline__ float block_sum(float v, float* red) {
   v = wave_sum(v);

@@ -111,6 +111,25 @@ __device__ __forceinline__ float lane_xor32(float x) {
   return __uint_as_float((__lane_id() & 32) ? r[0] : r[1]);
 }
 
+// the value of another lane of the 16-lane row, chosen by a DPP control
+template <int CTRL>
+__device__ __forceinline__ float dpp_move(float x) {
+  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), CTRL, 0xf, 0xf, false));
+}
+// Sum over aligned groups of 8 lanes, in all of them: two quad permutes (xor 1,
+// xor 2), then the half-row mirror, which exchanges the two finished quads.
+__device__ __forceinline__ float sum8(float x) {
+  x += dpp_move<0xB1>(x);
+  x += dpp_move<0x4E>(x);
+  return x + dpp_move<0x141>(x);
+}
+// sum over the wave, in every lane (row mirror joins the two finished halves of a row)
+__device__ __forceinline__ float wave_sum(float x) {
+  x = sum8(x);
+  x += dpp_move<0x140>(x);
+  return xor32_sum(xor16_sum(x));
+}
+
 // 16-byte LDS-DMA: each lane's 16 global bytes land at lds_base + lane*16
 // (lds_base must be wave-uniform). The swizzle, if any, is applied to the
 // per-lane *source* address (cdna_hip_programming.md rule 21).

@@ -34,11 +34,6 @@ __device__ __forceinline__ void st(T* p, float v) {
   else *p = v;
 }
 
-__device__ __forceinline__ float wave_sum(float v) {
-#pragma unroll
-  for (int m = 8; m >= 1; m >>= 1) v += __shfl_xor(v, m, 64);
-  return xor32_sum(xor16_sum(v));
-}
 __device__ __forceinline__ float wave_max(float v) {
 #pragma unroll
   for (int m = 8; m >= 1; m >>= 1) v = fmaxf(v, __shfl_xor(v, m, 64));
@@ -59,26 +54,92 @@ struct NormArgs {
   float eps;
 };
 
-// one workgroup per token: wave 0 the query latent, wave 1 the cached one
-template <typename T>
-__global__ __launch_bounds__(128) void norm(NormArgs a) {
+// workgroup (token, 0): the query latent, (token, 1): the cached one; up to
+// NORM_REG values per thread stay in registers between the sum and the scaling
+constexpr int NORM_REG = 8;
+
+// bf16 rows in 16-B pieces: one wave per (token, latent), NV pieces per lane
+constexpr int NORM_NV = 4;  // up to 2048 values
+__global__ __launch_bounds__(256) void norm_vec(NormArgs a, int T) {
   const int lane = threadIdx.x & 63;
-  const long t = blockIdx.x;
-  const bool second = threadIdx.x >= 64;
+  const long t = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (t >= T) return;
+  const bool second = blockIdx.y == 1;
   const int n = second ? a.nc : a.nq, np = second ? a.rp : a.qp;
-  if (n == 0) return;
+  const int slot = second ? a.slots[t] : 0;
+  if (slot < 0) return;
+  const unsigned short* z = (const unsigned short*)a.z + t * a.ldz + (second ? a.oc : a.oq);
+  const float* w = second ? a.wc : a.wq;
+  unsigned short* out =
+      second ? (unsigned short*)a.cache + (long)slot * a.rp : (unsigned short*)a.cq + t * a.qp;
+  bf16x8 x[NORM_NV];
+  f32x4 wv[NORM_NV][2];  // loaded ahead of the sum
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NORM_NV; ++i) {
+    const int c = 8 * (lane + 64 * i);
+    if (c < n) {
+      x[i] = *(const bf16x8*)(z + c);
+      wv[i][0] = *(const f32x4*)(w + c);
+      wv[i][1] = *(const f32x4*)(w + c + 4);
+    } else {
+      x[i] = bf16x8{};
+      wv[i][0] = f32x4{};
+      wv[i][1] = f32x4{};
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < NORM_NV; ++i)
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const float v = bf2f((unsigned short)x[i][j]);
+      ss = __builtin_fmaf(v, v, ss);
+    }
+  const float r = 1.0f / sqrtf(wave_sum(ss) / n + a.eps);
+#pragma unroll
+  for (int i = 0; i < NORM_NV; ++i) {
+    const int c = 8 * (lane + 64 * i);
+    if (c >= np) continue;
+    float y[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) y[j] = bf2f((unsigned short)x[i][j]) * r * wv[i][j >> 2][j & 3];
+    *(bf16x8*)(out + c) = pack_bf16x8(y, 0);
+  }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void norm(NormArgs a) {
+  __shared__ float red[4];
+  const int tid = threadIdx.x;
+  const long t = blockIdx.x;
+  const bool second = blockIdx.y == 1;
+  const int n = second ? a.nc : a.nq, np = second ? a.rp : a.qp;
   const int slot = second ? a.slots[t] : 0;
   if (slot < 0) return;
   const T* z = (const T*)a.z + t * a.ldz + (second ? a.oc : a.oq);
   const float* w = second ? a.wc : a.wq;
   T* out = second ? (T*)a.cache + (long)slot * a.rp : (T*)a.cq + t * a.qp;
-  float ss = 0.f;
-  for (int i = lane; i < n; i += 64) {
-    const float v = ld(z + i);
+  float x[NORM_REG], ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NORM_REG; ++i) {
+    const int c = tid + 256 * i;
+    x[i] = c < n ? ld(z + c) : 0.f;
+    ss += x[i] * x[i];
+  }
+  for (int c = tid + 256 * NORM_REG; c < n; c += 256) {
+    const float v = ld(z + c);
     ss += v * v;
   }
-  const float r = 1.0f / sqrtf(wave_sum(ss) / n + a.eps);
-  for (int i = lane; i < np; i += 64) st(out + i, i < n ? ld(z + i) * r * w[i] : 0.f);
+  ss = wave_sum(ss);
+  if ((tid & 63) == 0) red[tid >> 6] = ss;
+  __syncthreads();
+  const float r = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / n + a.eps);
+#pragma unroll
+  for (int i = 0; i < NORM_REG; ++i) {
+    const int c = tid + 256 * i;
+    if (c < np) st(out + c, c < n ? x[i] * r * w[c] : 0.f);
+  }
+  for (int c = tid + 256 * NORM_REG; c < np; c += 256) st(out + c, c < n ? ld(z + c) * r * w[c] : 0.f);
 }
 
 // ------------------------------------------------------------------ head_proj
@@ -180,7 +241,7 @@ struct Geo {
 // are the B operand of O^T = C^T P^T, whose A operand is the page read
 // transposed (ds_read_b64_tr_b16) in that key order.
 template <int RT>
-__global__ __launch_bounds__(512) void attn(Args a) {
+__global__ __launch_bounds__(RT > 8 ? 256 : 512) void attn(Args a) {
   using G = Geo<RT>;
   extern __shared__ __attribute__((aligned(16))) char smem[];  // two pages
   const int lane = threadIdx.x & 63, nw = blockDim.x >> 6;
@@ -320,28 +381,30 @@ __global__ __launch_bounds__(512) void attn(Args a) {
   }
 }
 
-// one wave per row: o = sum_s 2^((m_s - m) sl2) acc_s / sum_s 2^(..) l_s
-__global__ __launch_bounds__(256) void merge(Args a) {
-  const int lane = threadIdx.x & 63;
-  const long nrows = (long)a.Nt * a.H, row = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (row >= nrows) return;
-  float m = NEG;
-  for (int s = 0; s < a.nsplit; ++s) {
-    const float* ml = a.part_ml + 2 * (s * nrows + row);
-    if (ml[1] > 0.f) m = fmaxf(m, ml[0]);
+// one workgroup per row: o = sum_s 2^((m_s - m) sl2) acc_s / sum_s 2^((m_s - m) sl2) l_s
+constexpr int MAX_SPLIT = 64;
+__global__ __launch_bounds__(128) void merge(Args a) {
+  __shared__ float wt[MAX_SPLIT];
+  const int tid = threadIdx.x;
+  const long nrows = (long)a.Nt * a.H, row = blockIdx.x;
+  if (tid < 64) {
+    float m = NEG, l = 0.f;
+    if (tid < a.nsplit) {
+      const float* ml = a.part_ml + 2 * (tid * nrows + row);
+      l = ml[1];
+      m = l > 0.f ? ml[0] : NEG;
+    }
+    const float mx = wave_max(m);
+    const float e = l > 0.f ? __builtin_amdgcn_exp2f((m - mx) * a.sl2) : 0.f;
+    wt[tid] = e / wave_sum(e * l);
   }
-  float l = 0.f;
-  for (int s = 0; s < a.nsplit; ++s) {
-    const float* ml = a.part_ml + 2 * (s * nrows + row);
-    if (ml[1] > 0.f) l += ml[1] * __builtin_amdgcn_exp2f((ml[0] - m) * a.sl2);
-  }
-  const float inv = 1.0f / l;
-  for (int c = 4 * lane; c < a.RP; c += 256) {
+  __syncthreads();
+  for (int c = 4 * tid; c < a.RP; c += 512) {
     f32x4 v = f32x4{};
+#pragma unroll 4
     for (int s = 0; s < a.nsplit; ++s) {
-      const long pr = s * nrows + row;
-      if (a.part_ml[2 * pr + 1] > 0.f)
-        v += *(const f32x4*)(a.part_o + pr * a.RP + c) * (__builtin_amdgcn_exp2f((a.part_ml[2 * pr] - m) * a.sl2) * inv);
+      const float w = wt[s];
+      if (w > 0.f) v += *(const f32x4*)(a.part_o + (s * nrows + row) * a.RP + c) * w;
     }
     uint2 o;
     o.x = pack_bf16x2(v[0], v[1]);
@@ -438,8 +501,11 @@ KGS_EXPORT int kgs_latent_norm(const void* z, long ldz, int oq, int nq, int qp, 
       (nc && ldz < oc + nc))
     return KGS_ERR_SHAPE;
   NormArgs a{z, ldz, oq, nq, qp, oc, nc, rp, (const float*)wq, (const float*)wc, cq, cache, (const int*)slots, eps};
-  if (f32) hipLaunchKernelGGL(norm<float>, dim3(T), dim3(128), 0, s, a);
-  else hipLaunchKernelGGL(norm<unsigned short>, dim3(T), dim3(128), 0, s, a);
+  const bool vec = !f32 && ((nq | qp | nc | rp | oq | oc) & 7) == 0 && ldz % 8 == 0 && qp <= 512 * NORM_NV &&
+                   (!nc || rp <= 512 * NORM_NV) && (((uintptr_t)z | (uintptr_t)cq | (uintptr_t)cache | (uintptr_t)wq | (uintptr_t)wc) & 15) == 0;
+  if (vec) hipLaunchKernelGGL(norm_vec, dim3((T + 3) / 4, nc ? 2 : 1), dim3(256), 0, s, a, T);
+  else if (f32) hipLaunchKernelGGL(norm<float>, dim3(T, nc ? 2 : 1), dim3(256), 0, s, a);
+  else hipLaunchKernelGGL(norm<unsigned short>, dim3(T, nc ? 2 : 1), dim3(256), 0, s, a);
   return (int)hipGetLastError();
 }
 
@@ -474,10 +540,11 @@ KGS_EXPORT int kgs_latent_attn(const void* q, const void* cache, void* o, void* 
                                int tiles, int nw, int nsplit, int H, int W, int Nt, int RP, float scale,
                                hipStream_t s) {
   using namespace kgs::latent;
-  if (ntiles <= 0 || H <= 0 || W <= 0 || Nt <= 0 || nw < 1 || nw > 8 || nsplit < 1 || nsplit > 1024 ||
+  if (ntiles <= 0 || H <= 0 || W <= 0 || Nt <= 0 || nw < 1 || nw > 8 || nsplit < 1 || nsplit > MAX_SPLIT ||
       (!items && tiles <= 0))
     return KGS_ERR_SHAPE;
   if (nsplit > 1 && (!part_o || !part_ml)) return KGS_ERR_ARG;
+  if (RP > 256 && nw > 4) return KGS_ERR_SHAPE;  // a wave holds 16 x RP outputs in registers
   if (((uintptr_t)q | (uintptr_t)cache | (uintptr_t)o | (uintptr_t)part_o) & 15) return KGS_ERR_ALIGN;
   Args a{q, cache, o, (float*)part_o, (float*)part_ml, (const int*)q0, (const int*)n, (const int*)pos0,
          (const int*)bt, (const int*)items, nullptr, nullptr, H, W, tiles, nsplit, Nt, RP, scale,
@@ -495,7 +562,7 @@ KGS_EXPORT int kgs_latent_attn(const void* q, const void* cache, void* o, void* 
     default: return KGS_ERR_SHAPE;
   }
   if (e == hipSuccess && nsplit > 1) {
-    hipLaunchKernelGGL(merge, dim3(((long)Nt * H + 3) / 4), dim3(256), 0, s, a);
+    hipLaunchKernelGGL(merge, dim3((unsigned)((long)Nt * H)), dim3(128), 0, s, a);
     e = hipGetLastError();
   }
   return (int)e;

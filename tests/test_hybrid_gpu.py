@@ -19,7 +19,7 @@ pytestmark = pytest.mark.gpu
 
 # (median row, worst row): rms over the vocabulary, against the logits' own. In bf16 a
 # row whose scores nearly tie moves several times as far as the others.
-TOL = {"float32": (2e-6, 5e-6), "bfloat16": (1.6e-2, 8e-2)}
+TOL = {"float32": (3e-6, 2e-5), "bfloat16": (1.6e-2, 8e-2)}
 NAMES = sorted(HM.MODELS)
 
 
