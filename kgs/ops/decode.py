@@ -83,7 +83,8 @@ FP8_MAX = 448.0
 class PackedWeight:
     """A projection weight in skinny-GEMM fragment order (plus its shape).
 
-    * ``swiglu=True``: a fused gate|up weight whose GEMM emits ``silu(g) * u``;
+    * ``swiglu=True``: a fused gate|up weight whose GEMM emits ``act(g) * u``
+      (``act``: ``"silu"`` or ``"gelu_tanh"``);
     * ``fold``: an RMSNorm weight ``[K]`` folded into the columns (``W * fold``),
       for GEMMs that apply the norm in their epilogue (``rms=``);
     * ``fp8=True``: weight-only fp8 (W8A16): OCP e4m3 with one scale per output
@@ -92,11 +93,14 @@ class PackedWeight:
       GEMM whose epilogue applies RoPE and writes the KV cache (``rope=`` of
       :func:`skinny_gemm`); its output is in the original order."""
 
-    __slots__ = ("data", "n", "k", "swiglu", "fp8", "wscale", "rope")
+    __slots__ = ("data", "n", "k", "swiglu", "fp8", "wscale", "rope", "act")
 
     def __init__(self, w: torch.Tensor, swiglu: bool = False, fold: torch.Tensor | None = None, fp8: bool = False,
-                 rope: tuple | None = None):
+                 rope: tuple | None = None, act: str = "silu"):
         self.n, self.k = w.shape
+        if act not in ("silu", "gelu_tanh"):
+            raise ValueError(f"unknown gate activation {act!r}")
+        self.act = act
         self.swiglu, self.fp8, self.rope = swiglu, fp8, rope
         if swiglu and rope:
             raise ValueError("a weight is either SwiGLU- or RoPE-packed")
@@ -387,7 +391,7 @@ def _workspace(device: torch.device, floats: int, ints: int):
     return ws, cnt
 
 
-EPI_SWIGLU, EPI_RMS, EPI_RESID = 1, 2, 4
+EPI_SWIGLU, EPI_RMS, EPI_RESID, EPI_GELU = 1, 2, 4, 16
 
 
 def skinny_gemm(x: torch.Tensor, w: PackedWeight, out: torch.Tensor | None = None,
@@ -426,7 +430,7 @@ def skinny_gemm(x: torch.Tensor, w: PackedWeight, out: torch.Tensor | None = Non
     rps, kpc, mpad = skinny_geometry(m, variant)
     if w.n % rps or k % kpc:
         raise ValueError(f"skinny GEMM needs N % {rps} == 0 and K % {kpc} == 0 (N={w.n}, K={k})")
-    epi = (EPI_SWIGLU if w.swiglu else 0) | (EPI_RMS if rms is not None else 0) | \
+    epi = (EPI_SWIGLU | (EPI_GELU if w.act == "gelu_tanh" else 0) if w.swiglu else 0) | (EPI_RMS if rms is not None else 0) | \
         (EPI_RESID if resid_ss is not None else 0)
     for t, name in ((rms, "rms"), (resid_ss, "resid_ss"), (zero, "zero")):
         if t is not None and (t.dtype != torch.float32 or t.numel() < m or not t.is_contiguous()):

@@ -11,7 +11,7 @@ A sublayer is ``h -> mixer or feed-forward -> y`` between two launches of
 :func:`kgs.ops.hyper.hyper_step`, which writes ``y`` back into the fp32 streams and
 produces the next sublayer's normed input in one pass. Weights are laid out once
 at load: the projections of one input fused into one matrix, every dimension
-that a GEMM sees padded with zeros to a multiple of 64.
+that a GEMM sees padded with zeros to a multiple of 64 (larger ones of 128).
 
 ``dtype="float32"``: the same steps with fp32 weights, activations and caches.
 """
@@ -23,13 +23,14 @@ import numpy as np
 import torch
 
 from kgs.models.ruruzen import DeltaSpec, LatentSpec, RuruzenConfig
-from kgs.ops.activation import act_mul, softcap
+from kgs.ops.activation import softcap
+from kgs.ops import decode as D
 from kgs.ops.decode import PAGE
 from kgs.ops.delta import DeltaShape, DeltaState, RaggedSeqs, chunk_plan, delta_forward, delta_out
 from kgs.ops.hyper import MAX_STREAMS, hyper_embed, hyper_step
 from kgs.ops.latent import (KERNEL_SIZES, LatentCache, LatentRows, head_proj, latent_attention, latent_norm,
                             padded_latent, split_count, waves_for)
-from kgs.ops.linear import project
+from kgs.ops.linear import Projection
 from kgs.ops.transformer import attention_ragged
 
 from .trace import TRACE as T
@@ -41,6 +42,12 @@ QBLOCK = 128  # query rows of one attention_ragged item
 
 def pad64(n: int) -> int:
     return (n + 63) // 64 * 64
+
+
+def padk(n: int) -> int:
+    """Padded size of a GEMM's inner dimension: the MFMA GEMMs step by 128, which a
+    small one is not padded to."""
+    return pad64(n) if n <= 512 else (n + 127) // 128 * 128
 
 
 def _pad(w: torch.Tensor, *sizes: int) -> torch.Tensor:
@@ -127,8 +134,11 @@ class Geometry:
 class _Weights:
     """Checkpoint tensors on their way to the device layout."""
 
-    def __init__(self, w: dict, device, dtype):
-        self.w, self.device, self.dtype = w, device, dtype
+    def __init__(self, w: dict, device, dtype, pack: bool):
+        self.w, self.device, self.dtype, self.pack = w, device, dtype, pack
+
+    def proj(self, t: torch.Tensor, gated: str | None = None) -> Projection:
+        return Projection(t, gated, pack=self.pack)
 
     def f32(self, name: str) -> torch.Tensor:
         return self.w[name].to(self.device).float().contiguous()
@@ -158,12 +168,13 @@ class LatentMixer:
         self.layer = i
         self.eps = cfg.eps
         names = ["dq", "g"] + (["dkv"] if m.kv_from is None else [])
-        self.win, offs = w.stack([p + n for n in names], model.wp)
+        win, offs = w.stack([p + n for n in names], model.wp)
+        self.win = w.proj(win)
         self.oq, self.og = offs[0], offs[1]
         self.oc = offs[2] if m.kv_from is None else 0
         self.wq = w.f32(p + "dq.norm")
         self.wc = w.f32(p + "dkv.norm") if m.kv_from is None else None
-        self.qp = pad64(m.q_rank)
+        self.qp = padk(m.q_rank)
         rp = padded_latent(m.kv_rank)
         both = max(m.dim, m.vdim)
         hd = (64 if both <= 64 else 128 if both <= 128 else 0) if w.dtype == torch.bfloat16 else 0
@@ -175,21 +186,21 @@ class LatentMixer:
             t = w.w[p + name].to(w.device).to(w.dtype).reshape(H, d, rank)
             return _pad(t, dp, rankp)
 
-        self.uq = heads("uq", m.dim, self.hq, m.q_rank, self.qp).reshape(H * self.hq, self.qp).contiguous()
+        self.uq = w.proj(heads("uq", m.dim, self.hq, m.q_rank, self.qp).reshape(H * self.hq, self.qp))
         uk = heads("uk", m.dim, self.hq, m.kv_rank, rp)
         self.uv = heads("uv", m.vdim, self.hv, m.kv_rank, rp).contiguous()          # [H, HV, RP]
         self.ukt = uk.transpose(1, 2).contiguous()                                  # [H, RP, HQ]
-        self.ukv = torch.cat([uk.reshape(-1, rp), self.uv.reshape(-1, rp)]).contiguous() if hd else None
+        self.ukv = Projection(torch.cat([uk.reshape(-1, rp), self.uv.reshape(-1, rp)]), pack=False) if hd else None
         o = w.w[p + "o"].to(w.device).to(w.dtype).reshape(cfg.width, H, m.vdim)
-        self.o = _pad(_pad(o, self.hv).reshape(cfg.width, H * self.hv), model.wp, H * self.hv).contiguous()
+        self.o = w.proj(_pad(_pad(o, self.hv).reshape(cfg.width, H * self.hv), model.wp, H * self.hv))
 
     def __call__(self, model, h: torch.Tensor, b: Batch) -> torch.Tensor:
         m, geo = self.m, self.geo
-        z = project(h, self.win)
+        z = self.win(h)
         pages = model.cache.pages[self.owner]
         cq = latent_norm(z, self.oq, self.wq, self.qp, self.oc, self.wc, pages if self.wc is not None else None,
                          b.slots, self.eps)
-        q = project(cq, self.uq)
+        q = self.uq(cq)
         T.op(f"L{self.layer} latent projections")
         gate = z[:, self.og:self.og + m.heads]
         plan = b.plans[geo]
@@ -197,7 +208,7 @@ class LatentMixer:
         if plan.expanded is not None:
             e = plan.expanded
             c = pages.view(-1, geo.rp).index_select(0, e.ctx_slots)
-            kv = project(c, self.ukv)
+            kv = self.ukv(c)
             n = m.heads * geo.hd
             attention_ragged(q, kv[:, :n], kv[:, n:], e.items, m.heads, geo.hd, m.scale, a, gate=gate)
             T.op(f"L{self.layer} expanded attention")
@@ -208,7 +219,7 @@ class LatentMixer:
             ol = latent_attention(ql, pages, r, m.heads, m.scale)
             head_proj(ol, self.uv, r.nt, a, rows_out=r.rows, gate=gate)
             T.op(f"L{self.layer} latent attention")
-        return project(a, self.o)
+        return self.o(a)
 
 
 class DeltaMixer:
@@ -216,38 +227,40 @@ class DeltaMixer:
         p = f"l{i}.mix."
         cfg = model.cfg
         self.layer, self.eps, self.shape = i, cfg.eps, delta_shape(m)
-        self.win, offs = w.stack([p + n for n in ("q", "k", "v", "b", "a1", "g1")], model.wp)
+        win, offs = w.stack([p + n for n in ("q", "k", "v", "b", "a1", "g1")], model.wp)
+        self.win = w.proj(win)
         self.offs, self.oa, self.og = tuple(offs[:4]), offs[4], offs[5]
         self.ra, self.rg = pad64(w.w[p + "a1"].shape[0]), pad64(w.w[p + "g1"].shape[0])
         hk, hv = m.heads * m.dim, m.heads * m.vdim
-        self.a2 = w.mat(p + "a2", pad64(hk), self.ra)
-        self.g2 = w.mat(p + "g2", pad64(hv), self.rg)
+        self.a2 = w.proj(w.mat(p + "a2", pad64(hk), self.ra))
+        self.g2 = w.proj(w.mat(p + "g2", pad64(hv), self.rg))
         self.cw = torch.cat([w.f32(f"{p}{n}.conv") for n in "qkv"]).T.contiguous()
         self.a_log, self.dt_bias, self.norm = w.f32(p + "A_log"), w.f32(p + "dt_bias"), w.f32(p + "norm")
-        self.ld = pad64(hv)
-        self.o = w.mat(p + "o", model.wp, self.ld)
+        self.ld = padk(hv)
+        self.o = w.proj(w.mat(p + "o", model.wp, self.ld))
 
     def __call__(self, model, h: torch.Tensor, b: Batch) -> torch.Tensor:
-        z = project(h, self.win)
-        a2 = project(z[:, self.oa:self.oa + self.ra], self.a2)
-        g2 = project(z[:, self.og:self.og + self.rg], self.g2)
+        z = self.win(h)
+        a2 = self.a2(z[:, self.oa:self.oa + self.ra])
+        g2 = self.g2(z[:, self.og:self.og + self.rg])
         T.op(f"L{self.layer} delta projections")
         o = delta_forward(z, self.offs, a2, self.cw, self.a_log, self.dt_bias, self.shape, model.state[self.layer],
                           b.seqs)
         y = delta_out(o, self.norm, g2, self.eps, self.ld)
         T.op(f"L{self.layer} delta rule")
-        return project(y, self.o)
+        return self.o(y)
 
 
 class DenseFF:
     def __init__(self, model, i: int, ff: int, w: _Weights):
         p = f"l{i}.mlp."
         self.layer = i
-        self.gate_up, _ = w.stack([p + "gate", p + "up"], model.wp)
-        self.down = w.mat(p + "down", model.wp, pad64(ff))
+        fp = padk(ff)
+        self.gate_up = w.proj(torch.cat([w.mat(p + n, fp, model.wp) for n in ("gate", "up")]), gated="gelu_tanh")
+        self.down = w.proj(w.mat(p + "down", model.wp, fp))
 
     def __call__(self, model, h: torch.Tensor, b: Batch) -> torch.Tensor:
-        y = project(act_mul(project(h, self.gate_up), "gelu_tanh"), self.down)
+        y = self.down(self.gate_up(h))
         T.op(f"L{self.layer} feed-forward")
         return y
 
@@ -263,15 +276,19 @@ class HybridModel:
     pad_multiple = 1  # portions are not padded
 
     def __init__(self, cfg: RuruzenConfig, device="cuda", dtype: str = "bfloat16", seed: int = 0,
-                 num_pages: int = 1024, state_slots: int = 256, weights: dict | None = None):
+                 num_pages: int = 1024, state_slots: int = 256, weights: dict | None = None,
+                 packed_decode: bool = True):
         if cfg.streams > MAX_STREAMS:
             raise ValueError(f"streams {cfg.streams} is above {MAX_STREAMS}")
         self.cfg, self.device, self.dtype = cfg, torch.device(device), DTYPES[dtype]
         self.has_state = cfg.has_state
-        self.wp = pad64(cfg.width)
+        self.wp = padk(cfg.width)
         raw = weights if weights is not None else cfg.load_weights(seed, self.device)
-        w = _Weights(raw, self.device, self.dtype)
-        self.embed = w.mat("embed", pad64(cfg.vocab), self.wp).contiguous()
+        w = _Weights(raw, self.device, self.dtype, packed_decode)
+        if self.dtype == torch.bfloat16:
+            D.reserve_workspace(self.device)  # split-K partials, before any hipGraph capture
+        self.head = w.proj(w.mat("embed", pad64(cfg.vocab), self.wp))
+        self.embed = self.head.w
         self.embed_norm = w.f32("embed.norm")
         one = torch.ones(cfg.streams, dtype=torch.float32, device=self.device)
         self.subs = []    # (sublayer, layer, last of its layer, write-back mix, write-back out)
@@ -303,7 +320,8 @@ class HybridModel:
                 raise ValueError(f"{name}={getattr(ec, name)!r} is not available for this model")
         if ec.prefix_caching and cfg.has_state:
             raise ValueError("prefix caching shares cache pages, not recurrent state: off for this model")
-        return cls(cfg, device=device, dtype=ec.dtype, seed=ec.seed, num_pages=num_pages, state_slots=ec.max_batch)
+        return cls(cfg, device=device, dtype=ec.dtype, seed=ec.seed, num_pages=num_pages, state_slots=ec.max_batch,
+                   packed_decode=ec.packed_decode)
 
     @staticmethod
     def memory(cfg: RuruzenConfig, dtype: str, slots: int) -> dict:
@@ -314,7 +332,7 @@ class HybridModel:
         n = sum(int(np.prod(s)) for s in tensor_shapes(cfg).values())
         state = sum(DeltaState.bytes_per_slot(delta_shape(x.mixer)) for x in cfg.layers
                     if isinstance(x.mixer, DeltaSpec))
-        return {"weights": 2 * size * n, "state": (slots + 1) * state,
+        return {"weights": 3 * size * n, "state": (slots + 1) * state,
                 "page": LatentCache.bytes_per_page(latent_sizes(cfg), size) or 1}
 
     def weight_bytes(self) -> int:
@@ -338,7 +356,7 @@ class HybridModel:
             if b.logit_rows.shape[0] == 0:
                 return torch.empty((0, cfg.vocab), dtype=torch.float32, device=self.device)
             h = h.index_select(0, b.logit_rows)
-        logits = softcap(project(h, self.embed), cfg.vocab, cfg.logit_softcap)
+        logits = softcap(self.head(h), cfg.vocab, cfg.logit_softcap)
         T.op("logits")
         return logits
 

@@ -118,7 +118,7 @@ struct SkinnyCfg {
 //               paged cache slot slot[m] -- the rope_cache launch, folded in.
 // Together they remove both add_rmsnorm launches, the SwiGLU launch and the
 // RoPE / KV-write launch from a decode layer (kgs/serve/model.py fused path).
-enum { EPI_SWIGLU = 1, EPI_RMS = 2, EPI_RESID = 4, EPI_ROPE = 8 };
+enum { EPI_SWIGLU = 1, EPI_RMS = 2, EPI_RESID = 4, EPI_ROPE = 8, EPI_GELU = 16 };
 struct SkinnyEpi {
   int mode;
   const float* ss_in;
@@ -362,7 +362,8 @@ __global__ __launch_bounds__(256, (MT * KC_ > 32 || R * MT >= 16) ? 1 : 2) void 
       if (m < M && g < 2) {
         f32x4v o;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) o[i] = v[i] / (1.0f + __expf(-v[i])) * u[i];
+        for (int i = 0; i < 4; ++i)
+          o[i] = ((ep.mode & EPI_GELU) ? gate_act<GATE_GELU>(v[i]) : gate_act<GATE_SILU>(v[i])) * u[i];
         uint2 pk;
         pk.x = pack_bf16x2(o[0], o[1]);
         pk.y = pack_bf16x2(o[2], o[3]);
@@ -1201,7 +1202,7 @@ int skinny_fused(const void* wp, const void* x, void* y, float* ws, int* cnt, in
   const int rc = kgs_skinny_variant_geometry(variant, M, &rps, &kpc, &mpad);
   if (rc) return rc;
   if (variant == 0) variant = default_variant(mt_for(M));
-  if (epi & ~(EPI_SWIGLU | EPI_RMS | EPI_RESID | EPI_ROPE) || ((epi & EPI_SWIGLU) && (epi & EPI_RESID)))
+  if (epi & ~(EPI_SWIGLU | EPI_RMS | EPI_RESID | EPI_ROPE | EPI_GELU) || ((epi & EPI_GELU) && !(epi & EPI_SWIGLU)) || ((epi & EPI_SWIGLU) && (epi & EPI_RESID)))
     return KGS_ERR_ARG;
   if ((epi & EPI_ROPE) && (rope == nullptr || (epi & (EPI_SWIGLU | EPI_RESID)) || wscale != nullptr))
     return KGS_ERR_ARG;

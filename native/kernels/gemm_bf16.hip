@@ -167,7 +167,7 @@ static int cu_count() {
 
 // gemm_persistent.hip
 hipError_t launch_w4p_swiglu(const unsigned short* A, const unsigned short* B, unsigned short* C, int M, int N,
-                             int K, int lda, int ldb, int ldc, int cus, int* tq, hipStream_t s);
+                             int K, int lda, int ldb, int ldc, int cus, int* tq, bool gelu, hipStream_t s);
 template <int EPI>
 hipError_t launch_w4p(const unsigned short* A, const unsigned short* B, unsigned short* C, const unsigned short* bias,
                       int M, int N, int K, int lda, int ldb, int ldc, int cus, int* tq, hipStream_t s);
@@ -757,6 +757,12 @@ int launch_w4sw(dim3 grid, hipStream_t s, const unsigned short* a, const unsigne
                 int N, int K, int lda, int ldb, int ldc, bool aligned_m, int flags) {
   constexpr int BM = kgs::w4::tile_m<TM>();
   const bool packed = flags & 1;
+  if (flags & 0x40) {  // tanh gelu: row-major weights, two LDS stages
+    if (flags & 0x31) return KGS_ERR_ARG;
+    if (flags & 2) launch_w4sw_x<BN, TM, 2005200>(grid, s, a, b, c, M, N, K, lda, ldb, ldc, aligned_m);
+    else launch_w4sw_x<BN, TM, 2000000>(grid, s, a, b, c, M, N, K, lda, ldb, ldc, aligned_m);
+    return 0;
+  }
   if (flags & 2) {  // weights (B) non-temporal: two LDS stages only
     if (flags & 0x30) return KGS_ERR_ARG;
     if (packed) launch_w4sw_x<BN, TM, 1001005200>(grid, s, a, b, c, M, N, K, lda, ldb, ldc, aligned_m);
@@ -851,11 +857,13 @@ KGS_EXPORT int kgs_gemm_bf16_nt_w4x_swiglu(const void* A, const void* B, void* C
 
 // flags bit 0: B is the SwiGLU-packed copy of the fused gate|up weight
 // (kgs.ops.gemm.pack_w4x_weight(..., swiglu=True)), ldb must be K; bits 4-5:
-// LDS stages - 2 (as kgs_gemm_bf16_nt_w4x_ex)
+// LDS stages - 2 (as kgs_gemm_bf16_nt_w4x_ex); bit 6: tanh gelu instead of silu
+// (row-major B, two stages)
 KGS_EXPORT int kgs_gemm_bf16_nt_w4x_swiglu_ex(const void* A, const void* B, void* C, int M, int N, int K, int lda,
                                               int ldb, int ldc, int bn, int bm, int flags, hipStream_t stream) {
   using namespace kgs;
-  if (flags & ~0x33 || (flags & 0x30) == 0x30) return KGS_ERR_ARG;
+  if (flags & ~0x73 || (flags & 0x30) == 0x30) return KGS_ERR_ARG;
+  const bool gelu = flags & 0x40;
   if ((flags & 1) && ldb != K) return KGS_ERR_SHAPE;
   if (M <= 0 || N <= 0 || K <= 0 || lda < K || ldb < K || ldc < N / 2) return KGS_ERR_SHAPE;
   if ((bn != 128 && bn != 256) || (bm != 128 && bm != 256)) return KGS_ERR_ARG;
@@ -869,9 +877,9 @@ KGS_EXPORT int kgs_gemm_bf16_nt_w4x_swiglu_ex(const void* A, const void* B, void
   const bool aligned_m = M % bm == 0;
   // prompt-pass shapes (256 x 256 tiles, aligned M, more tiles than CUs): the
   // persistent kernel with the same K-step (bitwise the one-shot result)
-  if (bm == 256 && bn == 256 && aligned_m && flags == 0 && K >= 384 && (long)(M / 256) * (N / 256) > cu_count()) {
+  if (bm == 256 && bn == 256 && aligned_m && (flags & ~0x40) == 0 && K >= 384 && (long)(M / 256) * (N / 256) > cu_count()) {
     if (int* tq = tile_queue(stream)) {
-      const hipError_t e = launch_w4p_swiglu(a, b, c, M, N, K, lda, ldb, ldc, cu_count(), tq, stream);
+      const hipError_t e = launch_w4p_swiglu(a, b, c, M, N, K, lda, ldb, ldc, cu_count(), tq, gelu, stream);
       return e == hipSuccess ? 0 : (int)e;
     }
   }

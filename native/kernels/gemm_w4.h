@@ -576,7 +576,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     return;
   }
   if constexpr (SW) {
-    // out fragment q (16 columns) = silu(gate fragment ng) * up fragment ng + 2,
+    // out fragment q (16 columns) = act(gate fragment ng) * up fragment ng + 2 (SW 1: silu, 2: tanh gelu),
     // ng = 4 (q / 2) + q % 2; pairs (q, q + 1) share one 16-B store per lane
     static_for<0, MA>([&](auto ic) {
       constexpr int i = decltype(ic)::value;
@@ -596,7 +596,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
 #pragma unroll
           for (int e = 0; e < 4; ++e) {
             const float gf = bf2f(f2bf(g[e]));
-            r[e] = gf / (1.0f + __expf(-gf)) * bf2f(f2bf(u[e]));
+            r[e] = gate_act<(X / 1000000) % 10>(gf) * bf2f(f2bf(u[e]));
           }
           o[h].x = pack_bf16x2(r[0], r[1]);
           o[h].y = pack_bf16x2(r[2], r[3]);

@@ -174,6 +174,14 @@ __device__ __forceinline__ float gelu_tanh(float x) {
   return 0.5f * x * (1.0f + t);
 }
 
+// activation of a gated feed-forward's gate: 1 silu, 2 tanh gelu
+enum GateAct { GATE_SILU = 1, GATE_GELU = 2 };
+template <int ACT>
+__device__ __forceinline__ float gate_act(float g) {
+  if constexpr (ACT == GATE_GELU) return gelu_tanh(g);
+  return g / (1.0f + __expf(-g));
+}
+
 template <int EPI>
 __device__ __forceinline__ float epilogue(float v, float b) {
   if constexpr (EPI == EPI_NONE || EPI == EPI_ADDC) return v;

@@ -29,7 +29,7 @@ MODELS = {
         latent(1, 32, 32, 32, 32, 0.2, ff=64), delta(1, 1, 32, 32, 1, ff=64), latent(1, 32, 32, 32, 32, 0.3, kv_from=0)]),
     # latent wide against the heads: prompts of some 90 tokens run expanded
     "wide": dict(vocab=320, width=192, streams=2, logit_softcap=20.0, norm={"eps": 1e-5}, layers=[
-        latent(4, 32, 48, 64, 250, 0.18, ff=128), delta(4, 2, 64, 64, 4), latent(9, 16, 8, 24, 250, 0.3, kv_from=0, ff=96),
+        latent(4, 32, 48, 64, 250, 0.18, ff=128), delta(4, 2, 64, 64, 4), latent(9, 16, 8, 24, 250, 0.3, kv_from=0, ff=700),
         latent(2, 100, 128, 48, 512, 0.1)]),
     # no delta layer: no recurrent state anywhere
     "attention": dict(vocab=128, width=96, streams=5, logit_softcap=8.0, norm={"eps": 1e-4}, layers=[
