@@ -65,6 +65,10 @@ CXX = os.environ.get("CXX", "g++")
 # reports that it does not know the feature; harmless)
 NO_PACKED_F32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
+# kernels whose MFMA accumulators the VALU also touches (softmax rescales, decays)
+# keep them in VGPRs instead of copying them from and to AGPRs around every use
+MFMA_IN_VGPRS = ["-mllvm", "-amdgpu-mfma-vgpr-form=1"]
+
 HIP_FLAGS = [
     f"--offload-arch={ARCH}",
     "-O3",
@@ -88,6 +92,7 @@ class Target:
     link_flags: list[str] = field(default_factory=list)
     shared: bool = True
     headers: list[Path] = field(default_factory=list)
+    source_flags: dict = field(default_factory=dict)  # file name -> extra compiler flags
     optional: bool = False  # skip (with a warning) if a dependency is missing
 
     def stale(self) -> bool:
@@ -161,6 +166,7 @@ def targets(out: Path | None = None) -> list[Target]:
             HIPCC,
             flags=HIP_FLAGS + ["-fvisibility=hidden", f"-I{kdir}"],
             headers=k_headers,
+            source_flags={"latent.hip": MFMA_IN_VGPRS, "delta.hip": MFMA_IN_VGPRS},
         ),
         Target(
             "gpuprobe",
@@ -247,7 +253,7 @@ def targets(out: Path | None = None) -> list[Target]:
 
 
 def _compile_one(t: Target, src: Path, obj: Path) -> None:
-    cmd = [t.compiler, *t.flags, "-c", str(src), "-o", str(obj)]
+    cmd = [t.compiler, *t.flags, *t.source_flags.get(src.name, []), "-c", str(src), "-o", str(obj)]
     r = subprocess.run(cmd, capture_output=True, text=True)
     if r.returncode != 0:
         raise RuntimeError(f"compile failed: {' '.join(cmd)}\n{r.stdout}\n{r.stderr}")
@@ -346,7 +352,7 @@ def _toolchain(compiler: str) -> str:
 def _record(t: Target) -> dict:
     return {"output": _rel(t.output), "output_sha256": _sha256(t.output),
             "inputs": {_rel(p): _sha256(p) for p in [*t.sources, *t.headers] if p.exists()},
-            "compile": [Path(t.compiler).name, *t.flags], "link": t.link_flags,
+            "compile": [Path(t.compiler).name, *t.flags], "source_flags": t.source_flags, "link": t.link_flags,
             "toolchain": _toolchain(t.compiler)}
 
 

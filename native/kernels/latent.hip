@@ -172,12 +172,22 @@ __global__ __launch_bounds__(256) void head_proj(ProjArgs p) {
   f32x4 acc[TT];
 #pragma unroll
   for (int i = 0; i < TT; ++i) acc[i] = f32x4{};
-#pragma unroll 4
-  for (int k = 0; k < p.K; k += 32) {
-    const bf16x8 wf = *(const bf16x8*)(wp + k);
+  for (int k = 0; k < p.K; k += 128) {  // four steps' loads are in flight together
+    bf16x8 wf[4], af[4][TT];
 #pragma unroll
-    for (int i = 0; i < TT; ++i)
-      acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, *(const bf16x8*)(ap[i] + k), acc[i], 0, 0, 0);
+    for (int j = 0; j < 4; ++j)
+      if (k + 32 * j < p.K) {
+        wf[j] = *(const bf16x8*)(wp + k + 32 * j);
+#pragma unroll
+        for (int i = 0; i < TT; ++i) af[j][i] = *(const bf16x8*)(ap[i] + k + 32 * j);
+      }
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (k + 32 * j < p.K) {
+#pragma unroll
+        for (int i = 0; i < TT; ++i)
+          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[j], af[j][i], acc[i], 0, 0, 0);
+      }
   }
 #pragma unroll
   for (int i = 0; i < TT; ++i) {
@@ -235,6 +245,31 @@ struct Geo {
   __device__ static __forceinline__ int off(int r, int c) { return PITCH * r + 16 * (c ^ swz(r)); }
 };
 
+// Two 16-column tiles of a page's 32 keys, transposed: four ds_read_b64_tr_b16
+// (keys k0 .. and 16 + k0 .. of each), see tr_frag
+struct TrBatch {
+  bf16x4 lo[2], hi[2];
+  template <int RT>
+  __device__ __forceinline__ void read(unsigned base, int j, int k0, int tp) {
+    using G = Geo<RT>;
+#pragma unroll
+    for (int x = 0; x < 2; ++x) {
+      const unsigned at = base + G::off(k0, 2 * (2 * j + x) + (tp >> 1)) + 8 * (tp & 1);
+      asm volatile("ds_read_b64_tr_b16 %0, %2\n\tds_read_b64_tr_b16 %1, %2 offset:%3"
+                   : "=&v"(lo[x]), "=&v"(hi[x])
+                   : "v"(at), "n"(16 * G::PITCH));
+    }
+  }
+  // all but the N newest LDS operations have arrived
+  template <int N>
+  __device__ __forceinline__ void wait() {
+    asm volatile("s_waitcnt lgkmcnt(%4)" : "+v"(lo[0]), "+v"(hi[0]), "+v"(lo[1]), "+v"(hi[1]) : "n"(N));
+  }
+  __device__ __forceinline__ bf16x8 frag(int x) const {
+    return __builtin_shufflevector(lo[x], hi[x], 0, 1, 2, 3, 4, 5, 6, 7);
+  }
+};
+
 // Workgroup: 16 rows per wave of one sequence's (token, head) rows, head fastest,
 // over the pages of one context split. S^T = C Q^T, so a lane owns row
 // (lane & 15) and keys 16 t + 4 (lane >> 4) + r of a page; the same registers
@@ -247,12 +282,12 @@ __global__ __launch_bounds__(RT > 8 ? 256 : 512) void attn(Args a) {
   const int lane = threadIdx.x & 63, nw = blockDim.x >> 6;
   const int w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int l16 = lane & 15, g = lane >> 4, tq = (lane >> 2) & 3, tp = lane & 3;
-  int b, tile;
+  int b, tile;  // uniform: page ids then come by scalar loads
   if (a.items) {
     b = a.items[2 * blockIdx.x];
     tile = a.items[2 * blockIdx.x + 1];
   } else {
-    b = blockIdx.x / a.tiles;
+    b = __builtin_amdgcn_readfirstlane(blockIdx.x / a.tiles);
     tile = blockIdx.x - b * a.tiles;
   }
   const int rows = a.n[b] * a.H, pos0 = a.pos0[b];
@@ -264,8 +299,8 @@ __global__ __launch_bounds__(RT > 8 ? 256 : 512) void attn(Args a) {
   const int row = min(myrow, last);
   const int pos = pos0 + row / a.H;
   const int wmax = pos0 + min(r0 + 16 * w + 15, last) / a.H;  // this wave's last position
-  const int npages = (pos0 + last / a.H) / PAGE + 1;
-  const int pps = (npages + a.nsplit - 1) / a.nsplit;
+  const int npages = __builtin_amdgcn_readfirstlane((pos0 + last / a.H) / PAGE + 1);
+  const int pps = __builtin_amdgcn_readfirstlane((npages + a.nsplit - 1) / a.nsplit);
   const int p0 = blockIdx.y * pps, p1 = min(p0 + pps, npages);
   const int* bt = a.bt + (long)b * a.W;
   const unsigned short* cache = (const unsigned short*)a.cache;
@@ -295,8 +330,10 @@ __global__ __launch_bounds__(RT > 8 ? 256 : 512) void attn(Args a) {
     for (int k = 0; k < RT; ++k) qf[k] = qp[4 * k];
   }
   dma(bt[p0], 0);
+  int next = bt[min(p0 + 1, p1 - 1)];
   __builtin_amdgcn_s_waitcnt(0x0f70);  // vmcnt(0)
   __syncthreads();
+  const unsigned lds0 = (unsigned)(uintptr_t)(KGS_LDS char*)smem;
 
   f32x4 acc[2 * RT];
 #pragma unroll
@@ -306,7 +343,10 @@ __global__ __launch_bounds__(RT > 8 ? 256 : 512) void attn(Args a) {
 
   for (int p = p0; p < p1; ++p) {
     const int buf = (p - p0) & 1;
-    if (p + 1 < p1) dma(bt[p + 1], buf ^ 1);  // that buffer was released by the last barrier
+    if (p + 1 < p1) {  // that buffer was released by the last barrier
+      dma(next, buf ^ 1);
+      next = bt[min(p + 2, p1 - 1)];
+    }
     const char* C = smem + buf * G::PAGEB;
     if (p * PAGE <= wmax) {
       f32x4 s[2];
@@ -347,11 +387,23 @@ __global__ __launch_bounds__(RT > 8 ? 256 : 512) void attn(Args a) {
           l += e;
         }
       const bf16x8 pf = pack_bf16x8(pr, 0);
+      // C^T fragments two output tiles at a time, one batch ahead of its MFMAs. By
+      // hand: the compiler takes a transposed read for a reader of the page being
+      // filled and would wait for the whole DMA in front of it.
+      const unsigned base = lds0 + buf * G::PAGEB;
+      TrBatch v[2];
+      v[0].template read<RT>(base, 0, 4 * g + tq, tp);
 #pragma unroll
-      for (int i = 0; i < 2 * RT; ++i) {
-        const int c0 = 2 * i + (tp >> 1), k0 = 4 * g + tq;
-        const bf16x8 vf = tr_frag(C + G::off(k0, c0) + 8 * (tp & 1), C + G::off(16 + k0, c0) + 8 * (tp & 1));
-        acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf, acc[i], 0, 0, 0);
+      for (int j = 0; j < RT; ++j) {
+        if (j + 1 < RT) {
+          v[(j + 1) & 1].template read<RT>(base, j + 1, 4 * g + tq, tp);
+          v[j & 1].template wait<4>();
+        } else {
+          v[j & 1].template wait<0>();
+        }
+#pragma unroll
+        for (int x = 0; x < 2; ++x)
+          acc[2 * j + x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v[j & 1].frag(x), pf, acc[2 * j + x], 0, 0, 0);
       }
     }
     __builtin_amdgcn_s_waitcnt(0x0f70);  // vmcnt(0): the next page has landed
