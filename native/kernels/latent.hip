@@ -14,6 +14,8 @@
 //   * attn          rows x pages on v_mfma_f32_16x16x32_bf16, split over the
 //                   context, + merge;
 //   * attn_simple   the same on the VALU for any RP and for fp32 caches.
+#include <type_traits>
+
 #include "kgs_common.h"
 
 namespace kgs {
@@ -232,6 +234,14 @@ struct Args {
   float scale, sl2;  // sl2 = scale * log2(e)
 };
 
+template <int I, int N, class F>
+__device__ __forceinline__ void static_for(F f) {
+  if constexpr (I < N) {
+    f(std::integral_constant<int, I>{});
+    static_for<I + 1, N>(f);
+  }
+}
+
 template <int RT>
 struct Geo {
   static constexpr int RP = 32 * RT, CH = 4 * RT, PITCH = 64 * RT, PAGEB = PAGE * PITCH;
@@ -243,6 +253,28 @@ struct Geo {
     else return (r >> 2) & 3;
   }
   __device__ static __forceinline__ int off(int r, int c) { return PITCH * r + 16 * (c ^ swz(r)); }
+};
+
+// LDS reads by hand, several batches ahead of their MFMAs: a wave has its SIMD to
+// itself here, so nothing else hides their latency, and the compiler takes a
+// transposed read for a reader of the page being filled and would wait for the
+// whole DMA in front of it. wait<N>: all but the N newest LDS operations are done.
+
+// one 32-column step of a page's keys 0-15 and 16-31 (A operands)
+struct KeyBatch {
+  bf16x8 f[2];
+  template <int RT>
+  __device__ __forceinline__ void read(unsigned base, int k, int l16, int g) {
+    using G = Geo<RT>;
+    const unsigned at = base + G::off(l16, 4 * k + g);
+    asm volatile("ds_read_b128 %0, %2\n\tds_read_b128 %1, %2 offset:%3"
+                 : "=&v"(f[0]), "=&v"(f[1])
+                 : "v"(at), "n"(16 * G::PITCH));
+  }
+  template <int N>
+  __device__ __forceinline__ void wait() {
+    asm volatile("s_waitcnt lgkmcnt(%2)" : "+v"(f[0]), "+v"(f[1]) : "n"(N));
+  }
 };
 
 // Two 16-column tiles of a page's 32 keys, transposed: four ds_read_b64_tr_b16
@@ -260,7 +292,6 @@ struct TrBatch {
                    : "v"(at), "n"(16 * G::PITCH));
     }
   }
-  // all but the N newest LDS operations have arrived
   template <int N>
   __device__ __forceinline__ void wait() {
     asm volatile("s_waitcnt lgkmcnt(%4)" : "+v"(lo[0]), "+v"(hi[0]), "+v"(lo[1]), "+v"(hi[1]) : "n"(N));
@@ -347,17 +378,23 @@ __global__ __launch_bounds__(RT > 8 ? 256 : 512) void attn(Args a) {
       dma(next, buf ^ 1);
       next = bt[min(p + 2, p1 - 1)];
     }
-    const char* C = smem + buf * G::PAGEB;
+    const unsigned base = lds0 + buf * G::PAGEB;
     if (p * PAGE <= wmax) {
-      f32x4 s[2];
+      constexpr int KD = RT < 5 ? RT : 5;  // batches in flight
+      KeyBatch kb[KD];
+      f32x4 s2[2][2] = {};  // even and odd steps: two chains per key tile
 #pragma unroll
-      for (int t = 0; t < 2; ++t) {
-        s[t] = f32x4{};
+      for (int k = 0; k < KD - 1; ++k) kb[k].template read<RT>(base, k, l16, g);
+      static_for<0, RT>([&](auto kc) {
+        constexpr int k = decltype(kc)::value;
+        if constexpr (k + KD - 1 < RT) kb[(k + KD - 1) % KD].template read<RT>(base, k + KD - 1, l16, g);
+        constexpr int newer = (k + KD - 1 < RT ? KD - 1 : RT - 1 - k) * 2;
+        kb[k % KD].template wait<newer>();
 #pragma unroll
-        for (int k = 0; k < RT; ++k)
-          s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(C + G::off(16 * t + l16, 4 * k + g)), qf[k],
-                                                         s[t], 0, 0, 0);
-      }
+        for (int t = 0; t < 2; ++t)
+          s2[t][k & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kb[k % KD].f[t], qf[k], s2[t][k & 1], 0, 0, 0);
+      });
+      f32x4 s[2] = {s2[0][0] + s2[0][1], s2[1][0] + s2[1][1]};
       float mx = m;
 #pragma unroll
       for (int t = 0; t < 2; ++t)
@@ -386,25 +423,21 @@ __global__ __launch_bounds__(RT > 8 ? 256 : 512) void attn(Args a) {
           pr[4 * t + r] = e;
           l += e;
         }
-      const bf16x8 pf = pack_bf16x8(pr, 0);
-      // C^T fragments two output tiles at a time, one batch ahead of its MFMAs. By
-      // hand: the compiler takes a transposed read for a reader of the page being
-      // filled and would wait for the whole DMA in front of it.
-      const unsigned base = lds0 + buf * G::PAGEB;
-      TrBatch v[2];
-      v[0].template read<RT>(base, 0, 4 * g + tq, tp);
+      // the first C^T fragments are on their way under the packing of P
+      constexpr int PD = RT < 4 ? RT : 4;
+      TrBatch v[PD];
 #pragma unroll
-      for (int j = 0; j < RT; ++j) {
-        if (j + 1 < RT) {
-          v[(j + 1) & 1].template read<RT>(base, j + 1, 4 * g + tq, tp);
-          v[j & 1].template wait<4>();
-        } else {
-          v[j & 1].template wait<0>();
-        }
+      for (int j = 0; j < PD - 1; ++j) v[j].template read<RT>(base, j, 4 * g + tq, tp);
+      const bf16x8 pf = pack_bf16x8(pr, 0);
+      static_for<0, RT>([&](auto jc) {
+        constexpr int j = decltype(jc)::value;
+        if constexpr (j + PD - 1 < RT) v[(j + PD - 1) % PD].template read<RT>(base, j + PD - 1, 4 * g + tq, tp);
+        constexpr int newer = (j + PD - 1 < RT ? PD - 1 : RT - 1 - j) * 4;
+        v[j % PD].template wait<newer>();
 #pragma unroll
         for (int x = 0; x < 2; ++x)
-          acc[2 * j + x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v[j & 1].frag(x), pf, acc[2 * j + x], 0, 0, 0);
-      }
+          acc[2 * j + x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v[j % PD].frag(x), pf, acc[2 * j + x], 0, 0, 0);
+      });
     }
     __builtin_amdgcn_s_waitcnt(0x0f70);  // vmcnt(0): the next page has landed
     __syncthreads();
