@@ -70,11 +70,11 @@ class RaggedSeqs:
     step_seqs: torch.Tensor | None = None
 
 
-def chunk_plan(row0, n) -> dict:
-    """Host arrays of a batch's split: ``chunks [c, 4]`` (first row, rows, sequence,
-    0), ``cseqs [s, 4]`` (sequence, first chunk, chunks, first row; longest first),
+def chunk_plan(row0, n, pos0, slot) -> dict:
+    """Host arrays of a batch's split: ``chunks [c, 8]`` (first row, rows, sequence, 0,
+    then its sequence's first row, first position and state slot, 0), ``cseqs [s, 4]`` (sequence, first chunk, chunks, first row; longest first),
     ``step_rows``, ``step_seqs``. Empty when every sequence steps."""
-    row0, n = np.asarray(row0), np.asarray(n)
+    row0, n, pos0, slot = (np.asarray(x) for x in (row0, n, pos0, slot))
     big = np.flatnonzero(n >= CHUNK_MIN)
     if not len(big):
         return {}
@@ -82,7 +82,9 @@ def chunk_plan(row0, n) -> dict:
     first = np.cumsum(nc) - nc
     seq = np.repeat(big, nc)
     at = (np.arange(nc.sum()) - np.repeat(first, nc)) * CHUNK
-    chunks = np.stack([row0[seq] + at, np.minimum(CHUNK, n[seq] - at), seq, np.zeros_like(seq)], 1)
+    zero = np.zeros_like(seq)
+    chunks = np.stack([row0[seq] + at, np.minimum(CHUNK, n[seq] - at), seq, zero, row0[seq], pos0[seq], slot[seq], zero],
+                      1)
     cseqs = np.stack([big, first, nc, row0[big]], 1)[np.argsort(-nc, kind="stable")]
     small = np.flatnonzero(n < CHUNK_MIN)
     rows = np.concatenate([np.arange(row0[s], row0[s] + n[s]) for s in small]) if len(small) else np.zeros(0, np.int64)

@@ -394,7 +394,7 @@ class HybridModel:
         row_seq = np.repeat(order, n[order])
         pos = pos0[row_seq] + np.arange(len(tokens)) - row0[row_seq]
         refs = [pk.add(a) for a in (tokens, slots, row_seq, row0, n, pos0, slot, bt, logit_rows)]
-        split = {k: pk.add(v) for k, v in chunk_plan(row0, n).items()} if self.has_state else {}
+        split = {k: pk.add(v) for k, v in chunk_plan(row0, n, pos0, slot).items()} if self.has_state else {}
         host = {g: self._host_plan(pk, g, row0, n, pos0, bt, row_seq, pos, refs) for g in self.geometries}
         get = pk.send()
         d = [get(r) for r in refs]

@@ -68,7 +68,7 @@ struct Args {
   // null when all are) and chunked ones
   const int *rows, *seqs;
   int nrows, nseqs;
-  const int4* chunks;  // (first row, rows, sequence, -)
+  const int4* chunks;  // per chunk (first row, rows, sequence, -), (sequence's first row, position, slot, -)
   const int4* cseqs;   // (sequence, first chunk, chunks, first row)
   int nchunks, ncseqs;
   float *cW, *cQ, *cK, *cE, *cU, *cP;  // per (chunk, head): [16][KP] x 2, [KP][16], [KP], [16][V], [16][16]
@@ -114,8 +114,8 @@ __device__ __forceinline__ void conv_in(const Args& a, long src, int c, int col,
                                         float (&x)[N]) {
 #pragma unroll
   for (int i = 0; i < N; ++i) x[i] = 0.f;
-  if (src >= r0) ldn((const T*)a.z + src * a.ldz + col, x);
-  else if (p0 > 0) ldn(a.conv + (slot * (a.taps - 1) + (src - r0 + a.taps - 1)) * a.C + c, x);
+  if (src >= r0) ldn((const T*)a.z + src * a.ldz + (unsigned)col, x);
+  else if (p0 > 0) ldn(a.conv + (slot * (a.taps - 1) + (src - r0 + a.taps - 1)) * a.C + (unsigned)c, x);
 }
 
 // ... of row t after the convolution and silu. TAPS 0: any number.
@@ -369,19 +369,27 @@ constexpr int CH = 16;  // tokens per chunk
 // LDS row pitch: two rows apart are 32 banks apart for n a multiple of 32
 __host__ __device__ __forceinline__ int chunk_ld(int n) { return n + 16; }
 
-// one workgroup per (chunk, head)
-template <typename T, int N, int TAPS>
+// 1 / sqrt
+template <bool FAST>
+__device__ __forceinline__ float rsqrt_(float x) {
+  if constexpr (FAST) return __builtin_amdgcn_rsqf(x);
+  return 1.0f / sqrtf(x);
+}
+
+// one workgroup per (chunk, head). FIX: K = V = FIX, known to the compiler (0: any)
+template <typename T, int N, int TAPS, int FIX>
 __global__ __launch_bounds__(256, 4) void chunk_prep(Args a) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
   __shared__ __attribute__((aligned(16))) float sA[CH][CH + 4], sT[CH][CH + 4], sbeta[CH], srq[CH], srk[CH];
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
-  const int KP = a.KP, V = a.V, H = a.H, ldk = chunk_ld(KP), ldv = chunk_ld(V);
+  const int K = FIX ? FIX : a.K, KP = FIX ? FIX : a.KP, V = FIX ? FIX : a.V, H = a.H;
+  const int ldk = chunk_ld(KP), ldv = chunk_ld(V);
   float *sq = sm, *sk = sq + CH * ldk, *sb = sk + CH * ldk, *sv = sb + CH * ldk;
   const int ck = __builtin_amdgcn_readfirstlane(blockIdx.x / H), h = blockIdx.x - ck * H;
-  const int4 it = a.chunks[ck];  // first row, rows, sequence
-  const int b = it.z, n = it.y, gh = __builtin_amdgcn_readfirstlane(h / (H / a.G));
-  const int r0 = a.row0[b], p0 = a.pos0[b], K = a.K;
-  const long slot = a.slot[b], t0 = it.x;
+  const int4 it = a.chunks[2 * ck], sq4 = a.chunks[2 * ck + 1];
+  const int n = it.y, gh = __builtin_amdgcn_readfirstlane(h / (H / a.G));
+  const int r0 = sq4.x, p0 = sq4.y;
+  const long slot = sq4.z, t0 = it.x;
   constexpr bool FAST = sizeof(T) == 2;
   // threads by channel groups of N: q, k, v convolutions, then the decays
   const int nk = KP / N, nv = (V + N - 1) / N;
@@ -415,7 +423,7 @@ __global__ __launch_bounds__(256, 4) void chunk_prep(Args a) {
       for (int t = 0; t < CH; ++t) {
 #pragma unroll
         for (int i = 0; i < N; ++i) x[t][i] = 0.f;
-        if (t < n && c < K) ldn((const T*)a.a2 + (t0 + t) * a.lda + h * K + c, x[t]);
+        if (t < n && c < K) ldn((const T*)a.a2 + (t0 + t) * a.lda + h * K + (unsigned)c, x[t]);
       }
 #pragma unroll
       for (int t = 0; t < CH; ++t)
@@ -440,7 +448,7 @@ __global__ __launch_bounds__(256, 4) void chunk_prep(Args a) {
     ssk = wave_sum(ssk);
     sqk = wave_sum(sqk);
     if (lane == 0) {
-      const float rq = 1.0f / sqrtf(ssq + 1e-6f) / sqrtf((float)K), rk = 1.0f / sqrtf(ssk + 1e-6f);
+      const float rq = rsqrt_<FAST>(ssq + 1e-6f) * rsqrt_<FAST>((float)K), rk = rsqrt_<FAST>(ssk + 1e-6f);
       srq[i] = rq;
       srk[i] = rk;
       a.cP[((long)ck * H + h) * CH * CH + i * CH + i] = sqk * rq * rk;  // P's diagonal has no decay
@@ -532,14 +540,13 @@ __global__ __launch_bounds__(256, 4) void chunk_prep(Args a) {
   for (int c = tid; c < KP + V; c += 256) {
     float x[CH];
     if (c < KP) {
-      float* Q = a.cQ + base * CH * KP + c;
-      float* Kt = a.cK + (base * KP + c) * CH;
+      float *Q = a.cQ + base * CH * KP, *Kt = a.cK + base * KP * CH;
       const float bc = sb[(CH - 1) * ldk + c];
 #pragma unroll
       for (int i = 0; i < CH; ++i) {
         const float bi = sb[i * ldk + c], k = sk[i * ldk + c] * srk[i], e = __builtin_amdgcn_exp2f(bi);
         x[i] = k * e;
-        Q[i * KP] = sq[i * ldk + c] * srq[i] * e;
+        Q[(unsigned)(i * KP + c)] = sq[i * ldk + c] * srq[i] * e;
       }
 #pragma unroll
       for (int i = 0; i < CH; i += 4) {
@@ -547,15 +554,15 @@ __global__ __launch_bounds__(256, 4) void chunk_prep(Args a) {
 #pragma unroll
         for (int y = 0; y < 4; ++y)
           v[y] = sk[(i + y) * ldk + c] * srk[i + y] * __builtin_amdgcn_exp2f(bc - sb[(i + y) * ldk + c]);
-        *(f32x4*)(Kt + i) = v;
+        *(f32x4*)(Kt + (unsigned)(c * CH + i)) = v;
       }
       a.cE[base * KP + c] = __builtin_amdgcn_exp2f(bc);
     } else {
 #pragma unroll
       for (int i = 0; i < CH; ++i) x[i] = sv[i * ldv + c - KP];
     }
-    float* o = c < KP ? a.cW + base * CH * KP + c : a.cU + base * CH * V + c - KP;
-    const int ldo = c < KP ? KP : V;
+    float* W = a.cW + base * CH * KP;
+    float* U = a.cU + base * CH * V;
 #pragma unroll
     for (int i = 0; i < CH; ++i) {
       asm volatile("" ::: "memory");  // T's rows are read here, not all kept in registers
@@ -566,7 +573,8 @@ __global__ __launch_bounds__(256, 4) void chunk_prep(Args a) {
 #pragma unroll
         for (int y = 0; y < 4; ++y) s = __builtin_fmaf(t[y], x[j + y], s);
       }
-      o[i * ldo] = s;
+      if (c < KP) W[(unsigned)(i * KP + c)] = s;
+      else U[(unsigned)(i * V + c - KP)] = s;
     }
   }
 }
@@ -799,12 +807,15 @@ static hipError_t run(const Args& a, hipStream_t s) {
   }
   if (a.nchunks > 0) {
     const size_t lds = sizeof(float) * CH * (3 * chunk_ld(a.KP) + chunk_ld(a.V));
+    auto prep_k = chunk_prep<T, N, TAPS, 0>;
+    if constexpr (N == 2 && TAPS == 4)
+      if (a.K == 128 && a.KP == 128 && a.V == 128) prep_k = chunk_prep<T, N, TAPS, 128>;
     if (lds > 48 * 1024) {
       const hipError_t e =
-          hipFuncSetAttribute((const void*)chunk_prep<T, N, TAPS>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+          hipFuncSetAttribute((const void*)prep_k, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
       if (e != hipSuccess) return e;
     }
-    hipLaunchKernelGGL((chunk_prep<T, N, TAPS>), dim3((unsigned)(a.nchunks * a.H)), dim3(256), lds, s, a);
+    hipLaunchKernelGGL(prep_k, dim3((unsigned)(a.nchunks * a.H)), dim3(256), lds, s, a);
     const long wide = (long)((a.V + 31) / 32) * a.H * a.ncseqs;
     if (a.V > 16 && wide >= 256) run_chunk_scan<T, 2>(a, s);
     else run_chunk_scan<T, 1>(a, s);

@@ -203,11 +203,13 @@ def test_delta_chunk_plan():
 
     n = np.array([3, 40, 1, 16])
     row0 = np.array([0, 3, 43, 44])
-    p = chunk_plan(row0, n)
-    assert p["chunks"].tolist() == [[3, 16, 1, 0], [19, 16, 1, 0], [35, 8, 1, 0], [44, 16, 3, 0]]
+    pos0, slot = np.array([5, 6, 7, 0]), np.array([4, 3, 2, 1])
+    p = chunk_plan(row0, n, pos0, slot)
+    assert p["chunks"].tolist() == [[3, 16, 1, 0, 3, 6, 3, 0], [19, 16, 1, 0, 3, 6, 3, 0], [35, 8, 1, 0, 3, 6, 3, 0],
+                                    [44, 16, 3, 0, 44, 0, 1, 0]]
     assert p["cseqs"].tolist() == [[1, 0, 3, 3], [3, 3, 1, 44]]
     assert p["step_rows"].tolist() == [0, 1, 2, 43] and p["step_seqs"].tolist() == [0, 2]
-    assert chunk_plan(row0[:1], n[:1]) == {}
+    assert chunk_plan(row0[:1], n[:1], pos0[:1], slot[:1]) == {}
 
 
 # -------------------------------------------------------------------- oracle

@@ -246,11 +246,7 @@ def test_engine_refuses_what_the_model_has_not():
 
 def test_trace_run_program(tmp_path):
     """bin/trace_run as a program: steps on standard input, logits in files."""
-    from kgs.utils.safetensors import save_file
-
-    cfg = HM.config("odd")
-    (tmp_path / "config.json").write_text(json.dumps(cfg.raw))
-    save_file(HM.weights(cfg), tmp_path / "model.safetensors")
+    _folder(tmp_path)
     toks = {k: tokens("odd", n, seed=n) for k, n in (("x", 40), ("y", 9))}
     steps = [{"step": 0, "entries": [{"id": "x", "tokens": toks["x"][:30], "want": [0, 29]},
                                      {"id": "y", "tokens": toks["y"][:8], "want": []}], "end": []},
@@ -265,3 +261,55 @@ def test_trace_run_program(tmp_path):
     assert not (tmp_path / "1.f32").exists()
     got = np.concatenate([np.fromfile(tmp_path / f"{i}.f32", dtype="<f4") for i in (0, 2)]).reshape(3, -1)
     check(torch.from_numpy(got), HM.oracle_logits("odd", toks["x"])[[0, 29, 39]], "float32")
+
+
+def _folder(tmp_path, name="odd"):
+    from kgs.utils.safetensors import save_file
+
+    cfg = HM.config(name)
+    (tmp_path / "config.json").write_text(json.dumps(cfg.raw))
+    save_file(HM.weights(cfg), tmp_path / "model.safetensors")
+    return str(tmp_path)
+
+
+def test_serving_benchmark_on_a_model_folder(tmp_path, capsys):
+    from kgs.serve.bench import main
+
+    assert main(["--model", _folder(tmp_path), "--requests", "5", "--input-len", "33", "--output-len", "6", "--max-batch",
+                 "4", "--max-model-len", "256", "--chunked-prefill", "48"]) == 0
+    out = json.loads(capsys.readouterr().out.strip().splitlines()[-1])
+    assert out["output_tok_per_s"] > 0 and out["stats"]["decode_tokens"] >= 5 * 5
+
+
+def test_engine_process_serves_a_model_folder(tmp_path):
+    """The HTTP server's engine process, started from a model folder's description."""
+    import asyncio
+
+    from kgs.models.registry import load_config, to_spec
+    from kgs.serve import EngineConfig, SamplingParams
+    from kgs.serve.dp import DPEngineLoop
+
+    ec = EngineConfig(num_pages=40, max_batch=2, max_model_len=256, dtype="float32", chunked_prefill=64)
+    runner = DPEngineLoop(1, to_spec(load_config(_folder(tmp_path))), ec, device="cuda", start_timeout=100)
+    prompt = tokens("odd", 20, seed=3)
+
+    async def one():
+        q: asyncio.Queue = asyncio.Queue()
+        runner.submit(prompt, SamplingParams(max_tokens=8, ignore_eos=True), asyncio.get_running_loop(), q)
+        assert (await q.get())[0] == "id"
+        out = []
+        while True:
+            _, t, fin, _, _ = await q.get()
+            out.append(t)
+            if fin:
+                return out
+
+    try:
+        got = asyncio.run(one())
+    finally:
+        runner.shutdown()
+
+    class R:
+        output = got
+
+    _greedy_ok("odd", [prompt], [R], "float32")

@@ -270,7 +270,8 @@ class DeltaCase:
             row0 = [sum(n[:i]) for i in range(len(n))]
             seqs = RaggedSeqs(i32([b for b, m in enumerate(n) for _ in range(m)]), i32(row0), i32(n),
                               i32([c[2] for c in call]), i32([c[3] for c in call]),
-                              **{k: i32(v.tolist()).reshape(v.shape) for k, v in chunk_plan(row0, n).items()})
+                              **{k: i32(v.tolist()).reshape(v.shape) for k, v in chunk_plan(row0, n, [c[2] for c in call],
+                                                                                        [c[3] for c in call]).items()})
             o = delta_forward(self.z[rows].cuda(), self.offs, self.a2[rows].cuda(), self.cw.cuda(), self.a_log.cuda(),
                               self.dt_bias.cuda(), self.sh, self.state, seqs)
             out[rows] = o.cpu()
