@@ -95,23 +95,6 @@ KGS_EXPORT int kgs_exp_gemm_w4h(const void* A, const void* B, void* C, int M, in
         hipLaunchKernelGGL((kgs::w4p::gemm_nt_w4p<kgs::EPI_NONE, 140000000, 1, false, false, 1>), pg, dim3(256), 0, s,
                            a, b, c, nullptr, M, N, K, lda, ldb, ldc, tq);
         break;
-      // round 4: MFMA order inside a k-sub (gemm_w4p.h ord_of): i-major / n-major, default and mirror G8 maps
-      case 139:
-        hipLaunchKernelGGL((kgs::w4p::gemm_nt_w4p<kgs::EPI_NONE, 0, 1, false, false, 10>), pg, dim3(256), 0, s, a, b, c,
-                           nullptr, M, N, K, lda, ldb, ldc, tq);
-        break;
-      case 140:
-        hipLaunchKernelGGL((kgs::w4p::gemm_nt_w4p<kgs::EPI_NONE, 0, 1, false, false, 30>), pg, dim3(256), 0, s, a, b, c,
-                           nullptr, M, N, K, lda, ldb, ldc, tq);
-        break;
-      case 141:
-        hipLaunchKernelGGL((kgs::w4p::gemm_nt_w4p<kgs::EPI_NONE, 140000008, 1, false, false, 10>), pg, dim3(256), 0, s,
-                           a, b, c, nullptr, M, N, K, lda, ldb, ldc, tq);
-        break;
-      case 142:
-        hipLaunchKernelGGL((kgs::w4p::gemm_nt_w4p<kgs::EPI_NONE, 140000008, 1, false, false, 30>), pg, dim3(256), 0, s,
-                           a, b, c, nullptr, M, N, K, lda, ldb, ldc, tq);
-        break;
       // round 5: C store measurement builds (gemm_w4p.h (L / 100) % 10): no store / drain after the stores
       case 143:
         hipLaunchKernelGGL((kgs::w4p::gemm_nt_w4p<kgs::EPI_NONE, 0, 1, false, false, 100>), pg, dim3(256), 0, s, a, b,

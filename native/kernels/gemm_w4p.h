@@ -106,9 +106,6 @@ struct Lay<1> {
   }
 };
 
-// L / 10 (experiments): the MFMA order inside a k-sub, L / 10 - 1 (gemm_w4.h
-// make_order: 0 i-major, 1 growing square, 2 n-major); 0 = Knobs (growing square).
-constexpr int ord_of(int L) { return (L / 10) % 10 ? (L / 10) % 10 - 1 : Kn::ORD; }
 // (L / 10^7) % 10 (experiments): the K-step schedule, barrier 1 after MFMA B1 and R MFMAs after
 // barrier 2 (the DMA window is [B1, KM - R)); 0 = Knobs (B1 24, R 20). 1: 20 / 20, 2: 24 / 16,
 // 3: 20 / 16, 4: 18 / 16 (a wider DMA window; the f1 reads end at MFMA NR = 16); 5: 20 / 24,
@@ -190,7 +187,7 @@ __device__ __forceinline__ auto make_tick(int* qx, int* slot) {
 template <int ST, int X, bool ZERO, int TK, int K, int L = 0, int WX = 0, int CAT = 1, class TQ = Tick>
 __device__ __forceinline__ void pbody(const Ctx& c, const Ctx& cd, const StepPtrs& sp, Frag<MA, NB>& f0,
                                       Frag<MA, NB>& f1, TQ& tq) {
-  constexpr int B1 = b1_of(L), R = r_of(L), P = Kn::P, ORD = ord_of(L);
+  constexpr int B1 = b1_of(L), R = r_of(L), P = Kn::P, ORD = Kn::ORD;
   constexpr int KM = S::KM, HM = S::HM, NR = S::NR, ND = w4::dma_per_stage<BM, BN>();
   static_assert(B1 >= NR && B1 + ND <= KM - R && NR <= R * P, "bad K-step schedule");
   if constexpr (K < KM) {
@@ -501,7 +498,7 @@ __device__ __forceinline__ void set_b(Ctx& c, const unsigned short* B, int tn, i
 // XCC_ID << 32, [2 + j] the end of its j-th tile's epilogue (j < 11), [13] its
 // exit (after the queue's exit counter / reset), [14] the end of its last tile,
 // [15] tiles.
-// L: LDS image layout (L % 10, Lay above) and MFMA order ((L / 10) % 10, ord_of); 0 = production.
+// L: LDS image layout (L % 10, Lay above); 0 = production.
 // (L / 100) % 10, the C store (experiments only, EPI_NONE): 1 = no store (output not written),
 // 2 = s_waitcnt vmcnt(0) right after each tile's stores (measurement builds: how much of a tile
 // change waits on its stores -- gfx950 counts stores and loads in one vmcnt, so the next tile's
@@ -627,8 +624,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     const char* pb = pbbase<L>(c, 0, 0);
 #pragma unroll
     for (int e = 0; e < S::NR; ++e) {
-      const int x = w4::rd_idx(ord_of(L), MA, NB, e);
-      if (w4::rd_isa(ord_of(L), MA, NB, e)) f0.a[x] = w4::frag(pa + Lay<L % 10>::frag_off(x));
+      const int x = w4::rd_idx(Kn::ORD, MA, NB, e);
+      if (w4::rd_isa(Kn::ORD, MA, NB, e)) f0.a[x] = w4::frag(pa + Lay<L % 10>::frag_off(x));
       else f0.b[x] = w4::frag(pb + Lay<L % 10>::frag_off(x));
     }
   }

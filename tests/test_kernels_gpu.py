@@ -755,11 +755,9 @@ def test_gemm_small_grid_routing_is_bitwise_the_256_tile(M, N, K):
 @pytest.mark.parametrize("M,N,K,variant", [(8192, 8192, 384, "w4p_0"), (4608, 4096, 384, "w4p_0"),
                                            (8192, 2304, 512, "w4p_140000000"), (1024, 768, 1024, "w4p_0"),
                                            (4608, 4096, 384, "w4pn_0"), (8192, 2304, 9216, "w4pn_140000008"),
-                                           # round 4: LDS layout 1 and the MFMA-order knobs
+                                           # round 4: LDS layout 1
                                            (4608, 4096, 384, "w4pl_0"), (8192, 2304, 9216, "w4pl_140000008"),
                                            (8192, 2304, 512, "w4pl_140000000"), (4096, 4608, 8320, "w4pl_8"),
-                                           (4608, 4096, 384, "w4po0_0"), (4608, 4096, 384, "w4po2_0"),
-                                           (8192, 2304, 9216, "w4po2_140000008"),
                                            # round 5: drain after each tile's stores (measurement build)
                                            (8192, 8192, 384, "w4pd_0"), (8192, 8192, 384, "w4pw_0"),
                                            (8192, 2304, 9216, "w4pw_0"), (4608, 4096, 384, "w4pw_0"),
