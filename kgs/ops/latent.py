@@ -69,9 +69,10 @@ class LatentRows:
     nsplit: int
 
 
-def split_count(ntiles: int, max_pages: int) -> int:
-    """Context splits: about two workgroups per CU, at least two pages each."""
-    return max(1, min(2 * CUS // max(1, ntiles), (max_pages + 1) // 2, 64))
+def split_count(ntiles: int, max_pages: int, rp: int = 0) -> int:
+    """Context splits: as many workgroups as the CUs hold at once (two each, one
+    where the page ring takes most of the LDS), at least two pages each."""
+    return max(1, min((1 if rp > 384 else 2) * CUS // max(1, ntiles), (max_pages + 1) // 2, 64))
 
 
 def waves_for(rows: int, rp: int) -> int:

@@ -438,7 +438,7 @@ class HybridModel:
                          "tok_seq": pk.add(np.repeat(np.arange(len(sel)), ns)), "tok_pos": pk.add(pos[at]),
                          "rows": None if order is None else pk.add(order), "items": pk.add(items)},
                         {"nt": int(ns.sum()), "ntiles": len(items), "tiles": 0, "waves": waves,
-                         "nsplit": split_count(len(items), maxp)})
+                         "nsplit": split_count(len(items), maxp, g.rp)})
         sel = np.flatnonzero(big)
         if len(sel):
             items, ctx, base = [], [], 0
@@ -473,6 +473,6 @@ class HybridModel:
             plans[g] = LatentPlan(LatentRows(
                 nt=nb, q0=f["ar"], n=f["one"], pos0=positions, bt=block_tables, tok_seq=f["ar"], tok_pos=positions,
                 rows=None, items=None, ntiles=nb * tiles, tiles=tiles, waves=waves,
-                nsplit=split_count(nb * tiles, W)), None)
+                nsplit=split_count(nb * tiles, W, g.rp)), None)
         seqs = RaggedSeqs(f["ar"], f["ar"], f["one"], positions, state_slots if self.has_state else f["zero"])
         return self.forward(Batch(tokens, slots, seqs, plans, None))

@@ -246,6 +246,8 @@ template <int RT>
 struct Geo {
   static constexpr int RP = 32 * RT, CH = 4 * RT, PITCH = 64 * RT, PAGEB = PAGE * PITCH;
   static constexpr int LOW = CH & -CH, P = LOW > 16 ? 16 : LOW;
+  static constexpr int NP = P / 4;             // column steps whose swizzled addresses differ in more than an offset
+  static constexpr int NB = RT == 12 ? 3 : 4;  // pages in the ring: two workgroups per CU up to 384, one at 512
   // XOR of a row's 16-B chunk index: rows that share banks land on other chunks
   __device__ static __forceinline__ int swz(int r) {
     if constexpr (P == 16) return ((r & 3) << 2) | ((r >> 1) & 2) | ((r >> 3) & 1);
@@ -263,13 +265,14 @@ struct Geo {
 // one 32-column step of a page's keys 0-15 and 16-31 (A operands)
 struct KeyBatch {
   bf16x8 f[2];
-  template <int RT>
-  __device__ __forceinline__ void read(unsigned base, int k, int l16, int g) {
+  // at: address of step k % NP
+  template <int RT, int K>
+  __device__ __forceinline__ void read(unsigned at) {
     using G = Geo<RT>;
-    const unsigned at = base + G::off(l16, 4 * k + g);
-    asm volatile("ds_read_b128 %0, %2\n\tds_read_b128 %1, %2 offset:%3"
+    constexpr int o = 16 * G::P * (K / G::NP);
+    asm volatile("ds_read_b128 %0, %2 offset:%3\n\tds_read_b128 %1, %2 offset:%4"
                  : "=&v"(f[0]), "=&v"(f[1])
-                 : "v"(at), "n"(16 * G::PITCH));
+                 : "v"(at), "n"(o), "n"(o + 16 * G::PITCH));
   }
   template <int N>
   __device__ __forceinline__ void wait() {
@@ -281,16 +284,16 @@ struct KeyBatch {
 // (keys k0 .. and 16 + k0 .. of each), see tr_frag
 struct TrBatch {
   bf16x4 lo[2], hi[2];
-  template <int RT>
-  __device__ __forceinline__ void read(unsigned base, int j, int k0, int tp) {
+  // at: addresses of the two tiles of step j % NP
+  template <int RT, int J>
+  __device__ __forceinline__ void read(const unsigned (&at)[2]) {
     using G = Geo<RT>;
+    constexpr int o = 16 * G::P * (J / G::NP);
 #pragma unroll
-    for (int x = 0; x < 2; ++x) {
-      const unsigned at = base + G::off(k0, 2 * (2 * j + x) + (tp >> 1)) + 8 * (tp & 1);
-      asm volatile("ds_read_b64_tr_b16 %0, %2\n\tds_read_b64_tr_b16 %1, %2 offset:%3"
+    for (int x = 0; x < 2; ++x)
+      asm volatile("ds_read_b64_tr_b16 %0, %2 offset:%3\n\tds_read_b64_tr_b16 %1, %2 offset:%4"
                    : "=&v"(lo[x]), "=&v"(hi[x])
-                   : "v"(at), "n"(16 * G::PITCH));
-    }
+                   : "v"(at[x]), "n"(o), "n"(o + 16 * G::PITCH));
   }
   template <int N>
   __device__ __forceinline__ void wait() {
@@ -301,15 +304,41 @@ struct TrBatch {
   }
 };
 
+// one wave's part of a page into its slot of the ring, swizzled
+template <int RT>
+__device__ __forceinline__ void page_dma(const unsigned short* page, char* dst, int w, int nw, int lane) {
+  using G = Geo<RT>;
+  const __amdgpu_buffer_rsrc_t src = __builtin_amdgcn_make_buffer_rsrc((void*)page, 0, G::PAGEB, 0x00020000);
+#pragma unroll 4
+  for (int i = w; i < 2 * RT; i += nw) {
+    const int L = 64 * i + lane, r = L / G::CH, c = (L % G::CH) ^ G::swz(r);
+    __builtin_amdgcn_raw_ptr_buffer_load_lds(src, (KGS_LDS void*)(dst + 1024 * i), 16, r * G::PITCH + 16 * c, 0, 0, 0);
+  }
+}
+
+// All but the n newest vector memory operations of this wave are done (or fewer left).
+__device__ __forceinline__ void vm_wait(int n) {
+  if (n >= 32) asm volatile("s_waitcnt vmcnt(32)" ::: "memory");
+  else if (n >= 24) asm volatile("s_waitcnt vmcnt(24)" ::: "memory");
+  else if (n >= 16) asm volatile("s_waitcnt vmcnt(16)" ::: "memory");
+  else if (n >= 12) asm volatile("s_waitcnt vmcnt(12)" ::: "memory");
+  else if (n >= 8) asm volatile("s_waitcnt vmcnt(8)" ::: "memory");
+  else if (n >= 4) asm volatile("s_waitcnt vmcnt(4)" ::: "memory");
+  else if (n >= 2) asm volatile("s_waitcnt vmcnt(2)" ::: "memory");
+  else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+}
+
 // Workgroup: 16 rows per wave of one sequence's (token, head) rows, head fastest,
 // over the pages of one context split. S^T = C Q^T, so a lane owns row
 // (lane & 15) and keys 16 t + 4 (lane >> 4) + r of a page; the same registers
 // are the B operand of O^T = C^T P^T, whose A operand is the page read
-// transposed (ds_read_b64_tr_b16) in that key order.
+// transposed (ds_read_b64_tr_b16) in that key order. Pages come through a ring of
+// NB, NB - 1 of them in flight; one barrier per page says both that it has landed
+// for every wave and that the page before it has been read by every wave.
 template <int RT>
 __global__ __launch_bounds__(RT > 8 ? 256 : 512) void attn(Args a) {
   using G = Geo<RT>;
-  extern __shared__ __attribute__((aligned(16))) char smem[];  // two pages
+  extern __shared__ __attribute__((aligned(16))) char smem[];  // NB pages
   const int lane = threadIdx.x & 63, nw = blockDim.x >> 6;
   const int w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int l16 = lane & 15, g = lane >> 4, tq = (lane >> 2) & 3, tp = lane & 3;
@@ -346,25 +375,33 @@ __global__ __launch_bounds__(RT > 8 ? 256 : 512) void attn(Args a) {
     return;
   }
 
-  auto dma = [&](int page, int buf) {
-    const unsigned short* src = cache + (long)page * PAGE * G::RP;
-    for (int i = w; i < 2 * RT; i += nw) {
-      const int L = 64 * i + lane, r = L / G::CH, c = (L % G::CH) ^ G::swz(r);
-      glds16(src + r * G::RP + 8 * c, smem + buf * G::PAGEB + 1024 * i);
-    }
-  };
-
   bf16x8 qf[RT];
   {
     const bf16x8* qp = (const bf16x8*)((const unsigned short*)a.q + (base + row) * G::RP + 8 * g);
 #pragma unroll
     for (int k = 0; k < RT; ++k) qf[k] = qp[4 * k];
   }
-  dma(bt[p0], 0);
-  int next = bt[min(p0 + 1, p1 - 1)];
-  __builtin_amdgcn_s_waitcnt(0x0f70);  // vmcnt(0)
-  __syncthreads();
+
+  int ids = 0;  // lane j: the id of page pb + j
+  int pb = p0 - 64;
+  const int per = 2 * RT / nw;  // DMA instructions per page and wave, rounded down
+  auto dma = [&](int p) {
+    if (p - pb >= 64) {
+      pb = p;
+      ids = bt[min(p + lane, p1 - 1)];
+    }
+    const int page = __builtin_amdgcn_readlane(ids, p - pb);
+    page_dma<RT>(cache + (long)page * PAGE * G::RP, smem + (p - p0) % G::NB * G::PAGEB, w, nw, lane);
+  };
+  for (int p = p0; p < min(p0 + G::NB - 1, p1); ++p) dma(p);
   const unsigned lds0 = (unsigned)(uintptr_t)(KGS_LDS char*)smem;
+  unsigned ka[G::NP], va[G::NP][2];
+#pragma unroll
+  for (int k = 0; k < G::NP; ++k) {
+    ka[k] = lds0 + G::off(l16, 4 * k + g);
+#pragma unroll
+    for (int x = 0; x < 2; ++x) va[k][x] = lds0 + G::off(4 * g + tq, 2 * (2 * k + x) + (tp >> 1)) + 8 * (tp & 1);
+  }
 
   f32x4 acc[2 * RT];
 #pragma unroll
@@ -373,21 +410,28 @@ __global__ __launch_bounds__(RT > 8 ? 256 : 512) void attn(Args a) {
   const float sl2 = a.sl2;
 
   for (int p = p0; p < p1; ++p) {
-    const int buf = (p - p0) & 1;
-    if (p + 1 < p1) {  // that buffer was released by the last barrier
-      dma(next, buf ^ 1);
-      next = bt[min(p + 2, p1 - 1)];
-    }
-    const unsigned base = lds0 + buf * G::PAGEB;
+    vm_wait(min(G::NB - 2, p1 - 1 - p) * per);
+    asm volatile("s_barrier" ::: "memory");
+    if (p + G::NB - 1 < p1) dma(p + G::NB - 1);
     if (p * PAGE <= wmax) {
+      const unsigned slot = (p - p0) % G::NB * G::PAGEB;
+      unsigned kp[G::NP], vp[G::NP][2];
+#pragma unroll
+      for (int k = 0; k < G::NP; ++k) {
+        kp[k] = ka[k] + slot;
+        vp[k][0] = va[k][0] + slot;
+        vp[k][1] = va[k][1] + slot;
+      }
       constexpr int KD = RT < 5 ? RT : 5;  // batches in flight
       KeyBatch kb[KD];
       f32x4 s2[2][2] = {};  // even and odd steps: two chains per key tile
-#pragma unroll
-      for (int k = 0; k < KD - 1; ++k) kb[k].template read<RT>(base, k, l16, g);
+      static_for<0, KD - 1>([&](auto kc) {
+        constexpr int k = decltype(kc)::value;
+        kb[k].template read<RT, k>(kp[k % G::NP]);
+      });
       static_for<0, RT>([&](auto kc) {
         constexpr int k = decltype(kc)::value;
-        if constexpr (k + KD - 1 < RT) kb[(k + KD - 1) % KD].template read<RT>(base, k + KD - 1, l16, g);
+        if constexpr (k + KD - 1 < RT) kb[(k + KD - 1) % KD].template read<RT, k + KD - 1>(kp[(k + KD - 1) % G::NP]);
         constexpr int newer = (k + KD - 1 < RT ? KD - 1 : RT - 1 - k) * 2;
         kb[k % KD].template wait<newer>();
 #pragma unroll
@@ -426,12 +470,14 @@ __global__ __launch_bounds__(RT > 8 ? 256 : 512) void attn(Args a) {
       // the first C^T fragments are on their way under the packing of P
       constexpr int PD = RT < 4 ? RT : 4;
       TrBatch v[PD];
-#pragma unroll
-      for (int j = 0; j < PD - 1; ++j) v[j].template read<RT>(base, j, 4 * g + tq, tp);
+      static_for<0, PD - 1>([&](auto jc) {
+        constexpr int j = decltype(jc)::value;
+        v[j].template read<RT, j>(vp[j % G::NP]);
+      });
       const bf16x8 pf = pack_bf16x8(pr, 0);
       static_for<0, RT>([&](auto jc) {
         constexpr int j = decltype(jc)::value;
-        if constexpr (j + PD - 1 < RT) v[(j + PD - 1) % PD].template read<RT>(base, j + PD - 1, 4 * g + tq, tp);
+        if constexpr (j + PD - 1 < RT) v[(j + PD - 1) % PD].template read<RT, j + PD - 1>(vp[(j + PD - 1) % G::NP]);
         constexpr int newer = (j + PD - 1 < RT ? PD - 1 : RT - 1 - j) * 4;
         v[j % PD].template wait<newer>();
 #pragma unroll
@@ -439,8 +485,6 @@ __global__ __launch_bounds__(RT > 8 ? 256 : 512) void attn(Args a) {
           acc[2 * j + x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v[j % PD].frag(x), pf, acc[2 * j + x], 0, 0, 0);
       });
     }
-    __builtin_amdgcn_s_waitcnt(0x0f70);  // vmcnt(0): the next page has landed
-    __syncthreads();
   }
   l = xor32_sum(xor16_sum(l));
   if (myrow > last) return;
@@ -565,7 +609,7 @@ __global__ __launch_bounds__(256) void attn_simple(Args a) {
 
 template <int RT>
 static hipError_t launch_attn(const Args& a, int ntiles, int nw, hipStream_t s) {
-  const size_t lds = 2 * Geo<RT>::PAGEB;
+  const size_t lds = Geo<RT>::NB * Geo<RT>::PAGEB;
   if (lds > 48 * 1024) {
     const hipError_t e =
         hipFuncSetAttribute((const void*)attn<RT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
