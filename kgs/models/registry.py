@@ -30,6 +30,7 @@ class Architecture:
 ARCHITECTURES = {a.name: a for a in (
     Architecture("Llama", "kgs.models.llama:LlamaConfig", "kgs.serve.model:ServingModel"),
     Architecture("Ruruzen", "kgs.models.ruruzen:RuruzenConfig", "kgs.serve.hybrid:HybridModel"),
+    Architecture("Nufusun", "kgs.models.nufusun:NufusunConfig", "kgs.serve.nufusun:NufusunModel"),
 )}
 
 

@@ -111,6 +111,21 @@ _SIGS = {
                                                                                 _c_void_p], _c_int),
     "kgs_head_proj": ([_c_void_p] * 6 + [_c_long] * 5 + [_c_int] * 5 + [_c_void_p], _c_int),
     "kgs_latent_attn": ([_c_void_p] * 10 + [_c_int] * 8 + [ctypes.c_float, _c_void_p], _c_int),
+    # residual, talking-heads attention, mixture of experts (residual.hip, talking.hip, moe.hip)
+    "kgs_residual_embed": ([_c_void_p] * 3 + [_c_long, ctypes.c_float] + [_c_void_p] * 2 + [_c_long, _c_void_p]
+                           + [_c_int] * 4 + [ctypes.c_float, _c_int, _c_void_p], _c_int),
+    "kgs_residual_add": ([_c_void_p] * 2 + [_c_long] + [_c_void_p] * 2 + [_c_long] * 2 + [_c_int] * 2
+                         + [_c_void_p, _c_int] + [_c_void_p] * 2 + [_c_long, _c_void_p] + [_c_int] * 4
+                         + [ctypes.c_float, _c_int, _c_void_p], _c_int),
+    "kgs_talking_write": ([_c_void_p, _c_long] + [_c_void_p] * 3 + [_c_int] * 8 + [_c_void_p], _c_int),
+    "kgs_talking_rows": ([_c_void_p, _c_long, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_int] + [_c_void_p] * 8
+                         + [_c_int] * 10 + [_c_void_p], _c_int),
+    "kgs_talking_tiles": ([_c_void_p, _c_long, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_int, _c_void_p, _c_int]
+                          + [_c_void_p] * 3 + [_c_int] * 6 + [_c_void_p], _c_int),
+    "kgs_moe_route": ([_c_void_p, _c_long] + [_c_void_p] * 6 + [_c_int] * 6 + [_c_void_p], _c_int),
+    "kgs_moe_plan": ([_c_void_p] * 9 + [_c_int] * 4 + [_c_void_p], _c_int),
+    "kgs_moe_grouped": ([_c_void_p, _c_long, _c_void_p, _c_void_p, _c_long] + [_c_void_p] * 4 + [_c_int] * 7
+                        + [ctypes.c_float] + [_c_int] * 2 + [_c_void_p], _c_int),
     "kgs_latent_attn_simple": ([_c_void_p] * 6 + [_c_int] * 4 + [ctypes.c_float, _c_int, _c_void_p], _c_int),
     "kgs_attn_fwd_ragged_bf16": ([_c_void_p] * 5 + [_c_int] * 3 + [_c_long] * 4 + [ctypes.c_float, _c_void_p, _c_long,
                                                                                   _c_void_p], _c_int),

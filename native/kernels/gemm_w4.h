@@ -65,7 +65,8 @@
 //               I + tn BN/2 ..), so every wave holds the gate and up columns of
 //               the same outputs, and the epilogue stores silu(g) * u: a
 //               [M, I] activation with no [M, 2I] round trip and no silu_mul
-//               launch. Same roundings as gate|up GEMM + silu_mul.
+//               launch. Same roundings as gate|up GEMM + silu_mul. (1: silu, 2: tanh
+//               gelu; 3: the grouped expert GEMM of moe.hip, whose A rows are gathered.)
 
 namespace kgs {
 namespace w4 {
@@ -97,6 +98,7 @@ struct Ctx {
   __amdgpu_buffer_rsrc_t ra, rb;
   __amdgpu_buffer_rsrc_t rb2;  // SwiGLU: the up block (rb holds the gate block)
   int voa, vob;     // per-lane DMA byte offsets (row, swizzled chunk)
+  int vog[8];       // gathered A rows (SW digit 3, moe.hip): the offset of every DMA row group
   int sa32, sb32;   // bytes between DMA row groups (32 rows)
   int w, wr, wc;
   int ro0, ro1;     // per-lane fragment byte offsets, k-sub 0 / 1
@@ -119,11 +121,13 @@ __device__ __forceinline__ void bar() {
 // K-tile starting at k0 into stage st: rows j*32 + w*8 + lane/8, 1 KiB = 8 rows
 // of 128 B. AUX: cache-policy bits of the load (0 = default; 16 = sc1). SW:
 // SwiGLU staging of B (groups alternate gate / up, see the MODE notes above).
-template <int BM, int BN, int OP, int AUX = 0, bool SW = false, bool PK = false>
+template <int BM, int BN, int OP, int AUX = 0, bool SW = false, bool PK = false, bool GA = false>
 __device__ __forceinline__ void dma(const Ctx& c, int st, int j, int k0) {
   using S = Shape<BM, BN>;
   char* dst = c.smem + st * S::STAGE + OP * S::OPA + (j * 4 + c.w) * 1024;
-  if constexpr (OP == 1 && PK) {
+  if constexpr (OP == 0 && GA) {
+    __builtin_amdgcn_raw_ptr_buffer_load_lds(c.ra, (KGS_LDS void*)dst, 16, c.vog[j], k0 * 2, 0, AUX);
+  } else if constexpr (OP == 1 && PK) {
     // packed B ([N/BN][K/BK][BN][BK], see PACKB): K-tile k0 / BK of this
     // panel is one contiguous BN x 128 B block
     const int so = j * c.sb32 + k0 * BN * 2;
@@ -150,15 +154,16 @@ __device__ __forceinline__ void dma_any(const Ctx& c, int st, int j, int k0) {
   constexpr int AUX = AUXX >= 50 ? AUXX - 50 : AUXX;   // B
   constexpr int AUXA = AUXX >= 50 ? 0 : AUXX;          // A
   constexpr bool SW = (X / 1000000) % 10 != 0;
+  constexpr bool GA = (X / 1000000) % 10 == 3;
   constexpr int ORDB = (X / 100000000) % 10;  // 1: the B operand's DMAs first, 2: A and B interleaved
   constexpr bool PK = (X / 1000000000) == 1;  // B packed by K-tile (PACKB)
   constexpr int JA = BM / 32, JB = BN / 32;
   if constexpr (ORDB == 1) {
-    if (j < JB) dma<BM, BN, 1, AUX, SW, PK>(c, st, j, k0); else dma<BM, BN, 0, AUXA>(c, st, j - JB, k0);
+    if (j < JB) dma<BM, BN, 1, AUX, SW, PK>(c, st, j, k0); else dma<BM, BN, 0, AUXA, false, false, GA>(c, st, j - JB, k0);
   } else if constexpr (ORDB == 2 && JA == JB) {
-    if (j & 1) dma<BM, BN, 1, AUX, SW, PK>(c, st, j >> 1, k0); else dma<BM, BN, 0, AUXA>(c, st, j >> 1, k0);
+    if (j & 1) dma<BM, BN, 1, AUX, SW, PK>(c, st, j >> 1, k0); else dma<BM, BN, 0, AUXA, false, false, GA>(c, st, j >> 1, k0);
   } else {
-    if (j < JA) dma<BM, BN, 0, AUXA>(c, st, j, k0); else dma<BM, BN, 1, AUX, SW, PK>(c, st, j - JA, k0);
+    if (j < JA) dma<BM, BN, 0, AUXA, false, false, GA>(c, st, j, k0); else dma<BM, BN, 1, AUX, SW, PK>(c, st, j - JA, k0);
   }
 }
 

@@ -1,0 +1,175 @@
+// The fp32 residual of models whose layers add all their sublayers at once: one
+// launch adds a layer's outputs (the mixer's projection and its bias, and every
+// token's chosen experts' rows) and produces the next layer's normed input; another
+// starts the residual from the embedding table. RMS norm with a weight stored
+// around zero: x / sqrt(mean x^2 + eps) * (1 + w). Activations bf16 or fp32.
+//
+// One workgroup per token. Rows are padded to a multiple of 8 columns whose weights
+// and inputs are zero, so only the mean knows the true width.
+#include "kgs_common.h"
+
+namespace kgs {
+namespace residual {
+
+constexpr int MAX_NV = 8;  // 8-column chunks per thread
+
+struct Args {
+  float* x;           // [T, wp]
+  const int* tokens;  // start of the residual
+  const void* embed;
+  long lde;
+  float scale;
+  const void* a;      // mixer output [T, lda] or null, and its bias [wp] or null
+  long lda;
+  const float* ab;
+  const void* y;      // expert rows [nslice][nrows][ldy] or null
+  const int* pos;     // [T, top]: each choice's row, -1: none
+  int top, y32, nslice;
+  long ldy, yslice;
+  const float* w;     // [wp]
+  void* h;            // [T, ldh]
+  long ldh;
+  int* zero;          // counters the next launches use, cleared here
+  int nzero;
+  int width, wp;
+  float eps;
+};
+
+__device__ __forceinline__ void load8(const float* p, float (&v)[8]) {
+  const f32x4 a = *(const f32x4*)p, b = *(const f32x4*)(p + 4);
+#pragma unroll
+  for (int i = 0; i < 4; ++i) v[i] = a[i], v[4 + i] = b[i];
+}
+__device__ __forceinline__ void load8(const unsigned short* p, float (&v)[8]) {
+  const bf16x8 a = *(const bf16x8*)p;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) v[i] = bf2f((unsigned short)a[i]);
+}
+__device__ __forceinline__ void store8(float* p, const float (&v)[8]) {
+  *(f32x4*)p = f32x4{v[0], v[1], v[2], v[3]};
+  *(f32x4*)(p + 4) = f32x4{v[4], v[5], v[6], v[7]};
+}
+__device__ __forceinline__ void store8(unsigned short* p, const float (&v)[8]) { *(bf16x8*)p = pack_bf16x8(v, 0); }
+
+template <typename T, int NV, bool EMBED>
+__global__ __launch_bounds__(256) void step(Args a) {
+  const long t = blockIdx.x;
+  const int tid = threadIdx.x, nt = blockDim.x, nc = a.wp / 8;
+  __shared__ float part[4];
+  if (blockIdx.x == 0)
+    for (int i = tid; i < a.nzero; i += nt) a.zero[i] = 0;
+  float v[NV][8], ss = 0.f;
+  const T* src = EMBED ? (const T*)a.embed + (long)a.tokens[t] * a.lde : (const T*)a.a + t * a.lda;
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int c = tid + k * nt;
+    if (c >= nc) continue;
+    float* xp = a.x + t * a.wp + 8 * c;
+    if constexpr (EMBED) {
+      load8(src + 8 * c, v[k]);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[k][i] *= a.scale;
+    } else {
+      float s[8] = {};
+      if (a.a) load8(src + 8 * c, s);
+      if (a.ab) {
+        float b[8];
+        load8(a.ab + 8 * c, b);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) s[i] += b[i];
+      }
+      if (a.y) {
+        for (int j = 0; j < a.top; ++j) {
+          const int p = a.pos[t * a.top + j];
+          if (p < 0) continue;
+          for (int sl = 0; sl < a.nslice; ++sl) {
+            float e[8];
+            const long o = sl * a.yslice + p * a.ldy + 8 * c;
+            if (a.y32) load8((const float*)a.y + o, e);
+            else load8((const unsigned short*)a.y + o, e);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) s[i] += e[i];
+          }
+        }
+      }
+      load8(xp, v[k]);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[k][i] += s[i];
+    }
+    store8(xp, v[k]);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) ss = __builtin_fmaf(v[k][i], v[k][i], ss);
+  }
+  ss = wave_sum(ss);
+  if (nt > 64) {
+    if ((tid & 63) == 0) part[tid >> 6] = ss;
+    __syncthreads();
+    ss = part[0];
+    for (int i = 1; i < nt / 64; ++i) ss += part[i];
+  }
+  const float inv = 1.0f / sqrtf(ss / a.width + a.eps);
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int c = tid + k * nt;
+    if (c >= nc) continue;
+    float w[8];
+    load8(a.w + 8 * c, w);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) w[i] = v[k][i] * inv * (1.0f + w[i]);
+    store8((T*)a.h + t * a.ldh + 8 * c, w);
+  }
+}
+
+template <typename T, bool EMBED>
+int launch(const Args& a, int rows, hipStream_t s) {
+  const int nc = a.wp / 8;
+  const int nt = nc >= 256 ? 256 : (nc + 63) / 64 * 64;
+  const int nv = (nc + nt - 1) / nt;
+  const dim3 grid(rows), block(nt);
+  if (nv <= 1) hipLaunchKernelGGL((step<T, 1, EMBED>), grid, block, 0, s, a);
+  else if (nv <= 2) hipLaunchKernelGGL((step<T, 2, EMBED>), grid, block, 0, s, a);
+  else if (nv <= 4) hipLaunchKernelGGL((step<T, 4, EMBED>), grid, block, 0, s, a);
+  else hipLaunchKernelGGL((step<T, 8, EMBED>), grid, block, 0, s, a);
+  return (int)hipGetLastError();
+}
+
+int check(const Args& a, int rows, int f32) {
+  if (rows <= 0 || a.width <= 0 || a.wp < a.width || a.wp > 256 * 8 * MAX_NV || a.ldh < a.wp) return KGS_ERR_SHAPE;
+  if (a.wp % 8 || a.ldh % 8 || (((uintptr_t)a.x | (uintptr_t)a.h | (uintptr_t)a.w) & 15)) return KGS_ERR_ALIGN;
+  return KGS_OK;
+}
+
+}  // namespace residual
+}  // namespace kgs
+
+// x [T, wp] fp32 = scale * embed[token]; h = norm(x). zero: counters to clear, or null.
+KGS_EXPORT int kgs_residual_embed(void* x, const void* tokens, const void* embed, long lde, float scale, const void* w,
+                                  void* h, long ldh, void* zero, int nzero, int rows, int width, int wp, float eps,
+                                  int f32, hipStream_t s) {
+  using namespace kgs::residual;
+  Args a{};
+  a.x = (float*)x, a.tokens = (const int*)tokens, a.embed = embed, a.lde = lde, a.scale = scale;
+  a.w = (const float*)w, a.h = h, a.ldh = ldh, a.zero = (int*)zero, a.nzero = zero ? nzero : 0;
+  a.width = width, a.wp = wp, a.eps = eps;
+  if (int rc = check(a, rows, f32)) return rc;
+  if (lde < wp) return KGS_ERR_SHAPE;
+  if (lde % 8 || ((uintptr_t)embed & 15)) return KGS_ERR_ALIGN;
+  return f32 ? launch<float, true>(a, rows, s) : launch<unsigned short, true>(a, rows, s);
+}
+
+// x += a + ab + sum of each token's expert rows y[pos[t][j]] (over nslice partial
+// products, yslice elements apart); h = norm(x).
+KGS_EXPORT int kgs_residual_add(void* x, const void* a_, long lda, const void* ab, const void* y, long ldy, long yslice,
+                                int nslice, int y32, const void* pos, int top, const void* w, void* h, long ldh,
+                                void* zero, int nzero, int rows, int width, int wp, float eps, int f32, hipStream_t s) {
+  using namespace kgs::residual;
+  Args a{};
+  a.x = (float*)x, a.a = a_, a.lda = lda, a.ab = (const float*)ab;
+  a.y = y, a.ldy = ldy, a.yslice = yslice, a.nslice = nslice, a.y32 = y32, a.pos = (const int*)pos, a.top = top;
+  a.w = (const float*)w, a.h = h, a.ldh = ldh, a.zero = (int*)zero, a.nzero = zero ? nzero : 0;
+  a.width = width, a.wp = wp, a.eps = eps;
+  if (int rc = check(a, rows, f32)) return rc;
+  if ((a_ && lda < wp) || (y && (ldy < wp || top <= 0 || nslice <= 0 || !pos))) return KGS_ERR_SHAPE;
+  if (lda % 8 || ldy % 8 || yslice % 8 || (((uintptr_t)a_ | (uintptr_t)y | (uintptr_t)ab) & 15)) return KGS_ERR_ALIGN;
+  return f32 ? launch<float, false>(a, rows, s) : launch<unsigned short, false>(a, rows, s);
+}
