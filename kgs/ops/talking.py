@@ -8,7 +8,7 @@ learned bias per distance bucket, one added to the softmax's denominator.
   temperatures and the distance table;
 * :func:`write_kv` -- the projections' biases and the cache write;
 * :func:`attention_rows` -- single query tokens (decode, short portions), split over
-  the context; :func:`attention_tiles` -- prompt portions, 16 queries per workgroup.
+  the context; :func:`attention_tiles` -- prompt portions, 16 or 32 queries per workgroup.
 """
 from __future__ import annotations
 
@@ -27,7 +27,6 @@ LOG2E = 1.4426950408889634
 MFMA_DIMS = (64, 128)   # head sizes of the MFMA kernels (others are padded up, larger ones run plain)
 MAX_ROW_HEADS = 64      # heads of the MFMA rows kernel
 MAX_SLOTS = 8           # slots of 4 heads of the tiles kernel
-TILE = 16               # queries per tile
 
 
 def padded_dim(n: int) -> int:
@@ -54,6 +53,11 @@ class Heads:
     @property
     def tiled(self) -> bool:
         return self.mfma and self.slots <= MAX_SLOTS
+
+    @property
+    def tile(self) -> int:
+        """Queries of one tile."""
+        return 32 if self.slots <= 4 else 16
 
     def slot_heads(self) -> list[int]:
         """Head at every position of the slots (-1: empty), padded to whole 16s."""
@@ -142,8 +146,10 @@ class TalkingWeights:
             self.talk = mix_fragments(tb, plain)
             if heads.tiled:
                 order = heads.slot_heads()
-                self.bias_slots = table(order)
-                self.talk_slots = mix_fragments(tb, order)
+                b = table(order)
+                self.bias_far = b[-1].clone()
+                self.bias_slots = (b - self.bias_far).contiguous()
+                self.talk_slots = mix_fragments(tb.to(torch.float16), order)  # exact down to 2^-14
         else:
             self.talk = talk.to(device).float().contiguous()
 
@@ -162,7 +168,7 @@ class QueryRows:
 
 @dataclass
 class QueryTiles:
-    """Blocks of up to 16 consecutive queries: int32 ``[n, 4]`` (first batch row,
+    """Blocks of up to ``Heads.tile`` consecutive queries: int32 ``[n, 4]`` (first batch row,
     block-table row, position of the first, queries)."""
     items: torch.Tensor
     bt: torch.Tensor
@@ -221,7 +227,7 @@ def attention_tiles(q: torch.Tensor, pages: torch.Tensor, w: TalkingWeights, t: 
                                       pages.data_ptr(), _act(out, out.shape[0], h.heads * h.dvp, torch.bfloat16, "out"),
                                       out.stride(0), t.bt.data_ptr(), t.bt.shape[1], t.items.data_ptr(),
                                       t.items.shape[0], w.sc.data_ptr(), w.talk_slots.data_ptr(),
-                                      w.bias_slots.data_ptr(), w.bias_slots.shape[1], w.nfar, h.heads, h.kv_heads,
+                                      w.bias_slots.data_ptr(), w.bias_far.data_ptr(), w.bias_slots.shape[1], w.nfar, h.heads, h.kv_heads,
                                       h.dkp, h.dvp, _lib.stream_handle(q.device))
     _lib.check(rc, f"talking_tiles[{t.items.shape[0]}x{h.heads}]")
     return out

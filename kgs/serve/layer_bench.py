@@ -1,6 +1,7 @@
-"""Prefill and decode throughput of a Ruruzen layer stack at sizes that resemble a
-real model's layers (random weights), beside a Llama stack of the same width,
-heads, feed-forward and depth: ``python bench.py --workload ruruzen``.
+"""Prefill and decode throughput of a Ruruzen or Nufusun layer stack at sizes that
+resemble a real model's layers (random weights), beside a Llama stack of the same
+width, heads, feed-forward (Nufusun: the experts that a token uses) and depth:
+``python bench.py --workload ruruzen|nufusun``.
 
 Both run through :class:`LLMEngine`'s own step runners: prefill a whole prompt
 batch in one step, decode a hipGraph replay per step. Per case the median of
@@ -16,11 +17,14 @@ import numpy as np
 import torch
 
 from kgs.models.llama import LlamaConfig
+from kgs.models.nufusun import NufusunConfig
 from kgs.models.ruruzen import RuruzenConfig
 from kgs.ops.decode import PAGE
 
 # name -> width, heads, q_rank, kv_rank, ff, Llama kv heads (head size 128 everywhere)
 SIZES = {"w2048": (2048, 16, 768, 512, 8192, 4), "w4096": (4096, 32, 1536, 512, 14336, 8)}
+EXPERTS, TOP = 16, 4     # Nufusun: experts of a layer and those a token uses, together as wide as ff
+LAYERS = {"ruruzen": "LDSD", "nufusun": "AAAA"}
 VOCAB = 32000
 PREFILL = ((1, 8192), (8, 1024), (64, 128))              # sequences x tokens
 DECODE = ((1, 1024), (16, 1024), (64, 1024), (256, 1024), (16, 8192))  # batch x context
@@ -42,6 +46,16 @@ def ruruzen(size: str, layers: str) -> RuruzenConfig:
         out.append({**e, "mlp": {"kind": "dense", "ff": ff}})
     return RuruzenConfig.from_dict({"architecture": "Ruruzen", "vocab": VOCAB, "width": width, "streams": 4,
                                     "logit_softcap": 30.0, "norm": {"eps": 1e-5}, "layers": out})
+
+
+def nufusun(size: str, layers: str) -> NufusunConfig:
+    """``layers``: one letter per layer -- A attention and experts, N attention alone."""
+    width, heads, _, _, ff, kv = SIZES[size]
+    mixer = {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "bias_max": 128}
+    mlp = {"kind": "moe", "router": {"experts": EXPERTS, "top": TOP}, "expert": {"ff": ff // TOP, "limit": 7.0}}
+    return NufusunConfig.from_dict({
+        "architecture": "Nufusun", "vocab": VOCAB, "width": width, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-5},
+        "layers": [{"type": "attention", "mixer": mixer, "mlp": mlp if ch == "A" else None} for ch in layers]})
 
 
 def llama(size: str, layers: str) -> LlamaConfig:
@@ -89,6 +103,7 @@ def _time(run, steps: int) -> float:
 
 def run(sizes=("w2048", "w4096"), layers: str = "LDSD", rounds: int = 3, prefill=PREFILL, decode=DECODE,
         models=("ruruzen", "llama"), progress=lambda s: None) -> list[dict]:
+    """``models``: "ruruzen", "nufusun", "llama"."""
     from .engine import EngineConfig, LLMEngine
 
     out = []
@@ -98,7 +113,7 @@ def run(sizes=("w2048", "w4096"), layers: str = "LDSD", rounds: int = 3, prefill
         ec = dict(num_pages=most // PAGE + 2 * nb + 2, max_batch=max(256, nb), max_model_len=16384)
         engines = {}
         for m in models:
-            cfg = ruruzen(size, layers) if m == "ruruzen" else llama(size, layers)
+            cfg = {"ruruzen": ruruzen, "nufusun": nufusun, "llama": llama}[m](size, layers)
             engines[m] = LLMEngine(cfg, EngineConfig(**ec))
             progress(f"{size} {m} ready")
         for kind, cases in (("prefill", prefill), ("decode", decode)):

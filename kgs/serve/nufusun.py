@@ -3,7 +3,7 @@ experts (:mod:`kgs.models.nufusun`).
 
 Every step is one ragged batch (:class:`kgs.serve.ragged.Batch`): the projections'
 biases are added where keys and values go to their pages, prompt portions attend in
-tiles of 16 queries, decoded tokens and short portions row by row with the context
+tiles of 16 or 32 queries, decoded tokens and short portions row by row with the context
 split over the CUs. A layer's two sublayers read the same normed input; one launch
 (:func:`kgs.ops.residual.residual_add`) adds both to the fp32 residual, gathering
 every token's expert rows, and produces the next layer's input.
@@ -24,7 +24,7 @@ from kgs.ops import moe as M
 from kgs.ops.activation import softcap
 from kgs.ops.decode import PAGE
 from kgs.ops.residual import MAX_WIDTH, ExpertRows, residual_add, residual_embed
-from kgs.ops.talking import (TILE, HeadPages, Heads, QueryRows, QueryTiles, TalkingWeights, attention_rows,
+from kgs.ops.talking import (HeadPages, Heads, QueryRows, QueryTiles, TalkingWeights, attention_rows,
                              attention_tiles, heads_of, split_count, write_kv)
 
 from .ragged import DTYPES, Batch, HostPack, RaggedModel, Weights, _pad, pad64
@@ -70,8 +70,9 @@ class Geometry:
                      "tok_pos": refs[9] if whole else pk.add(pos[at]),
                      "rows": None if whole else pk.add(at)}, len(at), split_count(len(at), pages))
         if tiled.any():
-            items = [(row0[s] + q, s, pos0[s] + q, min(TILE, n[s] - q))
-                     for s in np.flatnonzero(tiled) for q in range(0, int(n[s]), TILE)]
+            tile = self.heads.tile
+            items = [(row0[s] + q, s, pos0[s] + q, min(tile, n[s] - q))
+                     for s in np.flatnonzero(tiled) for q in range(0, int(n[s]), tile)]
             items = np.array(items, np.int64)
             tiles = pk.add(items[np.argsort(-(items[:, 2] + items[:, 3]), kind="stable")])  # longest context first
 

@@ -9,10 +9,11 @@
 // = log2(e) sum_g talk[h, g] rel_g[n], whose last row serves every distance from
 // its number on.
 //
-// The mixture is an MFMA over heads. talk is exact in bf16; a score enters as
-// three bf16 parts (truncated, truncated, rest) that together hold its 24 bits, so
-// the product is an fp32 one. What makes it cheap is that no score leaves the
-// registers for it:
+// The mixture is an MFMA over heads whose products are exact: talk is a bf16 number, and
+// a score enters in parts that hold its bits -- three bf16 parts (rows: all 24 bits) or
+// two fp16 parts (tiles: 22 bits or 2^-24, less than the fp32 sum of the score itself
+// loses; beyond fp16's range a part saturates). What makes it cheap is that no score
+// leaves the registers for it:
 //   rows   (decoded tokens, short portions) S = q K^T with heads on the MFMA's rows
 //          leaves a lane 4 heads of one key; an MFMA contracts in any order both
 //          operands share, so those registers are its operand as they are, and with
@@ -28,6 +29,9 @@
 //
 // The running maximum starts at 0, the score of the `1 +`, so it never needs a
 // first tile; each row's sum gets 2^(0 - max) once, at the end.
+#include <type_traits>
+
+#include "acc_regs.h"
 #include "kgs_common.h"
 
 namespace kgs {
@@ -51,10 +55,21 @@ __device__ __forceinline__ void split3(float s, unsigned (&u)[3]) {
   u[1] = __float_as_uint(r1);
   u[2] = __float_as_uint(r1 - __uint_as_float(u[1] & 0xffff0000u));
 }
+// two fp16 parts of two fp32 values: parts truncated, so a value out of range saturates
+typedef _Float16 f16x2 __attribute__((ext_vector_type(2)));
+typedef _Float16 f16x8 __attribute__((ext_vector_type(8)));
+__device__ __forceinline__ void split2(float a, float b, unsigned& hi, unsigned& lo) {
+  const f16x2 h = __builtin_bit_cast(f16x2, __builtin_amdgcn_cvt_pkrtz(a, b));
+  // one v_fma_mix_f32 each
+  const float ra = __builtin_fmaf((float)h[0], -1.0f, a), rb = __builtin_fmaf((float)h[1], -1.0f, b);
+  hi = __builtin_bit_cast(unsigned, h);
+  lo = __builtin_bit_cast(unsigned, __builtin_amdgcn_cvt_pkrtz(ra, rb));
+}
 // upper halves of (lo, hi) as one word
 __device__ __forceinline__ unsigned pack_hi(unsigned lo, unsigned hi) { return __builtin_amdgcn_perm(hi, lo, 0x07060302u); }
 
 typedef unsigned u32x4 __attribute__((ext_vector_type(4)));
+typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
 
 // ------------------------------------------------------- biases and cache write
 struct WriteArgs {
@@ -147,13 +162,14 @@ struct Args {
   const int* tok_seq;  // per query: its block-table row and its position
   const int* tok_pos;
   const int* rows;     // its batch row, or null: the same
-  const int4* items;   // tiles: (first batch row, block-table row, position, queries <= 16)
+  const int4* items;   // tiles: (first batch row, block-table row, position, queries)
   float* po;           // partial results of split rows: [row, split][heads][dvp]
   float* pml;          // [row, split][heads][2]
   const float* sc;     // [heads]
-  const unsigned short* talk;  // bf16 MFMA fragments (rows: [HT][NC][64][8]; tiles: [MT][64][8])
+  const unsigned short* talk;  // MFMA fragments (rows: bf16 [HT][NC][64][8]; tiles: fp16 [MT][64][8])
   const float* talk32; // [heads][heads], the plain kernel's
-  const float* bias;   // [nfar + 1][ldb]
+  const float* bias;   // [nfar + 1][ldb] (tiles: less the last row)
+  const float* bfar;   // tiles: the last row
   int ldb, nfar;
   int H, G, R, dkp, dvp, nsplit;
 };
@@ -411,240 +427,371 @@ __device__ __forceinline__ void transpose4(unsigned (&x)[4]) {
   x[0] = c[0], x[1] = c[1], x[2] = d[0], x[3] = d[1];
 }
 
-// 16 queries of one portion, all heads. Wave w: queries 4w .. 4w + 3. Heads sit in
-// slots of 4 that share a key head (slot s: key head s / QPG, its heads
-// 4 (s % QPG) .., those past the group's end empty). K and V pages come by LDS-DMA:
-// the next K while the scores are mixed, the next V while they are computed.
-template <int NS, int NK, int ND>
-__global__ __launch_bounds__(256, NS * (NK + ND) > 64 ? 1 : 2) void attn_tiles(Args a) {
-  constexpr int MT = (NS + 3) / 4;
-  constexpr bool QRES = NS * ND < 64;  // queries stay in registers
-  __shared__ __attribute__((aligned(1024))) char smem[NS * (2 * NK + ND + 4) * 1024];
+// Compile-time loop: f(std::integral_constant<int, i>) for i in [B, E).
+template <int B, int E, class F>
+__device__ __forceinline__ void static_for(F&& f) {
+  if constexpr (B < E) {
+    f(std::integral_constant<int, B>{});
+    static_for<B + 1, E>(f);
+  }
+}
+
+__device__ __forceinline__ void fence() { __builtin_amdgcn_sched_barrier(0); }
+// every wave's LDS accesses are done; loads stay in flight
+__device__ __forceinline__ void bar() {
+  fence();
+  asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+  fence();
+}
+// ... and every wave's LDS-DMA has landed
+__device__ __forceinline__ void bar_vm() {
+  fence();
+  asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)\n\ts_barrier" ::: "memory");
+  fence();
+}
+
+// 16 QT queries of one portion, all heads; wave w has queries 4 QT w .. in QT blocks of
+// 4. Heads sit in slots of 4 that share a key head (slot s: key head s / QPG, its heads
+// 4 (s % QPG) .., those past the group's end empty), so a row tile is 4 queries x 4 heads.
+//
+// Per page: S = Q K^T for every row tile (K fragments are read two half slots ahead of
+// their MFMAs, Q row tiles a ring ahead, the first of the next page during P V), the
+// next K and this V on their way by LDS-DMA, mix and softmax, P through this wave's
+// corner of LDS into operand order, P V. The outputs live in named AGPRs
+// (acc_regs.h, accumulator (s QT + qt) ND + d): they take half the register file, and the compiler would
+// move them about. Rescales are collected over the page and applied before P V.
+template <int NS, int QT, int NK, int ND>
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) void attn_tiles(Args a) {
+  constexpr int MT = (NS + 3) / 4, RT = NS * QT;
+  constexpr int RQ = RT * NK <= 16 ? RT : 16 / NK;  // Q row tiles in registers
+  static_assert(RT * ND <= 64, "outputs exceed the AGPRs");
+  __shared__ __attribute__((aligned(1024))) char smem[(NS * (2 * NK + ND) + 4 * RT) * 1024];
   char* const ks = smem;
   char* const vs = smem + NS * 2 * NK * 1024;
   const int lane = threadIdx.x & 63, w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), n = lane & 15, q = lane >> 4;
-  char* const ps = vs + NS * ND * 1024 + w * NS * 1024;  // this wave's P: [slot][16 rows][32 keys]
+  char* const ps = vs + NS * ND * 1024 + w * RT * 1024;  // this wave's P: [qt][slot][16 rows][32 keys]
   const int4 it = a.items[blockIdx.x];
   const int qpg = (a.R + 3) / 4, nslot = a.G * qpg;
   const int* bt = a.bt + (long)it.y * a.W;
   const int npage = (it.z + it.w - 1) / PAGE + 1;
   const long hpage = (long)PAGE * (a.dkp + a.dvp) * 2;  // bytes of one head's page
-  const int posw = it.z + 4 * w;                        // position of the wave's first query
+  const int posw = it.z + 4 * QT * w;                   // position of the wave's first query
 
-  // this lane's query row of the S tiles: query n >> 2, head n & 3 of the slot
-  const unsigned short* qrow = (const unsigned short*)a.q + (long)(it.x + min(4 * w + (n >> 2), it.w - 1)) * a.ldq + 8 * q;
-  auto load_q = [&](bf16x8 (&f)[NK], int s) {
-    const int hr = 4 * (s % qpg) + (n & 3);
-    const unsigned short* p = qrow + (long)(s / qpg * a.R + hr) * a.dkp;
+  // this lane's row of the S tiles: query n >> 2 of the block, head n & 3 of the slot. A query
+  // past the portion's end reads its last one; an empty head reads what follows the
+  // group (zeros past the last row): its scale is 0.
+  const __amdgpu_buffer_rsrc_t qrsrc = __builtin_amdgcn_make_buffer_rsrc((void*)((const unsigned short*)a.q + (long)it.x * a.ldq), 0,
+                                                       it.w * (int)a.ldq * 2, 0x00020000);
+  int qoff[QT];
 #pragma unroll
-    for (int k = 0; k < NK; ++k) f[k] = s < nslot && hr < a.R ? *(const bf16x8*)(p + 32 * k) : bf16x8{};
+  for (int t = 0; t < QT; ++t)
+    qoff[t] = (min(4 * (QT * w + t) + (n >> 2), it.w - 1) * (int)a.ldq + (n & 3) * a.dkp + 8 * q) * 2;
+  auto load_q = [&](bf16x8 (&f)[NK], int rt) {
+    const int s = rt / QT, so = (min(s / qpg, a.G - 1) * a.R + 4 * (s % qpg)) * a.dkp * 2;
+#pragma unroll
+    for (int k = 0; k < NK; ++k)
+      f[k] = __builtin_bit_cast(bf16x8, __builtin_amdgcn_raw_buffer_load_b128(qrsrc, qoff[rt % QT] + 64 * k, so, 0));
   };
-  bf16x8 qf[QRES ? NS : 1][NK];
-  if constexpr (QRES) {
-#pragma unroll
-    for (int s = 0; s < NS; ++s) load_q(qf[s], s);
-  }
   float sc[NS][4];  // uniform
 #pragma unroll
   for (int s = 0; s < NS; ++s)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int hr = 4 * (s % qpg) + r;
-      sc[s][r] = s < nslot && hr < a.R ? a.sc[s / qpg * a.R + hr] : 0.f;
+      sc[s][r] = __uint_as_float(__builtin_amdgcn_readfirstlane(
+          __float_as_uint(s < nslot && hr < a.R ? a.sc[s / qpg * a.R + hr] : 0.f)));
     }
-  bf16x8 tf[MT];
-  f32x4 bfar[MT];
+  f16x8 tf[MT];
 #pragma unroll
-  for (int t = 0; t < MT; ++t) {
-    tf[t] = *(const bf16x8*)(a.talk + (t * 64 + lane) * 8);
-    bfar[t] = *(const f32x4*)(a.bias + (long)a.nfar * a.ldb + 16 * t + 4 * q);
-  }
+  for (int t = 0; t < MT; ++t) tf[t] = *(const f16x8*)(a.talk + (t * 64 + lane) * 8);
 
   // page chunks of 1 KB, dealt to the waves
-  auto dma_k = [&](int pg) {
-    const char* base = (const char*)a.pages + (long)bt[pg] * a.G * hpage + 16 * lane;
-    for (int i = w; i < a.G * 2 * NK; i += 4) glds16(base + (i / (2 * NK)) * hpage + (i % (2 * NK)) * 1024, ks + i * 1024);
+  const int pbytes = a.G * (int)hpage;
+  // chunk w + 4 c of `per` chunks a key head, from byte `first` of its page on (past the
+  // last one: that one again)
+  auto dma = [&](int page, char* dst, int per, int first, int c) {
+    const __amdgpu_buffer_rsrc_t r =
+        __builtin_amdgcn_make_buffer_rsrc((void*)((const char*)a.pages + (long)page * pbytes), 0, pbytes, 0x00020000);
+    const int i = min(w + 4 * c, a.G * per - 4 + w);
+    __builtin_amdgcn_raw_ptr_buffer_load_lds(r, (KGS_LDS void*)(dst + i * 1024), 16, 16 * lane,
+                                             (i / per) * (int)hpage + first + (i % per) * 1024, 0, 0);
   };
-  auto dma_v = [&](int pg) {
-    const char* base = (const char*)a.pages + (long)bt[pg] * a.G * hpage + PAGE * a.dkp * 2 + 16 * lane;
-    for (int i = w; i < a.G * ND; i += 4) glds16(base + (i / ND) * hpage + (i % ND) * 1024, vs + i * 1024);
-  };
-  auto drain = [&]() {
-    asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");
-    __syncthreads();
-  };
+  constexpr int CK = NS * 2 * NK / 4, CV = NS * ND / 4;  // chunks per wave of K and of V
+  auto page_id = [&](int pg) { return bt[min(pg, npage - 1)]; };
 
-  f32x4 acc[NS][ND];
-  f32x4 m[4][MT];  // running maxima of (query, slot 4t + q, head)
-  float l[NS];
+  // the far bias less the running maximum of (query, slot 4t + q, head): the mixture's addend
+  f32x4 cm[4 * QT][MT];
+  float l[RT];
 #pragma unroll
-  for (int s = 0; s < NS; ++s) {
-    l[s] = 0.f;
+  for (int i = 0; i < 4 * QT; ++i)
 #pragma unroll
-    for (int d = 0; d < ND; ++d) acc[s][d] = f32x4{};
-  }
+    for (int t = 0; t < MT; ++t) cm[i][t] = *(const f32x4*)(a.bfar + 16 * t + 4 * q);
 #pragma unroll
-  for (int i = 0; i < 4; ++i)
-#pragma unroll
-    for (int t = 0; t < MT; ++t) m[i][t] = f32x4{};
+  for (int i = 0; i < RT; ++i) l[i] = 0.f;
+  KGS_ACC_RESERVE();
+  static_for<0, RT * ND>([](auto i) { accr::zero<decltype(i)::value>(); });
 
-  dma_k(0);
-  drain();
+  bf16x8 qf[RQ][NK];
+#pragma unroll
+  for (int i = 0; i < RQ; ++i) load_q(qf[i], i);
+  int page = __builtin_amdgcn_readfirstlane(page_id(0));
+#pragma unroll
+  for (int c = 0; c < CK; ++c) dma(page, ks, 2 * NK, 0, c);
+  bar_vm();
   for (int pg = 0; pg < npage; ++pg) {
     const int tok0 = pg * PAGE;
-    if constexpr (QRES) dma_v(pg);
-    f32x4 S[NS][2];
+    const int next = page_id(pg + 1);
+    // ---- scores
+    f32x4 S[RT][2];
+    // K fragments of both 16-key halves, one 32-dim step at a time, PF steps ahead
+    constexpr int PF = 5, STEPS = NS * NK;
+    bf16x8 kf[PF + 1][2];
+    auto read_k = [&](int p) {
+      const char* kp = ks + (min((p / NK) / qpg, a.G - 1) * 2 * NK + p % NK) * 1024 + 16 * lane;
+      kf[p % (PF + 1)][0] = *(const bf16x8*)kp;
+      kf[p % (PF + 1)][1] = *(const bf16x8*)(kp + NK * 1024);
+    };
 #pragma unroll
-    for (int s = 0; s < NS; ++s) {
-      S[s][0] = S[s][1] = f32x4{};
-      if (s < nslot) {
-        if constexpr (!QRES) load_q(qf[0], s);
-        const char* kp = ks + (s / qpg) * (2 * NK * 1024) + 16 * lane;
+    for (int p = 0; p < PF; ++p) read_k(p);
+#pragma unroll
+    for (int p = 0; p < STEPS; ++p) {
+      if (p + PF < STEPS) read_k(p + PF);
+      fence();
+#pragma unroll
+      for (int t = 0; t < QT; ++t) {
+        const int rt = (p / NK) * QT + t;
+        if (p % NK == 0) S[rt][0] = S[rt][1] = f32x4{};
 #pragma unroll
         for (int kt = 0; kt < 2; ++kt)
-#pragma unroll
-          for (int k = 0; k < NK; ++k)
-            S[s][kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[QRES ? s : 0][k], *(const bf16x8*)(kp + (kt * NK + k) * 1024),
-                                                               S[s][kt], 0, 0, 0);
+          S[rt][kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[rt % RQ][p % NK], kf[p % (PF + 1)][kt], S[rt][kt], 0, 0, 0);
       }
+      if (p % NK == NK - 1) {
+        fence();
+#pragma unroll
+        for (int t = 0; t < QT; ++t)
+          if ((p / NK) * QT + t + RQ < RT) load_q(qf[((p / NK) * QT + t) % RQ], (p / NK) * QT + t + RQ);
+      }
+#pragma unroll
+      for (int c = 0; c < CV; ++c)
+        if (c * STEPS / CV == p) dma(page, vs, ND, PAGE * NK * 64, c);
+      fence();
     }
-    if constexpr (!QRES) dma_v(pg);
-    // K of this page is done with everywhere, V of it is there
-    drain();
-    if (pg + 1 < npage) dma_k(pg + 1);
+    bar();  // K of this page is done with everywhere
+    page = __builtin_amdgcn_readfirstlane(next);
 
+    // ---- mix, softmax
     const bool near = posw - (tok0 + PAGE - 1) < a.nfar, edge = tok0 + PAGE - 1 > posw;
-    float p0[4][MT][4];
+    bool grown = false;
+    float al[RT];
 #pragma unroll
-    for (int kt = 0; kt < 2; ++kt) {
-      unsigned x[3][2][2][4];  // [part][half][head pair][slot of the half, then query]
+    for (int i = 0; i < RT; ++i) al[i] = 1.f;
 #pragma unroll
-      for (int s = 0; s < 4 * MT; ++s) {
-        unsigned u[4][3];
+    for (int qt = 0; qt < QT; ++qt) {
+      unsigned p0[4][MT][2];  // keys 2n, heads (0, 1) and (2, 3)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          if (s < NS) split3(S[s < NS ? s : 0][kt][r] * sc[s < NS ? s : 0][r], u[r]);
-          else u[r][0] = u[r][1] = u[r][2] = 0;
+      for (int kt = 0; kt < 2; ++kt) {
+        unsigned x[2][MT][2][4];  // [part][half][head pair][slot of the half, then query]
+#pragma unroll
+        for (int s = 0; s < 4 * MT; ++s)
+#pragma unroll
+          for (int c = 0; c < 2; ++c) {
+            if (s < NS) {
+              const int s_ = s < NS ? s : 0;
+              const f32x4& v = S[s_ * QT + qt][kt];
+              split2(v[2 * c] * sc[s_][2 * c], v[2 * c + 1] * sc[s_][2 * c + 1], x[0][s >> 2][c][s & 3], x[1][s >> 2][c][s & 3]);
+            } else x[0][s >> 2][c][s & 3] = x[1][s >> 2][c][s & 3] = 0;
+          }
+#pragma unroll
+        for (int j = 0; j < 2; ++j)
+#pragma unroll
+          for (int hf = 0; hf < MT; ++hf) transpose4(x[j][hf][0]), transpose4(x[j][hf][1]);
+        fence();
+        if (pg + 1 < npage) {
+#pragma unroll
+          for (int c = 0; c < CK; ++c)
+            if (c * 2 * QT / CK == 2 * qt + kt) dma(page, ks, 2 * NK, 0, c);
         }
+        f32x4 D[4][MT];
 #pragma unroll
-        for (int j = 0; j < 3; ++j) {
-          x[j][s >> 2][0][s & 3] = pack_hi(u[0][j], u[1][j]);
-          x[j][s >> 2][1][s & 3] = pack_hi(u[2][j], u[3][j]);
-        }
-      }
+        for (int j = 1; j >= 0; --j)
 #pragma unroll
-      for (int j = 0; j < 3; ++j)
+          for (int i = 0; i < 4; ++i) {
+            const u32x4 b = {x[j][0][0][i], x[j][0][1][i], MT > 1 ? x[j][MT - 1][0][i] : 0u, MT > 1 ? x[j][MT - 1][1][i] : 0u};
 #pragma unroll
-        for (int hf = 0; hf < MT; ++hf) transpose4(x[j][hf][0]), transpose4(x[j][hf][1]);
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        f32x4 D[MT];
-#pragma unroll
-        for (int t = 0; t < MT; ++t) D[t] = bfar[t];
-        const int dist = posw + i - (tok0 + 2 * n + kt);
+            for (int t = 0; t < MT; ++t)
+              D[i][t] = __builtin_amdgcn_mfma_f32_16x16x32_f16(tf[t], __builtin_bit_cast(f16x8, b),
+                                                               j == 1 ? cm[4 * qt + i][t] : D[i][t], 0, 0, 0);
+          }
+        // lane: query i, key 2n + kt, slot 4t + q, head r; above the running maximum
+        const int dist = posw + 4 * qt - (tok0 + 2 * n + kt);  // of query 0
         if (near) {
-          const float* bp = a.bias + (long)min(max(dist, 0), a.nfar) * a.ldb + 4 * q;
 #pragma unroll
-          for (int t = 0; t < MT; ++t) D[t] = *(const f32x4*)(bp + 16 * t);
-        }
+          for (int i = 0; i < 4; ++i) {
+            const float* bp = a.bias + (long)min(max(dist + i, 0), a.nfar) * a.ldb + 4 * q;
 #pragma unroll
-        for (int j = 2; j >= 0; --j) {
-          const u32x4 b = {x[j][0][0][i], x[j][0][1][i], MT > 1 ? x[j][MT - 1][0][i] : 0u, MT > 1 ? x[j][MT - 1][1][i] : 0u};
-#pragma unroll
-          for (int t = 0; t < MT; ++t)
-            D[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tf[t], __builtin_bit_cast(bf16x8, b), D[t], 0, 0, 0);
-        }
-        // lane: key 2n + kt, slot 4t + q, head r
-        float over = -1.f;
-#pragma unroll
-        for (int t = 0; t < MT; ++t)
-#pragma unroll
-          for (int r = 0; r < 4; ++r) {
-            if (edge && dist < 0) D[t][r] = NEG;
-            D[t][r] -= m[i][t][r];
-            over = fmaxf(over, D[t][r]);
+            for (int t = 0; t < MT; ++t) D[i][t] += *(const f32x4*)(bp + 16 * t);
           }
-        if (__any(over > RESCALE)) {
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+#pragma unroll
+            for (int t = 0; t < MT; ++t) asm volatile("" : "+v"(D[i][t]));  // waited for here, not where far pages pass too
+        }
+        if (edge) {
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+#pragma unroll
+            for (int t = 0; t < MT; ++t)
+#pragma unroll
+              for (int r = 0; r < 4; ++r) D[i][t][r] = dist + i < 0 ? NEG : D[i][t][r];
+        }
+        float over = D[0][0][0];
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+#pragma unroll
+          for (int t = 0; t < MT; ++t) over = fmaxf(fmaxf(fmaxf(over, D[i][t][0]), fmaxf(D[i][t][1], D[i][t][2])), D[i][t][3]);
+        if (__builtin_expect(__any(over > RESCALE), 0)) {
           // new maxima over the 16 keys; sel: the factor of head n & 3, for the lanes that hold its row
-          float sel[MT];
+          grown = true;
+          int n_ = n;
+          asm volatile("" : "+v"(n_));  // nothing of this path is worth a register outside it
 #pragma unroll
-          for (int t = 0; t < MT; ++t)
+          for (int i = 0; i < 4; ++i) {
+            float sel[MT];
 #pragma unroll
-            for (int r = 0; r < 4; ++r) {
-              float up = fmaxf(D[t][r], 0.f);
+            for (int t = 0; t < MT; ++t) {
+              float fr[4];
 #pragma unroll
-              for (int b = 1; b < 16; b <<= 1) up = fmaxf(up, __shfl_xor(up, b, 16));
-              const float f = __builtin_amdgcn_exp2f(-up);
-              m[i][t][r] += up;
-              D[t][r] -= up;
-              if (kt == 1) p0[i][t][r] *= f;
-              sel[t] = r == 0 || (n & 3) == r ? f : sel[t];
+              for (int r = 0; r < 4; ++r) {
+                float up = fmaxf(D[i][t][r], 0.f);
+#pragma unroll
+                for (int b = 1; b < 16; b <<= 1)
+                  up = fmaxf(up, __int_as_float(__builtin_amdgcn_ds_bpermute(((n_ ^ b) + 16 * q) * 4, __float_as_int(up))));
+                fr[r] = __builtin_amdgcn_exp2f(-up);
+                cm[4 * qt + i][t][r] -= up;
+                D[i][t][r] -= up;
+              }
+              sel[t] = (n_ & 2) ? ((n_ & 1) ? fr[3] : fr[2]) : ((n_ & 1) ? fr[1] : fr[0]);
+              if (kt == 1) {
+#pragma unroll
+                for (int c = 0; c < 2; ++c)
+                  p0[i][t][c] = pack_bf16x2(__uint_as_float(p0[i][t][c] << 16) * fr[2 * c],
+                                            __uint_as_float(p0[i][t][c] & 0xffff0000u) * fr[2 * c + 1]);
+              }
             }
 #pragma unroll
-          for (int s = 0; s < NS; ++s) {
-            const float g = __shfl(sel[s >> 2], 16 * (s & 3) + (n & 3), 64), f = (n >> 2) == i ? g : 1.f;
-            l[s] *= f;
-#pragma unroll
-            for (int d = 0; d < ND; ++d) acc[s][d] *= f;
+            for (int s = 0; s < NS; ++s) {
+              const float g = __shfl(sel[s >> 2], 16 * (s & 3) + (n_ & 3), 64);
+              al[s * QT + qt] *= (n_ >> 2) == i ? g : 1.f;
+            }
           }
         }
 #pragma unroll
-        for (int t = 0; t < MT; ++t)
+        for (int i = 0; i < 4; ++i)
 #pragma unroll
-          for (int r = 0; r < 4; ++r) {
-            const float p = __builtin_amdgcn_exp2f(D[t][r]);
-            if (kt == 0) p0[i][t][r] = p;
-            else if (4 * t + q < NS) {
-              // P row 4i + r of slot 4t + q; rows permuted by the slot and 16-B chunks by the row: no bank twice
-              const int s = 4 * t + q, rw = 4 * i + r;
-              *(unsigned*)(ps + s * 1024 + ((rw ^ (s & 3)) * 64) + (((n >> 2) ^ ((rw >> 2) & 3)) * 16) + (n & 3) * 4) =
-                  pack_bf16x2(p0[i][t][r], p);
+          for (int t = 0; t < MT; ++t) {
+            float p[4];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) p[r] = __builtin_amdgcn_exp2f(D[i][t][r]);
+            const unsigned c0 = pack_bf16x2(p[0], p[1]), c1 = pack_bf16x2(p[2], p[3]);
+            if (kt == 0) p0[i][t][0] = c0, p0[i][t][1] = c1;
+            else if (NS >= 4 || q < NS) {
+              // row 4i + r of slot 4t + q, keys 2n and 2n + 1; rows permuted by the slot and 16-B
+              // chunks by the row: no bank twice
+              char* pp = ps + (qt * NS + 4 * t + q) * 1024 + 256 * i + (((n >> 2) ^ i) * 16) + (n & 3) * 4;
+              *(unsigned*)(pp + ((0 ^ q) * 64)) = __builtin_amdgcn_perm(c0, p0[i][t][0], 0x05040100u);
+              *(unsigned*)(pp + ((1 ^ q) * 64)) = __builtin_amdgcn_perm(c0, p0[i][t][0], 0x07060302u);
+              *(unsigned*)(pp + ((2 ^ q) * 64)) = __builtin_amdgcn_perm(c1, p0[i][t][1], 0x05040100u);
+              *(unsigned*)(pp + ((3 ^ q) * 64)) = __builtin_amdgcn_perm(c1, p0[i][t][1], 0x07060302u);
             }
           }
       }
     }
-    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-    __builtin_amdgcn_wave_barrier();
-#pragma unroll
-    for (int s = 0; s < NS; ++s) {
-      if (s >= nslot) continue;
-      const u32x4 pw = *(const u32x4*)(ps + s * 1024 + ((n ^ (s & 3)) * 64) + ((q ^ ((n >> 2) & 3)) * 16));
-#pragma unroll
-      for (int e = 0; e < 4; ++e) l[s] += __uint_as_float(pw[e] << 16) + __uint_as_float(pw[e] & 0xffff0000u);
-      const bf16x8 pb = __builtin_bit_cast(bf16x8, pw);
-      const char* vp = vs + (s / qpg) * (ND * 1024) + 16 * lane;
-#pragma unroll
-      for (int d = 0; d < ND; ++d)
-        acc[s][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(vp + d * 1024), pb, acc[s][d], 0, 0, 0);
+    if (__builtin_expect(grown, 0)) {
+      asm volatile("s_nop 7\n\ts_nop 7\n\ts_nop 3" ::: "memory");  // MFMA -> v_accvgpr_read hazard
+      static_for<0, RT>([&](auto rc) {
+        constexpr int rt = decltype(rc)::value;
+        l[rt] *= al[rt];
+        static_for<0, ND>([&](auto dc) {
+          constexpr int i = rt * ND + decltype(dc)::value;
+          accr::write<i>(accr::read<i>() * al[rt]);
+        });
+      });
+      asm volatile("s_nop 7" ::: "memory");
     }
-    drain();  // V is done with everywhere, the next K is there
+    bar_vm();  // V of this page and K of the next are there
+
+    // ---- P V
+#pragma unroll
+    for (int i = 0; i < RQ; ++i) load_q(qf[i], i);  // for the next page
+    bf16x8 vf[2][ND];
+    auto read_v = [&](bf16x8 (&f)[ND], int s) {
+      const char* vp = vs + min(s / qpg, a.G - 1) * (ND * 1024) + 16 * lane;
+#pragma unroll
+      for (int i = 0; i < ND; ++i) f[i] = *(const bf16x8*)(vp + i * 1024);
+    };
+    u32x4 pw[2][QT];
+    auto read_p = [&](u32x4 (&f)[QT], int s) {
+#pragma unroll
+      for (int t = 0; t < QT; ++t)
+        f[t] = *(const u32x4*)(ps + (t * NS + s) * 1024 + ((n ^ (s & 3)) * 64) + ((q ^ ((n >> 2) & 3)) * 16));
+    };
+    read_p(pw[0], 0);
+    read_v(vf[0], 0);
+    fence();
+    static_for<0, NS>([&](auto sc_) {
+      constexpr int s = decltype(sc_)::value;
+      if constexpr (s + 1 < NS) {
+        read_p(pw[(s + 1) & 1], s + 1);
+        read_v(vf[(s + 1) & 1], s + 1);
+      }
+      fence();
+      static_for<0, QT>([&](auto tc) {
+        constexpr int t = decltype(tc)::value, rt = s * QT + t;
+        const u32x4 pv = pw[s & 1][t];
+        const bf16x8 pb = __builtin_bit_cast(bf16x8, pv);
+        static_for<0, ND>([&](auto dc) {
+          constexpr int d = decltype(dc)::value;
+          accr::mfma<rt * ND + d>(vf[s & 1][d], pb);
+        });
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const unsigned two = pv[e], ones = 0x3f803f80u;
+          l[rt] = __builtin_amdgcn_fdot2_f32_bf16(__builtin_bit_cast(bf16x2, two), __builtin_bit_cast(bf16x2, ones), l[rt], false);
+        }
+      });
+      fence();
+    });
+    bar();  // V is done with everywhere
   }
 
-  // rows' maxima to the lanes that hold the rows: [slot][row]
+  // rows' maxima to the lanes that hold the rows: [qt][slot][row]
   float* mm = (float*)ps;
 #pragma unroll
-  for (int i = 0; i < 4; ++i)
+  for (int i = 0; i < 4 * QT; ++i)
 #pragma unroll
     for (int t = 0; t < MT; ++t)
-      if (n == 0 && 4 * t + q < NS) *(f32x4*)(mm + (4 * t + q) * 16 + 4 * i) = m[i][t];
+      if (NS >= 4 || q < NS) *(f32x4*)(mm + ((i >> 2) * NS + 4 * t + q) * 16 + 4 * (i & 3)) =
+                                  *(const f32x4*)(a.bfar + 16 * t + 4 * q) - cm[i][t];
   asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-  __builtin_amdgcn_wave_barrier();
-  const int qi = 4 * w + (n >> 2);
-#pragma unroll
-  for (int s = 0; s < NS; ++s) {
-    const int hr = 4 * (s % qpg) + (n & 3);
-    const float L = xor32_sum(xor16_sum(l[s])) + __builtin_amdgcn_exp2f(-mm[s * 16 + n]);
-    if (s >= nslot || hr >= a.R || qi >= it.w) continue;
-    const float inv = 1.0f / L;
-    unsigned short* op = (unsigned short*)a.o + (long)(it.x + qi) * a.ldo + (long)(s / qpg * a.R + hr) * a.dvp + 4 * q;
-#pragma unroll
-    for (int d = 0; d < ND; ++d) {
-      uint2 pk;
-      pk.x = pack_bf16x2(acc[s][d][0] * inv, acc[s][d][1] * inv);
-      pk.y = pack_bf16x2(acc[s][d][2] * inv, acc[s][d][3] * inv);
-      *(uint2*)(op + 16 * d) = pk;
-    }
-  }
+  asm volatile("s_nop 7\n\ts_nop 7\n\ts_nop 3" ::: "memory");  // MFMA -> v_accvgpr_read hazard
+  static_for<0, NS>([&](auto sc_) {
+    static_for<0, QT>([&](auto tc) {
+      constexpr int s = decltype(sc_)::value, t = decltype(tc)::value, rt = s * QT + t;
+      const int hr = 4 * (s % qpg) + (n & 3), qi = 4 * (QT * w + t) + (n >> 2);
+      const float L = xor32_sum(xor16_sum(l[rt])) + __builtin_amdgcn_exp2f(-mm[(t * NS + s) * 16 + n]);
+      const bool ok = s < nslot && hr < a.R && qi < it.w;
+      const float inv = 1.0f / L;
+      unsigned short* op = (unsigned short*)a.o + (long)(it.x + qi) * a.ldo + (long)(s / qpg * a.R + hr) * a.dvp + 4 * q;
+      static_for<0, ND>([&](auto dc) {
+        constexpr int d = decltype(dc)::value;
+        const f32x4 o = accr::read<rt * ND + d>() * inv;
+        uint2 pk;
+        pk.x = pack_bf16x2(o[0], o[1]);
+        pk.y = pack_bf16x2(o[2], o[3]);
+        if (ok) *(uint2*)(op + 16 * d) = pk;
+      });
+    });
+  });
 }
 
 // ----------------------------------------------------------------------- plain
@@ -739,9 +886,9 @@ void rows_ht(const Args& a, int nrows, hipStream_t s) {
 template <int NK, int ND>
 void tiles_ns(const Args& a, int nitems, int nslot, hipStream_t s) {
   const dim3 grid((unsigned)nitems), block(256);
-  if (nslot <= 2) hipLaunchKernelGGL((attn_tiles<2, NK, ND>), grid, block, 0, s, a);
-  else if (nslot <= 4) hipLaunchKernelGGL((attn_tiles<4, NK, ND>), grid, block, 0, s, a);
-  else hipLaunchKernelGGL((attn_tiles<8, NK, ND>), grid, block, 0, s, a);
+  if (nslot <= 2) hipLaunchKernelGGL((attn_tiles<2, 2, NK, ND>), grid, block, 0, s, a);
+  else if (nslot <= 4) hipLaunchKernelGGL((attn_tiles<4, 2, NK, ND>), grid, block, 0, s, a);
+  else hipLaunchKernelGGL((attn_tiles<8, 1, NK, ND>), grid, block, 0, s, a);
 }
 
 int check(const Args& a, int n) {
@@ -782,7 +929,7 @@ KGS_EXPORT int kgs_talking_rows(const void* q, long ldq, const void* pages, void
   using namespace kgs::talking;
   Args a{q, ldq, pages, o, ldo, (const int*)bt, W, (const int*)tok_seq, (const int*)tok_pos, (const int*)rows, nullptr,
          (float*)po, (float*)pml, (const float*)sc, (const unsigned short*)talk, (const float*)talk, (const float*)bias,
-         ldb, nfar, H, G, G ? H / G : 0, dkp, dvp, nsplit};
+         nullptr, ldb, nfar, H, G, G ? H / G : 0, dkp, dvp, nsplit};
   if (int rc = check(a, nrows)) return rc;
   if (plain || f32) {
     const size_t lds = ((size_t)H * (dkp + dvp + 128 + 3)) * 4;
@@ -804,22 +951,23 @@ KGS_EXPORT int kgs_talking_rows(const void* q, long ldq, const void* pages, void
   return (int)hipGetLastError();
 }
 
-// Prompt portions: nitems blocks of up to 16 consecutive queries (first batch row,
-// block-table row, first position, queries). bf16, dkp and dvp 64 or 128, at most 8 slots
-// of 4 heads (G ceil(H / G / 4)); talk and bias in slot order, ldb = 16 ceil(slots / 4).
+// Prompt portions: nitems blocks of consecutive queries (first batch row, block-table
+// row, first position, queries: up to 32, 16 above 4 slots). bf16, dkp and dvp 64 or 128, at most 8 slots
+// of 4 heads (G ceil(H / G / 4)); talk (fp16) and biases in slot order, ldb = 16 ceil(slots / 4);
+// bias is the table less its last row, bfar.
 KGS_EXPORT int kgs_talking_tiles(const void* q, long ldq, const void* pages, void* o, long ldo, const void* bt, int W,
                                  const void* items, int nitems, const void* sc, const void* talk, const void* bias,
-                                 int ldb, int nfar, int H, int G, int dkp, int dvp, hipStream_t s) {
+                                 const void* bfar, int ldb, int nfar, int H, int G, int dkp, int dvp, hipStream_t s) {
   using namespace kgs::talking;
   Args a{};
   a.q = q, a.ldq = ldq, a.pages = pages, a.o = o, a.ldo = ldo, a.bt = (const int*)bt, a.W = W;
   a.items = (const int4*)items, a.sc = (const float*)sc, a.talk = (const unsigned short*)talk;
-  a.bias = (const float*)bias, a.ldb = ldb, a.nfar = nfar, a.H = H, a.G = G, a.R = G ? H / G : 0;
+  a.bias = (const float*)bias, a.bfar = (const float*)bfar, a.ldb = ldb, a.nfar = nfar, a.H = H, a.G = G, a.R = G ? H / G : 0;
   a.dkp = dkp, a.dvp = dvp, a.nsplit = 1;
   if (int rc = check(a, nitems)) return rc;
   const int nslot = G * ((H / G + 3) / 4);
   if (nslot > 8 || (dkp != 64 && dkp != 128) || (dvp != 64 && dvp != 128)) return KGS_ERR_ARG;
-  if (ldb < (nslot + 3) / 4 * 16 || ((uintptr_t)items & 15)) return KGS_ERR_SHAPE;
+  if (ldb < (nslot + 3) / 4 * 16 || (((uintptr_t)items | (uintptr_t)bfar | (uintptr_t)talk) & 15)) return KGS_ERR_SHAPE;
   if (dkp == 64) dvp == 64 ? tiles_ns<2, 4>(a, nitems, nslot, s) : tiles_ns<2, 8>(a, nitems, nslot, s);
   else dvp == 64 ? tiles_ns<4, 4>(a, nitems, nslot, s) : tiles_ns<4, 8>(a, nitems, nslot, s);
   return (int)hipGetLastError();

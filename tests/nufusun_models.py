@@ -39,11 +39,14 @@ def config(name: str) -> NufusunConfig:
 
 
 def weights(cfg: NufusunConfig, buckets: int, seed: int = 0) -> dict:
-    """Random weights with spread-out scores: queries scaled so that far keys matter."""
+    """Random weights with spread-out scores: queries scaled so that far keys matter, and
+    experts scaled down, so that in bf16 a choice between two that nearly tie matters less."""
     w = random_weights(cfg, seed, buckets=buckets)
     for name in w:
         if name.endswith("mix.q"):
             w[name] = (w[name].float() * 2).to(torch.bfloat16)
+        elif name.endswith(".down"):
+            w[name] = (w[name].float() * 0.3).to(torch.bfloat16)
         elif name.endswith(".b"):
             w[name] = (w[name].float() * 4).to(torch.bfloat16)
     return w

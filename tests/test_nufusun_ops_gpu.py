@@ -213,7 +213,8 @@ class Case:
         from kgs.ops.talking import QueryTiles, attention_tiles
 
         base = np.cumsum([0] + self.lens)
-        items = [(base[s] + p + j, s, p + j, min(16, n - j)) for s, p, n in portions for j in range(0, n, 16)]
+        step = self.h.tile
+        items = [(base[s] + p + j, s, p + j, min(step, n - j)) for s, p, n in portions for j in range(0, n, step)]
         t = QueryTiles(torch.tensor(items, dtype=torch.int32).cuda(), torch.tensor(self.bt).cuda())
         return self.view(attention_tiles(self.z, self.pages, self.w, t, self.out()))
 
