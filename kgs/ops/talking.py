@@ -59,6 +59,12 @@ class Heads:
         """Queries of one tile."""
         return 32 if self.slots <= 4 else 16
 
+    @property
+    def tile_bytes(self) -> int:
+        """Scratch of one tile: its queries in operand order."""
+        form = 2 if self.slots <= 2 else 4 if self.slots <= 4 else 8
+        return form * (2 if form <= 4 else 1) * 4096 * (self.dkp // 32)
+
     def slot_heads(self) -> list[int]:
         """Head at every position of the slots (-1: empty), padded to whole 16s."""
         out = []
@@ -223,11 +229,13 @@ def attention_tiles(q: torch.Tensor, pages: torch.Tensor, w: TalkingWeights, t: 
         raise ValueError(f"{h} has no tiled kernel")
     if t.items.dtype != torch.int32 or t.items.dim() != 2 or t.items.shape[1] != 4 or not t.items.is_contiguous():
         raise ValueError("items must be contiguous int32 [n, 4]")
+    n = t.items.shape[0]
+    scratch = torch.empty((n, h.tile_bytes), dtype=torch.uint8, device=q.device)
     rc = _lib.lib().kgs_talking_tiles(_act(q, q.shape[0], h.heads * h.dkp, torch.bfloat16, "q"), q.stride(0),
                                       pages.data_ptr(), _act(out, out.shape[0], h.heads * h.dvp, torch.bfloat16, "out"),
                                       out.stride(0), t.bt.data_ptr(), t.bt.shape[1], t.items.data_ptr(),
-                                      t.items.shape[0], w.sc.data_ptr(), w.talk_slots.data_ptr(),
+                                      n, scratch.data_ptr(), w.sc.data_ptr(), w.talk_slots.data_ptr(),
                                       w.bias_slots.data_ptr(), w.bias_far.data_ptr(), w.bias_slots.shape[1], w.nfar, h.heads, h.kv_heads,
                                       h.dkp, h.dvp, _lib.stream_handle(q.device))
-    _lib.check(rc, f"talking_tiles[{t.items.shape[0]}x{h.heads}]")
+    _lib.check(rc, f"talking_tiles[{n}x{h.heads}]")
     return out

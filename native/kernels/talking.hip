@@ -163,6 +163,7 @@ struct Args {
   const int* tok_pos;
   const int* rows;     // its batch row, or null: the same
   const int4* items;   // tiles: (first batch row, block-table row, position, queries)
+  void* qs;            // tiles: the queries of a workgroup again, in operand order
   float* po;           // partial results of split rows: [row, split][heads][dvp]
   float* pml;          // [row, split][heads][2]
   const float* sc;     // [heads]
@@ -436,17 +437,26 @@ __device__ __forceinline__ void static_for(F&& f) {
   }
 }
 
+// 1 KB of buffer `base` (16 bytes per lane from byte so + vo on) to LDS
+__device__ __forceinline__ void dma_chunk(const char* base, int bytes, char* dst, int vo, int so) {
+  const __amdgpu_buffer_rsrc_t r = __builtin_amdgcn_make_buffer_rsrc((void*)base, 0, bytes, 0x00020000);
+  __builtin_amdgcn_raw_ptr_buffer_load_lds(r, (KGS_LDS void*)dst, 16, vo, so, 0, 0);
+}
+
+// ... or to a register
+__device__ __forceinline__ bf16x8 load_frag(const char* base, int bytes, int vo, int so) {
+  const __amdgpu_buffer_rsrc_t r = __builtin_amdgcn_make_buffer_rsrc((void*)base, 0, bytes, 0x00020000);
+  return __builtin_bit_cast(bf16x8, __builtin_amdgcn_raw_buffer_load_b128(r, vo, so, 0));
+}
+
 __device__ __forceinline__ void fence() { __builtin_amdgcn_sched_barrier(0); }
-// every wave's LDS accesses are done; loads stay in flight
+// every wave's LDS accesses are done and all but its last VM loads have landed (63: no wait for any)
+template <int VM>
 __device__ __forceinline__ void bar() {
   fence();
-  asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
-  fence();
-}
-// ... and every wave's LDS-DMA has landed
-__device__ __forceinline__ void bar_vm() {
-  fence();
-  asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)\n\ts_barrier" ::: "memory");
+  asm volatile("" ::: "memory");
+  __builtin_amdgcn_s_waitcnt(0x0070 | (VM & 15) | ((VM >> 4) << 14));  // vmcnt(VM) lgkmcnt(0)
+  asm volatile("s_barrier" ::: "memory");
   fence();
 }
 
@@ -474,7 +484,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
   const int qpg = (a.R + 3) / 4, nslot = a.G * qpg;
   const int* bt = a.bt + (long)it.y * a.W;
   const int npage = (it.z + it.w - 1) / PAGE + 1;
-  const long hpage = (long)PAGE * (a.dkp + a.dvp) * 2;  // bytes of one head's page
+  constexpr int DK = 32 * NK, DV = 16 * ND, HPAGE = PAGE * (DK + DV) * 2;  // bytes of one head's page
   const int posw = it.z + 4 * QT * w;                   // position of the wave's first query
 
   // this lane's row of the S tiles: query n >> 2 of the block, head n & 3 of the slot. A query
@@ -485,12 +495,19 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
   int qoff[QT];
 #pragma unroll
   for (int t = 0; t < QT; ++t)
-    qoff[t] = (min(4 * (QT * w + t) + (n >> 2), it.w - 1) * (int)a.ldq + (n & 3) * a.dkp + 8 * q) * 2;
-  auto load_q = [&](bf16x8 (&f)[NK], int rt) {
-    const int s = rt / QT, so = (min(s / qpg, a.G - 1) * a.R + 4 * (s % qpg)) * a.dkp * 2;
+    qoff[t] = (min(4 * (QT * w + t) + (n >> 2), it.w - 1) * (int)a.ldq + (n & 3) * DK + 8 * q) * 2;
+  auto first_q = [&](bf16x8 (&f)[NK], int rt) {
+    const int s = rt / QT, so = (min(s / qpg, a.G - 1) * a.R + 4 * (s % qpg)) * DK * 2;
 #pragma unroll
     for (int k = 0; k < NK; ++k)
       f[k] = __builtin_bit_cast(bf16x8, __builtin_amdgcn_raw_buffer_load_b128(qrsrc, qoff[rt % QT] + 64 * k, so, 0));
+  };
+  // Those rows lie 16 to a load. They are read again for every page, so the wave puts them down
+  // in operand order first, 1 KB a fragment.
+  char* const qs = (char*)a.qs + ((long)blockIdx.x * 4 + w) * (RT * NK * 1024);
+  auto load_q = [&](bf16x8 (&f)[NK], int rt) {
+#pragma unroll
+    for (int k = 0; k < NK; ++k) f[k] = load_frag(qs, RT * NK * 1024, 16 * lane, (rt * NK + k) * 1024);
   };
   float sc[NS][4];  // uniform
 #pragma unroll
@@ -505,18 +522,18 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
 #pragma unroll
   for (int t = 0; t < MT; ++t) tf[t] = *(const f16x8*)(a.talk + (t * 64 + lane) * 8);
 
-  // page chunks of 1 KB, dealt to the waves
-  const int pbytes = a.G * (int)hpage;
-  // chunk w + 4 c of `per` chunks a key head, from byte `first` of its page on (past the
-  // last one: that one again)
-  auto dma = [&](int page, char* dst, int per, int first, int c) {
-    const __amdgpu_buffer_rsrc_t r =
-        __builtin_amdgcn_make_buffer_rsrc((void*)((const char*)a.pages + (long)page * pbytes), 0, pbytes, 0x00020000);
-    const int i = min(w + 4 * c, a.G * per - 4 + w);
-    __builtin_amdgcn_raw_ptr_buffer_load_lds(r, (KGS_LDS void*)(dst + i * 1024), 16, 16 * lane,
-                                             (i / per) * (int)hpage + first + (i % per) * 1024, 0, 0);
+  // Every slot has a place for its key head's K and V. They come in chunks of 1 KB, dealt to the
+  // waves: chunk w + 4 c of `per` a slot.
+  const int pbytes = a.G * HPAGE;
+  int head[NS];  // where a slot's head begins in a page
+#pragma unroll
+  for (int s = 0; s < NS; ++s) head[s] = min(s / qpg, a.G - 1) * HPAGE + w * 1024;
+  auto dma = [&](int page, char* dst, int per, int first, int c) {  // per: 4 or 8
+    dma_chunk((const char*)a.pages + (long)page * pbytes, pbytes, dst + (w + 4 * c) * 1024, 16 * lane,
+              head[4 * c / per] + (first + 4 * c % per * 1024));
   };
   constexpr int CK = NS * 2 * NK / 4, CV = NS * ND / 4;  // chunks per wave of K and of V
+  constexpr int KPER = 2 * NK, VPER = ND;
   auto page_id = [&](int pg) { return bt[min(pg, npage - 1)]; };
 
   // the far bias less the running maximum of (query, slot 4t + q, head): the mixture's addend
@@ -533,11 +550,15 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
 
   bf16x8 qf[RQ][NK];
 #pragma unroll
-  for (int i = 0; i < RQ; ++i) load_q(qf[i], i);
+  for (int i = RT - 1; i >= 0; --i) {
+    first_q(qf[i % RQ], i);
+#pragma unroll
+    for (int k = 0; k < NK; ++k) *(bf16x8*)(qs + (i * NK + k) * 1024 + 16 * lane) = qf[i % RQ][k];
+  }
   int page = __builtin_amdgcn_readfirstlane(page_id(0));
 #pragma unroll
-  for (int c = 0; c < CK; ++c) dma(page, ks, 2 * NK, 0, c);
-  bar_vm();
+  for (int c = 0; c < CK; ++c) dma(page, ks, KPER, 0, c);
+  bar<0>();
   for (int pg = 0; pg < npage; ++pg) {
     const int tok0 = pg * PAGE;
     const int next = page_id(pg + 1);
@@ -547,7 +568,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     constexpr int PF = 5, STEPS = NS * NK;
     bf16x8 kf[PF + 1][2];
     auto read_k = [&](int p) {
-      const char* kp = ks + (min((p / NK) / qpg, a.G - 1) * 2 * NK + p % NK) * 1024 + 16 * lane;
+      const char* kp = ks + (p / NK * 2 * NK + p % NK) * 1024 + 16 * lane;
       kf[p % (PF + 1)][0] = *(const bf16x8*)kp;
       kf[p % (PF + 1)][1] = *(const bf16x8*)(kp + NK * 1024);
     };
@@ -571,13 +592,10 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
         for (int t = 0; t < QT; ++t)
           if ((p / NK) * QT + t + RQ < RT) load_q(qf[((p / NK) * QT + t) % RQ], (p / NK) * QT + t + RQ);
       }
-#pragma unroll
-      for (int c = 0; c < CV; ++c)
-        if (c * STEPS / CV == p) dma(page, vs, ND, PAGE * NK * 64, c);
       fence();
     }
-    bar();  // K of this page is done with everywhere
-    page = __builtin_amdgcn_readfirstlane(next);
+    bar<63>();  // K of this page is done with everywhere
+    const int pnext = __builtin_amdgcn_readfirstlane(next);
 
     // ---- mix, softmax
     const bool near = posw - (tok0 + PAGE - 1) < a.nfar, edge = tok0 + PAGE - 1 > posw;
@@ -605,12 +623,6 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
         for (int j = 0; j < 2; ++j)
 #pragma unroll
           for (int hf = 0; hf < MT; ++hf) transpose4(x[j][hf][0]), transpose4(x[j][hf][1]);
-        fence();
-        if (pg + 1 < npage) {
-#pragma unroll
-          for (int c = 0; c < CK; ++c)
-            if (c * 2 * QT / CK == 2 * qt + kt) dma(page, ks, 2 * NK, 0, c);
-        }
         f32x4 D[4][MT];
 #pragma unroll
         for (int j = 1; j >= 0; --j)
@@ -644,6 +656,13 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
 #pragma unroll
               for (int r = 0; r < 4; ++r) D[i][t][r] = dist + i < 0 ? NEG : D[i][t][r];
         }
+        // first the V of this page, then the K of the next (past the last one: that one again)
+#pragma unroll
+        for (int c = 0; c < CV + CK; ++c)
+          if (c * 2 * QT / (CV + CK) == 2 * qt + kt) {
+            if (c < CV) dma(page, vs, VPER, PAGE * DK * 2, c);
+            else dma(pnext, ks, KPER, 0, c - CV);
+          }
         float over = D[0][0][0];
 #pragma unroll
         for (int i = 0; i < 4; ++i)
@@ -718,14 +737,15 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
       });
       asm volatile("s_nop 7" ::: "memory");
     }
-    bar_vm();  // V of this page and K of the next are there
+    bar<CK>();  // V of this page is there
+    page = pnext;
 
     // ---- P V
 #pragma unroll
     for (int i = 0; i < RQ; ++i) load_q(qf[i], i);  // for the next page
     bf16x8 vf[2][ND];
     auto read_v = [&](bf16x8 (&f)[ND], int s) {
-      const char* vp = vs + min(s / qpg, a.G - 1) * (ND * 1024) + 16 * lane;
+      const char* vp = vs + s * (ND * 1024) + 16 * lane;
 #pragma unroll
       for (int i = 0; i < ND; ++i) f[i] = *(const bf16x8*)(vp + i * 1024);
     };
@@ -761,8 +781,9 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
       });
       fence();
     });
-    bar();  // V is done with everywhere
+    bar<RQ * NK>();  // V is done with everywhere, K of the next page is there
   }
+  bar<0>();
 
   // rows' maxima to the lanes that hold the rows: [qt][slot][row]
   float* mm = (float*)ps;
@@ -781,7 +802,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
       const float L = xor32_sum(xor16_sum(l[rt])) + __builtin_amdgcn_exp2f(-mm[(t * NS + s) * 16 + n]);
       const bool ok = s < nslot && hr < a.R && qi < it.w;
       const float inv = 1.0f / L;
-      unsigned short* op = (unsigned short*)a.o + (long)(it.x + qi) * a.ldo + (long)(s / qpg * a.R + hr) * a.dvp + 4 * q;
+      unsigned short* op = (unsigned short*)a.o + (long)(it.x + qi) * a.ldo + (long)(s / qpg * a.R + hr) * DV + 4 * q;
       static_for<0, ND>([&](auto dc) {
         constexpr int d = decltype(dc)::value;
         const f32x4 o = accr::read<rt * ND + d>() * inv;
@@ -928,7 +949,7 @@ KGS_EXPORT int kgs_talking_rows(const void* q, long ldq, const void* pages, void
                                 int G, int dkp, int dvp, int nsplit, int plain, int f32, hipStream_t s) {
   using namespace kgs::talking;
   Args a{q, ldq, pages, o, ldo, (const int*)bt, W, (const int*)tok_seq, (const int*)tok_pos, (const int*)rows, nullptr,
-         (float*)po, (float*)pml, (const float*)sc, (const unsigned short*)talk, (const float*)talk, (const float*)bias,
+         nullptr, (float*)po, (float*)pml, (const float*)sc, (const unsigned short*)talk, (const float*)talk, (const float*)bias,
          nullptr, ldb, nfar, H, G, G ? H / G : 0, dkp, dvp, nsplit};
   if (int rc = check(a, nrows)) return rc;
   if (plain || f32) {
@@ -954,20 +975,21 @@ KGS_EXPORT int kgs_talking_rows(const void* q, long ldq, const void* pages, void
 // Prompt portions: nitems blocks of consecutive queries (first batch row, block-table
 // row, first position, queries: up to 32, 16 above 4 slots). bf16, dkp and dvp 64 or 128, at most 8 slots
 // of 4 heads (G ceil(H / G / 4)); talk (fp16) and biases in slot order, ldb = 16 ceil(slots / 4);
-// bias is the table less its last row, bfar.
+// bias is the table less its last row, bfar. qs: scratch, slots (2, 4 or 8) x 4 KB x dkp / 32
+// per item, twice that up to 4 slots.
 KGS_EXPORT int kgs_talking_tiles(const void* q, long ldq, const void* pages, void* o, long ldo, const void* bt, int W,
-                                 const void* items, int nitems, const void* sc, const void* talk, const void* bias,
+                                 const void* items, int nitems, void* qs, const void* sc, const void* talk, const void* bias,
                                  const void* bfar, int ldb, int nfar, int H, int G, int dkp, int dvp, hipStream_t s) {
   using namespace kgs::talking;
   Args a{};
   a.q = q, a.ldq = ldq, a.pages = pages, a.o = o, a.ldo = ldo, a.bt = (const int*)bt, a.W = W;
-  a.items = (const int4*)items, a.sc = (const float*)sc, a.talk = (const unsigned short*)talk;
+  a.items = (const int4*)items, a.qs = qs, a.sc = (const float*)sc, a.talk = (const unsigned short*)talk;
   a.bias = (const float*)bias, a.bfar = (const float*)bfar, a.ldb = ldb, a.nfar = nfar, a.H = H, a.G = G, a.R = G ? H / G : 0;
   a.dkp = dkp, a.dvp = dvp, a.nsplit = 1;
   if (int rc = check(a, nitems)) return rc;
   const int nslot = G * ((H / G + 3) / 4);
   if (nslot > 8 || (dkp != 64 && dkp != 128) || (dvp != 64 && dvp != 128)) return KGS_ERR_ARG;
-  if (ldb < (nslot + 3) / 4 * 16 || (((uintptr_t)items | (uintptr_t)bfar | (uintptr_t)talk) & 15)) return KGS_ERR_SHAPE;
+  if (ldb < (nslot + 3) / 4 * 16 || (((uintptr_t)items | (uintptr_t)bfar | (uintptr_t)talk | (uintptr_t)qs) & 15)) return KGS_ERR_SHAPE;
   if (dkp == 64) dvp == 64 ? tiles_ns<2, 4>(a, nitems, nslot, s) : tiles_ns<2, 8>(a, nitems, nslot, s);
   else dvp == 64 ? tiles_ns<4, 4>(a, nitems, nslot, s) : tiles_ns<4, 8>(a, nitems, nslot, s);
   return (int)hipGetLastError();
