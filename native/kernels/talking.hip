@@ -479,6 +479,9 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
   char* const ks = smem;
   char* const vs = smem + NS * 2 * NK * 1024;
   const int lane = threadIdx.x & 63, w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), n = lane & 15, q = lane >> 4;
+  // where this lane reads V: an address of its own, within the reach of the reads' offsets
+  unsigned vl = (unsigned)(uintptr_t)(KGS_LDS char*)vs + 16 * lane;
+  asm volatile("" : "+v"(vl));
   char* const ps = vs + NS * ND * 1024 + w * RT * 1024;  // this wave's P: [qt][slot][16 rows][32 keys]
   const int4 it = a.items[blockIdx.x];
   const int qpg = (a.R + 3) / 4, nslot = a.G * qpg;
@@ -592,6 +595,9 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
         for (int t = 0; t < QT; ++t)
           if ((p / NK) * QT + t + RQ < RT) load_q(qf[((p / NK) * QT + t) % RQ], (p / NK) * QT + t + RQ);
       }
+#pragma unroll
+      for (int c = 0; c < CV / 2; ++c)  // half of this page's V
+        if (c * STEPS / (CV / 2) == p) dma(page, vs, VPER, PAGE * DK * 2, c);
       fence();
     }
     bar<63>();  // K of this page is done with everywhere
@@ -656,13 +662,6 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
 #pragma unroll
               for (int r = 0; r < 4; ++r) D[i][t][r] = dist + i < 0 ? NEG : D[i][t][r];
         }
-        // first the V of this page, then the K of the next (past the last one: that one again)
-#pragma unroll
-        for (int c = 0; c < CV + CK; ++c)
-          if (c * 2 * QT / (CV + CK) == 2 * qt + kt) {
-            if (c < CV) dma(page, vs, VPER, PAGE * DK * 2, c);
-            else dma(pnext, ks, KPER, 0, c - CV);
-          }
         float over = D[0][0][0];
 #pragma unroll
         for (int i = 0; i < 4; ++i)
@@ -705,7 +704,15 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
           }
         }
 #pragma unroll
-        for (int i = 0; i < 4; ++i)
+        for (int i = 0; i < 4; ++i) {
+          // a chunk or two at a time: the rest of this page's V, then half of the next one's K
+          fence();
+#pragma unroll
+          for (int c = CV / 2; c < CV + CK / 2; ++c)
+            if ((c - CV / 2) * 8 * QT / (CV - CV / 2 + CK / 2) == 4 * (2 * qt + kt) + i) {
+              if (c < CV) dma(page, vs, VPER, PAGE * DK * 2, c);
+              else dma(pnext, ks, KPER, 0, c - CV);
+            }
 #pragma unroll
           for (int t = 0; t < MT; ++t) {
             float p[4];
@@ -723,6 +730,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
               *(unsigned*)(pp + ((3 ^ q) * 64)) = __builtin_amdgcn_perm(c1, p0[i][t][1], 0x07060302u);
             }
           }
+        }
       }
     }
     if (__builtin_expect(grown, 0)) {
@@ -737,7 +745,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
       });
       asm volatile("s_nop 7" ::: "memory");
     }
-    bar<CK>();  // V of this page is there
+    bar<CK / 2>();  // V of this page is there
     page = pnext;
 
     // ---- P V
@@ -745,9 +753,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     for (int i = 0; i < RQ; ++i) load_q(qf[i], i);  // for the next page
     bf16x8 vf[2][ND];
     auto read_v = [&](bf16x8 (&f)[ND], int s) {
-      const char* vp = vs + s * (ND * 1024) + 16 * lane;
 #pragma unroll
-      for (int i = 0; i < ND; ++i) f[i] = *(const bf16x8*)(vp + i * 1024);
+      for (int i = 0; i < ND; ++i) f[i] = *(const KGS_LDS bf16x8*)(uintptr_t)(vl + (s * ND + i) * 1024);
     };
     u32x4 pw[2][QT];
     auto read_p = [&](u32x4 (&f)[QT], int s) {
@@ -765,6 +772,9 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
         read_v(vf[(s + 1) & 1], s + 1);
       }
       fence();
+#pragma unroll
+      for (int c = CK / 2; c < CK; ++c)  // the other half of K (past the last page: that one again)
+        if ((c - CK / 2) * NS / 2 / (CK - CK / 2) == s) dma(pnext, ks, KPER, 0, c);
       static_for<0, QT>([&](auto tc) {
         constexpr int t = decltype(tc)::value, rt = s * QT + t;
         const u32x4 pv = pw[s & 1][t];
@@ -781,9 +791,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
       });
       fence();
     });
-    bar<RQ * NK>();  // V is done with everywhere, K of the next page is there
+    bar<0>();  // V is done with everywhere, K of the next page is there
   }
-  bar<0>();
 
   // rows' maxima to the lanes that hold the rows: [qt][slot][row]
   float* mm = (float*)ps;
