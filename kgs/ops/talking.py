@@ -148,14 +148,14 @@ class TalkingWeights:
         plain = list(range(H)) + [-1] * ((16 if H <= 16 else 32 if H <= 32 else (H + 63) // 64 * 64) - H)
         self.bias = table(plain)
         if heads.mfma:
-            tb = talk.to(device).to(torch.bfloat16)
+            tb = talk.to(device).to(torch.bfloat16).to(torch.float16)  # exact down to 2^-14
             self.talk = mix_fragments(tb, plain)
             if heads.tiled:
                 order = heads.slot_heads()
                 b = table(order)
                 self.bias_far = b[-1].clone()
                 self.bias_slots = (b - self.bias_far).contiguous()
-                self.talk_slots = mix_fragments(tb.to(torch.float16), order)  # exact down to 2^-14
+                self.talk_slots = mix_fragments(tb, order)
         else:
             self.talk = talk.to(device).float().contiguous()
 

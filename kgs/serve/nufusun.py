@@ -145,8 +145,8 @@ class ExpertsFF:
 
     @staticmethod
     def _router_rows(n: int) -> int:
-        """Experts padded to a size the MFMA router has (above 128: any multiple of 16)."""
-        return next((s for s in (16, 32, 64, 128) if s >= n), (n + 15) // 16 * 16)
+        """Experts padded to a size the MFMA router has (above 64: any multiple of 16)."""
+        return next((s for s in (16, 32, 64) if s >= n), (n + 15) // 16 * 16)
 
     def __call__(self, model, h: torch.Tensor, b: Batch) -> ExpertRows:
         m = self.m

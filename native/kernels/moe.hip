@@ -37,38 +37,49 @@ struct RouteArgs {
 
 __device__ __forceinline__ float rcp_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
 
-// z[16 tokens][zs] in LDS -> choices; 16 lanes per token
+// the larger logit, the lower number on a tie, over the 16 lanes of a DPP row
+template <int CTRL>
+__device__ __forceinline__ void better(float& v, int& e) {
+  const float ov = dpp_move<CTRL>(v);
+  const int oe = __float_as_int(dpp_move<CTRL>(__int_as_float(e)));
+  if (ov > v || (ov == v && oe < e)) v = ov, e = oe;
+}
+
+// z[16 tokens][zs] in LDS -> choices; 16 lanes per token (the first 256 threads), each over
+// its own experts
 __device__ __forceinline__ void choose(const RouteArgs& a, float* z, int zs, int* lh, int t0) {
-  const int tid = threadIdx.x, tk = tid >> 4, n = tid & 15;
-  for (int e = tid; e < a.E; e += 256) lh[e] = 0;
+  const int tid = threadIdx.x, tk = tid >> 4, n = tid & 15, nt = blockDim.x;
+  for (int e = tid; e < a.E; e += nt) lh[e] = 0;
   __syncthreads();
   const int t = t0 + tk;
-  const bool real = t < a.T && (!a.slots || a.slots[t] >= 0);
-  float* row = z + tk * zs;
-  for (int k = 0; k < a.top; ++k) {
-    float best = -INFINITY;
-    int be = 0x7fffffff;
-    for (int e = n; e < a.E; e += 16)
-      if (row[e] > best || (be == 0x7fffffff && row[e] == best)) best = row[e], be = e;
-#pragma unroll
-    for (int x = 1; x < 16; x <<= 1) {
-      const float ob = __shfl_xor(best, x, 16);
-      const int oe = __shfl_xor(be, x, 16);
-      if (ob > best || (ob == best && oe < be)) best = ob, be = oe;
+  const bool real = tid < 256 && t < a.T && (!a.slots || a.slots[t] >= 0);
+  if (tid < 256) {
+    float* row = z + tk * zs;
+    for (int k = 0; k < a.top; ++k) {
+      float best = -INFINITY;
+      int be = 0x7fffffff;
+      for (int e = n; e < a.E; e += 16) {
+        const float v = row[e];
+        if (v > best || (be == 0x7fffffff && v == best)) best = v, be = e;
+      }
+      better<0x128>(best, be);  // row_ror 8, 4, 2, 1
+      better<0x124>(best, be);
+      better<0x122>(best, be);
+      better<0x121>(best, be);
+      // be is a valid expert unless every logit left is NaN: such a token takes none
+      const bool ok = be < a.E;
+      if (ok && (be & 15) == n) row[be] = __uint_as_float(0x7fc00000u);  // taken: compares false from now on
+      if (n == 0 && t < a.T) {
+        const long o = (long)t * a.top + k;
+        a.ids[o] = real && ok ? be : -1;
+        a.weight[o] = rcp_sigmoid(best);
+        a.rank[o] = real && ok ? atomicAdd(&lh[be], 1) : 0;
+      }
     }
-    // be is a valid expert unless every logit left is NaN: such a token takes none
-    const bool ok = be < a.E;
-    if (ok && (be & 15) == n) row[be] = __uint_as_float(0x7fc00000u);  // taken: compares false from now on
-    if (n == 0 && t < a.T) {
-      const long o = (long)t * a.top + k;
-      a.ids[o] = real && ok ? be : -1;
-      a.weight[o] = rcp_sigmoid(best);
-      a.rank[o] = real && ok ? atomicAdd(&lh[be], 1) : 0;
-    }
-    __syncthreads();
   }
+  __syncthreads();
   // local ranks -> ranks among all tokens
-  for (int e = tid; e < a.E; e += 256) {
+  for (int e = tid; e < a.E; e += nt) {
     const int c = lh[e];
     if (c) lh[e] = atomicAdd(&a.counts[e], c);
   }
@@ -80,39 +91,52 @@ __device__ __forceinline__ void choose(const RouteArgs& a, float* z, int zs, int
     }
 }
 
-// bf16: four waves split the width, ET 16-expert MFMA tiles each
+// bf16: eight waves split the width, ET 16-expert MFMA tiles each, U steps' loads at a time
 template <int ET>
-__global__ __launch_bounds__(256) void route_mfma(RouteArgs a) {
+__global__ __launch_bounds__(512) void route_mfma(RouteArgs a) {
+  constexpr int U = ET >= 8 ? 1 : ET >= 4 ? 2 : 4;
   extern __shared__ float lds[];
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, n = lane & 15, q = lane >> 4;
-  const int t0 = blockIdx.x * RT, t = min(t0 + n, a.T - 1), kw = a.wp / 4;
+  const int t0 = blockIdx.x * RT, t = min(t0 + n, a.T - 1), kw = a.wp / 8;
   const unsigned short* hp = (const unsigned short*)a.h + (long)t * a.ldh + w * kw + 8 * q;
   const unsigned short* wr = (const unsigned short*)a.w + (long)n * a.wp + w * kw + 8 * q;
   f32x4 acc[ET];
 #pragma unroll
   for (int e = 0; e < ET; ++e) acc[e] = f32x4{};
-  for (int k = 0; k < kw; k += 32) {
-    const bf16x8 hf = *(const bf16x8*)(hp + k);
+  auto steps = [&](int k, auto uc) {
+    constexpr int UU = decltype(uc)::value;
+    bf16x8 hf[UU], wf[UU][ET];
 #pragma unroll
-    for (int e = 0; e < ET; ++e)
-      acc[e] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(wr + (long)e * 16 * a.wp + k), hf, acc[e], 0, 0, 0);
-  }
-  // lane: token n, experts 16e + 4q + r
+    for (int u = 0; u < UU; ++u) {
+      hf[u] = *(const bf16x8*)(hp + k + 32 * u);
+#pragma unroll
+      for (int e = 0; e < ET; ++e) wf[u][e] = *(const bf16x8*)(wr + (long)e * 16 * a.wp + k + 32 * u);
+    }
+#pragma unroll
+    for (int u = 0; u < UU; ++u)
+#pragma unroll
+      for (int e = 0; e < ET; ++e) acc[e] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[u][e], hf[u], acc[e], 0, 0, 0);
+  };
+  int k = 0;
+  for (; k + 32 * U <= kw; k += 32 * U) steps(k, std::integral_constant<int, U>{});
+  for (; k < kw; k += 32) steps(k, std::integral_constant<int, 1>{});
+  // lane: token n, experts 16e + 4q + r; the waves' sums meet in LDS, added in wave order
   const int zs = a.ep + 1;
   float* z = lds;
-  int* lh = (int*)(lds + RT * zs);
-  for (int src = 0; src < 4; ++src) {  // waves add in a fixed order
-    if (w == src)
+  float* part = lds + RT * zs;  // [8][RT][zs]
+  int* lh = (int*)(part + 8 * RT * zs);
 #pragma unroll
-      for (int e = 0; e < ET; ++e)
+  for (int e = 0; e < ET; ++e)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          float* p = z + n * zs + 16 * e + 4 * q + r;
-          *p = src == 0 ? acc[e][r] : *p + acc[e][r];
-        }
-    __syncthreads();
+    for (int r = 0; r < 4; ++r) part[(w * RT + n) * zs + 16 * e + 4 * q + r] = acc[e][r];
+  __syncthreads();
+  for (int i = threadIdx.x; i < RT * zs; i += 512) {
+    float s = part[i];
+#pragma unroll
+    for (int j = 1; j < 8; ++j) s += part[j * RT * zs + i];
+    z[i] = s;
   }
-  choose(a, z, zs, lh, t0);
+  choose(a, z, zs, lh, t0);  // begins with a barrier
 }
 
 template <typename T>
@@ -389,20 +413,20 @@ __global__ __launch_bounds__(256) void grouped_f32(GroupedArgs a) {
 
 template <int ET>
 int launch_route(const RouteArgs& a, size_t lds, hipStream_t s) {
-  hipLaunchKernelGGL((route_mfma<ET>), dim3((a.T + RT - 1) / RT), dim3(256), lds, s, a);
+  hipLaunchKernelGGL((route_mfma<ET>), dim3((a.T + RT - 1) / RT), dim3(512), lds + 8 * RT * (a.ep + 1) * 4, s, a);
   return (int)hipGetLastError();
 }
 
 }  // namespace moe
 }  // namespace kgs
 
-// Router logits of h [T, wp] with w [ep, wp] (wp % 128, ep % 16), the top choices per
+// Router logits of h [T, wp] with w [ep, wp] (wp % 256, ep % 16), the top choices per
 // token (ids -1: a row whose slot is negative), their weights and their ranks;
 // counts [E] must be zero and ends as the tokens of every expert.
 KGS_EXPORT int kgs_moe_route(const void* h, long ldh, const void* w, const void* slots, void* counts, void* ids,
                              void* rank, void* weight, int T, int E, int ep, int wp, int top, int f32, hipStream_t s) {
   using namespace kgs::moe;
-  if (T <= 0 || E <= 0 || E > 1024 || ep < E || ep % 16 || top <= 0 || top > E || wp <= 0 || wp % 128 || ldh < wp)
+  if (T <= 0 || E <= 0 || E > 1024 || ep < E || ep % 16 || top <= 0 || top > E || wp <= 0 || wp % 256 || ldh < wp)
     return KGS_ERR_SHAPE;
   if (ldh % 8 || (((uintptr_t)h | (uintptr_t)w) & 15)) return KGS_ERR_ALIGN;
   RouteArgs a{h, ldh, w, (const int*)slots, (int*)counts, (int*)ids, (int*)rank, (float*)weight, T, E, ep, wp, top};
@@ -413,7 +437,6 @@ KGS_EXPORT int kgs_moe_route(const void* h, long ldh, const void* w, const void*
   else if (ep <= 16) return launch_route<1>(a, lds, s);
   else if (ep <= 32) return launch_route<2>(a, lds, s);
   else if (ep == 64) return launch_route<4>(a, lds, s);
-  else if (ep == 128) return launch_route<8>(a, lds, s);
   else hipLaunchKernelGGL(route_plain<unsigned short>, grid, dim3(256), lds, s, a);
   return (int)hipGetLastError();
 }

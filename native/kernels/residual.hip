@@ -11,7 +11,7 @@
 namespace kgs {
 namespace residual {
 
-constexpr int MAX_NV = 8;  // 8-column chunks per thread
+constexpr int MAX_NT = 512, MAX_NV = 4;  // 8-column chunks per thread
 
 struct Args {
   float* x;           // [T, wp]
@@ -52,10 +52,10 @@ __device__ __forceinline__ void store8(float* p, const float (&v)[8]) {
 __device__ __forceinline__ void store8(unsigned short* p, const float (&v)[8]) { *(bf16x8*)p = pack_bf16x8(v, 0); }
 
 template <typename T, int NV, bool EMBED>
-__global__ __launch_bounds__(256) void step(Args a) {
+__global__ __launch_bounds__(MAX_NT) void step(Args a) {
   const long t = blockIdx.x;
   const int tid = threadIdx.x, nt = blockDim.x, nc = a.wp / 8;
-  __shared__ float part[4];
+  __shared__ float part[MAX_NT / 64];
   if (blockIdx.x == 0)
     for (int i = tid; i < a.nzero; i += nt) a.zero[i] = 0;
   float v[NV][8], ss = 0.f;
@@ -78,21 +78,26 @@ __global__ __launch_bounds__(256) void step(Args a) {
 #pragma unroll
         for (int i = 0; i < 8; ++i) s[i] += b[i];
       }
-      if (a.y) {
-        for (int j = 0; j < a.top; ++j) {
-          const int p = a.pos[t * a.top + j];
-          if (p < 0) continue;
-          for (int sl = 0; sl < a.nslice; ++sl) {
-            float e[8];
-            const long o = sl * a.yslice + p * a.ldy + 8 * c;
-            if (a.y32) load8((const float*)a.y + o, e);
-            else load8((const unsigned short*)a.y + o, e);
+      load8(xp, v[k]);
+      // the chosen experts' rows, four choices' loads at a time
+      for (int j0 = 0; j0 < a.top; j0 += 4) {
+        int p[4];
 #pragma unroll
-            for (int i = 0; i < 8; ++i) s[i] += e[i];
+        for (int j = 0; j < 4; ++j) p[j] = j0 + j < a.top ? a.pos[t * a.top + j0 + j] : -1;
+        for (int sl = 0; sl < a.nslice; ++sl) {
+          float e[4][8];
+#pragma unroll
+          for (int j = 0; j < 4; ++j) {
+            const long o = sl * a.yslice + max(p[j], 0) * a.ldy + 8 * c;
+            if (a.y32) load8((const float*)a.y + o, e[j]);
+            else load8((const unsigned short*)a.y + o, e[j]);
           }
+#pragma unroll
+          for (int j = 0; j < 4; ++j)
+#pragma unroll
+            for (int i = 0; i < 8; ++i) s[i] += p[j] >= 0 ? e[j][i] : 0.f;
         }
       }
-      load8(xp, v[k]);
 #pragma unroll
       for (int i = 0; i < 8; ++i) v[k][i] += s[i];
     }
@@ -123,18 +128,17 @@ __global__ __launch_bounds__(256) void step(Args a) {
 template <typename T, bool EMBED>
 int launch(const Args& a, int rows, hipStream_t s) {
   const int nc = a.wp / 8;
-  const int nt = nc >= 256 ? 256 : (nc + 63) / 64 * 64;
+  const int nt = nc >= MAX_NT ? MAX_NT : (nc + 63) / 64 * 64;
   const int nv = (nc + nt - 1) / nt;
   const dim3 grid(rows), block(nt);
   if (nv <= 1) hipLaunchKernelGGL((step<T, 1, EMBED>), grid, block, 0, s, a);
   else if (nv <= 2) hipLaunchKernelGGL((step<T, 2, EMBED>), grid, block, 0, s, a);
-  else if (nv <= 4) hipLaunchKernelGGL((step<T, 4, EMBED>), grid, block, 0, s, a);
-  else hipLaunchKernelGGL((step<T, 8, EMBED>), grid, block, 0, s, a);
+  else hipLaunchKernelGGL((step<T, 4, EMBED>), grid, block, 0, s, a);
   return (int)hipGetLastError();
 }
 
 int check(const Args& a, int rows, int f32) {
-  if (rows <= 0 || a.width <= 0 || a.wp < a.width || a.wp > 256 * 8 * MAX_NV || a.ldh < a.wp) return KGS_ERR_SHAPE;
+  if (rows <= 0 || a.width <= 0 || a.wp < a.width || a.wp > MAX_NT * 8 * MAX_NV || a.ldh < a.wp) return KGS_ERR_SHAPE;
   if (a.wp % 8 || a.ldh % 8 || (((uintptr_t)a.x | (uintptr_t)a.h | (uintptr_t)a.w) & 15)) return KGS_ERR_ALIGN;
   return KGS_OK;
 }
@@ -165,7 +169,7 @@ KGS_EXPORT int kgs_residual_add(void* x, const void* a_, long lda, const void* a
   using namespace kgs::residual;
   Args a{};
   a.x = (float*)x, a.a = a_, a.lda = lda, a.ab = (const float*)ab;
-  a.y = y, a.ldy = ldy, a.yslice = yslice, a.nslice = nslice, a.y32 = y32, a.pos = (const int*)pos, a.top = top;
+  a.y = y, a.ldy = ldy, a.yslice = yslice, a.nslice = nslice, a.y32 = y32, a.pos = (const int*)pos, a.top = y ? top : 0;
   a.w = (const float*)w, a.h = h, a.ldh = ldh, a.zero = (int*)zero, a.nzero = zero ? nzero : 0;
   a.width = width, a.wp = wp, a.eps = eps;
   if (int rc = check(a, rows, f32)) return rc;

@@ -9,10 +9,10 @@
 // = log2(e) sum_g talk[h, g] rel_g[n], whose last row serves every distance from
 // its number on.
 //
-// The mixture is an MFMA over heads whose products are exact: talk is a bf16 number, and
-// a score enters in parts that hold its bits -- three bf16 parts (rows: all 24 bits) or
-// two fp16 parts (tiles: 22 bits or 2^-24, less than the fp32 sum of the score itself
-// loses; beyond fp16's range a part saturates). What makes it cheap is that no score
+// The mixture is an MFMA over heads whose products are exact: talk is a bf16 number
+// that fp16 holds (to 2^-25 where it is below 2^-14), and a score enters as two fp16 parts
+// that hold 22 of its bits, or 2^-24: less than the fp32 sum of the score itself
+// loses (beyond fp16's range a part saturates). What makes it cheap is that no score
 // leaves the registers for it:
 //   rows   (decoded tokens, short portions) S = q K^T with heads on the MFMA's rows
 //          leaves a lane 4 heads of one key; an MFMA contracts in any order both
@@ -48,13 +48,6 @@ __device__ __forceinline__ int v_at(int tok, int d) {
   return ((d >> 4) * 64 + (tok >> 3) * 16 + (d & 15)) * 8 + (tok & 7);
 }
 
-// three bf16 parts of an fp32 value, each in the upper half of its word; exact
-__device__ __forceinline__ void split3(float s, unsigned (&u)[3]) {
-  u[0] = __float_as_uint(s);
-  const float r1 = s - __uint_as_float(u[0] & 0xffff0000u);
-  u[1] = __float_as_uint(r1);
-  u[2] = __float_as_uint(r1 - __uint_as_float(u[1] & 0xffff0000u));
-}
 // two fp16 parts of two fp32 values: parts truncated, so a value out of range saturates
 typedef _Float16 f16x2 __attribute__((ext_vector_type(2)));
 typedef _Float16 f16x8 __attribute__((ext_vector_type(8)));
@@ -65,8 +58,6 @@ __device__ __forceinline__ void split2(float a, float b, unsigned& hi, unsigned&
   hi = __builtin_bit_cast(unsigned, h);
   lo = __builtin_bit_cast(unsigned, __builtin_amdgcn_cvt_pkrtz(ra, rb));
 }
-// upper halves of (lo, hi) as one word
-__device__ __forceinline__ unsigned pack_hi(unsigned lo, unsigned hi) { return __builtin_amdgcn_perm(hi, lo, 0x07060302u); }
 
 typedef unsigned u32x4 __attribute__((ext_vector_type(4)));
 typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
@@ -96,9 +87,11 @@ __global__ __launch_bounds__(256) void write_kv(WriteArgs a) {
   const int kind = col < a.nq ? 0 : col < a.nq + nk ? 1 : 2;
   const int c = kind == 0 ? col : kind == 1 ? col - a.nq : col - a.nq - nk;
   const int zc = kind == 0 ? c : kind == 1 ? a.ok + c : a.ov + c;
-  float b[8];
+  const f32x4 b0 = *(const f32x4*)(a.b + col), b1 = *(const f32x4*)(a.b + col + 4);
+  const float b[8] = {b0[0], b0[1], b0[2], b0[3], b1[0], b1[1], b1[2], b1[3]};
+  int sl[8];
 #pragma unroll
-  for (int i = 0; i < 8; ++i) b[i] = a.b[col + i];
+  for (int r = 0; r < 8; ++r) sl[r] = r < nr ? a.slots[r0 + r] : -1;
   Vec8<T> x[8];
 #pragma unroll
   for (int r = 0; r < 8; ++r) {
@@ -117,9 +110,6 @@ __global__ __launch_bounds__(256) void write_kv(WriteArgs a) {
   }
   const long per = (long)PAGE * (a.dkp + a.dvp);  // elements of one head's page
   const int g = c / (kind == 1 ? a.dkp : a.dvp), d = c - g * (kind == 1 ? a.dkp : a.dvp);
-  int sl[8];
-#pragma unroll
-  for (int r = 0; r < 8; ++r) sl[r] = r < nr ? a.slots[r0 + r] : -1;
   if (kind == 1) {
 #pragma unroll
     for (int r = 0; r < 8; ++r)
@@ -167,7 +157,7 @@ struct Args {
   float* po;           // partial results of split rows: [row, split][heads][dvp]
   float* pml;          // [row, split][heads][2]
   const float* sc;     // [heads]
-  const unsigned short* talk;  // MFMA fragments (rows: bf16 [HT][NC][64][8]; tiles: fp16 [MT][64][8])
+  const unsigned short* talk;  // fp16 MFMA fragments (rows: [HT][NC][64][8]; tiles: [MT][64][8])
   const float* talk32; // [heads][heads], the plain kernel's
   const float* bias;   // [nfar + 1][ldb] (tiles: less the last row)
   const float* bfar;   // tiles: the last row
@@ -178,7 +168,7 @@ struct Args {
 // Heads 16 ht + .. of one token per MFMA tile. Four waves take pages of the split in
 // turn, key heads one after another with the next one's fragments in flight.
 template <int HT, int NK, int ND>
-__global__ __launch_bounds__(256, 2) void attn_rows(Args a) {
+__global__ __launch_bounds__(256, HT > 2 ? 1 : 2) void attn_rows(Args a) {
   constexpr int NC = (HT + 1) / 2, NL = 2 * NK > ND ? 2 * NK : ND;
   const int lane = threadIdx.x & 63, w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), n = lane & 15, q = lane >> 4;
   const int row = blockIdx.x / a.nsplit, sp = blockIdx.x - row * a.nsplit;
@@ -188,16 +178,20 @@ __global__ __launch_bounds__(256, 2) void attn_rows(Args a) {
   const long brow = a.rows ? a.rows[row] : row;
   __shared__ __attribute__((aligned(16))) float lo[4][HT * ND * 256];
   __shared__ float lm[4][HT * 16][2];
+  __shared__ __attribute__((aligned(16))) unsigned short lq[HT * NK * 512];  // the query in operand order
 
-  bf16x8 qf[HT][NK];
   float sc[HT][4];
   int grp[HT][4], gcol[HT];  // key head of this lane's S rows and of its mixed column
 #pragma unroll
   for (int t = 0; t < HT; ++t) {
     const int h = 16 * t + n;
-    const unsigned short* qp = (const unsigned short*)a.q + brow * a.ldq + (long)h * a.dkp + 8 * q;
+    if ((t & 3) == w || HT < 4) {
+      const unsigned short* qp = (const unsigned short*)a.q + brow * a.ldq + (long)h * a.dkp + 8 * q;
 #pragma unroll
-    for (int ks = 0; ks < NK; ++ks) qf[t][ks] = h < a.H ? *(const bf16x8*)(qp + 32 * ks) : bf16x8{};
+      for (int ks = 0; ks < NK; ++ks)
+        if (HT >= 4 || ((t * NK + ks) & 3) == w)
+          *(bf16x8*)(lq + (t * NK + ks) * 512 + 8 * lane) = h < a.H ? *(const bf16x8*)(qp + 32 * ks) : bf16x8{};
+    }
     gcol[t] = h < a.H ? h / a.R : -1;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
@@ -206,11 +200,11 @@ __global__ __launch_bounds__(256, 2) void attn_rows(Args a) {
       grp[t][r] = hr < a.H ? hr / a.R : -1;
     }
   }
-  bf16x8 tf[HT][NC];
+  f16x8 tf[HT][NC];
 #pragma unroll
   for (int t = 0; t < HT; ++t)
 #pragma unroll
-    for (int c = 0; c < NC; ++c) tf[t][c] = *(const bf16x8*)(a.talk + ((t * NC + c) * 64 + lane) * 8);
+    for (int c = 0; c < NC; ++c) tf[t][c] = *(const f16x8*)(a.talk + ((t * NC + c) * 64 + lane) * 8);
 
   f32x4 acc[HT][ND];
   float m[HT], l[HT], bfar[HT];
@@ -252,38 +246,40 @@ __global__ __launch_bounds__(256, 2) void attn_rows(Args a) {
 #pragma unroll
       for (int t = 0; t < HT; ++t) {
         if (16 * t > h1 || 16 * t + 15 < h0) continue;
+        bf16x8 qf[NK];
+#pragma unroll
+        for (int ks = 0; ks < NK; ++ks) qf[ks] = *(const bf16x8*)(lq + (t * NK + ks) * 512 + 8 * lane);
 #pragma unroll
         for (int kt = 0; kt < 2; ++kt) {
           f32x4 s{};
 #pragma unroll
-          for (int ks = 0; ks < NK; ++ks) s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[t][ks], f[kt * NK + ks], s, 0, 0, 0);
+          for (int ks = 0; ks < NK; ++ks) s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[ks], f[kt * NK + ks], s, 0, 0, 0);
 #pragma unroll
           for (int r = 0; r < 4; ++r) S[t][kt][r] = grp[t][r] == g ? s[r] : S[t][kt][r];
         }
       }
       if (g == a.G - 1) {  // every head's scores of the page are there: mix, softmax
         const int tok0 = (p0 + w + 4 * cpage) * PAGE;
-        bf16x8 part[NC][2][3];
+        f16x8 part[NC][2][2];
 #pragma unroll
         for (int c = 0; c < NC; ++c)
 #pragma unroll
           for (int kt = 0; kt < 2; ++kt) {
-            u32x4 x[3] = {};
+            u32x4 x[2] = {};
 #pragma unroll
             for (int hf = 0; hf < 2; ++hf) {
               const int t = 2 * c + hf;
               if (t >= HT) continue;
-              unsigned u[4][3];
 #pragma unroll
-              for (int r = 0; r < 4; ++r) split3(S[t][kt][r] * sc[t][r], u[r]);
-#pragma unroll
-              for (int j = 0; j < 3; ++j) {
-                x[j][2 * hf] = pack_hi(u[0][j], u[1][j]);
-                x[j][2 * hf + 1] = pack_hi(u[2][j], u[3][j]);
+              for (int r = 0; r < 2; ++r) {
+                unsigned hi, lo;
+                split2(S[t][kt][2 * r] * sc[t][2 * r], S[t][kt][2 * r + 1] * sc[t][2 * r + 1], hi, lo);
+                x[0][2 * hf + r] = hi;
+                x[1][2 * hf + r] = lo;
               }
             }
-#pragma unroll
-            for (int j = 0; j < 3; ++j) part[c][kt][j] = __builtin_bit_cast(bf16x8, x[j]);
+            part[c][kt][0] = __builtin_bit_cast(f16x8, x[0]);
+            part[c][kt][1] = __builtin_bit_cast(f16x8, x[1]);
           }
         const bool near = pos - (tok0 + PAGE - 1) < a.nfar, edge = tok0 + PAGE - 1 > pos;
 #pragma unroll
@@ -302,8 +298,8 @@ __global__ __launch_bounds__(256, 2) void attn_rows(Args a) {
 #pragma unroll
             for (int c = 0; c < NC; ++c)
 #pragma unroll
-              for (int j = 2; j >= 0; --j)
-                D[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(part[c][kt][j], tf[t][c], D[kt], 0, 0, 0);
+              for (int j = 1; j >= 0; --j)
+                D[kt] = __builtin_amdgcn_mfma_f32_16x16x32_f16(part[c][kt][j], tf[t][c], D[kt], 0, 0, 0);
             if (edge) {
 #pragma unroll
               for (int r = 0; r < 4; ++r)
@@ -352,6 +348,7 @@ __global__ __launch_bounds__(256, 2) void attn_rows(Args a) {
     bf16x8 fa[NL], fb[NL];
 #pragma unroll
     for (int t = 0; t < HT; ++t) S[t][0] = S[t][1] = f32x4{}, pf[t] = u32x4{};
+    __syncthreads();
     load(fa);
     for (int st = 0; st < nst; st += 2) {  // nst is even
       load(fb);
@@ -396,25 +393,38 @@ __global__ __launch_bounds__(256, 2) void attn_rows(Args a) {
   }
 }
 
-// splits of one (row, head): 64 threads, 2 or 1 dims each (dvp 128 or 64)
+// splits (at most 64) of one (row, head): 64 threads, 2 or 1 dims each (dvp 128 or 64)
 __global__ __launch_bounds__(64) void merge(Args a) {
-  const int row = blockIdx.x / a.H, h = blockIdx.x - row * a.H, e = a.dvp / 64, d = threadIdx.x * e;
+  const int row = blockIdx.x / a.H, h = blockIdx.x - row * a.H, e = a.dvp / 64, lane = threadIdx.x;
   const long pr = (long)row * a.nsplit * a.H + h;
-  float M = 0.f;
-  for (int s = 0; s < a.nsplit; ++s) M = fmaxf(M, a.pml[2 * (pr + (long)s * a.H)]);
-  float L = __builtin_amdgcn_exp2f(-M), o0 = 0.f, o1 = 0.f;
-  for (int s = 0; s < a.nsplit; ++s) {
-    const long p = pr + (long)s * a.H;
-    const float f = __builtin_amdgcn_exp2f(a.pml[2 * p] - M);
-    L += f * a.pml[2 * p + 1];
-    const float* x = a.po + p * a.dvp + d;
-    o0 += f * x[0];
-    if (e == 2) o1 += f * x[1];
-  }
   const long brow = a.rows ? a.rows[row] : row;
-  unsigned short* op = (unsigned short*)a.o + brow * a.ldo + (long)h * a.dvp + d;
-  op[0] = f2bf(o0 / L);
-  if (e == 2) op[1] = f2bf(o1 / L);
+  float m = 0.f, l = 0.f;
+  if (lane < a.nsplit) m = a.pml[2 * (pr + (long)lane * a.H)], l = a.pml[2 * (pr + (long)lane * a.H) + 1];
+  float M = m;
+#pragma unroll
+  for (int b = 1; b < 64; b <<= 1) M = fmaxf(M, __shfl_xor(M, b, 64));
+  const float f = __builtin_amdgcn_exp2f(m - M);
+  const float inv = 1.0f / (wave_sum(f * l) + __builtin_amdgcn_exp2f(-M));
+  const float* x = a.po + pr * a.dvp + lane * e;
+  const long step = (long)a.H * a.dvp;
+  float o0 = 0.f, o1 = 0.f;
+  for (int s0 = 0; s0 < a.nsplit; s0 += 8) {  // eight splits' loads at a time
+    float2 v[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const float* p = x + min(s0 + j, a.nsplit - 1) * step;
+      v[j] = e == 2 ? *(const float2*)p : make_float2(*p, 0.f);
+    }
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const float g = s0 + j < a.nsplit ? __shfl(f, s0 + j, 64) : 0.f;
+      o0 += g * v[j].x;
+      o1 += g * v[j].y;
+    }
+  }
+  unsigned short* op = (unsigned short*)a.o + brow * a.ldo + (long)h * a.dvp + lane * e;
+  op[0] = f2bf(o0 * inv);
+  if (e == 2) op[1] = f2bf(o1 * inv);
 }
 
 // ----------------------------------------------------------------------- tiles
@@ -942,7 +952,7 @@ KGS_EXPORT int kgs_talking_write(void* z, long ldz, const void* b, void* pages, 
   if (T <= 0 || nq <= 0 || G <= 0 || dkp <= 0 || dvp <= 0 || dkp % 32 || dvp % 16 || nq % 8 || ok < nq ||
       ldz < ok + G * dkp || ldz < ov + G * dvp || T > 8 * 65535)
     return KGS_ERR_SHAPE;
-  if (ldz % 8 || ok % 8 || ov % 8 || (((uintptr_t)z | (uintptr_t)pages) & 15)) return KGS_ERR_ALIGN;
+  if (ldz % 8 || ok % 8 || ov % 8 || (((uintptr_t)z | (uintptr_t)pages | (uintptr_t)b) & 15)) return KGS_ERR_ALIGN;
   WriteArgs a{z, ldz, (const float*)b, pages, (const int*)slots, T, nq, G, dkp, dvp, ok, ov};
   const dim3 grid(((nq + G * (dkp + dvp)) / 8 + 255) / 256, (T + 7) / 8);
   if (f32) hipLaunchKernelGGL(write_kv<float>, grid, dim3(256), 0, s, a);

@@ -75,7 +75,7 @@ def test_experts(T, E, top, W, ff, limit, dtype):
     W256 = (W + 255) // 256 * 256
     pad = lambda t, n, d: torch.nn.functional.pad(t, (0, W256 - W) if d == 1 else (0, 0, 0, W256 - W))  # noqa: E731
     h = pad(rnd(T, W, seed=T, dtype=dtype), W256, 1)
-    ep = next((s for s in (16, 32, 64, 128) if s >= E), (E + 15) // 16 * 16)
+    ep = next((s for s in (16, 32, 64) if s >= E), (E + 15) // 16 * 16)
     router = torch.zeros(ep, W256, dtype=dtype)
     router[:E] = pad(rnd(E, W, seed=2, scale=W ** -0.5, dtype=BF).to(dtype), W256, 1)
     gu = pad(rnd(E * 2 * ff, W, seed=3, scale=2 * W ** -0.5, dtype=BF).to(dtype), W256, 1).reshape(E, 2 * ff, W256)
