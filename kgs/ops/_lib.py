@@ -120,8 +120,8 @@ _SIGS = {
     "kgs_talking_write": ([_c_void_p, _c_long] + [_c_void_p] * 3 + [_c_int] * 8 + [_c_void_p], _c_int),
     "kgs_talking_rows": ([_c_void_p, _c_long, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_int] + [_c_void_p] * 8
                          + [_c_int] * 10 + [_c_void_p], _c_int),
-    "kgs_talking_tiles": ([_c_void_p, _c_long, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_int, _c_void_p, _c_int]
-                          + [_c_void_p] * 5 + [_c_int] * 6 + [_c_void_p], _c_int),
+    "kgs_talking_tiles": ([_c_void_p, _c_long, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_int, _c_void_p, _c_int,
+                           _c_void_p, _c_int] + [_c_void_p] * 7 + [_c_int] * 6 + [_c_void_p], _c_int),
     "kgs_moe_route": ([_c_void_p, _c_long] + [_c_void_p] * 6 + [_c_int] * 6 + [_c_void_p], _c_int),
     "kgs_moe_plan": ([_c_void_p] * 9 + [_c_int] * 4 + [_c_void_p], _c_int),
     "kgs_moe_grouped": ([_c_void_p, _c_long, _c_void_p, _c_void_p, _c_long] + [_c_void_p] * 4 + [_c_int] * 7

@@ -174,10 +174,37 @@ class QueryRows:
 
 @dataclass
 class QueryTiles:
-    """Blocks of up to ``Heads.tile`` consecutive queries: int32 ``[n, 4]`` (first batch row,
-    block-table row, position of the first, queries)."""
+    """Blocks of up to ``Heads.tile`` consecutive queries over a range of their pages
+    (:func:`tile_items`): int32 ``[n, 8]`` (first batch row, block-table row, position of
+    the first, queries, first page, end, partial result or -1, 0), and ``merges [m, 4]``
+    (first batch row, queries, first part, parts) of the blocks that are split."""
     items: torch.Tensor
     bt: torch.Tensor
+    merges: torch.Tensor | None = None
+    parts: int = 0
+
+
+MIN_PAGES = 16  # pages of a part
+MAX_PARTS = 64  # parts that one merge takes
+
+
+def tile_items(portions, tile: int) -> tuple[np.ndarray, np.ndarray]:
+    """Items and merges of ``portions`` (first batch row, block-table row, position,
+    tokens). Blocks with more than an even share of all pages are split, so that a long
+    prompt's last blocks do not outlast the rest; the longest first."""
+    b = np.array([(r + j, s, p + j, min(tile, n - j)) for r, s, p, n in portions for j in range(0, n, tile)], np.int64)
+    pages = (b[:, 2] + b[:, 3] - 1) // PAGE + 1
+    cap = max(MIN_PAGES, -(-int(pages.sum()) // CUS))
+    parts = np.minimum(-(-pages // cap), MAX_PARTS) if len(b) < 2 * CUS else np.ones_like(pages)
+    at = np.repeat(np.arange(len(b)), parts)
+    k = np.arange(len(at)) - np.repeat(np.cumsum(parts) - parts, parts)
+    first, end = pages[at] * k // parts[at], pages[at] * (k + 1) // parts[at]
+    split = parts > 1
+    part0 = np.cumsum(np.where(split, parts, 0)) - np.where(split, parts, 0)
+    part = np.where(split[at], part0[at] + k, -1)
+    items = np.concatenate([b[at], np.stack([first, end, part, np.zeros_like(k)], 1)], 1)
+    merges = np.stack([b[:, 0], b[:, 3], part0, parts], 1)[split]
+    return items[np.argsort(first - end, kind="stable")], merges
 
 
 def split_count(n: int, max_pages: int) -> int:
@@ -227,14 +254,19 @@ def attention_tiles(q: torch.Tensor, pages: torch.Tensor, w: TalkingWeights, t: 
     h = w.heads
     if not h.tiled:
         raise ValueError(f"{h} has no tiled kernel")
-    if t.items.dtype != torch.int32 or t.items.dim() != 2 or t.items.shape[1] != 4 or not t.items.is_contiguous():
-        raise ValueError("items must be contiguous int32 [n, 4]")
+    if t.items.dtype != torch.int32 or t.items.dim() != 2 or t.items.shape[1] != 8 or not t.items.is_contiguous():
+        raise ValueError("items must be contiguous int32 [n, 8]")
+    m, po, pml = 0 if t.merges is None else t.merges.shape[0], None, None
+    if m:
+        po = torch.empty((t.parts * h.tile, h.heads, h.dvp), dtype=torch.float32, device=q.device)
+        pml = torch.empty((t.parts * h.tile, h.heads, 2), dtype=torch.float32, device=q.device)
     n = t.items.shape[0]
     scratch = torch.empty((n, h.tile_bytes), dtype=torch.uint8, device=q.device)
     rc = _lib.lib().kgs_talking_tiles(_act(q, q.shape[0], h.heads * h.dkp, torch.bfloat16, "q"), q.stride(0),
                                       pages.data_ptr(), _act(out, out.shape[0], h.heads * h.dvp, torch.bfloat16, "out"),
                                       out.stride(0), t.bt.data_ptr(), t.bt.shape[1], t.items.data_ptr(),
-                                      n, scratch.data_ptr(), w.sc.data_ptr(), w.talk_slots.data_ptr(),
+                                      n, t.merges.data_ptr() if m else 0, m, po.data_ptr() if m else 0,
+                                      pml.data_ptr() if m else 0, scratch.data_ptr(), w.sc.data_ptr(), w.talk_slots.data_ptr(),
                                       w.bias_slots.data_ptr(), w.bias_far.data_ptr(), w.bias_slots.shape[1], w.nfar, h.heads, h.kv_heads,
                                       h.dkp, h.dvp, _lib.stream_handle(q.device))
     _lib.check(rc, f"talking_tiles[{n}x{h.heads}]")

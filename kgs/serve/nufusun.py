@@ -25,7 +25,7 @@ from kgs.ops.activation import softcap
 from kgs.ops.decode import PAGE
 from kgs.ops.residual import MAX_WIDTH, ExpertRows, residual_add, residual_embed
 from kgs.ops.talking import (HeadPages, Heads, QueryRows, QueryTiles, TalkingWeights, attention_rows,
-                             attention_tiles, heads_of, split_count, write_kv)
+                             attention_tiles, heads_of, split_count, tile_items, write_kv)
 
 from .ragged import DTYPES, Batch, HostPack, RaggedModel, Weights, _pad, pad64
 from .trace import TRACE as T
@@ -70,18 +70,19 @@ class Geometry:
                      "tok_pos": refs[9] if whole else pk.add(pos[at]),
                      "rows": None if whole else pk.add(at)}, len(at), split_count(len(at), pages))
         if tiled.any():
-            tile = self.heads.tile
-            items = [(row0[s] + q, s, pos0[s] + q, min(tile, n[s] - q))
-                     for s in np.flatnonzero(tiled) for q in range(0, int(n[s]), tile)]
-            items = np.array(items, np.int64)
-            tiles = pk.add(items[np.argsort(-(items[:, 2] + items[:, 3]), kind="stable")])  # longest context first
+            sel = np.flatnonzero(tiled)
+            items, merges = tile_items([(row0[s], s, pos0[s], n[s]) for s in sel], self.heads.tile)
+            tiles = (pk.add(items), pk.add(merges) if len(merges) else None, int(merges[:, 3].sum()))
 
         def build(get):
             r = None
             if rows is not None:
                 r = QueryRows(n=rows[1], bt=get(refs[7]), nsplit=rows[2],
                               **{k: None if v is None else get(v) for k, v in rows[0].items()})
-            return TalkingPlan(r, None if tiles is None else QueryTiles(get(tiles), get(refs[7])))
+            if tiles is None:
+                return TalkingPlan(r, None)
+            items, merges, parts = tiles
+            return TalkingPlan(r, QueryTiles(get(items), get(refs[7]), None if merges is None else get(merges), parts))
 
         return build
 

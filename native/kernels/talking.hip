@@ -152,7 +152,10 @@ struct Args {
   const int* tok_seq;  // per query: its block-table row and its position
   const int* tok_pos;
   const int* rows;     // its batch row, or null: the same
-  const int4* items;   // tiles: (first batch row, block-table row, position, queries)
+  const int4* items;   // tiles, two each: (first batch row, block-table row, position, queries),
+                       // (first page, end, partial result or -1, 0)
+  const int4* merges;  // split tiles
+  int tile;            // queries of a tile
   void* qs;            // tiles: the queries of a workgroup again, in operand order
   float* po;           // partial results of split rows: [row, split][heads][dvp]
   float* pml;          // [row, split][heads][2]
@@ -393,31 +396,43 @@ __global__ __launch_bounds__(256, HT > 2 ? 1 : 2) void attn_rows(Args a) {
   }
 }
 
-// splits (at most 64) of one (row, head): 64 threads, 2 or 1 dims each (dvp 128 or 64)
+// splits (at most 64) of one (row, head): 64 threads, 2 or 1 dims each (dvp 128 or 64).
+// TILES: rows are the queries of split tiles, merges = (first batch row, queries, first
+// part, parts) of a tile; a part holds `tile` rows.
+template <bool TILES>
 __global__ __launch_bounds__(64) void merge(Args a) {
   const int row = blockIdx.x / a.H, h = blockIdx.x - row * a.H, e = a.dvp / 64, lane = threadIdx.x;
-  const long pr = (long)row * a.nsplit * a.H + h;
-  const long brow = a.rows ? a.rows[row] : row;
+  long pr = (long)row * a.nsplit * a.H + h, brow, between = a.H;
+  int nsplit = a.nsplit;
+  if constexpr (TILES) {
+    const int4 mt = a.merges[row / a.tile];
+    const int q = row % a.tile;
+    if (q >= mt.y) return;
+    brow = mt.x + q;
+    pr = ((long)mt.z * a.tile + q) * a.H + h;
+    between = (long)a.tile * a.H;
+    nsplit = mt.w;
+  } else brow = a.rows ? a.rows[row] : row;
   float m = 0.f, l = 0.f;
-  if (lane < a.nsplit) m = a.pml[2 * (pr + (long)lane * a.H)], l = a.pml[2 * (pr + (long)lane * a.H) + 1];
+  if (lane < nsplit) m = a.pml[2 * (pr + lane * between)], l = a.pml[2 * (pr + lane * between) + 1];
   float M = m;
 #pragma unroll
   for (int b = 1; b < 64; b <<= 1) M = fmaxf(M, __shfl_xor(M, b, 64));
   const float f = __builtin_amdgcn_exp2f(m - M);
   const float inv = 1.0f / (wave_sum(f * l) + __builtin_amdgcn_exp2f(-M));
   const float* x = a.po + pr * a.dvp + lane * e;
-  const long step = (long)a.H * a.dvp;
+  const long step = between * a.dvp;
   float o0 = 0.f, o1 = 0.f;
-  for (int s0 = 0; s0 < a.nsplit; s0 += 8) {  // eight splits' loads at a time
+  for (int s0 = 0; s0 < nsplit; s0 += 8) {  // eight splits' loads at a time
     float2 v[8];
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
-      const float* p = x + min(s0 + j, a.nsplit - 1) * step;
+      const float* p = x + min(s0 + j, nsplit - 1) * step;
       v[j] = e == 2 ? *(const float2*)p : make_float2(*p, 0.f);
     }
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
-      const float g = s0 + j < a.nsplit ? __shfl(f, s0 + j, 64) : 0.f;
+      const float g = s0 + j < nsplit ? __shfl(f, s0 + j, 64) : 0.f;
       o0 += g * v[j].x;
       o1 += g * v[j].y;
     }
@@ -493,10 +508,10 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
   unsigned vl = (unsigned)(uintptr_t)(KGS_LDS char*)vs + 16 * lane;
   asm volatile("" : "+v"(vl));
   char* const ps = vs + NS * ND * 1024 + w * RT * 1024;  // this wave's P: [qt][slot][16 rows][32 keys]
-  const int4 it = a.items[blockIdx.x];
+  const int4 it = a.items[2 * blockIdx.x], part = a.items[2 * blockIdx.x + 1];  // part: first page, end, result (-1: whole)
   const int qpg = (a.R + 3) / 4, nslot = a.G * qpg;
   const int* bt = a.bt + (long)it.y * a.W;
-  const int npage = (it.z + it.w - 1) / PAGE + 1;
+  const int pend = part.y;
   constexpr int DK = 32 * NK, DV = 16 * ND, HPAGE = PAGE * (DK + DV) * 2;  // bytes of one head's page
   const int posw = it.z + 4 * QT * w;                   // position of the wave's first query
 
@@ -547,7 +562,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
   };
   constexpr int CK = NS * 2 * NK / 4, CV = NS * ND / 4;  // chunks per wave of K and of V
   constexpr int KPER = 2 * NK, VPER = ND;
-  auto page_id = [&](int pg) { return bt[min(pg, npage - 1)]; };
+  auto page_id = [&](int pg) { return bt[min(pg, pend - 1)]; };
 
   // the far bias less the running maximum of (query, slot 4t + q, head): the mixture's addend
   f32x4 cm[4 * QT][MT];
@@ -568,11 +583,11 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
 #pragma unroll
     for (int k = 0; k < NK; ++k) *(bf16x8*)(qs + (i * NK + k) * 1024 + 16 * lane) = qf[i % RQ][k];
   }
-  int page = __builtin_amdgcn_readfirstlane(page_id(0));
+  int page = __builtin_amdgcn_readfirstlane(page_id(part.x));
 #pragma unroll
   for (int c = 0; c < CK; ++c) dma(page, ks, KPER, 0, c);
   bar<0>();
-  for (int pg = 0; pg < npage; ++pg) {
+  for (int pg = part.x; pg < pend; ++pg) {
     const int tok0 = pg * PAGE;
     const int next = page_id(pg + 1);
     // ---- scores
@@ -653,16 +668,22 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
         // lane: query i, key 2n + kt, slot 4t + q, head r; above the running maximum
         const int dist = posw + 4 * qt - (tok0 + 2 * n + kt);  // of query 0
         if (near) {
+          // all loads, then all sums: waited for here, not where far pages pass too
+          f32x4 b[4][MT];
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
-            const float* bp = a.bias + (long)min(max(dist + i, 0), a.nfar) * a.ldb + 4 * q;
+            const unsigned at = min(max(dist + i, 0), a.nfar) * a.ldb + 4 * q;
 #pragma unroll
-            for (int t = 0; t < MT; ++t) D[i][t] += *(const f32x4*)(bp + 16 * t);
+            for (int t = 0; t < MT; ++t) b[i][t] = *(const f32x4*)(a.bias + (at + 16 * t));
           }
+          fence();
 #pragma unroll
           for (int i = 0; i < 4; ++i)
 #pragma unroll
-            for (int t = 0; t < MT; ++t) asm volatile("" : "+v"(D[i][t]));  // waited for here, not where far pages pass too
+            for (int t = 0; t < MT; ++t) {
+              D[i][t] += b[i][t];
+              asm volatile("" : "+v"(D[i][t]));
+            }
         }
         if (edge) {
 #pragma unroll
@@ -818,18 +839,29 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     static_for<0, QT>([&](auto tc) {
       constexpr int s = decltype(sc_)::value, t = decltype(tc)::value, rt = s * QT + t;
       const int hr = 4 * (s % qpg) + (n & 3), qi = 4 * (QT * w + t) + (n >> 2);
-      const float L = xor32_sum(xor16_sum(l[rt])) + __builtin_amdgcn_exp2f(-mm[(t * NS + s) * 16 + n]);
+      const float m = mm[(t * NS + s) * 16 + n], L = xor32_sum(xor16_sum(l[rt]));
       const bool ok = s < nslot && hr < a.R && qi < it.w;
-      const float inv = 1.0f / L;
-      unsigned short* op = (unsigned short*)a.o + (long)(it.x + qi) * a.ldo + (long)(s / qpg * a.R + hr) * DV + 4 * q;
-      static_for<0, ND>([&](auto dc) {
-        constexpr int d = decltype(dc)::value;
-        const f32x4 o = accr::read<rt * ND + d>() * inv;
-        uint2 pk;
-        pk.x = pack_bf16x2(o[0], o[1]);
-        pk.y = pack_bf16x2(o[2], o[3]);
-        if (ok) *(uint2*)(op + 16 * d) = pk;
-      });
+      const int h = s / qpg * a.R + hr;
+      if (part.z < 0) {
+        const float inv = 1.0f / (L + __builtin_amdgcn_exp2f(-m));
+        unsigned short* op = (unsigned short*)a.o + (long)(it.x + qi) * a.ldo + (long)h * DV + 4 * q;
+        static_for<0, ND>([&](auto dc) {
+          constexpr int d = decltype(dc)::value;
+          const f32x4 o = accr::read<rt * ND + d>() * inv;
+          uint2 pk;
+          pk.x = pack_bf16x2(o[0], o[1]);
+          pk.y = pack_bf16x2(o[2], o[3]);
+          if (ok) *(uint2*)(op + 16 * d) = pk;
+        });
+      } else {
+        const long pr = ((long)part.z * (16 * QT) + qi) * a.H + h;
+        static_for<0, ND>([&](auto dc) {
+          constexpr int d = decltype(dc)::value;
+          const f32x4 o = accr::read<rt * ND + d>();
+          if (ok) *(f32x4*)(a.po + pr * DV + 16 * d + 4 * q) = o;
+        });
+        if (ok && q == 0) a.pml[2 * pr] = m, a.pml[2 * pr + 1] = L;
+      }
     });
   });
 }
@@ -915,7 +947,7 @@ __global__ __launch_bounds__(256) void attn_plain(Args a) {
 template <int HT, int NK, int ND>
 void run_rows(const Args& a, int nrows, hipStream_t s) {
   hipLaunchKernelGGL((attn_rows<HT, NK, ND>), dim3((unsigned)(nrows * a.nsplit)), dim3(256), 0, s, a);
-  if (a.nsplit > 1) hipLaunchKernelGGL(merge, dim3((unsigned)(nrows * a.H)), dim3(64), 0, s, a);
+  if (a.nsplit > 1) hipLaunchKernelGGL(merge<false>, dim3((unsigned)(nrows * a.H)), dim3(64), 0, s, a);
 }
 template <int NK, int ND>
 void rows_ht(const Args& a, int nrows, hipStream_t s) {
@@ -968,7 +1000,7 @@ KGS_EXPORT int kgs_talking_rows(const void* q, long ldq, const void* pages, void
                                 int G, int dkp, int dvp, int nsplit, int plain, int f32, hipStream_t s) {
   using namespace kgs::talking;
   Args a{q, ldq, pages, o, ldo, (const int*)bt, W, (const int*)tok_seq, (const int*)tok_pos, (const int*)rows, nullptr,
-         nullptr, (float*)po, (float*)pml, (const float*)sc, (const unsigned short*)talk, (const float*)talk, (const float*)bias,
+         nullptr, 0, nullptr, (float*)po, (float*)pml, (const float*)sc, (const unsigned short*)talk, (const float*)talk, (const float*)bias,
          nullptr, ldb, nfar, H, G, G ? H / G : 0, dkp, dvp, nsplit};
   if (int rc = check(a, nrows)) return rc;
   if (plain || f32) {
@@ -991,25 +1023,31 @@ KGS_EXPORT int kgs_talking_rows(const void* q, long ldq, const void* pages, void
   return (int)hipGetLastError();
 }
 
-// Prompt portions: nitems blocks of consecutive queries (first batch row, block-table
-// row, first position, queries: up to 32, 16 above 4 slots). bf16, dkp and dvp 64 or 128, at most 8 slots
-// of 4 heads (G ceil(H / G / 4)); talk (fp16) and biases in slot order, ldb = 16 ceil(slots / 4);
-// bias is the table less its last row, bfar. qs: scratch, slots (2, 4 or 8) x 4 KB x dkp / 32
-// per item, twice that up to 4 slots.
+// Prompt portions: nitems blocks of consecutive queries over a range of their pages, two
+// int4 each (Args::items): up to 32 queries, 16 above 4 slots. A block split over its pages
+// leaves partial results (po, pml: one part holds 32 or 16 rows of all heads) that
+// `merges` names. bf16, dkp and dvp 64 or 128, at most 8 slots of 4 heads
+// (G ceil(H / G / 4)); talk (fp16) and biases in slot order, ldb = 16 ceil(slots / 4); bias is
+// the table less its last row, bfar. qs: scratch, slots (2, 4 or 8) x 4 KB x dkp / 32 per
+// item, twice that up to 4 slots.
 KGS_EXPORT int kgs_talking_tiles(const void* q, long ldq, const void* pages, void* o, long ldo, const void* bt, int W,
-                                 const void* items, int nitems, void* qs, const void* sc, const void* talk, const void* bias,
+                                 const void* items, int nitems, const void* merges,
+                                 int nmerge, void* po, void* pml, void* qs, const void* sc, const void* talk, const void* bias,
                                  const void* bfar, int ldb, int nfar, int H, int G, int dkp, int dvp, hipStream_t s) {
   using namespace kgs::talking;
   Args a{};
   a.q = q, a.ldq = ldq, a.pages = pages, a.o = o, a.ldo = ldo, a.bt = (const int*)bt, a.W = W;
-  a.items = (const int4*)items, a.qs = qs, a.sc = (const float*)sc, a.talk = (const unsigned short*)talk;
+  a.items = (const int4*)items, a.merges = (const int4*)merges, a.po = (float*)po, a.pml = (float*)pml, a.qs = qs, a.sc = (const float*)sc, a.talk = (const unsigned short*)talk;
   a.bias = (const float*)bias, a.bfar = (const float*)bfar, a.ldb = ldb, a.nfar = nfar, a.H = H, a.G = G, a.R = G ? H / G : 0;
   a.dkp = dkp, a.dvp = dvp, a.nsplit = 1;
   if (int rc = check(a, nitems)) return rc;
   const int nslot = G * ((H / G + 3) / 4);
   if (nslot > 8 || (dkp != 64 && dkp != 128) || (dvp != 64 && dvp != 128)) return KGS_ERR_ARG;
   if (ldb < (nslot + 3) / 4 * 16 || (((uintptr_t)items | (uintptr_t)bfar | (uintptr_t)talk | (uintptr_t)qs) & 15)) return KGS_ERR_SHAPE;
+  a.tile = nslot <= 4 ? 32 : 16;
+  if (nmerge < 0 || (nmerge && (!merges || !po || !pml)) || (long)nmerge * a.tile * H > 0x7fffffff) return KGS_ERR_SHAPE;
   if (dkp == 64) dvp == 64 ? tiles_ns<2, 4>(a, nitems, nslot, s) : tiles_ns<2, 8>(a, nitems, nslot, s);
   else dvp == 64 ? tiles_ns<4, 4>(a, nitems, nslot, s) : tiles_ns<4, 8>(a, nitems, nslot, s);
+  if (nmerge) hipLaunchKernelGGL(merge<true>, dim3((unsigned)(nmerge * a.tile * H)), dim3(64), 0, s, a);
   return (int)hipGetLastError();
 }

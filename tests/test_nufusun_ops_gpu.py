@@ -208,14 +208,15 @@ class Case:
                       i32([base[s] + p for s, p in sel]), nsplit)
         return self.view(attention_rows(self.z, self.pages, self.w, r, self.out()))
 
-    def tiles(self, portions):
+    def tiles(self, portions, split=False):
         """``portions``: (sequence, first position, tokens)."""
-        from kgs.ops.talking import QueryTiles, attention_tiles
+        from kgs.ops.talking import QueryTiles, attention_tiles, tile_items
 
         base = np.cumsum([0] + self.lens)
-        step = self.h.tile
-        items = [(base[s] + p + j, s, p + j, min(step, n - j)) for s, p, n in portions for j in range(0, n, step)]
-        t = QueryTiles(torch.tensor(items, dtype=torch.int32).cuda(), torch.tensor(self.bt).cuda())
+        items, merges = tile_items([(base[s] + p, s, p, n) for s, p, n in portions], self.h.tile)
+        assert split == bool(len(merges))
+        i32 = lambda a: torch.tensor(a, dtype=torch.int32).cuda()  # noqa: E731
+        t = QueryTiles(i32(items), i32(self.bt), i32(merges) if split else None, int(merges[:, 3].sum()))
         return self.view(attention_tiles(self.z, self.pages, self.w, t, self.out()))
 
     def check(self, got, sel, what):
@@ -260,6 +261,16 @@ def test_scores_that_stand_out(shape, dtype):
     if c.h.tiled:
         c.check(c.tiles([(0, 0, 301)]), [(0, p) for p in range(301)], "tiles")
         c.check(c.tiles([(0, 110, 191)]), [(0, p) for p in range(110, 301)], "tiles")
+
+
+@pytest.mark.parametrize("shape", [(6, 2, 64, 48), (20, 4, 100, 50), (16, 4, 128, 128)], ids=str)
+def test_split_tiles(shape):
+    """Portions over many pages: blocks split over their pages and merged, beside whole ones."""
+    sharp = [(700, 3, 2.0), (690, 512, 2.0), (650, 300, 3.0), (700, 699, 1.0)]
+    c = Case(shape, [701, 40], BF, sharp=sharp)
+    got = c.tiles([(0, 600, 101), (1, 0, 40)], split=True)
+    c.check(got, [(0, p) for p in range(600, 701)] + [(1, p) for p in range(40)], "split tiles")
+    assert torch.isnan(got[:600]).all()
 
 
 @pytest.mark.parametrize("rows,far", [(16, 50.0), (32, 240.0), (2, 7.0), (64, 150.5)])
