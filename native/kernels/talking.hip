@@ -591,7 +591,26 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     const int tok0 = pg * PAGE;
     const int next = page_id(pg + 1);
     // ---- scores
-    f32x4 S[RT][2];
+    // A slot's scores become their fp16 parts while the next slot's MFMAs run.
+    unsigned x[QT][2][2][MT][2][4];  // [block][key half][part][half of the slots][head pair][slot of it, then query]
+    f32x4 S[2][QT][2];
+    auto split_slot = [&](int s, int u0, int u1) {  // units u0 .. u1 - 1 of 4 QT: (block, key half, head pair)
+#pragma unroll
+      for (int u = 0; u < 4 * QT; ++u) {
+        if (u < u0 || u >= u1) continue;
+        const int t = u >> 2, kt = u >> 1 & 1, c = u & 1;
+        const f32x4& v = S[s & 1][t][kt];
+        unsigned &hi = x[t][kt][0][s >> 2][c][s & 3], &lo = x[t][kt][1][s >> 2][c][s & 3];
+        split2(v[2 * c] * sc[s][2 * c], v[2 * c + 1] * sc[s][2 * c + 1], hi, lo);
+        asm volatile("" : "+v"(hi), "+v"(lo));  // here, not where they are used
+      }
+    };
+    if constexpr (NS < 4) {
+#pragma unroll
+      for (int i = 0; i < QT * 8; ++i)
+#pragma unroll
+        for (int s = NS; s < 4; ++s) x[i >> 3][i >> 2 & 1][i >> 1 & 1][0][i & 1][s] = 0;
+    }
     // K fragments of both 16-key halves, one 32-dim step at a time, PF steps ahead
     constexpr int PF = 5, STEPS = NS * NK;
     bf16x8 kf[PF + 1][2];
@@ -609,11 +628,13 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
 #pragma unroll
       for (int t = 0; t < QT; ++t) {
         const int rt = (p / NK) * QT + t;
-        if (p % NK == 0) S[rt][0] = S[rt][1] = f32x4{};
+        f32x4(&c)[2] = S[(p / NK) & 1][t];
+        if (p % NK == 0) c[0] = c[1] = f32x4{};
 #pragma unroll
         for (int kt = 0; kt < 2; ++kt)
-          S[rt][kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[rt % RQ][p % NK], kf[p % (PF + 1)][kt], S[rt][kt], 0, 0, 0);
+          c[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[rt % RQ][p % NK], kf[p % (PF + 1)][kt], c[kt], 0, 0, 0);
       }
+      if (p >= NK) split_slot(p / NK - 1, p % NK * 4 * QT / NK, (p % NK + 1) * 4 * QT / NK);
       if (p % NK == NK - 1) {
         fence();
 #pragma unroll
@@ -625,6 +646,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
         if (c * STEPS / (CV / 2) == p) dma(page, vs, VPER, PAGE * DK * 2, c);
       fence();
     }
+    split_slot(NS - 1, 0, 4 * QT);
     bar<63>();  // K of this page is done with everywhere
     const int pnext = __builtin_amdgcn_readfirstlane(next);
 
@@ -639,27 +661,17 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
       unsigned p0[4][MT][2];  // keys 2n, heads (0, 1) and (2, 3)
 #pragma unroll
       for (int kt = 0; kt < 2; ++kt) {
-        unsigned x[2][MT][2][4];  // [part][half][head pair][slot of the half, then query]
-#pragma unroll
-        for (int s = 0; s < 4 * MT; ++s)
-#pragma unroll
-          for (int c = 0; c < 2; ++c) {
-            if (s < NS) {
-              const int s_ = s < NS ? s : 0;
-              const f32x4& v = S[s_ * QT + qt][kt];
-              split2(v[2 * c] * sc[s_][2 * c], v[2 * c + 1] * sc[s_][2 * c + 1], x[0][s >> 2][c][s & 3], x[1][s >> 2][c][s & 3]);
-            } else x[0][s >> 2][c][s & 3] = x[1][s >> 2][c][s & 3] = 0;
-          }
 #pragma unroll
         for (int j = 0; j < 2; ++j)
 #pragma unroll
-          for (int hf = 0; hf < MT; ++hf) transpose4(x[j][hf][0]), transpose4(x[j][hf][1]);
+          for (int hf = 0; hf < MT; ++hf) transpose4(x[qt][kt][j][hf][0]), transpose4(x[qt][kt][j][hf][1]);
         f32x4 D[4][MT];
 #pragma unroll
         for (int j = 1; j >= 0; --j)
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
-            const u32x4 b = {x[j][0][0][i], x[j][0][1][i], MT > 1 ? x[j][MT - 1][0][i] : 0u, MT > 1 ? x[j][MT - 1][1][i] : 0u};
+            const unsigned(&y)[MT][2][4] = x[qt][kt][j];
+            const u32x4 b = {y[0][0][i], y[0][1][i], MT > 1 ? y[MT - 1][0][i] : 0u, MT > 1 ? y[MT - 1][1][i] : 0u};
 #pragma unroll
             for (int t = 0; t < MT; ++t)
               D[i][t] = __builtin_amdgcn_mfma_f32_16x16x32_f16(tf[t], __builtin_bit_cast(f16x8, b),
