@@ -38,6 +38,7 @@ namespace kgs {
 namespace talking {
 
 constexpr int PAGE = 32;
+constexpr int TILE = 16;  // queries of a tile
 constexpr float NEG = -1.0e30f;
 constexpr float RESCALE = 8.0f;  // log2 units a score may exceed the running maximum by
 
@@ -496,9 +497,11 @@ __device__ __forceinline__ void bar() {
 // (acc_regs.h, accumulator (s QT + qt) ND + d): they take half the register file, and the compiler would
 // move them about. Rescales are collected over the page and applied before P V.
 template <int NS, int QT, int NK, int ND>
-__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) void attn_tiles(Args a) {
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(NS * QT > 4 ? 1 : 2, NS * QT > 4 ? 1 : 2)))
+void attn_tiles(Args a) {
   constexpr int MT = (NS + 3) / 4, RT = NS * QT;
-  constexpr int RQ = RT * NK <= 16 ? RT : 16 / NK;  // Q row tiles in registers
+  constexpr bool TWO = RT <= 4;  // two waves per SIMD: half the registers
+  constexpr int RQ = TWO ? 1 : RT * NK <= 16 ? RT : 16 / NK;  // Q row tiles in registers
   static_assert(RT * ND <= 64, "outputs exceed the AGPRs");
   __shared__ __attribute__((aligned(1024))) char smem[(NS * (2 * NK + ND) + 4 * RT) * 1024];
   char* const ks = smem;
@@ -573,7 +576,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     for (int t = 0; t < MT; ++t) cm[i][t] = *(const f32x4*)(a.bfar + 16 * t + 4 * q);
 #pragma unroll
   for (int i = 0; i < RT; ++i) l[i] = 0.f;
-  KGS_ACC_RESERVE();
+  if constexpr (TWO) KGS_ACC_RESERVE_HALF();
+  else KGS_ACC_RESERVE();
   static_for<0, RT * ND>([](auto i) { accr::zero<decltype(i)::value>(); });
 
   bf16x8 qf[RQ][NK];
@@ -612,7 +616,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
         for (int s = NS; s < 4; ++s) x[i >> 3][i >> 2 & 1][i >> 1 & 1][0][i & 1][s] = 0;
     }
     // K fragments of both 16-key halves, one 32-dim step at a time, PF steps ahead
-    constexpr int PF = 5, STEPS = NS * NK;
+    constexpr int PF = TWO ? 1 : 5, STEPS = NS * NK;
     bf16x8 kf[PF + 1][2];
     auto read_k = [&](int p) {
       const char* kp = ks + (p / NK * 2 * NK + p % NK) * 1024 + 16 * lane;
@@ -794,12 +798,13 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     // ---- P V
 #pragma unroll
     for (int i = 0; i < RQ; ++i) load_q(qf[i], i);  // for the next page
-    bf16x8 vf[2][ND];
+    constexpr int VB = TWO ? 1 : 2;  // slots' V in registers
+    bf16x8 vf[VB][ND];
     auto read_v = [&](bf16x8 (&f)[ND], int s) {
 #pragma unroll
       for (int i = 0; i < ND; ++i) f[i] = *(const KGS_LDS bf16x8*)(uintptr_t)(vl + (s * ND + i) * 1024);
     };
-    u32x4 pw[2][QT];
+    u32x4 pw[VB][QT];
     auto read_p = [&](u32x4 (&f)[QT], int s) {
 #pragma unroll
       for (int t = 0; t < QT; ++t)
@@ -810,7 +815,10 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     fence();
     static_for<0, NS>([&](auto sc_) {
       constexpr int s = decltype(sc_)::value;
-      if constexpr (s + 1 < NS) {
+      if constexpr (TWO && s > 0) {
+        read_p(pw[0], s);
+        read_v(vf[0], s);
+      } else if constexpr (!TWO && s + 1 < NS) {
         read_p(pw[(s + 1) & 1], s + 1);
         read_v(vf[(s + 1) & 1], s + 1);
       }
@@ -820,11 +828,11 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
         if ((c - CK / 2) * NS / 2 / (CK - CK / 2) == s) dma(pnext, ks, KPER, 0, c);
       static_for<0, QT>([&](auto tc) {
         constexpr int t = decltype(tc)::value, rt = s * QT + t;
-        const u32x4 pv = pw[s & 1][t];
+        const u32x4 pv = pw[s % VB][t];
         const bf16x8 pb = __builtin_bit_cast(bf16x8, pv);
         static_for<0, ND>([&](auto dc) {
           constexpr int d = decltype(dc)::value;
-          accr::mfma<rt * ND + d>(vf[s & 1][d], pb);
+          accr::mfma<rt * ND + d>(vf[s % VB][d], pb);
         });
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
@@ -970,8 +978,8 @@ void rows_ht(const Args& a, int nrows, hipStream_t s) {
 template <int NK, int ND>
 void tiles_ns(const Args& a, int nitems, int nslot, hipStream_t s) {
   const dim3 grid((unsigned)nitems), block(256);
-  if (nslot <= 2) hipLaunchKernelGGL((attn_tiles<2, 2, NK, ND>), grid, block, 0, s, a);
-  else if (nslot <= 4) hipLaunchKernelGGL((attn_tiles<4, 2, NK, ND>), grid, block, 0, s, a);
+  if (nslot <= 2) hipLaunchKernelGGL((attn_tiles<2, 1, NK, ND>), grid, block, 0, s, a);
+  else if (nslot <= 4) hipLaunchKernelGGL((attn_tiles<4, 1, NK, ND>), grid, block, 0, s, a);
   else hipLaunchKernelGGL((attn_tiles<8, 1, NK, ND>), grid, block, 0, s, a);
 }
 
@@ -1036,12 +1044,12 @@ KGS_EXPORT int kgs_talking_rows(const void* q, long ldq, const void* pages, void
 }
 
 // Prompt portions: nitems blocks of consecutive queries over a range of their pages, two
-// int4 each (Args::items): up to 32 queries, 16 above 4 slots. A block split over its pages
-// leaves partial results (po, pml: one part holds 32 or 16 rows of all heads) that
+// int4 each (Args::items): up to 16 queries. A block split over its pages
+// leaves partial results (po, pml: one part holds 16 rows of all heads) that
 // `merges` names. bf16, dkp and dvp 64 or 128, at most 8 slots of 4 heads
 // (G ceil(H / G / 4)); talk (fp16) and biases in slot order, ldb = 16 ceil(slots / 4); bias is
 // the table less its last row, bfar. qs: scratch, slots (2, 4 or 8) x 4 KB x dkp / 32 per
-// item, twice that up to 4 slots.
+// item.
 KGS_EXPORT int kgs_talking_tiles(const void* q, long ldq, const void* pages, void* o, long ldo, const void* bt, int W,
                                  const void* items, int nitems, const void* merges,
                                  int nmerge, void* po, void* pml, void* qs, const void* sc, const void* talk, const void* bias,
@@ -1056,7 +1064,7 @@ KGS_EXPORT int kgs_talking_tiles(const void* q, long ldq, const void* pages, voi
   const int nslot = G * ((H / G + 3) / 4);
   if (nslot > 8 || (dkp != 64 && dkp != 128) || (dvp != 64 && dvp != 128)) return KGS_ERR_ARG;
   if (ldb < (nslot + 3) / 4 * 16 || (((uintptr_t)items | (uintptr_t)bfar | (uintptr_t)talk | (uintptr_t)qs) & 15)) return KGS_ERR_SHAPE;
-  a.tile = nslot <= 4 ? 32 : 16;
+  a.tile = TILE;
   if (nmerge < 0 || (nmerge && (!merges || !po || !pml)) || (long)nmerge * a.tile * H > 0x7fffffff) return KGS_ERR_SHAPE;
   if (dkp == 64) dvp == 64 ? tiles_ns<2, 4>(a, nitems, nslot, s) : tiles_ns<2, 8>(a, nitems, nslot, s);
   else dvp == 64 ? tiles_ns<4, 4>(a, nitems, nslot, s) : tiles_ns<4, 8>(a, nitems, nslot, s);

@@ -213,7 +213,7 @@ class Case:
         from kgs.ops.talking import QueryTiles, attention_tiles, tile_items
 
         base = np.cumsum([0] + self.lens)
-        items, merges = tile_items([(base[s] + p, s, p, n) for s, p, n in portions], self.h.tile)
+        items, merges = tile_items([(base[s] + p, s, p, n) for s, p, n in portions], self.h.tiles_at_once)
         assert split == bool(len(merges))
         i32 = lambda a: torch.tensor(a, dtype=torch.int32).cuda()  # noqa: E731
         t = QueryTiles(i32(items), i32(self.bt), i32(merges) if split else None, int(merges[:, 3].sum()))
