@@ -501,7 +501,10 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(NS * QT > 4
 void attn_tiles(Args a) {
   constexpr int MT = (NS + 3) / 4, RT = NS * QT;
   constexpr bool TWO = RT <= 4;  // two waves per SIMD: half the registers
-  constexpr int RQ = TWO ? 1 : RT * NK <= 16 ? RT : 16 / NK;  // Q row tiles in registers
+  // Q row tiles in registers: the first RES for good, the others through a ring of RB
+  constexpr int RQ = TWO ? 1 : RT * NK <= 16 ? RT : 16 / NK;
+  constexpr int RES = TWO || NK == 2 ? 0 : 1, RB = RQ - RES;
+  auto ring = [](int rt) { return rt < RES ? rt : RES + (rt - RES) % (RB ? RB : 1); };
   static_assert(RT * ND <= 64, "outputs exceed the AGPRs");
   __shared__ __attribute__((aligned(1024))) char smem[(NS * (2 * NK + ND) + 4 * RT) * 1024];
   char* const ks = smem;
@@ -583,9 +586,9 @@ void attn_tiles(Args a) {
   bf16x8 qf[RQ][NK];
 #pragma unroll
   for (int i = RT - 1; i >= 0; --i) {
-    first_q(qf[i % RQ], i);
+    first_q(qf[ring(i)], i);
 #pragma unroll
-    for (int k = 0; k < NK; ++k) *(bf16x8*)(qs + (i * NK + k) * 1024 + 16 * lane) = qf[i % RQ][k];
+    for (int k = 0; k < NK; ++k) *(bf16x8*)(qs + (i * NK + k) * 1024 + 16 * lane) = qf[ring(i)][k];
   }
   int page = __builtin_amdgcn_readfirstlane(page_id(part.x));
 #pragma unroll
@@ -616,7 +619,7 @@ void attn_tiles(Args a) {
         for (int s = NS; s < 4; ++s) x[i >> 3][i >> 2 & 1][i >> 1 & 1][0][i & 1][s] = 0;
     }
     // K fragments of both 16-key halves, one 32-dim step at a time, PF steps ahead
-    constexpr int PF = TWO ? 1 : 5, STEPS = NS * NK;
+    constexpr int PF = TWO ? 1 : 3, STEPS = NS * NK;
     bf16x8 kf[PF + 1][2];
     auto read_k = [&](int p) {
       const char* kp = ks + (p / NK * 2 * NK + p % NK) * 1024 + 16 * lane;
@@ -636,14 +639,16 @@ void attn_tiles(Args a) {
         if (p % NK == 0) c[0] = c[1] = f32x4{};
 #pragma unroll
         for (int kt = 0; kt < 2; ++kt)
-          c[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[rt % RQ][p % NK], kf[p % (PF + 1)][kt], c[kt], 0, 0, 0);
+          c[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[ring(rt)][p % NK], kf[p % (PF + 1)][kt], c[kt], 0, 0, 0);
       }
       if (p >= NK) split_slot(p / NK - 1, p % NK * 4 * QT / NK, (p % NK + 1) * 4 * QT / NK);
       if (p % NK == NK - 1) {
         fence();
 #pragma unroll
-        for (int t = 0; t < QT; ++t)
-          if ((p / NK) * QT + t + RQ < RT) load_q(qf[((p / NK) * QT + t) % RQ], (p / NK) * QT + t + RQ);
+        for (int t = 0; t < QT; ++t) {
+          const int rt = (p / NK) * QT + t;
+          if (rt >= RES && rt + RB < RT) load_q(qf[ring(rt)], rt + RB);
+        }
       }
 #pragma unroll
       for (int c = 0; c < CV / 2; ++c)  // half of this page's V
@@ -797,7 +802,7 @@ void attn_tiles(Args a) {
 
     // ---- P V
 #pragma unroll
-    for (int i = 0; i < RQ; ++i) load_q(qf[i], i);  // for the next page
+    for (int i = RES; i < RQ; ++i) load_q(qf[i], i);  // for the next page
     constexpr int VB = TWO ? 1 : 2;  // slots' V in registers
     bf16x8 vf[VB][ND];
     auto read_v = [&](bf16x8 (&f)[ND], int s) {
