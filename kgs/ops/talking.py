@@ -8,7 +8,7 @@ learned bias per distance bucket, one added to the softmax's denominator.
   temperatures and the distance table;
 * :func:`write_kv` -- the projections' biases and the cache write;
 * :func:`attention_rows` -- single query tokens (decode, short portions), split over
-  the context; :func:`attention_tiles` -- prompt portions, 16 queries per workgroup.
+  the context; :func:`attention_tiles` -- prompt portions, 16 or 32 queries per workgroup.
 """
 from __future__ import annotations
 
@@ -27,7 +27,6 @@ LOG2E = 1.4426950408889634
 MFMA_DIMS = (64, 128)   # head sizes of the MFMA kernels (others are padded up, larger ones run plain)
 MAX_ROW_HEADS = 64      # heads of the MFMA rows kernel
 MAX_SLOTS = 8           # slots of 4 heads of the tiles kernel
-TILE = 16               # queries per tile
 
 
 def padded_dim(n: int) -> int:
@@ -56,15 +55,15 @@ class Heads:
         return self.mfma and self.slots <= MAX_SLOTS
 
     @property
-    def tiles_at_once(self) -> int:
-        """Tile workgroups the chip holds: two per CU where the registers allow it."""
-        return CUS * (2 if self.slots <= 4 else 1)
+    def tile(self) -> int:
+        """Queries of one tile (a workgroup, one per CU)."""
+        return 32 if self.slots <= 4 else 16
 
     @property
     def tile_bytes(self) -> int:
         """Scratch of one tile: its queries in operand order."""
         form = 2 if self.slots <= 2 else 4 if self.slots <= 4 else 8
-        return form * 4096 * (self.dkp // 32)
+        return form * 256 * self.tile * (self.dkp // 32)
 
     def slot_heads(self) -> list[int]:
         """Head at every position of the slots (-1: empty), padded to whole 16s."""
@@ -175,7 +174,7 @@ class QueryRows:
 
 @dataclass
 class QueryTiles:
-    """Blocks of up to ``TILE`` consecutive queries over a range of their pages
+    """Blocks of up to ``Heads.tile`` consecutive queries over a range of their pages
     (:func:`tile_items`): int32 ``[n, 8]`` (first batch row, block-table row, position of
     the first, queries, first page, end, partial result or -1, 0), and ``merges [m, 4]``
     (first batch row, queries, first part, parts) of the blocks that are split."""
@@ -189,19 +188,23 @@ MIN_PAGES = 16  # pages of a part
 MAX_PARTS = 64  # parts that one merge takes
 
 
-def tile_items(portions, slots: int) -> tuple[np.ndarray, np.ndarray]:
+def tile_items(portions, tile: int) -> tuple[np.ndarray, np.ndarray]:
     """Items and merges of ``portions`` (first batch row, block-table row, position,
-    tokens) for ``slots`` workgroups at a time. Blocks with more than an even share of
-    all pages are split, so that a long prompt's last blocks do not outlast the rest; the
-    longest first."""
-    b = np.array([(r + j, s, p + j, min(TILE, n - j)) for r, s, p, n in portions for j in range(0, n, TILE)], np.int64)
+    tokens). Blocks with more than an even share of all pages are split, so that a long
+    prompt's last blocks do not outlast the others: evenly where all items run at once,
+    else into such shares and a rest, which fill up the last round; the longest first."""
+    b = np.array([(r + j, s, p + j, min(tile, n - j)) for r, s, p, n in portions for j in range(0, n, tile)], np.int64)
     pages = (b[:, 2] + b[:, 3] - 1) // PAGE + 1
-    cap = max(MIN_PAGES, -(-int(pages.sum()) // slots))
-    parts = np.minimum(-(-pages // cap), MAX_PARTS) if len(b) < 2 * slots else np.ones_like(pages)
+    share = max(MIN_PAGES, -(-int(pages.sum()) // CUS)) if len(b) < 2 * CUS else int(pages.max())
+    cap = np.maximum(share, -(-pages // MAX_PARTS))
+    parts = -(-pages // cap)
+    split = parts > 1
     at = np.repeat(np.arange(len(b)), parts)
     k = np.arange(len(at)) - np.repeat(np.cumsum(parts) - parts, parts)
-    first, end = pages[at] * k // parts[at], pages[at] * (k + 1) // parts[at]
-    split = parts > 1
+    if len(at) <= CUS:
+        first, end = pages[at] * k // parts[at], pages[at] * (k + 1) // parts[at]
+    else:
+        first, end = k * cap[at], np.minimum((k + 1) * cap[at], pages[at])
     part0 = np.cumsum(np.where(split, parts, 0)) - np.where(split, parts, 0)
     part = np.where(split[at], part0[at] + k, -1)
     items = np.concatenate([b[at], np.stack([first, end, part, np.zeros_like(k)], 1)], 1)
@@ -260,8 +263,8 @@ def attention_tiles(q: torch.Tensor, pages: torch.Tensor, w: TalkingWeights, t: 
         raise ValueError("items must be contiguous int32 [n, 8]")
     m, po, pml = 0 if t.merges is None else t.merges.shape[0], None, None
     if m:
-        po = torch.empty((t.parts * TILE, h.heads, h.dvp), dtype=torch.float32, device=q.device)
-        pml = torch.empty((t.parts * TILE, h.heads, 2), dtype=torch.float32, device=q.device)
+        po = torch.empty((t.parts * h.tile, h.heads, h.dvp), dtype=torch.float32, device=q.device)
+        pml = torch.empty((t.parts * h.tile, h.heads, 2), dtype=torch.float32, device=q.device)
     n = t.items.shape[0]
     scratch = torch.empty((n, h.tile_bytes), dtype=torch.uint8, device=q.device)
     rc = _lib.lib().kgs_talking_tiles(_act(q, q.shape[0], h.heads * h.dkp, torch.bfloat16, "q"), q.stride(0),

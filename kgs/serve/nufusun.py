@@ -3,7 +3,7 @@ experts (:mod:`kgs.models.nufusun`).
 
 Every step is one ragged batch (:class:`kgs.serve.ragged.Batch`): the projections'
 biases are added where keys and values go to their pages, prompt portions attend in
-tiles of 16 queries, decoded tokens and short portions row by row with the context
+tiles of 16 or 32 queries, decoded tokens and short portions row by row with the context
 split over the CUs. A layer's two sublayers read the same normed input; one launch
 (:func:`kgs.ops.residual.residual_add`) adds both to the fp32 residual, gathering
 every token's expert rows, and produces the next layer's input.
@@ -71,7 +71,7 @@ class Geometry:
                      "rows": None if whole else pk.add(at)}, len(at), split_count(len(at), pages))
         if tiled.any():
             sel = np.flatnonzero(tiled)
-            items, merges = tile_items([(row0[s], s, pos0[s], n[s]) for s in sel], self.heads.tiles_at_once)
+            items, merges = tile_items([(row0[s], s, pos0[s], n[s]) for s in sel], self.heads.tile)
             tiles = (pk.add(items), pk.add(merges) if len(merges) else None, int(merges[:, 3].sum()))
 
         def build(get):

@@ -38,7 +38,6 @@ namespace kgs {
 namespace talking {
 
 constexpr int PAGE = 32;
-constexpr int TILE = 16;  // queries of a tile
 constexpr float NEG = -1.0e30f;
 constexpr float RESCALE = 8.0f;  // log2 units a score may exceed the running maximum by
 
@@ -486,62 +485,69 @@ __device__ __forceinline__ void bar() {
   fence();
 }
 
-// 16 QT queries of one portion, all heads; wave w has queries 4 QT w .. in QT blocks of
-// 4. Heads sit in slots of 4 that share a key head (slot s: key head s / QPG, its heads
-// 4 (s % QPG) .., those past the group's end empty), so a row tile is 4 queries x 4 heads.
+// 4 NW queries of one portion, all heads; wave w has queries 4w .. 4w + 3. Heads sit in
+// slots of 4 that share a key head (slot s: key head s / QPG, its heads 4 (s % QPG) ..,
+// those past the group's end empty), so a row tile is the wave's 4 queries x a slot's heads.
 //
-// Per page: S = Q K^T for every row tile (K fragments are read two half slots ahead of
-// their MFMAs, Q row tiles a ring ahead, the first of the next page during P V), the
-// next K and this V on their way by LDS-DMA, mix and softmax, P through this wave's
-// corner of LDS into operand order, P V. The outputs live in named AGPRs
-// (acc_regs.h, accumulator (s QT + qt) ND + d): they take half the register file, and the compiler would
-// move them about. Rescales are collected over the page and applied before P V.
-template <int NS, int QT, int NK, int ND>
-__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(NS * QT > 4 ? 1 : 2, NS * QT > 4 ? 1 : 2)))
+// Per page: S = Q K^T slot by slot (K fragments are read some steps ahead of their
+// MFMAs), the next K and this V on their way by LDS-DMA, mix and softmax, P through this
+// wave's corner of LDS into operand order, P V. The outputs live in named AGPRs
+// (acc_regs.h, accumulator s ND + d): they take half the register file, and the compiler
+// would move them about. Rescales are collected over the page and applied before P V.
+//
+// Q is too large for what is left of the registers. Up to four slots, eight waves (two per
+// SIMD) share K and V, and LDS has room for the first LQ row tiles' Q. Above, four waves
+// have all registers, and RES row tiles' stay there. The others come from memory again
+// for every page, the first of them during the last page's P V: what counts is that all
+// workgroups of an XCD together fit its L2.
+template <int NS>
+constexpr int waves() { return NS <= 4 ? 8 : 4; }
+
+template <int NS, int NK, int ND>
+__global__ __launch_bounds__(64 * waves<NS>()) __attribute__((amdgpu_waves_per_eu(waves<NS>() / 4, waves<NS>() / 4)))
 void attn_tiles(Args a) {
-  constexpr int MT = (NS + 3) / 4, RT = NS * QT;
-  constexpr bool TWO = RT <= 4;  // two waves per SIMD: half the registers
-  // Q row tiles in registers: the first RES for good, the others through a ring of RB
-  constexpr int RQ = TWO ? 1 : RT * NK <= 16 ? RT : 16 / NK;
+  constexpr int MT = (NS + 3) / 4, NW = waves<NS>();
+  constexpr bool TWO = NW == 8;  // two waves per SIMD: half the registers
+  constexpr int LQ = !TWO ? 0 : NS < 8 / NK ? NS : 8 / NK;
+  constexpr int RQ = TWO ? 1 : NS * NK <= 16 ? NS : 16 / NK;  // row tiles' Q in registers
   constexpr int RES = TWO || NK == 2 ? 0 : 1, RB = RQ - RES;
-  auto ring = [](int rt) { return rt < RES ? rt : RES + (rt - RES) % (RB ? RB : 1); };
-  static_assert(RT * ND <= 64, "outputs exceed the AGPRs");
-  __shared__ __attribute__((aligned(1024))) char smem[(NS * (2 * NK + ND) + 4 * RT) * 1024];
+  // register place of a row tile past LQ: the first RES for good, the others through a ring of RB
+  auto ring = [](int rt) { return rt - LQ < RES ? rt - LQ : RES + (rt - LQ - RES) % RB; };
+  static_assert(NS * ND <= 64, "outputs exceed the AGPRs");
+  __shared__ __attribute__((aligned(1024))) char smem[(NS * (2 * NK + ND) + NW * (NS + LQ * NK)) * 1024];
   char* const ks = smem;
   char* const vs = smem + NS * 2 * NK * 1024;
   const int lane = threadIdx.x & 63, w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), n = lane & 15, q = lane >> 4;
   // where this lane reads V: an address of its own, within the reach of the reads' offsets
   unsigned vl = (unsigned)(uintptr_t)(KGS_LDS char*)vs + 16 * lane;
   asm volatile("" : "+v"(vl));
-  char* const ps = vs + NS * ND * 1024 + w * RT * 1024;  // this wave's P: [qt][slot][16 rows][32 keys]
+  char* const ps = vs + NS * ND * 1024 + w * NS * 1024;  // this wave's P: [slot][16 rows][32 keys]
+  char* const lq = vs + NS * (ND + NW) * 1024 + w * LQ * NK * 1024 + 16 * lane;  // and its Q
   const int4 it = a.items[2 * blockIdx.x], part = a.items[2 * blockIdx.x + 1];  // part: first page, end, result (-1: whole)
   const int qpg = (a.R + 3) / 4, nslot = a.G * qpg;
   const int* bt = a.bt + (long)it.y * a.W;
   const int pend = part.y;
   constexpr int DK = 32 * NK, DV = 16 * ND, HPAGE = PAGE * (DK + DV) * 2;  // bytes of one head's page
-  const int posw = it.z + 4 * QT * w;                   // position of the wave's first query
+  const int posw = it.z + 4 * w;                        // position of the wave's first query
 
   // this lane's row of the S tiles: query n >> 2 of the block, head n & 3 of the slot. A query
   // past the portion's end reads its last one; an empty head reads what follows the
   // group (zeros past the last row): its scale is 0.
   const __amdgpu_buffer_rsrc_t qrsrc = __builtin_amdgcn_make_buffer_rsrc((void*)((const unsigned short*)a.q + (long)it.x * a.ldq), 0,
                                                        it.w * (int)a.ldq * 2, 0x00020000);
-  int qoff[QT];
-#pragma unroll
-  for (int t = 0; t < QT; ++t)
-    qoff[t] = (min(4 * (QT * w + t) + (n >> 2), it.w - 1) * (int)a.ldq + (n & 3) * DK + 8 * q) * 2;
-  auto first_q = [&](bf16x8 (&f)[NK], int rt) {
-    const int s = rt / QT, so = (min(s / qpg, a.G - 1) * a.R + 4 * (s % qpg)) * DK * 2;
+  const int qoff = (min(4 * w + (n >> 2), it.w - 1) * (int)a.ldq + (n & 3) * DK + 8 * q) * 2;
+  auto first_q = [&](bf16x8 (&f)[NK], int s) {
+    const int so = (min(s / qpg, a.G - 1) * a.R + 4 * (s % qpg)) * DK * 2;
 #pragma unroll
     for (int k = 0; k < NK; ++k)
-      f[k] = __builtin_bit_cast(bf16x8, __builtin_amdgcn_raw_buffer_load_b128(qrsrc, qoff[rt % QT] + 64 * k, so, 0));
+      f[k] = __builtin_bit_cast(bf16x8, __builtin_amdgcn_raw_buffer_load_b128(qrsrc, qoff + 64 * k, so, 0));
   };
   // Those rows lie 16 to a load. They are read again for every page, so the wave puts them down
   // in operand order first, 1 KB a fragment.
-  char* const qs = (char*)a.qs + ((long)blockIdx.x * 4 + w) * (RT * NK * 1024);
+  char* const qs = (char*)a.qs + ((long)blockIdx.x * NW + w) * (NS * NK * 1024);
   auto load_q = [&](bf16x8 (&f)[NK], int rt) {
 #pragma unroll
-    for (int k = 0; k < NK; ++k) f[k] = load_frag(qs, RT * NK * 1024, 16 * lane, (rt * NK + k) * 1024);
+    for (int k = 0; k < NK; ++k) f[k] = load_frag(qs, NS * NK * 1024, 16 * lane, (rt * NK + k) * 1024);
   };
   float sc[NS][4];  // uniform
 #pragma unroll
@@ -557,35 +563,43 @@ void attn_tiles(Args a) {
   for (int t = 0; t < MT; ++t) tf[t] = *(const f16x8*)(a.talk + (t * 64 + lane) * 8);
 
   // Every slot has a place for its key head's K and V. They come in chunks of 1 KB, dealt to the
-  // waves: chunk w + 4 c of `per` a slot.
+  // waves: chunk w + NW c of `per` a slot.
   const int pbytes = a.G * HPAGE;
   int head[NS];  // where a slot's head begins in a page
 #pragma unroll
-  for (int s = 0; s < NS; ++s) head[s] = min(s / qpg, a.G - 1) * HPAGE + w * 1024;
+  for (int s = 0; s < NS; ++s) head[s] = min(s / qpg, a.G - 1) * HPAGE;
   auto dma = [&](int page, char* dst, int per, int first, int c) {  // per: 4 or 8
-    dma_chunk((const char*)a.pages + (long)page * pbytes, pbytes, dst + (w + 4 * c) * 1024, 16 * lane,
-              head[4 * c / per] + (first + 4 * c % per * 1024));
+    const int lo = NW * c / per, so = per < NW && w >= per ? head[lo + 1] : head[lo];
+    dma_chunk((const char*)a.pages + (long)page * pbytes, pbytes, dst + (w + NW * c) * 1024, 16 * lane,
+              so + first + (NW * c + w) % per * 1024);
   };
-  constexpr int CK = NS * 2 * NK / 4, CV = NS * ND / 4;  // chunks per wave of K and of V
+  constexpr int CK = NS * 2 * NK / NW, CV = NS * ND / NW;  // chunks per wave of K and of V
+  constexpr int CV1 = CV / 2, CK1 = CK / 2;                // V: before the mixture and in it; K: in it and after
   constexpr int KPER = 2 * NK, VPER = ND;
   auto page_id = [&](int pg) { return bt[min(pg, pend - 1)]; };
 
   // the far bias less the running maximum of (query, slot 4t + q, head): the mixture's addend
-  f32x4 cm[4 * QT][MT];
-  float l[RT];
+  f32x4 cm[4][MT];
+  float l[NS];
 #pragma unroll
-  for (int i = 0; i < 4 * QT; ++i)
+  for (int i = 0; i < 4; ++i)
 #pragma unroll
     for (int t = 0; t < MT; ++t) cm[i][t] = *(const f32x4*)(a.bfar + 16 * t + 4 * q);
 #pragma unroll
-  for (int i = 0; i < RT; ++i) l[i] = 0.f;
+  for (int i = 0; i < NS; ++i) l[i] = 0.f;
   if constexpr (TWO) KGS_ACC_RESERVE_HALF();
   else KGS_ACC_RESERVE();
-  static_for<0, RT * ND>([](auto i) { accr::zero<decltype(i)::value>(); });
+  static_for<0, NS * ND>([](auto i) { accr::zero<decltype(i)::value>(); });
 
   bf16x8 qf[RQ][NK];
 #pragma unroll
-  for (int i = RT - 1; i >= 0; --i) {
+  for (int i = 0; i < LQ; ++i) {
+    first_q(qf[0], i);
+#pragma unroll
+    for (int k = 0; k < NK; ++k) *(bf16x8*)(lq + (i * NK + k) * 1024) = qf[0][k];
+  }
+#pragma unroll
+  for (int i = NS - 1; i >= LQ; --i) {
     first_q(qf[ring(i)], i);
 #pragma unroll
     for (int k = 0; k < NK; ++k) *(bf16x8*)(qs + (i * NK + k) * 1024 + 16 * lane) = qf[ring(i)][k];
@@ -598,33 +612,34 @@ void attn_tiles(Args a) {
     const int tok0 = pg * PAGE;
     const int next = page_id(pg + 1);
     // ---- scores
-    // A slot's scores become their fp16 parts while the next slot's MFMAs run.
-    unsigned x[QT][2][2][MT][2][4];  // [block][key half][part][half of the slots][head pair][slot of it, then query]
-    f32x4 S[2][QT][2];
-    auto split_slot = [&](int s, int u0, int u1) {  // units u0 .. u1 - 1 of 4 QT: (block, key half, head pair)
+    // A slot's scores become its fp16 parts while the next slot's MFMAs run.
+    unsigned x[2][2][MT][2][4];  // [key half][part][half of the slots][head pair][slot of it, then query]
+    f32x4 S[2][2];
+    auto split_slot = [&](int s, int u0, int u1) {  // units u0 .. u1 - 1 of 4: (key half, head pair)
 #pragma unroll
-      for (int u = 0; u < 4 * QT; ++u) {
+      for (int u = 0; u < 4; ++u) {
         if (u < u0 || u >= u1) continue;
-        const int t = u >> 2, kt = u >> 1 & 1, c = u & 1;
-        const f32x4& v = S[s & 1][t][kt];
-        unsigned &hi = x[t][kt][0][s >> 2][c][s & 3], &lo = x[t][kt][1][s >> 2][c][s & 3];
+        const int kt = u >> 1, c = u & 1;
+        const f32x4& v = S[s & 1][kt];
+        unsigned &hi = x[kt][0][s >> 2][c][s & 3], &lo = x[kt][1][s >> 2][c][s & 3];
         split2(v[2 * c] * sc[s][2 * c], v[2 * c + 1] * sc[s][2 * c + 1], hi, lo);
         asm volatile("" : "+v"(hi), "+v"(lo));  // here, not where they are used
       }
     };
     if constexpr (NS < 4) {
 #pragma unroll
-      for (int i = 0; i < QT * 8; ++i)
+      for (int i = 0; i < 8; ++i)
 #pragma unroll
-        for (int s = NS; s < 4; ++s) x[i >> 3][i >> 2 & 1][i >> 1 & 1][0][i & 1][s] = 0;
+        for (int s = NS; s < 4; ++s) x[i >> 2][i >> 1 & 1][0][i & 1][s] = 0;
     }
     // K fragments of both 16-key halves, one 32-dim step at a time, PF steps ahead
     constexpr int PF = TWO ? 1 : 3, STEPS = NS * NK;
-    bf16x8 kf[PF + 1][2];
+    bf16x8 kf[PF + 1][2], ql[PF + 1];
     auto read_k = [&](int p) {
       const char* kp = ks + (p / NK * 2 * NK + p % NK) * 1024 + 16 * lane;
       kf[p % (PF + 1)][0] = *(const bf16x8*)kp;
       kf[p % (PF + 1)][1] = *(const bf16x8*)(kp + NK * 1024);
+      if (p / NK < LQ) ql[p % (PF + 1)] = *(const bf16x8*)(lq + p * 1024);
     };
 #pragma unroll
     for (int p = 0; p < PF; ++p) read_k(p);
@@ -632,62 +647,55 @@ void attn_tiles(Args a) {
     for (int p = 0; p < STEPS; ++p) {
       if (p + PF < STEPS) read_k(p + PF);
       fence();
+      const int s = p / NK;
+      f32x4(&c)[2] = S[s & 1];
+      if (p % NK == 0) c[0] = c[1] = f32x4{};
 #pragma unroll
-      for (int t = 0; t < QT; ++t) {
-        const int rt = (p / NK) * QT + t;
-        f32x4(&c)[2] = S[(p / NK) & 1][t];
-        if (p % NK == 0) c[0] = c[1] = f32x4{};
-#pragma unroll
-        for (int kt = 0; kt < 2; ++kt)
-          c[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[ring(rt)][p % NK], kf[p % (PF + 1)][kt], c[kt], 0, 0, 0);
-      }
-      if (p >= NK) split_slot(p / NK - 1, p % NK * 4 * QT / NK, (p % NK + 1) * 4 * QT / NK);
+      for (int kt = 0; kt < 2; ++kt)
+        c[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(s < LQ ? ql[p % (PF + 1)] : qf[s < LQ ? 0 : ring(s)][p % NK],
+                                                        kf[p % (PF + 1)][kt], c[kt], 0, 0, 0);
+      if (s > 0) split_slot(s - 1, p % NK * 4 / NK, (p % NK + 1) * 4 / NK);
       if (p % NK == NK - 1) {
         fence();
-#pragma unroll
-        for (int t = 0; t < QT; ++t) {
-          const int rt = (p / NK) * QT + t;
-          if (rt >= RES && rt + RB < RT) load_q(qf[ring(rt)], rt + RB);
-        }
+        if (s >= LQ + RES && s + RB < NS) load_q(qf[ring(s)], s + RB);
       }
 #pragma unroll
-      for (int c = 0; c < CV / 2; ++c)  // half of this page's V
-        if (c * STEPS / (CV / 2) == p) dma(page, vs, VPER, PAGE * DK * 2, c);
+      for (int c = 0; c < CV1; ++c)  // half of this page's V
+        if (c * STEPS / (CV1 ? CV1 : 1) == p) dma(page, vs, VPER, PAGE * DK * 2, c);
       fence();
     }
-    split_slot(NS - 1, 0, 4 * QT);
+    split_slot(NS - 1, 0, 4);
     bar<63>();  // K of this page is done with everywhere
     const int pnext = __builtin_amdgcn_readfirstlane(next);
 
     // ---- mix, softmax
     const bool near = posw - (tok0 + PAGE - 1) < a.nfar, edge = tok0 + PAGE - 1 > posw;
     bool grown = false;
-    float al[RT];
+    float al[NS];
 #pragma unroll
-    for (int i = 0; i < RT; ++i) al[i] = 1.f;
-#pragma unroll
-    for (int qt = 0; qt < QT; ++qt) {
+    for (int i = 0; i < NS; ++i) al[i] = 1.f;
+    {
       unsigned p0[4][MT][2];  // keys 2n, heads (0, 1) and (2, 3)
 #pragma unroll
       for (int kt = 0; kt < 2; ++kt) {
 #pragma unroll
         for (int j = 0; j < 2; ++j)
 #pragma unroll
-          for (int hf = 0; hf < MT; ++hf) transpose4(x[qt][kt][j][hf][0]), transpose4(x[qt][kt][j][hf][1]);
+          for (int hf = 0; hf < MT; ++hf) transpose4(x[kt][j][hf][0]), transpose4(x[kt][j][hf][1]);
         f32x4 D[4][MT];
 #pragma unroll
         for (int j = 1; j >= 0; --j)
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
-            const unsigned(&y)[MT][2][4] = x[qt][kt][j];
+            const unsigned(&y)[MT][2][4] = x[kt][j];
             const u32x4 b = {y[0][0][i], y[0][1][i], MT > 1 ? y[MT - 1][0][i] : 0u, MT > 1 ? y[MT - 1][1][i] : 0u};
 #pragma unroll
             for (int t = 0; t < MT; ++t)
               D[i][t] = __builtin_amdgcn_mfma_f32_16x16x32_f16(tf[t], __builtin_bit_cast(f16x8, b),
-                                                               j == 1 ? cm[4 * qt + i][t] : D[i][t], 0, 0, 0);
+                                                               j == 1 ? cm[i][t] : D[i][t], 0, 0, 0);
           }
         // lane: query i, key 2n + kt, slot 4t + q, head r; above the running maximum
-        const int dist = posw + 4 * qt - (tok0 + 2 * n + kt);  // of query 0
+        const int dist = posw - (tok0 + 2 * n + kt);  // of query 0
         if (near) {
           // all loads, then all sums: waited for here, not where far pages pass too
           f32x4 b[4][MT];
@@ -737,7 +745,7 @@ void attn_tiles(Args a) {
                 for (int b = 1; b < 16; b <<= 1)
                   up = fmaxf(up, __int_as_float(__builtin_amdgcn_ds_bpermute(((n_ ^ b) + 16 * q) * 4, __float_as_int(up))));
                 fr[r] = __builtin_amdgcn_exp2f(-up);
-                cm[4 * qt + i][t][r] -= up;
+                cm[i][t][r] -= up;
                 D[i][t][r] -= up;
               }
               sel[t] = (n_ & 2) ? ((n_ & 1) ? fr[3] : fr[2]) : ((n_ & 1) ? fr[1] : fr[0]);
@@ -751,7 +759,7 @@ void attn_tiles(Args a) {
 #pragma unroll
             for (int s = 0; s < NS; ++s) {
               const float g = __shfl(sel[s >> 2], 16 * (s & 3) + (n_ & 3), 64);
-              al[s * QT + qt] *= (n_ >> 2) == i ? g : 1.f;
+              al[s] *= (n_ >> 2) == i ? g : 1.f;
             }
           }
         }
@@ -760,8 +768,8 @@ void attn_tiles(Args a) {
           // a chunk or two at a time: the rest of this page's V, then half of the next one's K
           fence();
 #pragma unroll
-          for (int c = CV / 2; c < CV + CK / 2; ++c)
-            if ((c - CV / 2) * 8 * QT / (CV - CV / 2 + CK / 2) == 4 * (2 * qt + kt) + i) {
+          for (int c = CV1; c < CV + CK1; ++c)
+            if ((c - CV1) * 8 / (CV - CV1 + CK1) == 4 * kt + i) {
               if (c < CV) dma(page, vs, VPER, PAGE * DK * 2, c);
               else dma(pnext, ks, KPER, 0, c - CV);
             }
@@ -775,7 +783,7 @@ void attn_tiles(Args a) {
             else if (NS >= 4 || q < NS) {
               // row 4i + r of slot 4t + q, keys 2n and 2n + 1; rows permuted by the slot and 16-B
               // chunks by the row: no bank twice
-              char* pp = ps + (qt * NS + 4 * t + q) * 1024 + 256 * i + (((n >> 2) ^ i) * 16) + (n & 3) * 4;
+              char* pp = ps + (4 * t + q) * 1024 + 256 * i + (((n >> 2) ^ i) * 16) + (n & 3) * 4;
               *(unsigned*)(pp + ((0 ^ q) * 64)) = __builtin_amdgcn_perm(c0, p0[i][t][0], 0x05040100u);
               *(unsigned*)(pp + ((1 ^ q) * 64)) = __builtin_amdgcn_perm(c0, p0[i][t][0], 0x07060302u);
               *(unsigned*)(pp + ((2 ^ q) * 64)) = __builtin_amdgcn_perm(c1, p0[i][t][1], 0x05040100u);
@@ -787,33 +795,32 @@ void attn_tiles(Args a) {
     }
     if (__builtin_expect(grown, 0)) {
       asm volatile("s_nop 7\n\ts_nop 7\n\ts_nop 3" ::: "memory");  // MFMA -> v_accvgpr_read hazard
-      static_for<0, RT>([&](auto rc) {
-        constexpr int rt = decltype(rc)::value;
-        l[rt] *= al[rt];
+      static_for<0, NS>([&](auto rc) {
+        constexpr int s = decltype(rc)::value;
+        l[s] *= al[s];
         static_for<0, ND>([&](auto dc) {
-          constexpr int i = rt * ND + decltype(dc)::value;
-          accr::write<i>(accr::read<i>() * al[rt]);
+          constexpr int i = s * ND + decltype(dc)::value;
+          accr::write<i>(accr::read<i>() * al[s]);
         });
       });
       asm volatile("s_nop 7" ::: "memory");
     }
-    bar<CK / 2>();  // V of this page is there
+    bar<CK1>();  // V of this page is there
     page = pnext;
 
     // ---- P V
 #pragma unroll
-    for (int i = RES; i < RQ; ++i) load_q(qf[i], i);  // for the next page
+    for (int i = RES; i < RQ; ++i)
+      if (LQ + i < NS) load_q(qf[i], LQ + i);  // for the next page
     constexpr int VB = TWO ? 1 : 2;  // slots' V in registers
     bf16x8 vf[VB][ND];
     auto read_v = [&](bf16x8 (&f)[ND], int s) {
 #pragma unroll
       for (int i = 0; i < ND; ++i) f[i] = *(const KGS_LDS bf16x8*)(uintptr_t)(vl + (s * ND + i) * 1024);
     };
-    u32x4 pw[VB][QT];
-    auto read_p = [&](u32x4 (&f)[QT], int s) {
-#pragma unroll
-      for (int t = 0; t < QT; ++t)
-        f[t] = *(const u32x4*)(ps + (t * NS + s) * 1024 + ((n ^ (s & 3)) * 64) + ((q ^ ((n >> 2) & 3)) * 16));
+    u32x4 pw[VB];
+    auto read_p = [&](u32x4& f, int s) {
+      f = *(const u32x4*)(ps + s * 1024 + ((n ^ (s & 3)) * 64) + ((q ^ ((n >> 2) & 3)) * 16));
     };
     read_p(pw[0], 0);
     read_v(vf[0], 0);
@@ -829,42 +836,38 @@ void attn_tiles(Args a) {
       }
       fence();
 #pragma unroll
-      for (int c = CK / 2; c < CK; ++c)  // the other half of K (past the last page: that one again)
-        if ((c - CK / 2) * NS / 2 / (CK - CK / 2) == s) dma(pnext, ks, KPER, 0, c);
-      static_for<0, QT>([&](auto tc) {
-        constexpr int t = decltype(tc)::value, rt = s * QT + t;
-        const u32x4 pv = pw[s % VB][t];
-        const bf16x8 pb = __builtin_bit_cast(bf16x8, pv);
-        static_for<0, ND>([&](auto dc) {
-          constexpr int d = decltype(dc)::value;
-          accr::mfma<rt * ND + d>(vf[s % VB][d], pb);
-        });
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          const unsigned two = pv[e], ones = 0x3f803f80u;
-          l[rt] = __builtin_amdgcn_fdot2_f32_bf16(__builtin_bit_cast(bf16x2, two), __builtin_bit_cast(bf16x2, ones), l[rt], false);
-        }
+      for (int c = CK1; c < CK; ++c)  // the other half of K (past the last page: that one again)
+        if ((c - CK1) * NS / 2 / (CK - CK1) == s) dma(pnext, ks, KPER, 0, c);
+      const u32x4 pv = pw[s % VB];
+      const bf16x8 pb = __builtin_bit_cast(bf16x8, pv);
+      static_for<0, ND>([&](auto dc) {
+        constexpr int d = decltype(dc)::value;
+        accr::mfma<s * ND + d>(vf[s % VB][d], pb);
       });
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const unsigned two = pv[e], ones = 0x3f803f80u;
+        l[s] = __builtin_amdgcn_fdot2_f32_bf16(__builtin_bit_cast(bf16x2, two), __builtin_bit_cast(bf16x2, ones), l[s], false);
+      }
       fence();
     });
     bar<0>();  // V is done with everywhere, K of the next page is there
   }
 
-  // rows' maxima to the lanes that hold the rows: [qt][slot][row]
+  // rows' maxima to the lanes that hold the rows: [slot][row]
   float* mm = (float*)ps;
 #pragma unroll
-  for (int i = 0; i < 4 * QT; ++i)
+  for (int i = 0; i < 4; ++i)
 #pragma unroll
     for (int t = 0; t < MT; ++t)
-      if (NS >= 4 || q < NS) *(f32x4*)(mm + ((i >> 2) * NS + 4 * t + q) * 16 + 4 * (i & 3)) =
+      if (NS >= 4 || q < NS) *(f32x4*)(mm + (4 * t + q) * 16 + 4 * i) =
                                   *(const f32x4*)(a.bfar + 16 * t + 4 * q) - cm[i][t];
   asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
   asm volatile("s_nop 7\n\ts_nop 7\n\ts_nop 3" ::: "memory");  // MFMA -> v_accvgpr_read hazard
   static_for<0, NS>([&](auto sc_) {
-    static_for<0, QT>([&](auto tc) {
-      constexpr int s = decltype(sc_)::value, t = decltype(tc)::value, rt = s * QT + t;
-      const int hr = 4 * (s % qpg) + (n & 3), qi = 4 * (QT * w + t) + (n >> 2);
-      const float m = mm[(t * NS + s) * 16 + n], L = xor32_sum(xor16_sum(l[rt]));
+      constexpr int s = decltype(sc_)::value;
+      const int hr = 4 * (s % qpg) + (n & 3), qi = 4 * w + (n >> 2);
+      const float m = mm[s * 16 + n], L = xor32_sum(xor16_sum(l[s]));
       const bool ok = s < nslot && hr < a.R && qi < it.w;
       const int h = s / qpg * a.R + hr;
       if (part.z < 0) {
@@ -872,22 +875,21 @@ void attn_tiles(Args a) {
         unsigned short* op = (unsigned short*)a.o + (long)(it.x + qi) * a.ldo + (long)h * DV + 4 * q;
         static_for<0, ND>([&](auto dc) {
           constexpr int d = decltype(dc)::value;
-          const f32x4 o = accr::read<rt * ND + d>() * inv;
+          const f32x4 o = accr::read<s * ND + d>() * inv;
           uint2 pk;
           pk.x = pack_bf16x2(o[0], o[1]);
           pk.y = pack_bf16x2(o[2], o[3]);
           if (ok) *(uint2*)(op + 16 * d) = pk;
         });
       } else {
-        const long pr = ((long)part.z * (16 * QT) + qi) * a.H + h;
+        const long pr = ((long)part.z * (4 * NW) + qi) * a.H + h;
         static_for<0, ND>([&](auto dc) {
           constexpr int d = decltype(dc)::value;
-          const f32x4 o = accr::read<rt * ND + d>();
+          const f32x4 o = accr::read<s * ND + d>();
           if (ok) *(f32x4*)(a.po + pr * DV + 16 * d + 4 * q) = o;
         });
         if (ok && q == 0) a.pml[2 * pr] = m, a.pml[2 * pr + 1] = L;
       }
-    });
   });
 }
 
@@ -982,10 +984,10 @@ void rows_ht(const Args& a, int nrows, hipStream_t s) {
 }
 template <int NK, int ND>
 void tiles_ns(const Args& a, int nitems, int nslot, hipStream_t s) {
-  const dim3 grid((unsigned)nitems), block(256);
-  if (nslot <= 2) hipLaunchKernelGGL((attn_tiles<2, 1, NK, ND>), grid, block, 0, s, a);
-  else if (nslot <= 4) hipLaunchKernelGGL((attn_tiles<4, 1, NK, ND>), grid, block, 0, s, a);
-  else hipLaunchKernelGGL((attn_tiles<8, 1, NK, ND>), grid, block, 0, s, a);
+  const dim3 grid((unsigned)nitems);
+  if (nslot <= 2) hipLaunchKernelGGL((attn_tiles<2, NK, ND>), grid, dim3(64 * waves<2>()), 0, s, a);
+  else if (nslot <= 4) hipLaunchKernelGGL((attn_tiles<4, NK, ND>), grid, dim3(64 * waves<4>()), 0, s, a);
+  else hipLaunchKernelGGL((attn_tiles<8, NK, ND>), grid, dim3(64 * waves<8>()), 0, s, a);
 }
 
 int check(const Args& a, int n) {
@@ -1049,12 +1051,12 @@ KGS_EXPORT int kgs_talking_rows(const void* q, long ldq, const void* pages, void
 }
 
 // Prompt portions: nitems blocks of consecutive queries over a range of their pages, two
-// int4 each (Args::items): up to 16 queries. A block split over its pages
-// leaves partial results (po, pml: one part holds 16 rows of all heads) that
+// int4 each (Args::items): up to 32 queries, 16 above 4 slots. A block split over its pages
+// leaves partial results (po, pml: one part holds 32 or 16 rows of all heads) that
 // `merges` names. bf16, dkp and dvp 64 or 128, at most 8 slots of 4 heads
 // (G ceil(H / G / 4)); talk (fp16) and biases in slot order, ldb = 16 ceil(slots / 4); bias is
 // the table less its last row, bfar. qs: scratch, slots (2, 4 or 8) x 4 KB x dkp / 32 per
-// item.
+// item, twice that up to 4 slots.
 KGS_EXPORT int kgs_talking_tiles(const void* q, long ldq, const void* pages, void* o, long ldo, const void* bt, int W,
                                  const void* items, int nitems, const void* merges,
                                  int nmerge, void* po, void* pml, void* qs, const void* sc, const void* talk, const void* bias,
@@ -1069,7 +1071,7 @@ KGS_EXPORT int kgs_talking_tiles(const void* q, long ldq, const void* pages, voi
   const int nslot = G * ((H / G + 3) / 4);
   if (nslot > 8 || (dkp != 64 && dkp != 128) || (dvp != 64 && dvp != 128)) return KGS_ERR_ARG;
   if (ldb < (nslot + 3) / 4 * 16 || (((uintptr_t)items | (uintptr_t)bfar | (uintptr_t)talk | (uintptr_t)qs) & 15)) return KGS_ERR_SHAPE;
-  a.tile = TILE;
+  a.tile = nslot <= 4 ? 32 : 16;
   if (nmerge < 0 || (nmerge && (!merges || !po || !pml)) || (long)nmerge * a.tile * H > 0x7fffffff) return KGS_ERR_SHAPE;
   if (dkp == 64) dvp == 64 ? tiles_ns<2, 4>(a, nitems, nslot, s) : tiles_ns<2, 8>(a, nitems, nslot, s);
   else dvp == 64 ? tiles_ns<4, 4>(a, nitems, nslot, s) : tiles_ns<4, 8>(a, nitems, nslot, s);

@@ -80,7 +80,7 @@ def test_checkpoint_shapes_are_checked():
 
 
 # ------------------------------------------------------------------ distances
-@pytest.mark.parametrize("rows,far", [(32, 240), (32, 128), (8, 20), (16, 100.5), (2, 5), (6, 10), (64, 1000)])
+@pytest.mark.parametrize("rows,far", [(24, 200), (32, 128), (8, 20), (16, 100.5), (2, 5), (6, 10), (64, 1000)])
 def test_buckets(rows, far):
     n = math.ceil(far) + 50
     b, half = buckets(rows, far, n), rows // 2
@@ -157,17 +157,17 @@ def _plan(heads, n, pos0):
 
 
 def test_plan_splits_tiles_and_rows():
-    h = heads_of(6, 2, 64, 64, torch.bfloat16)
+    h = heads_of(6, 3, 64, 64, torch.bfloat16)
     p, row0 = _plan(h, [1, 40, 2, 16, 15], [70, 3, 9, 500, 0])
     items = sorted(p.tiles.items.tolist())
-    assert items == [[1, 1, 3, 16, 0, 1, -1, 0], [17, 1, 19, 16, 0, 2, -1, 0], [33, 1, 35, 8, 0, 2, -1, 0], [43, 3, 500, 16, 0, 17 // 2, 0, 0],
+    assert items == [[1, 1, 3, 32, 0, 2, -1, 0], [33, 1, 35, 8, 0, 2, -1, 0], [43, 3, 500, 16, 0, 17 // 2, 0, 0],
                      [43, 3, 500, 16, 8, 17, 1, 0]]
     pages = [i[5] - i[4] for i in p.tiles.items.tolist()]
     assert pages == sorted(pages, reverse=True)
     assert p.tiles.merges.tolist() == [[43, 16, 0, 2]] and p.tiles.parts == 2
     assert p.rows.n == 18 and p.rows.rows.tolist() == [0, 41, 42, *range(59, 74)]
     assert p.rows.tok_seq.tolist() == [0, 2, 2] + [4] * 15 and p.rows.tok_pos.tolist() == [70, 9, 10, *range(15)]
-    p, _ = _plan(heads_of(32, 8, 64, 64, torch.bfloat16), [40], [3])
+    p, _ = _plan(heads_of(32, 8, 64, 64, torch.bfloat16), [40], [3])  # eight slots: tiles of 16
     assert sorted(p.tiles.items.tolist()) == [[0, 0, 3, 16, 0, 1, -1, 0], [16, 0, 19, 16, 0, 2, -1, 0], [32, 0, 35, 8, 0, 2, -1, 0]]
     assert p.tiles.merges is None
     p, _ = _plan(h, [1, 1], [5, 900])
@@ -179,12 +179,12 @@ def test_plan_splits_tiles_and_rows():
 
 
 def test_tile_items_cover_every_page_once():
-    for portions in ([(0, 0, 0, 8192)], [(i * 700, i, 50 * i, 700) for i in range(9)], [(5, 2, 9000, 17)], [(0, 0, 0, 3)]):
-        for slots in (256, 512):
-            items, merges = tile_items(portions, slots)
+    for portions in ([(0, 0, 0, 8192)], [(0, 0, 33000, 700)], [(i * 700, i, 50 * i, 700) for i in range(9)], [(5, 2, 9000, 17)], [(0, 0, 0, 3)]):
+        for tile in (16, 32):
+            items, merges = tile_items(portions, tile)
             seen, parts = {}, {}
             for r, s, p, n, a, b, part, _ in items.tolist():
-                assert 0 <= a < b <= (p + n - 1) // 32 + 1 and 0 < n <= 16
+                assert 0 <= a < b <= (p + n - 1) // 32 + 1 and 0 < n <= tile
                 seen.setdefault((r, s, p, n), []).append((a, b))
                 if part >= 0:
                     parts.setdefault(r, []).append(part)
@@ -195,7 +195,7 @@ def test_tile_items_cover_every_page_once():
             assert sorted(x for v in parts.values() for x in v) == list(range(sum(map(len, parts.values()))))
             assert {m[0]: (m[2], m[3]) for m in merges.tolist()} == {r: (min(v), len(v)) for r, v in parts.items()}
             assert sum(k[3] for k in seen) == sum(x[3] for x in portions) and (merges[:, 3] <= 64).all()
-    items, _ = tile_items([(0, 0, 0, 8192)], 512)
+    items, _ = tile_items([(0, 0, 0, 8192)], 32)
     assert (items[:, 5] - items[:, 4]).max() <= 129
 
 

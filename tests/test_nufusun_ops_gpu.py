@@ -136,7 +136,7 @@ def test_router_reads_32_bit_sums():
 
 # ------------------------------------------------------------------ attention
 SHAPES = [  # heads, kv_heads, dim, vdim
-    (6, 2, 64, 48), (1, 1, 16, 16), (5, 1, 80, 128), (8, 8, 64, 64), (12, 3, 128, 64), (20, 4, 100, 50), (32, 8, 128, 128),
+    (9, 3, 56, 40), (1, 1, 16, 16), (5, 1, 80, 128), (8, 8, 64, 64), (12, 3, 128, 64), (20, 4, 100, 50), (32, 8, 128, 128),
     (16, 4, 128, 128), (28, 7, 40, 120), (18, 18, 32, 64), (40, 5, 64, 100), (64, 16, 128, 128), (4, 2, 160, 32),
     (66, 6, 20, 40)]
 
@@ -213,7 +213,7 @@ class Case:
         from kgs.ops.talking import QueryTiles, attention_tiles, tile_items
 
         base = np.cumsum([0] + self.lens)
-        items, merges = tile_items([(base[s] + p, s, p, n) for s, p, n in portions], self.h.tiles_at_once)
+        items, merges = tile_items([(base[s] + p, s, p, n) for s, p, n in portions], self.h.tile)
         assert split == bool(len(merges))
         i32 = lambda a: torch.tensor(a, dtype=torch.int32).cuda()  # noqa: E731
         t = QueryTiles(i32(items), i32(self.bt), i32(merges) if split else None, int(merges[:, 3].sum()))
@@ -249,7 +249,7 @@ def test_attention(shape, dtype):
 
 
 @pytest.mark.parametrize("dtype", [F32, BF])
-@pytest.mark.parametrize("shape", [(6, 2, 64, 48), (32, 8, 128, 128), (20, 4, 100, 50)], ids=str)
+@pytest.mark.parametrize("shape", [(9, 3, 56, 40), (32, 8, 128, 128), (20, 4, 100, 50)], ids=str)
 def test_scores_that_stand_out(shape, dtype):
     """Keys that one query finds by far the best -- the first, at page borders, far back,
     the last -- in rising order, so the running maximum moves in late tiles."""
@@ -263,7 +263,7 @@ def test_scores_that_stand_out(shape, dtype):
         c.check(c.tiles([(0, 110, 191)]), [(0, p) for p in range(110, 301)], "tiles")
 
 
-@pytest.mark.parametrize("shape", [(6, 2, 64, 48), (20, 4, 100, 50), (16, 4, 128, 128)], ids=str)
+@pytest.mark.parametrize("shape", [(9, 3, 56, 40), (20, 4, 100, 50), (16, 4, 128, 128)], ids=str)
 def test_split_tiles(shape):
     """Portions over many pages: blocks split over their pages and merged, beside whole ones."""
     sharp = [(700, 3, 2.0), (690, 512, 2.0), (650, 300, 3.0), (700, 699, 1.0)]
@@ -273,7 +273,7 @@ def test_split_tiles(shape):
     assert torch.isnan(got[:600]).all()
 
 
-@pytest.mark.parametrize("rows,far", [(16, 50.0), (32, 240.0), (2, 7.0), (64, 150.5)])
+@pytest.mark.parametrize("rows,far", [(16, 50.0), (24, 200.0), (2, 7.0), (64, 150.5)])
 @pytest.mark.parametrize("dtype", [F32, BF])
 def test_every_bucket_edge(rows, far, dtype):
     """One bucket at a time much higher than the others: a distance counted to the
@@ -295,9 +295,9 @@ def test_every_bucket_edge(rows, far, dtype):
 @pytest.mark.parametrize("level", [-30.0, 0.0, 30.0])
 def test_the_one_in_the_denominator(level, dtype):
     """All scores far below, about and far above the added term's 0."""
-    c = Case((6, 2, 64, 48), [100], dtype)
+    c = Case((9, 3, 56, 40), [100], dtype)
     c.rel = torch.full_like(c.rel, level)
-    c.talk = torch.eye(6, dtype=BF)
+    c.talk = torch.eye(9, dtype=BF)
     from kgs.ops.talking import TalkingWeights
 
     c.w = TalkingWeights(c.h, c.talk, c.temp, c.rel, c.scale, c.far, "cuda")
