@@ -396,12 +396,13 @@ __global__ __launch_bounds__(256, HT > 2 ? 1 : 2) void attn_rows(Args a) {
   }
 }
 
-// splits (at most 64) of one (row, head): 64 threads, 2 or 1 dims each (dvp 128 or 64).
+// splits (at most 64) of one (row, head): a wave, 2 or 1 dims a lane (dvp 128 or 64).
 // TILES: rows are the queries of split tiles, merges = (first batch row, queries, first
 // part, parts) of a tile; a part holds `tile` rows.
 template <bool TILES>
-__global__ __launch_bounds__(64) void merge(Args a) {
-  const int row = blockIdx.x / a.H, h = blockIdx.x - row * a.H, e = a.dvp / 64, lane = threadIdx.x;
+__global__ __launch_bounds__(TILES ? 256 : 64) void merge(Args a) {
+  const int unit = TILES ? 4 * blockIdx.x + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6) : blockIdx.x;
+  const int row = unit / a.H, h = unit - row * a.H, e = a.dvp / 64, lane = threadIdx.x & 63;
   long pr = (long)row * a.nsplit * a.H + h, brow, between = a.H;
   int nsplit = a.nsplit;
   if constexpr (TILES) {
@@ -413,6 +414,18 @@ __global__ __launch_bounds__(64) void merge(Args a) {
     between = (long)a.tile * a.H;
     nsplit = mt.w;
   } else brow = a.rows ? a.rows[row] : row;
+  const float* x = a.po + pr * a.dvp + lane * e;
+  const long step = between * a.dvp;
+  constexpr int CH = TILES ? 4 : 8;  // splits' loads at a time, the first ahead of the sums
+  float2 v[CH];
+  auto load = [&](int s0) {
+#pragma unroll
+    for (int j = 0; j < CH; ++j) {
+      const float* p = x + min(s0 + j, nsplit - 1) * step;
+      v[j] = e == 2 ? *(const float2*)p : make_float2(*p, 0.f);
+    }
+  };
+  load(0);
   float m = 0.f, l = 0.f;
   if (lane < nsplit) m = a.pml[2 * (pr + lane * between)], l = a.pml[2 * (pr + lane * between) + 1];
   float M = m;
@@ -420,18 +433,11 @@ __global__ __launch_bounds__(64) void merge(Args a) {
   for (int b = 1; b < 64; b <<= 1) M = fmaxf(M, __shfl_xor(M, b, 64));
   const float f = __builtin_amdgcn_exp2f(m - M);
   const float inv = 1.0f / (wave_sum(f * l) + __builtin_amdgcn_exp2f(-M));
-  const float* x = a.po + pr * a.dvp + lane * e;
-  const long step = between * a.dvp;
   float o0 = 0.f, o1 = 0.f;
-  for (int s0 = 0; s0 < nsplit; s0 += 8) {  // eight splits' loads at a time
-    float2 v[8];
+  for (int s0 = 0; s0 < nsplit; s0 += CH) {
+    if (s0) load(s0);
 #pragma unroll
-    for (int j = 0; j < 8; ++j) {
-      const float* p = x + min(s0 + j, nsplit - 1) * step;
-      v[j] = e == 2 ? *(const float2*)p : make_float2(*p, 0.f);
-    }
-#pragma unroll
-    for (int j = 0; j < 8; ++j) {
+    for (int j = 0; j < CH; ++j) {
       const float g = s0 + j < nsplit ? __shfl(f, s0 + j, 64) : 0.f;
       o0 += g * v[j].x;
       o1 += g * v[j].y;
@@ -1075,6 +1081,6 @@ KGS_EXPORT int kgs_talking_tiles(const void* q, long ldq, const void* pages, voi
   if (nmerge < 0 || (nmerge && (!merges || !po || !pml)) || (long)nmerge * a.tile * H > 0x7fffffff) return KGS_ERR_SHAPE;
   if (dkp == 64) dvp == 64 ? tiles_ns<2, 4>(a, nitems, nslot, s) : tiles_ns<2, 8>(a, nitems, nslot, s);
   else dvp == 64 ? tiles_ns<4, 4>(a, nitems, nslot, s) : tiles_ns<4, 8>(a, nitems, nslot, s);
-  if (nmerge) hipLaunchKernelGGL(merge<true>, dim3((unsigned)(nmerge * a.tile * H)), dim3(64), 0, s, a);
+  if (nmerge) hipLaunchKernelGGL(merge<true>, dim3((unsigned)(nmerge * a.tile / 4 * H)), dim3(256), 0, s, a);  // tile: whole 4s
   return (int)hipGetLastError();
 }
