@@ -190,12 +190,13 @@ MAX_PARTS = 64  # parts that one merge takes
 
 def tile_items(portions, tile: int) -> tuple[np.ndarray, np.ndarray]:
     """Items and merges of ``portions`` (first batch row, block-table row, position,
-    tokens). Blocks with more than an even share of all pages are split, so that a long
-    prompt's last blocks do not outlast the others: evenly where all items run at once,
-    else into such shares and a rest, which fill up the last round; the longest first."""
+    tokens). Blocks with more than 1.2 even shares of all pages are split, so that a long
+    prompt's last blocks do not outlast the others (a part costs a merge): evenly where
+    all items run at once,
+    else into such parts and a rest, which fill up the last round; the longest first."""
     b = np.array([(r + j, s, p + j, min(tile, n - j)) for r, s, p, n in portions for j in range(0, n, tile)], np.int64)
     pages = (b[:, 2] + b[:, 3] - 1) // PAGE + 1
-    share = max(MIN_PAGES, -(-int(pages.sum()) // CUS)) if len(b) < 2 * CUS else int(pages.max())
+    share = max(MIN_PAGES, -(-6 * int(pages.sum()) // (5 * CUS))) if len(b) < 2 * CUS else int(pages.max())
     cap = np.maximum(share, -(-pages // MAX_PARTS))
     parts = -(-pages // cap)
     split = parts > 1

@@ -78,9 +78,9 @@ class Geometry:
         pairs = n * (pos0 + 0.5 * n)
         return self.hd > 0 and n >= EXPAND_MIN and pos0 * self.rp * self.hd < (self.rp - self.hd) * pairs
 
-    def host_plan(self, pk: HostPack, row0, n, pos0, bt, row_seq, pos, refs):
-        """Splits the sequences between the absorbed and the expanded form and lays
-        out both launches; returns the plan's builder, to be called once ``pk`` is sent."""
+    def lay_out(self, pk: HostPack, row0, n, pos0, bt, row_seq, pos, refs):
+        """Splits the sequences between the absorbed and the expanded form and adds
+        both launches' arrays to ``pk``."""
         big = np.array([self.expand(int(x), int(p)) for x, p in zip(n, pos0)], bool)
         absorbed = expanded = None
         sel = np.flatnonzero(~big)
@@ -119,6 +119,11 @@ class Geometry:
             items = np.array(items, np.int64)
             items = items[np.argsort(-(items[:, 2] + items[:, 3]), kind="stable")]
             expanded = (pk.add(items), pk.add(np.concatenate(ctx)))
+        return absorbed, expanded
+
+    def host_plan(self, pk: HostPack, *layout):
+        """The builder of the plan, to be called once ``pk`` is sent."""
+        absorbed, expanded = self.lay_out(pk, *layout)
 
         def build(get):
             a = e = None

@@ -170,7 +170,7 @@ def test_state_slots_follow_random_traffic(chunk):
 
 # --------------------------------------------------------------------- plans
 def test_launch_plan_splits_portions_and_orders_rows():
-    from kgs.serve.hybrid import Geometry, HostPack, HybridModel
+    from kgs.serve.hybrid import Geometry, HostPack
 
     g = Geometry(heads=4, rp=256, hd=64)
     # behind a long context a portion is worth expanding from rp hd / (rp - hd) = 85 tokens on, at the start from 16
@@ -184,7 +184,7 @@ def test_launch_plan_splits_portions_and_orders_rows():
     pos = pos0[row_seq] + np.arange(n.sum()) - row0[row_seq]
     pk = HostPack(torch.device("cpu"))
     refs = [None] * 9
-    (r, shape), e = HybridModel._host_plan(pk, g, row0, n, pos0, bt, row_seq, pos, refs)
+    (r, shape), e = g.lay_out(pk, row0, n, pos0, bt, row_seq, pos, refs)
     get = pk.send()
     assert shape["nt"] == 4 and get(r["rows"]).tolist() == [300, 301, 302, 433]
     assert get(r["q0"]).tolist() == [0, 3] and get(r["n"]).tolist() == [3, 1]

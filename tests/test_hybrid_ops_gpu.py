@@ -141,7 +141,7 @@ def test_head_proj(dt, nt):
 def run_latent(q, c, lens, n, H, scale, dt, nsplit=None):
     """q [sum n, H, R], c [B][len, R]: the last n[b] positions of each sequence."""
     from kgs.ops.latent import LatentRows, latent_attention, padded_latent, split_count, waves_for
-    from kgs.serve.hybrid import Geometry, HostPack, HybridModel
+    from kgs.serve.hybrid import Geometry, HostPack
 
     R, rp = q.shape[2], padded_latent(q.shape[2])
     lens, n = np.asarray(lens), np.asarray(n)
@@ -157,7 +157,7 @@ def run_latent(q, c, lens, n, H, scale, dt, nsplit=None):
     pos = pos0[seq] + np.arange(n.sum()) - row0[seq]
     pk = HostPack(torch.device("cuda"))
     refs = [None] * 7 + [pk.add(bt), None]
-    (r, shape), _ = HybridModel._host_plan(pk, Geometry(H, rp, 0), row0, n, pos0, bt, seq, pos, refs)
+    (r, shape), _ = Geometry(H, rp, 0).lay_out(pk, row0, n, pos0, bt, seq, pos, refs)
     get = pk.send()
     if nsplit:
         shape["nsplit"] = nsplit
