@@ -61,7 +61,7 @@ def faults(lines: list[str]) -> list[str]:
     return bad
 
 
-def test_checker_sees_faults():
+def test_scan_sees_faults():
     ok = [" ;;#ASMSTART", " v_mfma_f32_16x16x32_bf16 a[0:3], v[0:3], v[4:7], a[0:3]", " s_nop 7", " s_nop 7", " s_nop 3",
           " v_accvgpr_read_b32 v0, a0", " ;;#ASMEND", " v_add_f32_e32 v0, v0, v1"]
     assert not faults(ok)
