@@ -31,6 +31,7 @@ ARCHITECTURES = {a.name: a for a in (
     Architecture("Llama", "kgs.models.llama:LlamaConfig", "kgs.serve.model:ServingModel"),
     Architecture("Ruruzen", "kgs.models.ruruzen:RuruzenConfig", "kgs.serve.hybrid:HybridModel"),
     Architecture("Nufusun", "kgs.models.nufusun:NufusunConfig", "kgs.serve.nufusun:NufusunModel"),
+    Architecture("Nokipel", "kgs.models.nokipel:NokipelConfig", "kgs.serve.nokipel:NokipelModel"),
 )}
 
 

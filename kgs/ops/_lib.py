@@ -83,12 +83,13 @@ _SIGS = {
     "kgs_skinny_gemm_bf16_ex": ([_c_void_p] * 5 + [_c_int] * 3 + [_c_long, _c_long] + [_c_int] * 3 + [_c_void_p],
                                 _c_int),
     "kgs_skinny_gemm_bf16_fused": ([_c_void_p] * 5 + [_c_int] * 3 + [_c_long, _c_long] + [_c_int] * 3 +
-                                   [_c_void_p] * 3 + [ctypes.c_float, ctypes.c_float, _c_void_p, _c_void_p], _c_int),
+                                   [_c_void_p] * 3 + [ctypes.c_float, ctypes.c_float, _c_void_p, ctypes.c_float,
+                                                      _c_void_p], _c_int),
     "kgs_skinny_variant_geometry": ([_c_int, _c_int] + [ctypes.POINTER(_c_int)] * 3, _c_int),
     "kgs_rope_cache_bf16": ([_c_void_p] * 6 + [_c_long, _c_int, _c_int, _c_int, _c_long, _c_int, _c_void_p, _c_int,
                                                   _c_void_p], _c_int),
     "kgs_gemm_bf16_nt_w4x_swiglu": ([_c_void_p] * 3 + [_c_int] * 8 + [_c_void_p], _c_int),
-    "kgs_gemm_bf16_nt_w4x_swiglu_ex": ([_c_void_p] * 3 + [_c_int] * 9 + [_c_void_p], _c_int),
+    "kgs_gemm_bf16_nt_w4x_swiglu_ex": ([_c_void_p] * 3 + [_c_int] * 9 + [_c_void_p] * 2, _c_int),
     "kgs_skinny_gemm_bf16_rope": ([_c_void_p] * 5 + [_c_int] * 3 + [_c_long, _c_long] + [_c_int] * 3 +
                                   [_c_void_p, ctypes.c_float, ctypes.c_float] + [_c_void_p] * 5 + [_c_int, _c_int,
                                                                                                   _c_void_p], _c_int),
@@ -105,7 +106,7 @@ _SIGS = {
     # hyper-connections, latent attention, delta rule (hyper.hip, latent.hip, delta.hip, activation.hip)
     "kgs_hyper_step": ([_c_void_p] * 7 + [_c_int] * 3 + [_c_long] * 2 + [ctypes.c_float, _c_int, _c_void_p], _c_int),
     "kgs_hyper_embed": ([_c_void_p] * 7 + [_c_int] * 3 + [_c_long] * 2 + [ctypes.c_float, _c_int, _c_void_p], _c_int),
-    "kgs_act_mul": ([_c_void_p] * 2 + [_c_int] * 2 + [_c_long] * 2 + [_c_int] * 2 + [_c_void_p], _c_int),
+    "kgs_act_mul": ([_c_void_p] * 2 + [_c_int] * 2 + [_c_long] * 2 + [_c_int, ctypes.c_float, _c_int, _c_void_p], _c_int),
     "kgs_softcap": ([_c_void_p] * 2 + [_c_int] * 2 + [_c_long, ctypes.c_float, _c_int, _c_void_p], _c_int),
     "kgs_latent_norm": ([_c_void_p, _c_long] + [_c_int] * 6 + [_c_void_p] * 5 + [_c_int, ctypes.c_float, _c_int,
                                                                                 _c_void_p], _c_int),
@@ -113,19 +114,32 @@ _SIGS = {
     "kgs_latent_attn": ([_c_void_p] * 10 + [_c_int] * 8 + [ctypes.c_float, _c_void_p], _c_int),
     # residual, talking-heads attention, mixture of experts (residual.hip, talking.hip, moe.hip)
     "kgs_residual_embed": ([_c_void_p] * 3 + [_c_long, ctypes.c_float] + [_c_void_p] * 2 + [_c_long, _c_void_p]
-                           + [_c_int] * 4 + [ctypes.c_float, _c_int, _c_void_p], _c_int),
+                           + [_c_int] * 5 + [ctypes.c_float] * 2 + [_c_int, _c_void_p], _c_int),
     "kgs_residual_add": ([_c_void_p] * 2 + [_c_long] + [_c_void_p] * 2 + [_c_long] * 2 + [_c_int] * 2
-                         + [_c_void_p, _c_int] + [_c_void_p] * 2 + [_c_long, _c_void_p] + [_c_int] * 4
-                         + [ctypes.c_float, _c_int, _c_void_p], _c_int),
-    "kgs_talking_write": ([_c_void_p, _c_long] + [_c_void_p] * 3 + [_c_int] * 8 + [_c_void_p], _c_int),
+                         + [_c_void_p, _c_int] + [_c_void_p, _c_long, _c_void_p] * 2
+                         + [_c_void_p] * 2 + [_c_long, ctypes.c_float] + [_c_void_p] * 2 + [_c_long, _c_void_p]
+                         + [_c_int] * 5 + [ctypes.c_float] * 2 + [_c_int, _c_void_p], _c_int),
+    "kgs_talking_write": ([_c_void_p, _c_long] + [_c_void_p] * 3 + [_c_int] * 7 + [_c_void_p] * 2 + [_c_int] * 3
+                          + [_c_void_p], _c_int),
     "kgs_talking_rows": ([_c_void_p, _c_long, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_int] + [_c_void_p] * 8
                          + [_c_int] * 10 + [_c_void_p], _c_int),
     "kgs_talking_tiles": ([_c_void_p, _c_long, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_int, _c_void_p, _c_int,
                            _c_void_p, _c_int] + [_c_void_p] * 7 + [_c_int] * 6 + [_c_void_p], _c_int),
     "kgs_moe_route": ([_c_void_p, _c_long] + [_c_void_p] * 6 + [_c_int] * 6 + [_c_void_p], _c_int),
+    "kgs_moe_route_softmax": ([_c_void_p, _c_long] + [_c_void_p] * 9 + [_c_int] * 5 + [ctypes.c_float] + [_c_int] * 4
+                              + [_c_void_p], _c_int),
     "kgs_moe_plan": ([_c_void_p] * 9 + [_c_int] * 4 + [_c_void_p], _c_int),
     "kgs_moe_grouped": ([_c_void_p, _c_long, _c_void_p, _c_void_p, _c_long] + [_c_void_p] * 4 + [_c_int] * 7
-                        + [ctypes.c_float] + [_c_int] * 2 + [_c_void_p], _c_int),
+                        + [ctypes.c_float] + [_c_int] * 3 + [_c_void_p], _c_int),
+    # softmax attention over head pages, lightning attention (paged.hip, lightning.hip)
+    "kgs_paged_rows": ([_c_void_p, _c_long, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_int] + [_c_void_p] * 5
+                       + [ctypes.c_float] + [_c_int] * 9 + [_c_void_p], _c_int),
+    "kgs_paged_tiles": ([_c_void_p, _c_long, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_int, _c_void_p, _c_int,
+                         ctypes.c_float] + [_c_int] * 5 + [_c_void_p], _c_int),
+    "kgs_lightning_forward": ([_c_void_p, _c_long] + [_c_int] * 3 + [_c_void_p] * 5 + [_c_int, _c_void_p] * 2
+                              + [_c_int, _c_void_p, _c_void_p, _c_int] + [_c_void_p] * 3 + [_c_int] * 4 + [_c_void_p], _c_int),
+    "kgs_lightning_out": ([_c_void_p] * 3 + [_c_long, _c_void_p, _c_long] + [_c_int] * 3 + [ctypes.c_float, _c_int,
+                                                                                             _c_void_p], _c_int),
     "kgs_latent_attn_simple": ([_c_void_p] * 6 + [_c_int] * 4 + [ctypes.c_float, _c_int, _c_void_p], _c_int),
     "kgs_attn_fwd_ragged_bf16": ([_c_void_p] * 5 + [_c_int] * 3 + [_c_long] * 4 + [ctypes.c_float, _c_void_p, _c_long,
                                                                                   _c_void_p], _c_int),

@@ -2,11 +2,40 @@
 bf16 or fp32: the gated feed-forward product and the logits' soft cap."""
 from __future__ import annotations
 
+from dataclasses import dataclass
+from functools import lru_cache
+
 import torch
 
 from . import _lib
 
-ACTS = {"silu": 0, "gelu_tanh": 1}
+ACTS = {"silu": 0, "gelu_tanh": 1, "clamped": 2}
+
+
+@dataclass(frozen=True)
+class Gate:
+    """How a gated feed-forward joins its two projections: ``silu(gate) * up``,
+    ``gelu_tanh(gate) * up``, or ``clamped``: ``g sigmoid(1.702 g) (u + 1)`` with
+    ``g = min(gate, limit)``, ``u = clamp(up, -limit, limit)``."""
+    act: str
+    limit: float = 0.0
+
+    def __post_init__(self):
+        if self.act not in ACTS:
+            raise ValueError(f"unknown gate activation {self.act!r}")
+
+    @classmethod
+    def of(cls, act) -> "Gate":
+        return act if isinstance(act, Gate) else cls(act)
+
+    def limit_ptr(self, device) -> int:
+        """The limit on the device, for epilogues that read it there (0: none)."""
+        return _limit(self.limit, str(device)).data_ptr() if self.act == "clamped" else 0
+
+
+@lru_cache(maxsize=None)
+def _limit(limit: float, device: str) -> torch.Tensor:
+    return torch.tensor([limit], dtype=torch.float32, device=device)
 
 
 def _mat(t: torch.Tensor, name: str) -> None:
@@ -14,12 +43,14 @@ def _mat(t: torch.Tensor, name: str) -> None:
         raise ValueError(f"{name} must be a row-major bf16 or fp32 GPU matrix")
 
 
-def act_mul(gu: torch.Tensor, act: str) -> torch.Tensor:
-    """``act(gu[:, :n]) * gu[:, n:]`` for a fused gate|up output of width 2n."""
+def act_mul(gu: torch.Tensor, act) -> torch.Tensor:
+    """``act(gu[:, :n]) * gu[:, n:]`` for a fused gate|up output of width 2n (``act``: a
+    name or a :class:`Gate`)."""
     _mat(gu, "gu")
+    gate = Gate.of(act)
     rows, n = gu.shape[0], gu.shape[1] // 2
     out = torch.empty((rows, n), dtype=gu.dtype, device=gu.device)
-    rc = _lib.lib().kgs_act_mul(gu.data_ptr(), out.data_ptr(), rows, n, gu.stride(0), n, ACTS[act],
+    rc = _lib.lib().kgs_act_mul(gu.data_ptr(), out.data_ptr(), rows, n, gu.stride(0), n, ACTS[gate.act], float(gate.limit),
                                 int(gu.dtype == torch.float32), _lib.stream_handle(gu.device))
     _lib.check(rc, f"act_mul[{rows}x{n}]")
     return out

@@ -26,6 +26,7 @@ import os
 import torch
 
 from . import _lib
+from .activation import Gate
 
 PAGE = 32
 HEAD_DIM = 128
@@ -84,7 +85,7 @@ class PackedWeight:
     """A projection weight in skinny-GEMM fragment order (plus its shape).
 
     * ``swiglu=True``: a fused gate|up weight whose GEMM emits ``act(g) * u``
-      (``act``: ``"silu"`` or ``"gelu_tanh"``);
+      (``act``: ``"silu"``, ``"gelu_tanh"`` or a :class:`kgs.ops.activation.Gate`);
     * ``fold``: an RMSNorm weight ``[K]`` folded into the columns (``W * fold``),
       for GEMMs that apply the norm in their epilogue (``rms=``);
     * ``fp8=True``: weight-only fp8 (W8A16): OCP e4m3 with one scale per output
@@ -96,11 +97,9 @@ class PackedWeight:
     __slots__ = ("data", "n", "k", "swiglu", "fp8", "wscale", "rope", "act")
 
     def __init__(self, w: torch.Tensor, swiglu: bool = False, fold: torch.Tensor | None = None, fp8: bool = False,
-                 rope: tuple | None = None, act: str = "silu"):
+                 rope: tuple | None = None, act="silu"):
         self.n, self.k = w.shape
-        if act not in ("silu", "gelu_tanh"):
-            raise ValueError(f"unknown gate activation {act!r}")
-        self.act = act
+        self.act = Gate.of(act)
         self.swiglu, self.fp8, self.rope = swiglu, fp8, rope
         if swiglu and rope:
             raise ValueError("a weight is either SwiGLU- or RoPE-packed")
@@ -391,7 +390,8 @@ def _workspace(device: torch.device, floats: int, ints: int):
     return ws, cnt
 
 
-EPI_SWIGLU, EPI_RMS, EPI_RESID, EPI_GELU = 1, 2, 4, 16
+EPI_SWIGLU, EPI_RMS, EPI_RESID, EPI_GELU, EPI_CLAMPED = 1, 2, 4, 16, 32
+GATE_EPI = {"silu": 0, "gelu_tanh": EPI_GELU, "clamped": EPI_CLAMPED}
 
 
 def skinny_gemm(x: torch.Tensor, w: PackedWeight, out: torch.Tensor | None = None,
@@ -430,7 +430,7 @@ def skinny_gemm(x: torch.Tensor, w: PackedWeight, out: torch.Tensor | None = Non
     rps, kpc, mpad = skinny_geometry(m, variant)
     if w.n % rps or k % kpc:
         raise ValueError(f"skinny GEMM needs N % {rps} == 0 and K % {kpc} == 0 (N={w.n}, K={k})")
-    epi = (EPI_SWIGLU | (EPI_GELU if w.act == "gelu_tanh" else 0) if w.swiglu else 0) | (EPI_RMS if rms is not None else 0) | \
+    epi = (EPI_SWIGLU | GATE_EPI[w.act.act] if w.swiglu else 0) | (EPI_RMS if rms is not None else 0) | \
         (EPI_RESID if resid_ss is not None else 0)
     for t, name in ((rms, "rms"), (resid_ss, "resid_ss"), (zero, "zero")):
         if t is not None and (t.dtype != torch.float32 or t.numel() < m or not t.is_contiguous()):
@@ -465,7 +465,7 @@ def skinny_gemm(x: torch.Tensor, w: PackedWeight, out: torch.Tensor | None = Non
         w.data.data_ptr(), x.data_ptr(), out.data_ptr(), ws.data_ptr(), cnt.data_ptr(), m, w.n, k, x.stride(0),
         out.stride(0), ks, variant, epi, rms.data_ptr() if rms is not None else None,
         resid_ss.data_ptr() if resid_ss is not None else None, zero.data_ptr() if zero is not None else None,
-        1.0 / k, float(eps), w.wscale.data_ptr() if w.fp8 else None, _lib.stream_handle(x.device))
+        1.0 / k, float(eps), w.wscale.data_ptr() if w.fp8 else None, w.act.limit, _lib.stream_handle(x.device))
     _lib.check(rc, f"skinny_gemm[{m}x{w.n}x{k}, variant={variant}, ksplit={ks}, epi={epi}, fp8={w.fp8}]")
     return out
 

@@ -176,7 +176,7 @@ def pack_w4x_weight(w: torch.Tensor, bn: int, swiglu: bool = False) -> PanelWeig
     return PanelWeight(data, N, K, bn, swiglu)
 
 
-GATE_FLAGS = {"silu": 0, "gelu_tanh": 0x40}
+GATE_FLAGS = {"silu": 0, "gelu_tanh": 0x40, "clamped": 0x80}
 
 
 def _w4x_flags(packed: int, stages: int, nt_weights: bool = False) -> int:
@@ -301,9 +301,9 @@ def gemm_nt_w4x_partials(a: torch.Tensor, b, bn: int, nslice: int, bm: int = 256
 
 def gemm_nt_w4x_swiglu(a: torch.Tensor, w_gate_up, bn: int = 128,
                        out: torch.Tensor | None = None, bm: int = 256, stages: int = 2,
-                       nt_weights: bool = False, act: str = "silu") -> torch.Tensor:
-    """``act(a @ gate.T) * (a @ up.T)`` (``act``: silu, or gelu_tanh with a row-major
-    weight and two stages) for a fused gate|up weight ``[2I, K]``
+                       nt_weights: bool = False, act="silu") -> torch.Tensor:
+    """``act(a @ gate.T) * (a @ up.T)`` (``act``: silu, or gelu_tanh or a clamped
+    :class:`kgs.ops.activation.Gate` with a row-major weight and two stages) for a fused gate|up weight ``[2I, K]``
     (gate rows first) on the four-wave kernel, the SwiGLU applied in the GEMM
     epilogue: returns ``[M, I]`` (both products rounded to bf16 first, as
     ``gemm_nt`` + ``kgs.ops.transformer.silu_mul`` round them). Any M;
@@ -319,9 +319,13 @@ def gemm_nt_w4x_swiglu(a: torch.Tensor, w_gate_up, bn: int = 128,
         raise ValueError(f"inner dims differ: a {tuple(a.shape)} w {tuple(wshape)}")
     if out is None:
         out = torch.empty((M, N // 2), dtype=torch.bfloat16, device=a.device)
+    from .activation import Gate
+
+    gate = Gate.of(act)
     rc = _lib.lib().kgs_gemm_bf16_nt_w4x_swiglu_ex(a.data_ptr(), w.data_ptr(), out.data_ptr(), M, N, K,
                                                    a.stride(0), ldb, out.stride(0), int(bn), int(bm),
-                                                   _w4x_flags(packed, stages, nt_weights) | GATE_FLAGS[act],
+                                                   _w4x_flags(packed, stages, nt_weights) | GATE_FLAGS[gate.act],
+                                                   gate.limit_ptr(a.device),
                                                    _lib.stream_handle(a.device))
     _lib.check(rc, f"gemm_nt_w4x_swiglu[{M}x{N}x{K} {bm}x{bn}]")
     return out
@@ -352,16 +356,16 @@ def swiglu_fused_ok(a: torch.Tensor, w: torch.Tensor) -> bool:
             and a.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0 and a.shape[1] == K)
 
 
-def gemm_swiglu(a: torch.Tensor, w_gate_up: torch.Tensor, act: str = "silu") -> torch.Tensor:
+def gemm_swiglu(a: torch.Tensor, w_gate_up: torch.Tensor, act="silu") -> torch.Tensor:
     """Gated MLP input projection ``act(a @ gate.T) * (a @ up.T)`` -> ``[M, I]``:
     fused into the four-wave GEMM's epilogue (256x256 tiles; 256x128 when
     ``2I % 256 != 0``) when the shape allows, else GEMM + the elementwise product.
     Same bits either way (silu)."""
     if swiglu_fused_ok(a, w_gate_up):
         return gemm_nt_w4x_swiglu(a, w_gate_up, bn=256 if w_gate_up.shape[0] % 256 == 0 else 128, act=act)
-    if act != "silu":
-        from .activation import act_mul
+    from .activation import Gate, act_mul
 
+    if Gate.of(act).act != "silu":
         return act_mul(gemm_nt(a, w_gate_up), act)
     from .transformer import silu_mul
 

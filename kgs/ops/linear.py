@@ -5,7 +5,8 @@
 over a prepacked weight for small decode batches, split-K four-wave tiles for
 larger ones, the 256x256 pipeline for prompts, the library GEMM for shapes the
 kernels do not take. A gated projection (fused gate|up weight) applies
-``act(gate) * up`` in the epilogue where one exists. fp32 runs on the library's
+``act(gate) * up`` (``act``: a name or a :class:`kgs.ops.activation.Gate`) in the
+epilogue where one exists. fp32 runs on the library's
 true fp32 GEMM.
 """
 from __future__ import annotations
@@ -13,6 +14,7 @@ from __future__ import annotations
 import torch
 
 from . import decode as D
+from .activation import Gate
 
 SKINNY_MAX_ROWS = 32   # untuned shapes: skinny GEMM up to here
 SPLIT_MAX_ROWS = 512   # four-wave split-K tiles up to here
@@ -38,8 +40,10 @@ class Projection:
     ``w = [gate; up]``. ``pack``: keep a second copy of the weight in the skinny
     GEMM's order for decode."""
 
-    def __init__(self, w: torch.Tensor, gated: str | None = None, pack: bool = True):
-        self.w, self.gated = w.contiguous(), gated
+    def __init__(self, w: torch.Tensor, gated=None, pack: bool = True):
+        self.w, self.gated = w.contiguous(), None if gated is None else Gate.of(gated)
+        if gated is not None and w.is_cuda:
+            self.gated.limit_ptr(w.device)  # on the device before any hipGraph capture
         n, k = w.shape
         # every default skinny tile: 64 or 128 rows of w, 8 or 16 k-steps of 32
         fits = n % 128 == 0 and k % 512 == 0

@@ -219,17 +219,37 @@ def split_count(n: int, max_pages: int) -> int:
     return max(1, min(2 * CUS // max(1, n), -(-max_pages // 4), 64))
 
 
+class Rotary:
+    """Rotary positions of the pairs (0, 1), (2, 3), .. of each head's first ``dims`` dims:
+    the pair i turns by ``position * base ** (-2 i / dims)``. ``table`` fp32 ``[positions,
+    dims padded to 8]``: cos and sin of each pair."""
+
+    def __init__(self, dims: int, base: float, positions: int, device):
+        p = torch.arange(positions, dtype=torch.float64)[:, None]
+        a = p * base ** (-torch.arange(0, dims, 2, dtype=torch.float64) / dims)
+        t = torch.stack([a.cos(), a.sin()], -1).reshape(positions, dims)
+        if dims % 8:  # the pad's pairs stay as they are
+            t = torch.cat([t, torch.tensor([1.0, 0.0], dtype=torch.float64).repeat(positions, (8 - dims % 8) // 2)], 1)
+        self.table = t.float().to(device).contiguous()
+
+
 def write_kv(z: torch.Tensor, bias: torch.Tensor, pages: torch.Tensor, slots: torch.Tensor, h: Heads, ok: int,
-             ov: int) -> None:
+             ov: int, rotary: Rotary | None = None, pos: torch.Tensor | None = None) -> None:
     """``z [T, >=]`` holds q (columns 0 ..), k (``ok`` ..) and v (``ov`` ..), heads padded.
     Adds the biases (``bias``: q, k, v one after another): q in place, k and v into
-    ``pages`` at ``slots`` (-1: dropped)."""
+    ``pages`` at ``slots`` (-1: dropped). ``rotary``: q and k turned by the rows' ``pos``
+    (int32 ``[T]``)."""
     T, nq, nk, nv = z.shape[0], h.heads * h.dkp, h.kv_heads * h.dkp, h.kv_heads * h.dvp
     if pages.dtype != z.dtype or not pages.is_contiguous() or pages.shape[1:] != (h.kv_heads, PAGE * (h.dkp + h.dvp)):
         raise ValueError(f"pages {tuple(pages.shape)} {pages.dtype} do not fit {h}")
+    turn = (0, 0, 0, 0)
+    if rotary is not None:
+        if pos is None or pos.dtype != torch.int32 or not pos.is_contiguous() or pos.shape[0] != T:
+            raise ValueError("rotary positions need contiguous int32 positions of the rows")
+        turn = (rotary.table.data_ptr(), pos.data_ptr(), *rotary.table.shape)
     rc = _lib.lib().kgs_talking_write(_act(z, T, max(nq, ok + nk, ov + nv), z.dtype, "z"), z.stride(0),
                                       _f32(bias, (nq + nk + nv,), "bias"), pages.data_ptr(), slots.data_ptr(), T, nq,
-                                      h.kv_heads, h.dkp, h.dvp, ok, ov, int(z.dtype == torch.float32),
+                                      h.kv_heads, h.dkp, h.dvp, ok, ov, *turn, int(z.dtype == torch.float32),
                                       _lib.stream_handle(z.device))
     _lib.check(rc, f"talking_write[{T}]")
 

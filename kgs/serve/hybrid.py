@@ -260,7 +260,7 @@ class HybridModel(RaggedModel):
             raise ValueError(f"streams {cfg.streams} is above {MAX_STREAMS}")
         super().__init__()
         self.cfg, self.device, self.dtype = cfg, torch.device(device), DTYPES[dtype]
-        self.has_state = cfg.has_state
+        self.has_state = self.delta_chunks = cfg.has_state
         self.wp = padk(cfg.width)
         raw = weights if weights is not None else cfg.load_weights(seed, self.device)
         w = Weights(raw, self.device, self.dtype, packed_decode)

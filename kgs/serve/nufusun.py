@@ -21,24 +21,16 @@ import torch
 from kgs.models.nufusun import AttentionSpec, ExpertsSpec, NufusunConfig
 from kgs.ops import decode as D
 from kgs.ops import moe as M
-from kgs.ops.activation import softcap
+from kgs.ops.activation import Gate, softcap
 from kgs.ops.decode import PAGE
-from kgs.ops.residual import MAX_WIDTH, ExpertRows, residual_add, residual_embed
+from kgs.ops.residual import MAX_WIDTH, ExpertRows, Norm, residual_add, residual_embed
 from kgs.ops.talking import (HeadPages, Heads, QueryRows, QueryTiles, TalkingWeights, attention_rows,
                              attention_tiles, heads_of, split_count, tile_items, write_kv)
 
-from .ragged import DTYPES, Batch, HostPack, RaggedModel, Weights, _pad, pad64
+from .ragged import DTYPES, Batch, HostPack, RaggedModel, Weights, _pad, pad64, pad128, pad256
 from .trace import TRACE as T
 
 TILE_MIN = 16  # shorter portions run row by row
-
-
-def pad256(n: int) -> int:
-    return (n + 255) // 256 * 256
-
-
-def pad128(n: int) -> int:
-    return (n + 127) // 128 * 128
 
 
 def attention_heads(m: AttentionSpec, dtype) -> Heads:
@@ -139,22 +131,17 @@ class ExpertsFF:
     def __init__(self, model, i: int, m: ExpertsSpec, w: Weights, counts: torch.Tensor):
         p, wp, fp = f"l{i}.mlp.", model.wp, pad128(m.ff)
         self.layer, self.m, self.counts = i, m, counts
-        self.router = w.mat(p + "router", self._router_rows(m.experts), wp).contiguous()
+        self.router = w.mat(p + "router", M.router_rows(m.experts), wp).contiguous()
         self.gate_up = torch.stack([torch.cat([w.mat(f"{p}e{e}.{n}", fp, wp) for n in ("gate", "up")])
                                     for e in range(m.experts)])
         self.down = torch.stack([w.mat(f"{p}e{e}.down", wp, fp) for e in range(m.experts)])
-
-    @staticmethod
-    def _router_rows(n: int) -> int:
-        """Experts padded to a size the MFMA router has (above 64: any multiple of 16)."""
-        return next((s for s in (16, 32, 64) if s >= n), (n + 15) // 16 * 16)
 
     def __call__(self, model, h: torch.Tensor, b: Batch) -> ExpertRows:
         m = self.m
         c = M.route(h, self.router, self.counts, m.top, b.slots)
         p = M.plan(c, M.tile_rows(h.shape[0], m.top, m.experts, h.dtype))
         T.op(f"L{self.layer} router")
-        y = M.down(M.gate_up(h, self.gate_up, p, m.limit), self.down, p)
+        y = M.down(M.gate_up(h, self.gate_up, p, Gate("clamped", m.limit)), self.down, p)
         T.op(f"L{self.layer} experts")
         return ExpertRows(y, p.pos)
 
@@ -215,11 +202,12 @@ class NufusunModel(RaggedModel):
     def forward(self, b: Batch) -> torch.Tensor:
         """Runs the batch; fp32 logits ``[rows wanted, vocab]``."""
         cfg = self.cfg
-        x, h = residual_embed(b.tokens, self.embed, cfg.embed_scale, self.norms[0], cfg.width, cfg.eps, zero=self.counts)
+        norm = Norm(cfg.width, cfg.eps)
+        x, h = residual_embed(b.tokens, self.embed, cfg.embed_scale, self.norms[0], norm, zero=self.counts)
         for i, (mixer, ff) in enumerate(self.layers):
             a = mixer(self, h, b)
             e = None if ff is None else ff(self, h, b)
-            h = residual_add(x, a, mixer.o_bias, e, self.norms[i + 1], cfg.width, cfg.eps, self.dtype)
+            h = residual_add(x, a, mixer.o_bias, e, self.norms[i + 1], norm, self.dtype)
             T.op(f"L{i} residual")
             if self.on_layer is not None:
                 self.on_layer(i, x[:, :cfg.width])

@@ -28,6 +28,14 @@ def pad64(n: int) -> int:
     return (n + 63) // 64 * 64
 
 
+def pad128(n: int) -> int:
+    return (n + 127) // 128 * 128
+
+
+def pad256(n: int) -> int:
+    return (n + 255) // 256 * 256
+
+
 def padk(n: int) -> int:
     """Padded size of a GEMM's inner dimension: the MFMA GEMMs step by 128, which a
     small one is not padded to."""
@@ -73,6 +81,7 @@ class Batch:
     seqs: RaggedSeqs
     plans: dict                # attention geometry -> its launch plan
     logit_rows: torch.Tensor | None  # rows whose logits are wanted (None: every row)
+    pos: torch.Tensor | None = None  # [T] int32 position of each row
 
 
 # --------------------------------------------------------------------- weights
@@ -82,7 +91,7 @@ class Weights:
     def __init__(self, w: dict, device, dtype, pack: bool):
         self.w, self.device, self.dtype, self.pack = w, device, dtype, pack
 
-    def proj(self, t: torch.Tensor, gated: str | None = None) -> Projection:
+    def proj(self, t: torch.Tensor, gated=None) -> Projection:
         return Projection(t, gated, pack=self.pack)
 
     def f32(self, name: str) -> torch.Tensor:
@@ -116,6 +125,7 @@ class RaggedModel:
     ragged = True
     pad_multiple = 1  # portions are not padded
     has_state = False
+    delta_chunks = False  # batches carry the delta rule's split into chunks
 
     def __init__(self):
         self._fixed: dict = {}
@@ -165,13 +175,14 @@ class RaggedModel:
         row_seq = np.repeat(order, n[order])
         pos = pos0[row_seq] + np.arange(len(tokens)) - row0[row_seq]
         refs = [pk.add(a) for a in (tokens, slots, row_seq, row0, n, pos0, slot, bt, logit_rows, pos)]
-        split = {k: pk.add(v) for k, v in chunk_plan(row0, n, pos0, slot).items()} if self.has_state else {}
+        split = {k: pk.add(v) for k, v in chunk_plan(row0, n, pos0, slot).items()} if self.delta_chunks else {}
         host = {g: g.host_plan(pk, row0, n, pos0, bt, row_seq, pos, refs) for g in self.geometries}
         get = pk.send()
         d = [get(r) for r in refs]
         plans = {g: build(get) for g, build in host.items()}
         return Batch(dev_tokens.to(torch.int32).contiguous() if dev_tokens is not None else d[0], d[1],
-                     RaggedSeqs(d[2], d[3], d[4], d[5], d[6], **{k: get(r) for k, r in split.items()}), plans, d[8].long())
+                     RaggedSeqs(d[2], d[3], d[4], d[5], d[6], **{k: get(r) for k, r in split.items()}), plans, d[8].long(),
+                     d[9])
 
     # ------------------------------------------------------------------- decode
     def _fixed_seqs(self, nb: int) -> dict:
@@ -187,4 +198,4 @@ class RaggedModel:
         f = self._fixed_seqs(nb)
         plans = {g: g.decode_plan(f, nb, positions, block_tables) for g in self.geometries}
         seqs = RaggedSeqs(f["ar"], f["ar"], f["one"], positions, state_slots if self.has_state else f["zero"])
-        return self.forward(Batch(tokens, slots, seqs, plans, None))
+        return self.forward(Batch(tokens, slots, seqs, plans, None, positions))

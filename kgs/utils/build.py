@@ -166,7 +166,7 @@ def targets(out: Path | None = None) -> list[Target]:
             HIPCC,
             flags=HIP_FLAGS + ["-fvisibility=hidden", f"-I{kdir}"],
             headers=k_headers,
-            source_flags={"latent.hip": MFMA_IN_VGPRS, "delta.hip": MFMA_IN_VGPRS, "talking.hip": MFMA_IN_VGPRS},
+            source_flags={f: MFMA_IN_VGPRS for f in ("latent.hip", "delta.hip", "talking.hip", "paged.hip", "lightning.hip")},
         ),
         Target(
             "gpuprobe",

@@ -1,12 +1,12 @@
 // Elementwise steps around the projections, for any width and for bf16 or fp32
-// activations: the gated feed-forward product act(gate) * up from one fused
-// gate|up row, and the tanh soft cap of the logits.
+// activations: the gated feed-forward product act(gate) * up (or the clamped gate) from
+// one fused gate|up row, and the tanh soft cap of the logits.
 #include "kgs_common.h"
 
 namespace kgs {
 namespace act {
 
-enum { ACT_SILU = 0, ACT_GELU_TANH = 1 };
+enum { ACT_SILU = 0, ACT_GELU_TANH = 1, ACT_CLAMPED = 2 };
 
 template <int ACT>
 __device__ __forceinline__ float f(float z) {
@@ -15,15 +15,22 @@ __device__ __forceinline__ float f(float z) {
 }
 
 template <int ACT>
-__global__ __launch_bounds__(256) void mul_f32(const float* gu, float* o, int n, long ldi, long ldo) {
+__global__ __launch_bounds__(256) void mul_f32(const float* gu, float* o, int n, long ldi, long ldo, float limit) {
   const long r = blockIdx.y;
   const int c = blockIdx.x * 256 + threadIdx.x;
-  if (c < n) o[r * ldo + c] = f<ACT>(gu[r * ldi + c]) * gu[r * ldi + n + c];
+  if (c >= n) return;
+  float g = gu[r * ldi + c], u = gu[r * ldi + n + c];
+  if constexpr (ACT == ACT_CLAMPED) {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    o[r * ldo + c] = g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
+  } else o[r * ldo + c] = f<ACT>(g) * u;
 }
 
 // 8 columns per thread (n % 8 == 0, 16-B rows)
 template <int ACT>
-__global__ __launch_bounds__(256) void mul_bf16(const unsigned short* gu, unsigned short* o, int n, long ldi, long ldo) {
+__global__ __launch_bounds__(256) void mul_bf16(const unsigned short* gu, unsigned short* o, int n, long ldi, long ldo,
+                                                float limit) {
   const long r = blockIdx.y;
   const int c = (blockIdx.x * 256 + threadIdx.x) * 8;
   if (c >= n) return;
@@ -31,8 +38,8 @@ __global__ __launch_bounds__(256) void mul_bf16(const unsigned short* gu, unsign
   float v[8];
 #pragma unroll
   for (int i = 0; i < 8; ++i) {
-    const float z = bf2f((unsigned short)g[i]);
-    v[i] = (ACT == ACT_GELU_TANH ? gelu_tanh(z) : f<ACT>(z)) * bf2f((unsigned short)u[i]);
+    const float z = bf2f((unsigned short)g[i]), y = bf2f((unsigned short)u[i]);
+    v[i] = ACT == ACT_CLAMPED ? gate_clamped(z, y, limit) : (ACT == ACT_GELU_TANH ? gelu_tanh(z) : f<ACT>(z)) * y;
   }
   *(bf16x8*)(o + r * ldo + c) = pack_bf16x8(v, 0);
 }
@@ -52,23 +59,23 @@ __global__ __launch_bounds__(256) void softcap(const T* x, float* o, int n, long
 }  // namespace act
 }  // namespace kgs
 
-KGS_EXPORT int kgs_act_mul(const void* gu, void* o, int rows, int n, long ldi, long ldo, int act, int f32,
-                           hipStream_t s) {
+KGS_EXPORT int kgs_act_mul(const void* gu, void* o, int rows, int n, long ldi, long ldo, int act, float limit,
+                           int f32, hipStream_t s) {
   using namespace kgs::act;
   if (rows <= 0 || rows > 65535 * 16 || n <= 0 || ldi < 2l * n || ldo < n) return KGS_ERR_SHAPE;
-  if (act != ACT_SILU && act != ACT_GELU_TANH) return KGS_ERR_ARG;
+  if (act < ACT_SILU || act > ACT_CLAMPED) return KGS_ERR_ARG;
   if (!f32 && (n % 8 || ldi % 8 || ldo % 8 || (((uintptr_t)gu | (uintptr_t)o) & 15))) return KGS_ERR_ALIGN;
   const long per = 65535;
   for (long r0 = 0; r0 < rows; r0 += per) {
     const unsigned nr = (unsigned)(rows - r0 < per ? rows - r0 : per);
     if (f32) {
-      auto k = act == ACT_SILU ? mul_f32<ACT_SILU> : mul_f32<ACT_GELU_TANH>;
+      auto k = act == ACT_SILU ? mul_f32<ACT_SILU> : act == ACT_CLAMPED ? mul_f32<ACT_CLAMPED> : mul_f32<ACT_GELU_TANH>;
       hipLaunchKernelGGL(k, dim3((n + 255) / 256, nr), dim3(256), 0, s, (const float*)gu + r0 * ldi,
-                         (float*)o + r0 * ldo, n, ldi, ldo);
+                         (float*)o + r0 * ldo, n, ldi, ldo, limit);
     } else {
-      auto k = act == ACT_SILU ? mul_bf16<ACT_SILU> : mul_bf16<ACT_GELU_TANH>;
+      auto k = act == ACT_SILU ? mul_bf16<ACT_SILU> : act == ACT_CLAMPED ? mul_bf16<ACT_CLAMPED> : mul_bf16<ACT_GELU_TANH>;
       hipLaunchKernelGGL(k, dim3((n / 8 + 255) / 256, nr), dim3(256), 0, s, (const unsigned short*)gu + r0 * ldi,
-                         (unsigned short*)o + r0 * ldo, n, ldi, ldo);
+                         (unsigned short*)o + r0 * ldo, n, ldi, ldo, limit);
     }
   }
   return (int)hipGetLastError();

@@ -118,7 +118,7 @@ struct SkinnyCfg {
 //               paged cache slot slot[m] -- the rope_cache launch, folded in.
 // Together they remove both add_rmsnorm launches, the SwiGLU launch and the
 // RoPE / KV-write launch from a decode layer (kgs/serve/model.py fused path).
-enum { EPI_SWIGLU = 1, EPI_RMS = 2, EPI_RESID = 4, EPI_ROPE = 8, EPI_GELU = 16 };
+enum { EPI_SWIGLU = 1, EPI_RMS = 2, EPI_RESID = 4, EPI_ROPE = 8, EPI_GELU = 16, EPI_CLAMPED = 32 };
 struct SkinnyEpi {
   int mode;
   const float* ss_in;
@@ -126,6 +126,7 @@ struct SkinnyEpi {
   float* ss_zero;
   float inv_k, eps;
   const float* wscale;  // W8: per packed row dequant scale
+  float limit;          // EPI_CLAMPED
   // EPI_ROPE
   const float* cosv;
   const float* sinv;
@@ -363,7 +364,8 @@ __global__ __launch_bounds__(256, (MT * KC_ > 32 || R * MT >= 16) ? 1 : 2) void 
         f32x4v o;
 #pragma unroll
         for (int i = 0; i < 4; ++i)
-          o[i] = ((ep.mode & EPI_GELU) ? gate_act<GATE_GELU>(v[i]) : gate_act<GATE_SILU>(v[i])) * u[i];
+          o[i] = (ep.mode & EPI_CLAMPED) ? gate_clamped(v[i], u[i], ep.limit)
+                 : ((ep.mode & EPI_GELU) ? gate_act<GATE_GELU>(v[i]) : gate_act<GATE_SILU>(v[i])) * u[i];
         uint2 pk;
         pk.x = pack_bf16x2(o[0], o[1]);
         pk.y = pack_bf16x2(o[2], o[3]);
@@ -1155,16 +1157,18 @@ KGS_EXPORT int kgs_skinny_geometry(int M, int* rows_per_strip, int* k_per_chunk,
 namespace {
 int skinny_fused(const void* wp, const void* x, void* y, float* ws, int* cnt, int M, int N, int K, long ldx, long ldy,
                  int ksplit, int variant, int epi, const float* ss_in, float* ss_out, float* ss_zero, float inv_k,
-                 float eps, const float* wscale, const kgs::dec::SkinnyEpi* rope, hipStream_t s);
+                 float eps, const float* wscale, const kgs::dec::SkinnyEpi& rope, hipStream_t s);
 }
 
 KGS_EXPORT int kgs_skinny_gemm_bf16_fused(const void* wp, const void* x, void* y, float* ws, int* cnt, int M, int N,
                                          int K, long ldx, long ldy, int ksplit, int variant, int epi,
                                          const float* ss_in, float* ss_out, float* ss_zero, float inv_k, float eps,
-                                         const float* wscale, hipStream_t s) {
+                                         const float* wscale, float limit, hipStream_t s) {
   if (epi & kgs::dec::EPI_ROPE) return KGS_ERR_ARG;  // kgs_skinny_gemm_bf16_rope
+  kgs::dec::SkinnyEpi ep{};
+  ep.limit = limit;
   return skinny_fused(wp, x, y, ws, cnt, M, N, K, ldx, ldy, ksplit, variant, epi, ss_in, ss_out, ss_zero, inv_k, eps,
-                      wscale, nullptr, s);
+                      wscale, ep, s);
 }
 
 // The fused qkv projection with RoPE + the KV-cache write in its epilogue
@@ -1190,21 +1194,22 @@ KGS_EXPORT int kgs_skinny_gemm_bf16_rope(const void* wp, const void* x, void* y,
   r.H = H;
   r.HKV = HKV;
   return skinny_fused(wp, x, y, ws, cnt, M, N, K, ldx, ldy, ksplit, variant, epi | EPI_ROPE, ss_in, nullptr, nullptr,
-                      inv_k, eps, nullptr, &r, s);
+                      inv_k, eps, nullptr, r, s);
 }
 
 namespace {
 int skinny_fused(const void* wp, const void* x, void* y, float* ws, int* cnt, int M, int N, int K, long ldx, long ldy,
                  int ksplit, int variant, int epi, const float* ss_in, float* ss_out, float* ss_zero, float inv_k,
-                 float eps, const float* wscale, const kgs::dec::SkinnyEpi* rope, hipStream_t s) {
+                 float eps, const float* wscale, const kgs::dec::SkinnyEpi& rope, hipStream_t s) {
   using namespace kgs::dec;
   int rps, kpc, mpad;
   const int rc = kgs_skinny_variant_geometry(variant, M, &rps, &kpc, &mpad);
   if (rc) return rc;
   if (variant == 0) variant = default_variant(mt_for(M));
-  if (epi & ~(EPI_SWIGLU | EPI_RMS | EPI_RESID | EPI_ROPE | EPI_GELU) || ((epi & EPI_GELU) && !(epi & EPI_SWIGLU)) || ((epi & EPI_SWIGLU) && (epi & EPI_RESID)))
+  if (epi & ~(EPI_SWIGLU | EPI_RMS | EPI_RESID | EPI_ROPE | EPI_GELU | EPI_CLAMPED) ||
+      ((epi & (EPI_GELU | EPI_CLAMPED)) && !(epi & EPI_SWIGLU)) || ((epi & EPI_SWIGLU) && (epi & EPI_RESID)))
     return KGS_ERR_ARG;
-  if ((epi & EPI_ROPE) && (rope == nullptr || (epi & (EPI_SWIGLU | EPI_RESID)) || wscale != nullptr))
+  if ((epi & EPI_ROPE) && (rope.cache == nullptr || (epi & (EPI_SWIGLU | EPI_RESID)) || wscale != nullptr))
     return KGS_ERR_ARG;
   if (((epi & EPI_RMS) && ss_in == nullptr) || ((epi & EPI_RESID) && ss_out == nullptr)) return KGS_ERR_ARG;
   if (N <= 0 || K <= 0 || N % rps || K % kpc || ldx < K || ldy < ((epi & EPI_SWIGLU) ? N / 2 : N))
@@ -1214,7 +1219,7 @@ int skinny_fused(const void* wp, const void* x, void* y, float* ws, int* cnt, in
   if (ksplit > 1 && (ws == nullptr || cnt == nullptr)) return KGS_ERR_ARG;
   if (!al16(wp) || !al16(x) || ((uintptr_t)y & 7) || ((uintptr_t)ws & 15) || ldx % 8 || ldy % 4) return KGS_ERR_ALIGN;
   const int cps = nchunks / ksplit;
-  SkinnyEpi ep = rope ? *rope : SkinnyEpi{};
+  SkinnyEpi ep = rope;
   ep.mode = epi;
   ep.ss_in = ss_in;
   ep.ss_out = ss_out;
@@ -1249,7 +1254,7 @@ int skinny_fused(const void* wp, const void* x, void* y, float* ws, int* cnt, in
 KGS_EXPORT int kgs_skinny_gemm_bf16_ex(const void* wp, const void* x, void* y, float* ws, int* cnt, int M, int N,
                                       int K, long ldx, long ldy, int ksplit, int variant, int epi, hipStream_t s) {
   return kgs_skinny_gemm_bf16_fused(wp, x, y, ws, cnt, M, N, K, ldx, ldy, ksplit, variant, epi, nullptr, nullptr,
-                                    nullptr, 0.f, 0.f, nullptr, s);
+                                    nullptr, 0.f, 0.f, nullptr, 0.f, s);
 }
 
 KGS_EXPORT int kgs_skinny_gemm_bf16_v(const void* wp, const void* x, void* y, float* ws, int* cnt, int M, int N, int K,

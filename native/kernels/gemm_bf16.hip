@@ -167,7 +167,8 @@ static int cu_count() {
 
 // gemm_persistent.hip
 hipError_t launch_w4p_swiglu(const unsigned short* A, const unsigned short* B, unsigned short* C, int M, int N,
-                             int K, int lda, int ldb, int ldc, int cus, int* tq, bool gelu, hipStream_t s);
+                             int K, int lda, int ldb, int ldc, int cus, int* tq, int act, const float* limit,
+                             hipStream_t s);
 template <int EPI>
 hipError_t launch_w4p(const unsigned short* A, const unsigned short* B, unsigned short* C, const unsigned short* bias,
                       int M, int N, int K, int lda, int ldb, int ldc, int cus, int* tq, hipStream_t s);
@@ -740,23 +741,31 @@ int launch_w4x(dim3 grid, hipStream_t s, const unsigned short* a, const unsigned
 
 template <int BN, int TM, int X>
 void launch_w4sw_x(dim3 grid, hipStream_t s, const unsigned short* a, const unsigned short* b, unsigned short* c,
-                   int M, int N, int K, int lda, int ldb, int ldc, bool aligned_m) {
+                   int M, int N, int K, int lda, int ldb, int ldc, bool aligned_m,
+                   const unsigned short* limit = nullptr) {
   using namespace kgs;
   constexpr int BM = w4::tile_m<TM>();
   using Kn = w4::Knobs<BM, BN>;
   if (aligned_m)
     hipLaunchKernelGGL((w4::gemm_nt_w4<EPI_NONE, BN, TM, Kn::B1, Kn::R, Kn::P, Kn::ORD, X>), grid, dim3(256), 0, s, a,
-                       b, c, nullptr, M, N, K, lda, ldb, ldc);
+                       b, c, limit, M, N, K, lda, ldb, ldc);
   else
     hipLaunchKernelGGL((w4::gemm_nt_w4<EPI_NONE, BN, TM | 1, Kn::B1, Kn::R, Kn::P, Kn::ORD, X>), grid, dim3(256), 0, s,
-                       a, b, c, nullptr, M, N, K, lda, ldb, ldc);
+                       a, b, c, limit, M, N, K, lda, ldb, ldc);
 }
 
 template <int BN, int TM>
 int launch_w4sw(dim3 grid, hipStream_t s, const unsigned short* a, const unsigned short* b, unsigned short* c, int M,
-                int N, int K, int lda, int ldb, int ldc, bool aligned_m, int flags) {
+                int N, int K, int lda, int ldb, int ldc, bool aligned_m, int flags, const float* limit) {
   constexpr int BM = kgs::w4::tile_m<TM>();
   const bool packed = flags & 1;
+  if (flags & 0x80) {  // clamped: row-major weights, two LDS stages
+    if (flags & 0x31) return KGS_ERR_ARG;
+    const auto lim = (const unsigned short*)limit;
+    if (flags & 2) launch_w4sw_x<BN, TM, 4005200>(grid, s, a, b, c, M, N, K, lda, ldb, ldc, aligned_m, lim);
+    else launch_w4sw_x<BN, TM, 4000000>(grid, s, a, b, c, M, N, K, lda, ldb, ldc, aligned_m, lim);
+    return 0;
+  }
   if (flags & 0x40) {  // tanh gelu: row-major weights, two LDS stages
     if (flags & 0x31) return KGS_ERR_ARG;
     if (flags & 2) launch_w4sw_x<BN, TM, 2005200>(grid, s, a, b, c, M, N, K, lda, ldb, ldc, aligned_m);
@@ -848,22 +857,26 @@ KGS_EXPORT int kgs_gemm_bf16_nt_w4x_ex(const void* A, const void* B, void* C, fl
 // M; tiles bm x bn (256 / 128 each); N % bn == 0, K % 128 == 0, lda/ldb/ldc % 8,
 // 16-B aligned pointers.
 KGS_EXPORT int kgs_gemm_bf16_nt_w4x_swiglu_ex(const void* A, const void* B, void* C, int M, int N, int K, int lda,
-                                              int ldb, int ldc, int bn, int bm, int flags, hipStream_t stream);
+                                              int ldb, int ldc, int bn, int bm, int flags, const void* limit,
+                                              hipStream_t stream);
 
 KGS_EXPORT int kgs_gemm_bf16_nt_w4x_swiglu(const void* A, const void* B, void* C, int M, int N, int K, int lda,
                                            int ldb, int ldc, int bn, int bm, hipStream_t stream) {
-  return kgs_gemm_bf16_nt_w4x_swiglu_ex(A, B, C, M, N, K, lda, ldb, ldc, bn, bm, 0, stream);
+  return kgs_gemm_bf16_nt_w4x_swiglu_ex(A, B, C, M, N, K, lda, ldb, ldc, bn, bm, 0, nullptr, stream);
 }
 
 // flags bit 0: B is the SwiGLU-packed copy of the fused gate|up weight
 // (kgs.ops.gemm.pack_w4x_weight(..., swiglu=True)), ldb must be K; bits 4-5:
-// LDS stages - 2 (as kgs_gemm_bf16_nt_w4x_ex); bit 6: tanh gelu instead of silu
-// (row-major B, two stages)
+// LDS stages - 2 (as kgs_gemm_bf16_nt_w4x_ex); bit 6: tanh gelu instead of silu;
+// bit 7: the clamped gate with the limit at `limit` (fp32, on the device); both with
+// row-major B, two stages
 KGS_EXPORT int kgs_gemm_bf16_nt_w4x_swiglu_ex(const void* A, const void* B, void* C, int M, int N, int K, int lda,
-                                              int ldb, int ldc, int bn, int bm, int flags, hipStream_t stream) {
+                                              int ldb, int ldc, int bn, int bm, int flags, const void* limit,
+                                              hipStream_t stream) {
   using namespace kgs;
-  if (flags & ~0x73 || (flags & 0x30) == 0x30) return KGS_ERR_ARG;
-  const bool gelu = flags & 0x40;
+  if (flags & ~0xf3 || (flags & 0x30) == 0x30 || (flags & 0xc0) == 0xc0) return KGS_ERR_ARG;
+  if ((flags & 0x80) && (!limit || (uintptr_t)limit % 4)) return KGS_ERR_ARG;
+  const int act = flags & 0x80 ? GATE_CLAMPED : flags & 0x40 ? GATE_GELU : GATE_SILU;
   if ((flags & 1) && ldb != K) return KGS_ERR_SHAPE;
   if (M <= 0 || N <= 0 || K <= 0 || lda < K || ldb < K || ldc < N / 2) return KGS_ERR_SHAPE;
   if ((bn != 128 && bn != 256) || (bm != 128 && bm != 256)) return KGS_ERR_ARG;
@@ -877,19 +890,19 @@ KGS_EXPORT int kgs_gemm_bf16_nt_w4x_swiglu_ex(const void* A, const void* B, void
   const bool aligned_m = M % bm == 0;
   // prompt-pass shapes (256 x 256 tiles, aligned M, more tiles than CUs): the
   // persistent kernel with the same K-step (bitwise the one-shot result)
-  if (bm == 256 && bn == 256 && aligned_m && (flags & ~0x40) == 0 && K >= 384 && (long)(M / 256) * (N / 256) > cu_count()) {
+  if (bm == 256 && bn == 256 && aligned_m && (flags & ~0xc0) == 0 && K >= 384 && (long)(M / 256) * (N / 256) > cu_count()) {
     if (int* tq = tile_queue(stream)) {
-      const hipError_t e = launch_w4p_swiglu(a, b, c, M, N, K, lda, ldb, ldc, cu_count(), tq, gelu, stream);
+      const hipError_t e = launch_w4p_swiglu(a, b, c, M, N, K, lda, ldb, ldc, cu_count(), tq, act, (const float*)limit, stream);
       return e == hipSuccess ? 0 : (int)e;
     }
   }
   int rc;
   if (bm == 256) {
-    if (bn == 256) rc = launch_w4sw<256, 0>(grid, stream, a, b, c, M, N, K, lda, ldb, ldc, aligned_m, flags);
-    else rc = launch_w4sw<128, 0>(grid, stream, a, b, c, M, N, K, lda, ldb, ldc, aligned_m, flags);
+    if (bn == 256) rc = launch_w4sw<256, 0>(grid, stream, a, b, c, M, N, K, lda, ldb, ldc, aligned_m, flags, (const float*)limit);
+    else rc = launch_w4sw<128, 0>(grid, stream, a, b, c, M, N, K, lda, ldb, ldc, aligned_m, flags, (const float*)limit);
   } else {
-    if (bn == 256) rc = launch_w4sw<256, 8>(grid, stream, a, b, c, M, N, K, lda, ldb, ldc, aligned_m, flags);
-    else rc = launch_w4sw<128, 8>(grid, stream, a, b, c, M, N, K, lda, ldb, ldc, aligned_m, flags);
+    if (bn == 256) rc = launch_w4sw<256, 8>(grid, stream, a, b, c, M, N, K, lda, ldb, ldc, aligned_m, flags, (const float*)limit);
+    else rc = launch_w4sw<128, 8>(grid, stream, a, b, c, M, N, K, lda, ldb, ldc, aligned_m, flags, (const float*)limit);
   }
   if (rc) return rc;
   return (int)hipGetLastError();

@@ -57,10 +57,13 @@ hipError_t launch_w4p(const unsigned short* A, const unsigned short* B, unsigned
 // gate|up, with the one-shot SwiGLU kernel's K-step and tile order (X 1000000),
 // so the result is bitwise the one-shot kernel's
 hipError_t launch_w4p_swiglu(const unsigned short* A, const unsigned short* B, unsigned short* C, int M, int N,
-                             int K, int lda, int ldb, int ldc, int cus, int* tq, bool gelu, hipStream_t s) {
+                             int K, int lda, int ldb, int ldc, int cus, int* tq, int act, const float* limit, hipStream_t s) {
   const int tiles = (M / 256) * (N / 256);
   const dim3 pg(tiles < cus ? tiles : cus);
-  if (gelu)
+  if (act == GATE_CLAMPED)
+    hipLaunchKernelGGL((w4p::gemm_nt_w4p<EPI_NONE, 4000000>), pg, dim3(256), 0, s, A, B, C,
+                       (const unsigned short*)limit, M, N, K, lda, ldb, ldc, tq);
+  else if (act == GATE_GELU)
     hipLaunchKernelGGL((w4p::gemm_nt_w4p<EPI_NONE, 2000000>), pg, dim3(256), 0, s, A, B, C, nullptr, M, N, K, lda, ldb,
                        ldc, tq);
   else

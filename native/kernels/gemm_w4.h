@@ -573,8 +573,11 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     return;
   }
   if constexpr (SW) {
-    // out fragment q (16 columns) = act(gate fragment ng) * up fragment ng + 2 (SW 1: silu, 2: tanh gelu),
+    // out fragment q (16 columns) = act(gate fragment ng) * up fragment ng + 2 (SW 1: silu, 2: tanh gelu,
+    // 4: clamped, its limit where the bias would be),
     // ng = 4 (q / 2) + q % 2; pairs (q, q + 1) share one 16-B store per lane
+    constexpr int ACT = (X / 1000000) % 10;
+    const float limit = ACT == GATE_CLAMPED ? *(const float*)bias : 0.f;
     static_for<0, MA>([&](auto ic) {
       constexpr int i = decltype(ic)::value;
       const int row = tm * BM + c.wr * (BM / 2) + i * 16 + fr;
@@ -591,10 +594,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
           const f32x4 g = v[ng], u = v[ng + 2];
           float r[4];
 #pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            const float gf = bf2f(f2bf(g[e]));
-            r[e] = gate_act<(X / 1000000) % 10>(gf) * bf2f(f2bf(u[e]));
-          }
+          for (int e = 0; e < 4; ++e) r[e] = gated<ACT>(g[e], u[e], limit);
           o[h].x = pack_bf16x2(r[0], r[1]);
           o[h].y = pack_bf16x2(r[2], r[3]);
         }

@@ -417,35 +417,34 @@ __device__ __forceinline__ void pepi_addc(const Ctx& c, unsigned short* __restri
 // alternating 32-row DMA groups, so a wave's fragment columns ng = 0, 1, 4, 5
 // are gate and ng + 2 the matching up columns; output fragment pair (QQ, QQ + 1)
 // = silu(gate) * up (tanh gelu with digit 2) of fragments ng(QQ), ng(QQ + 1), both products rounded to
-// bf16 first (the roundings of GEMM + silu_mul). C is [M, N / 2].
+// bf16 first (the roundings of GEMM + silu_mul); digit 4: the clamped gate, its limit where the bias
+// would be. C is [M, N / 2].
 template <int Q, int ACT>
-__device__ __forceinline__ uint2 swiglu4() {
+__device__ __forceinline__ uint2 swiglu4(float limit) {
   constexpr int i = Q / NB, qh = Q % NB, ng = 4 * (qh / 2) + qh % 2;
   const f32x4 g = accr::read<i * NB + ng>(), u = accr::read<i * NB + ng + 2>();
   float r[4];
 #pragma unroll
-  for (int e = 0; e < 4; ++e) {
-    const float gf = bf2f(f2bf(g[e]));
-    r[e] = gate_act<ACT>(gf) * bf2f(f2bf(u[e]));
-  }
+  for (int e = 0; e < 4; ++e) r[e] = gated<ACT>(g[e], u[e], limit);
   return make_uint2(pack_bf16x2(r[0], r[1]), pack_bf16x2(r[2], r[3]));
 }
 
 template <int I, int QQ, int ACT>
-__device__ __forceinline__ void pepi_sw(const Ctx& c, unsigned short* __restrict__ C, int ldc, int tm, int tn) {
+__device__ __forceinline__ void pepi_sw(const Ctx& c, unsigned short* __restrict__ C, int ldc, int tm, int tn,
+                                        float limit) {
   if constexpr (I < MA) {
     if constexpr (QQ < NB / 2) {
       const int lane = threadIdx.x & 63, fr = lane & 15, fq = lane >> 4;
-      const uint2 o0 = swiglu4<I * NB + QQ, ACT>(), o1 = swiglu4<I * NB + QQ + 1, ACT>();
+      const uint2 o0 = swiglu4<I * NB + QQ, ACT>(limit), o1 = swiglu4<I * NB + QQ + 1, ACT>(limit);
       auto sx = __builtin_amdgcn_permlane16_swap(o0.x, o1.x, false, false);
       auto sy = __builtin_amdgcn_permlane16_swap(o0.y, o1.y, false, false);
       const uint4 qv = make_uint4(sx[0], sy[0], sx[1], sy[1]);
       const int row = tm * BM + c.wr * (BM / 2) + I * 16 + fr;
       const int col0 = tn * (BN / 2) + c.wc * (BN / 4) + QQ * 16;
       *(uint4*)(C + (long)row * ldc + col0 + (fq & 1) * 16 + (fq >> 1) * 8) = qv;
-      pepi_sw<I, QQ + 2, ACT>(c, C, ldc, tm, tn);
+      pepi_sw<I, QQ + 2, ACT>(c, C, ldc, tm, tn, limit);
     } else {
-      pepi_sw<I + 1, 0, ACT>(c, C, ldc, tm, tn);
+      pepi_sw<I + 1, 0, ACT>(c, C, ldc, tm, tn, limit);
     }
   }
 }
@@ -681,7 +680,10 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     pstep<0, X, false, 0, L, 0, 2>(c, cn, f0, f1, more ? 0 : nt - 1, tq);
     pstep<1, X, false, 0, L, 0, 2>(c, cn, f0, f1, more ? 1 : nt - 1, tq);
     asm volatile("s_nop 7\n\ts_nop 7\n\ts_nop 3" ::: "memory");  // MFMA -> v_accvgpr_read
-    if constexpr (SW) pepi_sw<0, 0, (X / 1000000) % 10>(c, C, ldc, tm, tn);
+    if constexpr (SW) {
+      constexpr int ACT = (X / 1000000) % 10;
+      pepi_sw<0, 0, ACT>(c, C, ldc, tm, tn, ACT == GATE_CLAMPED ? *(const float*)bias : 0.f);
+    }
     float bv[NB][4];
     if constexpr (!SW) {
       const int fq = lane >> 4;

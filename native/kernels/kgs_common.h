@@ -174,12 +174,28 @@ __device__ __forceinline__ float gelu_tanh(float x) {
   return 0.5f * x * (1.0f + t);
 }
 
-// activation of a gated feed-forward's gate: 1 silu, 2 tanh gelu
-enum GateAct { GATE_SILU = 1, GATE_GELU = 2 };
+// activation of a gated feed-forward: 1 silu, 2 tanh gelu of the gate, times up;
+// 4 the clamped gate (3: the grouped GEMMs' digit for gathered rows)
+enum GateAct { GATE_SILU = 1, GATE_GELU = 2, GATE_CLAMPED = 4 };
 template <int ACT>
 __device__ __forceinline__ float gate_act(float g) {
   if constexpr (ACT == GATE_GELU) return gelu_tanh(g);
   return g / (1.0f + __expf(-g));
+}
+
+// min(g, limit) sigmoid(1.702 min(g, limit)) (clamp(u) + 1)
+__device__ __forceinline__ float gate_clamped(float g, float u, float limit) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g / (1.0f + __expf(-1.702f * g)) * (u + 1.0f);
+}
+
+// a GEMM epilogue's gated product; silu and gelu take both factors rounded to bf16,
+// as a separate pass over the GEMM's output would
+template <int ACT>
+__device__ __forceinline__ float gated(float g, float u, float limit) {
+  if constexpr (ACT == GATE_CLAMPED) return gate_clamped(g, u, limit);
+  return gate_act<ACT>(bf2f(f2bf(g))) * bf2f(f2bf(u));
 }
 
 template <int EPI>

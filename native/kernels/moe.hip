@@ -3,7 +3,10 @@
 //   route    router logits (bf16: MFMA with fp32 sums; fp32: plain dot products), the
 //            `top` largest per token and their sigmoid weights, and each choice's rank
 //            among the tokens of its expert (counted in LDS per 16 tokens, one global
-//            add per expert and workgroup)
+//            add per expert and workgroup). The other choice: softmax scores, chosen by
+//            score + correction within the best groups of neighbours, weights normalised;
+//            outputs past the experts return the input (their weights' sum is put out)
+//            and one more router row can be a shared expert's gate
 //   plan     a prefix over the experts' counts turns ranks into rows of the sorted
 //            order: row -> token and weight, choice -> row, and the GEMM tiles
 //            (expert, first row, rows)
@@ -13,8 +16,9 @@
 //            epilogue; down reads the sorted rows. Neither reads anything back on the
 //            host: the grid covers the most tiles there can be and the rest leaves.
 //
-// A weight scales its expert's input. Both projections of an expert are linear in
-// it, so it multiplies their fp32 sums, before the clamps.
+// A weight scales its expert's input or its output. Both projections of an expert are
+// linear in the input, so there it multiplies their fp32 sums, before the clamps; down is
+// linear too, so a weight of the output multiplies the gated product in fp32.
 #include "gemm_w4.h"
 #include "kgs_common.h"
 
@@ -33,6 +37,12 @@ struct RouteArgs {
   int* rank;          // [T, top]
   float* weight;      // [T, top]
   int T, E, ep, wp, top;
+  // softmax scores: E experts and `extra` outputs that return the input
+  const float* corr;  // [E + extra], or null: sigmoid scores, nothing below is used
+  float* ident;       // [T] sum of the weights of the extra outputs a token chose, or null
+  float* gate;        // [T] sigmoid of router row E + extra, or null
+  int extra, groups, keep;
+  float scale;
 };
 
 __device__ __forceinline__ float rcp_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
@@ -91,6 +101,123 @@ __device__ __forceinline__ void choose(const RouteArgs& a, float* z, int zs, int
     }
 }
 
+__device__ __forceinline__ float row_max(float v) {  // over the 16 lanes of a DPP row
+  v = fmaxf(v, dpp_move<0x128>(v));
+  v = fmaxf(v, dpp_move<0x124>(v));
+  v = fmaxf(v, dpp_move<0x122>(v));
+  return fmaxf(v, dpp_move<0x121>(v));
+}
+__device__ __forceinline__ float row_sum(float v) {
+  v += dpp_move<0x128>(v);
+  v += dpp_move<0x124>(v);
+  v += dpp_move<0x122>(v);
+  return v + dpp_move<0x121>(v);
+}
+
+// The same for softmax scores (p: [16][zs], scratch): work [16][groups + 2 top] after the E counters
+__device__ __forceinline__ void choose_softmax(const RouteArgs& a, float* z, float* p, int zs, int* lh, int t0) {
+  const int tid = threadIdx.x, tk = tid >> 4, n = tid & 15, nt = blockDim.x, EA = a.E + a.extra;
+  float* best_of = (float*)(lh + a.E);           // [16][groups]
+  float* lw = best_of + RT * a.groups;           // [16][top]
+  int* lid = (int*)(lw + RT * a.top);            // [16][top]
+  for (int e = tid; e < a.E; e += nt) lh[e] = 0;
+  __syncthreads();
+  const int t = t0 + tk, per = EA / a.groups;
+  const bool on = tid < 256, real = on && t < a.T && (!a.slots || a.slots[t] >= 0);
+  float* row = z + tk * zs;
+  float* pr = p + tk * zs;
+  if (on) {
+    float m = -INFINITY, s = 0.f;
+    for (int e = n; e < EA; e += 16) m = fmaxf(m, row[e]);
+    m = row_max(m);
+    for (int e = n; e < EA; e += 16) s += pr[e] = expf(row[e] - m);
+    s = row_sum(s);
+    for (int e = n; e < EA; e += 16) {
+      pr[e] /= s;
+      row[e] = pr[e] + a.corr[e];  // choice score
+    }
+  }
+  __syncthreads();
+  if (a.keep < a.groups) {
+    if (on)
+      for (int g = n; g < a.groups; g += 16) {
+        float b = row[g * per];
+        for (int i = 1; i < per; ++i) b = fmaxf(b, row[g * per + i]);
+        best_of[tk * a.groups + g] = b;
+      }
+    __syncthreads();
+    if (on)
+      for (int g = n; g < a.groups; g += 16) {
+        const float b = best_of[tk * a.groups + g];
+        int ahead = 0;
+        for (int j = 0; j < a.groups; ++j) {
+          const float o = best_of[tk * a.groups + j];
+          ahead += o > b || (o == b && j < g);
+        }
+        if (ahead >= a.keep)
+          for (int i = 0; i < per; ++i) row[g * per + i] = __uint_as_float(0x7fc00000u);  // compares false
+      }
+    __syncthreads();
+  }
+  if (on) {
+    float sum = 0.f;
+    for (int k = 0; k < a.top; ++k) {
+      float best = -INFINITY;
+      int be = 0x7fffffff;
+      for (int e = n; e < EA; e += 16) {
+        const float v = row[e];
+        if (v > best || (be == 0x7fffffff && v == best)) best = v, be = e;
+      }
+      better<0x128>(best, be);
+      better<0x124>(best, be);
+      better<0x122>(best, be);
+      better<0x121>(best, be);
+      const bool ok = be < EA;
+      const float s = ok ? pr[be] : 0.f;
+      if (ok && (be & 15) == n) row[be] = __uint_as_float(0x7fc00000u);
+      sum += s;
+      if (n == 0) {
+        lid[tk * a.top + k] = ok ? be : -1;
+        lw[tk * a.top + k] = s;
+      }
+    }
+    if (n == 0) best_of[tk * a.groups] = a.scale / (sum + 1e-20f);
+  }
+  __syncthreads();
+  for (int i = tid; i < RT * a.top; i += nt) {
+    const int k = i / a.top, tt = t0 + k;
+    if (tt >= a.T) continue;
+    const int e = lid[i];
+    const bool ok = e >= 0 && e < a.E && (!a.slots || a.slots[tt] >= 0);
+    const long o = (long)tt * a.top + (i - k * a.top);
+    a.ids[o] = ok ? e : -1;
+    a.weight[o] = lw[i] * best_of[k * a.groups];
+    a.rank[o] = ok ? atomicAdd(&lh[e], 1) : 0;
+  }
+  if (on && n == 0 && t < a.T) {
+    if (a.ident) {
+      float w = 0.f;
+      for (int k = 0; k < a.top; ++k)
+        if (lid[tk * a.top + k] >= a.E) w += lw[tk * a.top + k];
+      a.ident[t] = real ? w * best_of[tk * a.groups] : 0.f;
+    }
+    if (a.gate) a.gate[t] = rcp_sigmoid(row[EA]);
+  }
+  __syncthreads();
+  for (int e = tid; e < a.E; e += nt) {  // local ranks -> ranks among all tokens
+    const int c = lh[e];
+    if (c) lh[e] = atomicAdd(&a.counts[e], c);
+  }
+  __syncthreads();
+  for (int i = tid; i < RT * a.top; i += nt) {  // the thread that wrote it
+    const int k = i / a.top, tt = t0 + k;
+    if (tt >= a.T) continue;
+    const long o = (long)tt * a.top + (i - k * a.top);
+    const int e = a.ids[o];
+    if (e >= 0) a.rank[o] += lh[e];
+  }
+}
+
 // bf16: eight waves split the width, ET 16-expert MFMA tiles each, U steps' loads at a time
 template <int ET>
 __global__ __launch_bounds__(512) void route_mfma(RouteArgs a) {
@@ -136,7 +263,9 @@ __global__ __launch_bounds__(512) void route_mfma(RouteArgs a) {
     for (int j = 1; j < 8; ++j) s += part[j * RT * zs + i];
     z[i] = s;
   }
-  choose(a, z, zs, lh, t0);  // begins with a barrier
+  // both begin with a barrier
+  if (a.corr) choose_softmax(a, z, part, zs, lh, t0);
+  else choose(a, z, zs, lh, t0);
 }
 
 template <typename T>
@@ -144,9 +273,11 @@ __global__ __launch_bounds__(256) void route_plain(RouteArgs a) {
   extern __shared__ float lds[];
   const int zs = a.ep + 1, t0 = blockIdx.x * RT, tk = threadIdx.x >> 4, n = threadIdx.x & 15;
   float* z = lds;
-  int* lh = (int*)(lds + RT * zs);
+  float* p = lds + RT * zs;
+  int* lh = (int*)(a.corr ? p + RT * zs : p);
+  const int nrow = a.E + a.extra + (a.gate ? 1 : 0);
   const T* hp = (const T*)a.h + (long)min(t0 + tk, a.T - 1) * a.ldh;
-  for (int e = 0; e < a.E; ++e) {
+  for (int e = 0; e < nrow; ++e) {
     const T* wr = (const T*)a.w + (long)e * a.wp;
     float s = 0.f;
     for (int k = n; k < a.wp; k += 16) {
@@ -158,7 +289,8 @@ __global__ __launch_bounds__(256) void route_plain(RouteArgs a) {
     if (n == 0) z[tk * zs + e] = s;
   }
   __syncthreads();
-  choose(a, z, zs, lh, t0);
+  if (a.corr) choose_softmax(a, z, p, zs, lh, t0);
+  else choose(a, z, zs, lh, t0);
 }
 
 struct PlanArgs {
@@ -217,13 +349,14 @@ struct GroupedArgs {
   long lda;
   int T, P, N, K, ldc, nslice;
   float limit;
+  int act;             // ACT_*
 };
 
-// min(g, limit) sigmoid(1.702 min(g, limit)) (clamp(u) + 1)
-__device__ __forceinline__ float gate_clamped(float g, float u, float limit) {
-  g = fminf(g, limit);
-  u = fminf(fmaxf(u, -limit), limit);
-  return g / (1.0f + __expf(-1.702f * g)) * (u + 1.0f);
+// the clamped gate of a weighted input; silu(gate) up, the product weighted
+enum { ACT_CLAMPED = 0, ACT_SILU = 1 };
+__device__ __forceinline__ float gated_weighted(float g, float u, float w, const GroupedArgs& a) {
+  if (a.act == ACT_SILU) return gate_act<GATE_SILU>(g) * u * w;
+  return gate_clamped(g * w, u * w, a.limit);
 }
 
 // GATED: gate|up with gathered rows and the gated epilogue; else the down projection,
@@ -339,7 +472,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
           if constexpr (GATED) {
             const int ng = 4 * ((n + h) / 2) + (n + h) % 2;
 #pragma unroll
-            for (int e = 0; e < 4; ++e) r[e] = gate_clamped(v[ng][e] * rw, v[ng + 2][e] * rw, a.limit);
+            for (int e = 0; e < 4; ++e) r[e] = gated_weighted(v[ng][e], v[ng + 2][e], rw, a);
           } else {
 #pragma unroll
             for (int e = 0; e < 4; ++e) r[e] = v[n + h][e];
@@ -404,8 +537,11 @@ __global__ __launch_bounds__(256) void grouped_f32(GroupedArgs a) {
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       if constexpr (GATED) {
-        const float gg = fminf(g[i][j] * rw, a.limit), uu = fminf(fmaxf(u[i][j] * rw, -a.limit), a.limit);
-        cp[j] = gg / (1.0f + expf(-1.702f * gg)) * (uu + 1.0f);
+        if (a.act == ACT_SILU) cp[j] = g[i][j] / (1.0f + expf(-g[i][j])) * u[i][j] * rw;
+        else {
+          const float gg = fminf(g[i][j] * rw, a.limit), uu = fminf(fmaxf(u[i][j] * rw, -a.limit), a.limit);
+          cp[j] = gg / (1.0f + expf(-1.702f * gg)) * (uu + 1.0f);
+        }
       } else cp[j] = g[i][j];
     }
   }
@@ -413,8 +549,32 @@ __global__ __launch_bounds__(256) void grouped_f32(GroupedArgs a) {
 
 template <int ET>
 int launch_route(const RouteArgs& a, size_t lds, hipStream_t s) {
-  hipLaunchKernelGGL((route_mfma<ET>), dim3((a.T + RT - 1) / RT), dim3(512), lds + 8 * RT * (a.ep + 1) * 4, s, a);
+  const size_t all = lds + 8 * RT * (a.ep + 1) * 4;
+  if (all > 64 * 1024) return KGS_ERR_SHAPE;
+  hipLaunchKernelGGL((route_mfma<ET>), dim3((a.T + RT - 1) / RT), dim3(512), all, s, a);
   return (int)hipGetLastError();
+}
+
+template <typename T>
+int launch_plain(const RouteArgs& a, size_t lds, hipStream_t s) {
+  if (lds > 160 * 1024) return KGS_ERR_SHAPE;
+  if (lds > 64 * 1024) {
+    const hipError_t e = hipFuncSetAttribute((const void*)route_plain<T>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    if (e != hipSuccess) return (int)e;
+  }
+  hipLaunchKernelGGL(route_plain<T>, dim3((a.T + RT - 1) / RT), dim3(256), lds, s, a);
+  return (int)hipGetLastError();
+}
+
+int route(const RouteArgs& a, int f32, hipStream_t s) {
+  const int zs = a.ep + 1;
+  const size_t work = a.corr ? (size_t)RT * (a.groups + 2 * a.top) * 4 : 0;
+  const size_t lds = ((size_t)RT * zs + a.E) * 4 + work, plain = lds + (a.corr ? (size_t)RT * zs * 4 : 0);
+  if (f32) return launch_plain<float>(a, plain, s);
+  if (a.ep <= 16) return launch_route<1>(a, lds, s);
+  if (a.ep <= 32) return launch_route<2>(a, lds, s);
+  if (a.ep == 64) return launch_route<4>(a, lds, s);
+  return launch_plain<unsigned short>(a, plain, s);
 }
 
 }  // namespace moe
@@ -430,15 +590,28 @@ KGS_EXPORT int kgs_moe_route(const void* h, long ldh, const void* w, const void*
     return KGS_ERR_SHAPE;
   if (ldh % 8 || (((uintptr_t)h | (uintptr_t)w) & 15)) return KGS_ERR_ALIGN;
   RouteArgs a{h, ldh, w, (const int*)slots, (int*)counts, (int*)ids, (int*)rank, (float*)weight, T, E, ep, wp, top};
-  const size_t lds = (RT * (ep + 1) + E) * 4;
-  if (lds > 64 * 1024) return KGS_ERR_SHAPE;
-  const dim3 grid((T + RT - 1) / RT);
-  if (f32) hipLaunchKernelGGL(route_plain<float>, grid, dim3(256), lds, s, a);
-  else if (ep <= 16) return launch_route<1>(a, lds, s);
-  else if (ep <= 32) return launch_route<2>(a, lds, s);
-  else if (ep == 64) return launch_route<4>(a, lds, s);
-  else hipLaunchKernelGGL(route_plain<unsigned short>, grid, dim3(256), lds, s, a);
-  return (int)hipGetLastError();
+  return route(a, f32, s);
+}
+
+// The same with softmax scores over E experts and `extra` outputs that return their
+// input: the `top` largest of score + corr [E + extra] among the best `keep` of `groups`
+// groups of neighbours (by their largest), weights scale s / (sum s + 1e-20). ids -1 also
+// for an extra output; ident [T]: the sum of a token's weights of those. gate [T]:
+// sigmoid of router row E + extra. ident and gate may be null.
+KGS_EXPORT int kgs_moe_route_softmax(const void* h, long ldh, const void* w, const void* slots, void* counts, void* ids,
+                                     void* rank, void* weight, const void* corr, void* ident, void* gate, int T, int E,
+                                     int extra, int groups, int keep, float scale, int ep, int wp, int top, int f32,
+                                     hipStream_t s) {
+  using namespace kgs::moe;
+  const int EA = E + extra;
+  if (T <= 0 || E <= 0 || extra < 0 || EA > 1024 || ep < EA + (gate ? 1 : 0) || ep % 16 || groups <= 0 || EA % groups ||
+      keep <= 0 || keep > groups || top <= 0 || top > EA / groups * keep || wp <= 0 || wp % 256 || ldh < wp)
+    return KGS_ERR_SHAPE;
+  if (!corr) return KGS_ERR_ARG;
+  if (ldh % 8 || (((uintptr_t)h | (uintptr_t)w) & 15)) return KGS_ERR_ALIGN;
+  RouteArgs a{h, ldh, w, (const int*)slots, (int*)counts, (int*)ids, (int*)rank, (float*)weight, T, E, ep, wp, top,
+              (const float*)corr, (float*)ident, (float*)gate, extra, groups, keep, scale};
+  return route(a, f32, s);
 }
 
 KGS_EXPORT int kgs_moe_plan(const void* counts, const void* ids, const void* rank, const void* weight, void* pos,
@@ -452,19 +625,21 @@ KGS_EXPORT int kgs_moe_plan(const void* counts, const void* ids, const void* ran
   return (int)hipGetLastError();
 }
 
-// The experts' products over the sorted order. gated: C[p] = gate(limit) of A[rows[p]] with
-// B [E][gate | up = N][K], N / 2 columns; else C[p] = B[e] A[p], nslice > 1: fp32
+// The experts' products over the sorted order. gated: C[p] = the gated product (act 0:
+// clamped at limit, 1: silu) of A[rows[p]] with B [E][gate | up = N][K], N / 2 columns; else C[p] = B[e] A[p], nslice > 1: fp32
 // partial products [slice][P][N] over K / nslice columns each. max_tiles: the most
 // tiles of bm rows there can be.
 KGS_EXPORT int kgs_moe_grouped(const void* A, long lda, const void* B, void* C, long ldc, const void* rows,
                                const void* roww, const void* tiles, const void* ntiles, int max_tiles, int bm, int T,
-                               int P, int N, int K, int nslice, float limit, int gated, int f32, hipStream_t s) {
+                               int P, int N, int K, int nslice, float limit, int act, int gated, int f32,
+                               hipStream_t s) {
   using namespace kgs::moe;
+  if (act != ACT_CLAMPED && act != ACT_SILU) return KGS_ERR_ARG;
   if (max_tiles <= 0 || T <= 0 || P <= 0 || N <= 0 || K <= 0 || nslice <= 0 || K % nslice) return KGS_ERR_SHAPE;
   const int kk = K / nslice, no = gated ? N / 2 : N;
   if (lda < K || (nslice == 1 && ldc < no) || (gated && nslice != 1)) return KGS_ERR_SHAPE;
   GroupedArgs a{A, B, C, (const int*)rows, (const float*)roww, (const int4*)tiles, (const int*)ntiles, lda,
-                T, P, N, kk, (int)ldc, nslice, limit};
+                T, P, N, kk, (int)ldc, nslice, limit, act};
   if (f32) {
     if (bm != 64 || no % 64 || K % 16 || nslice != 1 || lda % 4) return KGS_ERR_SHAPE;
     const long g = (long)max_tiles * (no / 64);

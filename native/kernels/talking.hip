@@ -70,6 +70,11 @@ struct WriteArgs {
   void* pages;
   const int* slots;    // [T], -1: not cached
   int T, nq, G, dkp, dvp, ok, ov;
+  // rotary positions of q and k, neighbouring dims paired: [npos][rot] (cos, sin) of the
+  // pairs of the first `rot` dims (a multiple of 8), or null
+  const float* cs;
+  const int* pos;      // [T]
+  int npos, rot;
 };
 
 template <typename T>
@@ -77,7 +82,7 @@ struct Vec8 {
   T v[8];
 };
 
-// One thread: 8 columns of 8 rows. q gets its bias in place; k and v get theirs and
+// One thread: 8 columns of 8 rows. q gets its bias (and rotation) in place; k and v get theirs and
 // go to the page, v as 8 tokens of a dim where the rows allow it.
 template <typename T>
 __global__ __launch_bounds__(256) void write_kv(WriteArgs a) {
@@ -89,6 +94,8 @@ __global__ __launch_bounds__(256) void write_kv(WriteArgs a) {
   const int zc = kind == 0 ? c : kind == 1 ? a.ok + c : a.ov + c;
   const f32x4 b0 = *(const f32x4*)(a.b + col), b1 = *(const f32x4*)(a.b + col + 4);
   const float b[8] = {b0[0], b0[1], b0[2], b0[3], b1[0], b1[1], b1[2], b1[3]};
+  const int dd = kind == 2 ? 0 : c % a.dkp;
+  const bool turn = a.cs && kind != 2 && dd < a.rot;
   int sl[8];
 #pragma unroll
   for (int r = 0; r < 8; ++r) sl[r] = r < nr ? a.slots[r0 + r] : -1;
@@ -96,10 +103,27 @@ __global__ __launch_bounds__(256) void write_kv(WriteArgs a) {
 #pragma unroll
   for (int r = 0; r < 8; ++r) {
     x[r] = *(const Vec8<T>*)((const T*)a.z + (long)(r0 + min(r, nr - 1)) * a.ldz + zc);
+    float y[8];
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
-      if constexpr (sizeof(T) == 2) x[r].v[i] = f2bf(bf2f(x[r].v[i]) + b[i]);
-      else x[r].v[i] += b[i];
+      if constexpr (sizeof(T) == 2) y[i] = bf2f(x[r].v[i]) + b[i];
+      else y[i] = x[r].v[i] + b[i];
+    }
+    if (turn) {
+      const float* p = a.cs + (long)min(max(a.pos[r0 + min(r, nr - 1)], 0), a.npos - 1) * a.rot + dd;
+      const f32x4 p0 = *(const f32x4*)p, p1 = *(const f32x4*)(p + 4);
+      const float cs[8] = {p0[0], p0[1], p0[2], p0[3], p1[0], p1[1], p1[2], p1[3]};
+#pragma unroll
+      for (int i = 0; i < 8; i += 2) {
+        const float u = y[i], v = y[i + 1];
+        y[i] = rope_lo(u, v, cs[i], cs[i + 1]);
+        y[i + 1] = rope_hi(u, v, cs[i], cs[i + 1]);
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      if constexpr (sizeof(T) == 2) x[r].v[i] = f2bf(y[i]);
+      else x[r].v[i] = y[i];
     }
   }
   if (kind == 0) {
@@ -1010,15 +1034,20 @@ int check(const Args& a, int n) {
 
 // z [T, ldz] holds q from column 0, k from ok, v from ov (heads padded to dkp / dvp);
 // b their biases one after another (nq + G dkp + G dvp). q += b in place, k + b and
-// v + b go to their slots.
+// v + b go to their slots. cs not null: q and k rotated by the row's position, the
+// pairs (0, 1), (2, 3), .. of each head's first `rot` dims by cs [npos][rot / 2][cos, sin].
 KGS_EXPORT int kgs_talking_write(void* z, long ldz, const void* b, void* pages, const void* slots, int T, int nq, int G,
-                                 int dkp, int dvp, int ok, int ov, int f32, hipStream_t s) {
+                                 int dkp, int dvp, int ok, int ov, const void* cs, const void* pos, int npos, int rot,
+                                 int f32, hipStream_t s) {
   using namespace kgs::talking;
   if (T <= 0 || nq <= 0 || G <= 0 || dkp <= 0 || dvp <= 0 || dkp % 32 || dvp % 16 || nq % 8 || ok < nq ||
       ldz < ok + G * dkp || ldz < ov + G * dvp || T > 8 * 65535)
     return KGS_ERR_SHAPE;
   if (ldz % 8 || ok % 8 || ov % 8 || (((uintptr_t)z | (uintptr_t)pages | (uintptr_t)b) & 15)) return KGS_ERR_ALIGN;
-  WriteArgs a{z, ldz, (const float*)b, pages, (const int*)slots, T, nq, G, dkp, dvp, ok, ov};
+  if (cs && (!pos || npos <= 0 || rot <= 0 || rot % 8 || rot > dkp || nq % dkp)) return KGS_ERR_SHAPE;
+  if ((uintptr_t)cs & 15) return KGS_ERR_ALIGN;
+  WriteArgs a{z, ldz, (const float*)b, pages, (const int*)slots, T, nq, G, dkp, dvp, ok, ov,
+              (const float*)cs, (const int*)pos, npos, rot};
   const dim3 grid(((nq + G * (dkp + dvp)) / 8 + 255) / 256, (T + 7) / 8);
   if (f32) hipLaunchKernelGGL(write_kv<float>, grid, dim3(256), 0, s, a);
   else hipLaunchKernelGGL(write_kv<unsigned short>, grid, dim3(256), 0, s, a);

@@ -30,14 +30,14 @@ def rel_err(got, want):
 @pytest.mark.parametrize("dtype", [F32, BF])
 @pytest.mark.parametrize("width,wp,T", [(140, 256, 5), (2048, 2048, 3), (5000, 5120, 2), (16384, 16384, 2)])
 def test_residual(dtype, width, wp, T):
-    from kgs.ops.residual import ExpertRows, residual_add, residual_embed
+    from kgs.ops.residual import ExpertRows, Norm, residual_add, residual_embed
 
     pad = lambda t: torch.nn.functional.pad(t, (0, wp - width))  # noqa: E731
     emb = pad(rnd(11, width, seed=1, dtype=dtype))
     w, w2, ab = (pad(rnd(width, seed=s, scale=0.3)) for s in (2, 3, 4))
     toks = torch.tensor([i % 11 for i in range(T)], dtype=torch.int32)
     zero = torch.full((7,), 5, dtype=torch.int32, device="cuda")
-    x, h = residual_embed(toks.cuda(), emb.cuda(), 3.25, w.cuda(), width, 1e-3, zero)
+    x, h = residual_embed(toks.cuda(), emb.cuda(), 3.25, w.cuda(), Norm(width, 1e-3), zero)
     want = 3.25 * emb[toks.long()].double()
     tol = 2e-6 if dtype == F32 else 5e-3
     assert rel_err(x, want) < 1e-6 and (zero == 0).all()
@@ -47,7 +47,7 @@ def test_residual(dtype, width, wp, T):
     for y in (pad(rnd(2 * T, width, seed=6, dtype=dtype)), pad(rnd(3, 2 * T, width, seed=7)), None):
         x2 = x.clone()
         e = None if y is None else ExpertRows(y.cuda(), pos.cuda())
-        h = residual_add(x2, a.cuda(), ab.cuda(), e, w2.cuda(), width, 1e-5, dtype)
+        h = residual_add(x2, a.cuda(), ab.cuda(), e, w2.cuda(), Norm(width, 1e-5), dtype)
         s = want + a.double() + ab.double()
         if y is not None:
             ys = y.double() if y.dim() == 2 else y.double().sum(0)
@@ -71,6 +71,7 @@ def test_experts(T, E, top, W, ff, limit, dtype):
     """Routing, the sorted order and both grouped products: every choice's row is its
     expert's output for the token's weighted input."""
     from kgs.ops import moe as M
+    from kgs.ops.activation import Gate
 
     W256 = (W + 255) // 256 * 256
     pad = lambda t, n, d: torch.nn.functional.pad(t, (0, W256 - W) if d == 1 else (0, 0, 0, W256 - W))  # noqa: E731
@@ -100,7 +101,7 @@ def test_experts(T, E, top, W, ff, limit, dtype):
     n = int(real.sum()) * top
     pos = p.pos.cpu()
     assert sorted(pos[real].reshape(-1).tolist()) == list(range(n)) and (pos[~real] == -1).all()
-    a = M.gate_up(h.cuda(), gu.cuda(), p, limit)
+    a = M.gate_up(h.cuda(), gu.cuda(), p, Gate("clamped", limit))
     y = M.down(a, dn.cuda(), p)
     y = (y if y.dim() == 2 else y.sum(0)).cpu()
     check = range(T) if T < 100 else np.random.default_rng(0).integers(0, T, 60).tolist()
@@ -115,7 +116,7 @@ def test_experts(T, E, top, W, ff, limit, dtype):
     got, want = torch.stack(got), torch.stack(want)
     assert rel_err(got, want) < (1e-5 if dtype == F32 else 2e-2)
     if dtype == BF:  # the split form and the whole one agree
-        full = M._grouped(a, dn.cuda(), torch.empty((a.shape[0], W256), dtype=BF, device="cuda"), p, a.shape[0], 1, 0.0, False)
+        full = M._grouped(a, dn.cuda(), torch.empty((a.shape[0], W256), dtype=BF, device="cuda"), p, a.shape[0], 1, None)
         assert rel_err(full[:n].cpu(), y[:n].double()) < 1e-2
 
 
