@@ -85,13 +85,14 @@ def parse(argv=None):
     ap.add_argument("--oversubscribe", action="store_true",
                     help="allow more ranks than GPUs (rank r on GPU r %% n): tests the multi-rank GPU path on a "
                          "1-GPU box, with --dist-backend gloo; not a benchmark configuration")
-    ap.add_argument("--workload", choices=("gemm", "ruruzen", "nufusun"), default="gemm",
-                    help="gemm = the benchmark; ruruzen, nufusun = prefill and decode throughput of that design's "
-                         "layer stack beside a Llama stack of equal size, one GPU (kgs/serve/layer_bench.py)")
+    ap.add_argument("--workload", choices=("gemm", "ruruzen", "nufusun", "nokipel"), default="gemm",
+                    help="gemm = the benchmark; ruruzen, nufusun, nokipel = prefill and decode throughput of that design's "
+                         "layer stack beside stacks of equal size, one GPU (kgs/serve/layer_bench.py)")
     ap.add_argument("--sizes", default="w2048,w4096", help="layer stacks: sizes, comma-separated")
     ap.add_argument("--layers", default=None, help="layer stacks: one letter per layer (ruruzen: L, S, D, default "
-                                                   "LDSD; nufusun: A, N, default AAAA)")
-    ap.add_argument("--models", default=None, help="layer stacks: which models run (default: the design and llama)")
+                                                   "LDSD; nufusun: A, N, default AAAA; nokipel: L, M, C, A, default LAMC)")
+    ap.add_argument("--models", default=None, help="layer stacks: which models run, comma-separated (default: the design and the "
+                                                   "closest others)")
     ap.add_argument("--cases", choices=("all", "prefill", "decode"), default="all", help="layer stacks: which steps")
     ap.add_argument("--dtype", choices=("bf16", "fp8"), default="bf16",
                     help="bf16 = the headline (BASELINE.json); fp8 = e4m3 operands on the scaled MFMA (extra)")
@@ -161,18 +162,18 @@ def main(argv=None) -> int:
 
 
 def layer_workload(args) -> int:
-    """``--workload ruruzen|nufusun``: one JSON line with every case of both models."""
+    """``--workload ruruzen|nufusun|nokipel``: one JSON line with every case of every model."""
     import json
 
     from kgs.serve import layer_bench as lb
 
     t0 = time.perf_counter()
     rows = lb.run(tuple(args.sizes.split(",")), args.layers or lb.LAYERS[args.workload],
-                  models=tuple((args.models or f"{args.workload},llama").split(",")),
+                  models=tuple(args.models.split(",")) if args.models else (args.workload, *lb.BESIDE[args.workload]),
                   prefill=lb.PREFILL if args.cases != "decode" else (),
                   decode=lb.DECODE if args.cases != "prefill" else (),
                   progress=lambda s: print(f"[bench {time.perf_counter() - t0:6.1f}] {s}", file=sys.stderr, flush=True))
-    print(json.dumps({"metric": f"{args.workload.capitalize()} layer-stack throughput beside an equal Llama stack", "unit": "tok/s",
+    print(json.dumps({"metric": f"{args.workload.capitalize()} layer-stack throughput beside equal stacks", "unit": "tok/s",
                       "n_gpus": 1, "dtype": "bf16", "data": "synthetic tokens, random-init weights", "cases": rows}),
           flush=True)
     return 0

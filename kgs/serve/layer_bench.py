@@ -1,12 +1,11 @@
-"""Prefill and decode throughput of a Ruruzen or Nufusun layer stack at sizes that
-resemble a real model's layers (random weights), beside a Llama stack of the same
-width, heads, feed-forward (Nufusun: the experts that a token uses) and depth:
-``python bench.py --workload ruruzen|nufusun``.
+"""Prefill and decode throughput of a Ruruzen, Nufusun or Nokipel layer stack at sizes
+that resemble a real model's layers (random weights), beside stacks of the closest other
+models of the same width, heads, feed-forward (where there are experts: those that a token
+uses) and depth: ``python bench.py --workload ruruzen|nufusun|nokipel``.
 
-Both run through :class:`LLMEngine`'s own step runners: prefill a whole prompt
+All run through :class:`LLMEngine`'s own step runners: prefill a whole prompt
 batch in one step, decode a hipGraph replay per step. Per case the median of
-several interleaved rounds (one of each model in turn) is reported, and the
-weights' and cache's bytes or the projections' flops that a step cannot avoid.
+several interleaved rounds (one of each model in turn) is reported.
 """
 from __future__ import annotations
 
@@ -17,14 +16,18 @@ import numpy as np
 import torch
 
 from kgs.models.llama import LlamaConfig
+from kgs.models.nokipel import NokipelConfig
 from kgs.models.nufusun import NufusunConfig
 from kgs.models.ruruzen import RuruzenConfig
 from kgs.ops.decode import PAGE
 
 # name -> width, heads, q_rank, kv_rank, ff, Llama kv heads (head size 128 everywhere)
 SIZES = {"w2048": (2048, 16, 768, 512, 8192, 4), "w4096": (4096, 32, 1536, 512, 14336, 8)}
-EXPERTS, TOP = 16, 4     # Nufusun: experts of a layer and those a token uses, together as wide as ff
-LAYERS = {"ruruzen": "LDSD", "nufusun": "AAAA"}
+EXPERTS, TOP = 16, 4     # experts of a layer and those a token uses, together as wide as ff
+IDENTITY = 2             # Nokipel: identity experts among them; one of the TOP is the shared expert
+ATTENTION_CHUNK = 4096   # Nokipel: positions of an attention chunk
+LAYERS = {"ruruzen": "LDSD", "nufusun": "AAAA", "nokipel": "LAMC"}
+BESIDE = {"ruruzen": ("llama",), "nufusun": ("llama",), "nokipel": ("nufusun", "ruruzen")}
 VOCAB = 32000
 PREFILL = ((1, 8192), (8, 1024), (64, 128))              # sequences x tokens
 DECODE = ((1, 1024), (16, 1024), (64, 1024), (256, 1024), (16, 8192))  # batch x context
@@ -56,6 +59,26 @@ def nufusun(size: str, layers: str) -> NufusunConfig:
     return NufusunConfig.from_dict({
         "architecture": "Nufusun", "vocab": VOCAB, "width": width, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-5},
         "layers": [{"type": "attention", "mixer": mixer, "mlp": mlp if ch == "A" else None} for ch in layers]})
+
+
+def nokipel(size: str, layers: str) -> NokipelConfig:
+    """``layers``: one letter per layer -- L lightning attention and a dense feed-forward,
+    M lightning attention and experts, C chunked attention and a dense feed-forward, A
+    chunked attention and experts."""
+    width, heads, _, _, ff, kv = SIZES[size]
+    attention = {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                 "mask": {"size": ATTENTION_CHUNK}, "rot": {"dims": 64, "base": 5e5}}
+    lightning = {"heads": heads, "dim": 128, "vdim": 128, "decay": [1 - 2.0 ** -(1 + 9 * i / heads) for i in range(heads)]}
+    dense = {"kind": "dense", "ff": ff, "limit": 7.0}
+    moe = {"kind": "moe", "expert": {"ff": ff // TOP}, "shared": {"ff": ff // TOP},
+           "router": {"experts": EXPERTS - IDENTITY, "identity": IDENTITY, "top": TOP - 1, "scale": 1.5,
+                      "groups": {"count": 4, "keep": 2}}}
+    kinds = {"L": ("lightning", lightning, dense), "M": ("lightning", lightning, moe),
+             "C": ("attention", attention, dense), "A": ("attention", attention, moe)}
+    return NokipelConfig.from_dict({
+        "architecture": "Nokipel", "vocab": VOCAB, "width": width, "embedding": {"scale": 1.0},
+        "norm": {"eps": 1e-5, "groups": 8},
+        "layers": [dict(zip(("type", "mixer", "mlp"), kinds[ch])) for ch in layers]})
 
 
 def llama(size: str, layers: str) -> LlamaConfig:
@@ -103,7 +126,8 @@ def _time(run, steps: int) -> float:
 
 def run(sizes=("w2048", "w4096"), layers: str = "LDSD", rounds: int = 3, prefill=PREFILL, decode=DECODE,
         models=("ruruzen", "llama"), progress=lambda s: None) -> list[dict]:
-    """``models``: "ruruzen", "nufusun", "llama"."""
+    """``models``: "ruruzen", "nufusun", "nokipel", "llama"; ``layers``: the first one's, a
+    further design has its own."""
     from .engine import EngineConfig, LLMEngine
 
     out = []
@@ -113,7 +137,8 @@ def run(sizes=("w2048", "w4096"), layers: str = "LDSD", rounds: int = 3, prefill
         ec = dict(num_pages=most // PAGE + 2 * nb + 2, max_batch=max(256, nb), max_model_len=16384)
         engines = {}
         for m in models:
-            cfg = {"ruruzen": ruruzen, "nufusun": nufusun, "llama": llama}[m](size, layers)
+            make = {"ruruzen": ruruzen, "nufusun": nufusun, "nokipel": nokipel, "llama": llama}[m]
+            cfg = make(size, layers if m in (models[0], "llama") else LAYERS[m])
             engines[m] = LLMEngine(cfg, EngineConfig(**ec))
             progress(f"{size} {m} ready")
         for kind, cases in (("prefill", prefill), ("decode", decode)):
