@@ -53,10 +53,10 @@ def portion_items(portions, tile: int, chunk: int) -> np.ndarray:
 
 
 def row_splits(n: int, kv_heads: int, group: int, pages: int) -> int:
-    """Splits of the visible pages: three workgroups of four waves per CU, at least two
+    """Splits of the visible pages: two workgroups of four waves per CU (what fits), at least two
     pages per wave."""
     units = n * kv_heads * -(-group // 16)
-    return max(1, min(3 * CUS // max(1, units), -(-pages // 8), 64))
+    return max(1, min(2 * CUS // max(1, units), -(-pages // 8), 64))
 
 
 def visible_pages(pos: int, chunk: int) -> int:

@@ -25,7 +25,7 @@ from kgs.ops.decode import PAGE
 SIZES = {"w2048": (2048, 16, 768, 512, 8192, 4), "w4096": (4096, 32, 1536, 512, 14336, 8)}
 EXPERTS, TOP = 16, 4     # experts of a layer and those a token uses, together as wide as ff
 IDENTITY = 2             # Nokipel: identity experts among them; one of the TOP is the shared expert
-ATTENTION_CHUNK = 4096   # Nokipel: positions of an attention chunk
+ATTENTION_CHUNK = 5120   # Nokipel: positions of an attention chunk (3072 keys at the longest context below)
 LAYERS = {"ruruzen": "LDSD", "nufusun": "AAAA", "nokipel": "LAMC"}
 BESIDE = {"ruruzen": ("llama",), "nufusun": ("llama",), "nokipel": ("nufusun", "ruruzen")}
 VOCAB = 32000

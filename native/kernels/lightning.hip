@@ -14,7 +14,7 @@
 //             S   = d^n S_0 + K^T V',             V'_j = d^(n-1-j) v_j
 //           q, k and v are bf16 MFMA operands; P, V' and S enter the products as two bf16
 //           parts each (16 bits) and S itself stays in the fp32 accumulators: a wave owns
-//           32 columns of V, and the accumulator layout of S is the operand layout of
+//           16 columns of V, and the accumulator layout of S is the operand layout of
 //           S^T for keys in the order Q is staged in.
 //           A long portion is cut into segments that run side by side: chunks without
 //           output give every segment's own contribution, `scan` turns them into the
@@ -155,18 +155,19 @@ __device__ __forceinline__ bf16x8 silu8(bf16x8 x) {
   return pack_bf16x8(y, 0);
 }
 
-// grid: (item, head, V slab of 32 NW); NK: 32-key blocks. OUT: with output, from the
+// grid: (item, head, V slab of 16 NW); NK: 32-key blocks; a wave has 16 columns of V. OUT: with output, from the
 // segment's starting state; else the segment's own contribution into its buffer.
 template <int NK, int NW, bool OUT>
-__global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void chunks(Args a) {
-  constexpr int KP = 32 * NK, QLD = KP + 8, VS = 32 * NW, VLD = VS + 8, NT = 64 * NW;
+__global__ __launch_bounds__(64 * NW, 4) void chunks(Args a) {
+  constexpr int KP = 32 * NK, QLD = KP + 8, VS = 16 * NW, VLD = VS + 8, NT = 64 * NW;
   constexpr int UK = C * KP / 8 / NT, UV = C * VS / 8 / NT;  // 16-B units per thread
   __shared__ __attribute__((aligned(16))) unsigned short Qs[OUT ? C * QLD : 8];
   __shared__ __attribute__((aligned(16))) unsigned short Ks[C * QLD];
   __shared__ __attribute__((aligned(16))) unsigned short Vs[C * VLD];
   __shared__ __attribute__((aligned(16))) unsigned short Ps[2][OUT ? C * PLD : 8];  // rows i, columns j; hi, lo
   __shared__ float dec[C + 1];
-  const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6), n = lane & 15, q = lane >> 4;
+  int tid = threadIdx.x, n = tid & 15, q = tid >> 4 & 3;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int nslab = a.VP / VS;
   int id = blockIdx.x;
   const int slab = id % nslab;
@@ -181,8 +182,8 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void chunks(Args a) {
 
   const long per = (long)KP * a.VP;
   float* pool = a.S + ((long)a.slot[it.x] * a.H + h) * per;
-  const int vcol = slab * VS + 32 * w + n;  // + 16 vt
-  f32x4 S[2 * NK][2];
+  const int vcol = slab * VS + 16 * w + n;
+  f32x4 S[2 * NK];
   bool live = false;  // the state is not zero
   {
     const float* src = nullptr;
@@ -191,9 +192,7 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void chunks(Args a) {
 #pragma unroll
     for (int kt = 0; kt < 2 * NK; ++kt)
 #pragma unroll
-      for (int vt = 0; vt < 2; ++vt)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) S[kt][vt][r] = live ? src[(long)(16 * kt + 4 * q + r) * a.VP + vcol + 16 * vt] : 0.f;
+      for (int r = 0; r < 4; ++r) S[kt][r] = live ? src[(long)(16 * kt + 4 * q + r) * a.VP + vcol] : 0.f;
   }
 
   const unsigned short* z = (const unsigned short*)a.z + row0 * a.ldz;
@@ -201,19 +200,20 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void chunks(Args a) {
   const unsigned short* zk = z + a.ok + h * KP;
   const unsigned short* zv = z + a.ov + h * a.VP + slab * VS;
   bf16x8 rq[OUT ? UK : 1], rk[UK], rv[UV];
+  const unsigned ld = a.ldz;  // a segment's rows are within 32-bit offsets
   auto fetch = [&](int c0) {  // a chunk's projections, rows past the end zero
     const int nr = it.z - c0;
 #pragma unroll
     for (int i = 0; i < UK; ++i) {
       const int u = tid + i * NT, r = u / (KP / 8), c = u % (KP / 8);
-      const long o = (long)(c0 + r) * a.ldz + 8 * c;
+      const unsigned o = (unsigned)(c0 + r) * ld + 8 * c;
       if constexpr (OUT) rq[i] = r < nr ? *(const bf16x8*)(zq + o) : bf16x8{};
       rk[i] = r < nr ? *(const bf16x8*)(zk + o) : bf16x8{};
     }
 #pragma unroll
     for (int i = 0; i < UV; ++i) {
       const int u = tid + i * NT, r = u / (VS / 8), c = u % (VS / 8);
-      rv[i] = r < nr ? *(const bf16x8*)(zv + (long)(c0 + r) * a.ldz + 8 * c) : bf16x8{};
+      rv[i] = r < nr ? *(const bf16x8*)(zv + (unsigned)(c0 + r) * ld + 8 * c) : bf16x8{};
     }
   };
   // 8 tokens (32 ks + 8 q ..) of column col + n of a row-major tile
@@ -225,6 +225,8 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void chunks(Args a) {
   fetch(0);
   for (int c0 = 0; c0 < it.z; c0 += C) {
     const int nc = min(C, it.z - c0);
+    // addresses are worked out anew for every chunk: kept over the loop they would not fit the registers
+    asm volatile("" : "+v"(tid), "+v"(n), "+v"(q));
 #pragma unroll
     for (int i = 0; i < UK; ++i) {
       const int u = tid + i * NT, r = u / (KP / 8), c = u % (KP / 8);
@@ -244,22 +246,21 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void chunks(Args a) {
       *(bf16x8*)(Vs + r * VLD + 8 * c) = silu8(rv[i]);
     }
     __syncthreads();
-    if (c0 + C < it.z) fetch(c0 + C);
+    if (!OUT && c0 + C < it.z) fetch(c0 + C);
 
-    bf16x8 vf[2][2];  // [ks][vt]
+    bf16x8 vf[2];
 #pragma unroll
-    for (int ks = 0; ks < 2; ++ks)
-#pragma unroll
-      for (int vt = 0; vt < 2; ++vt) vf[ks][vt] = column(Vs, VLD, ks, 32 * w + 16 * vt);
+    for (int ks = 0; ks < 2; ++ks) vf[ks] = column(Vs, VLD, ks, 16 * w);
 
     if constexpr (OUT) {
-      // rows 16 ti .. of P: P^T tiles, a lane has 4 neighbouring j of one i
-      for (int ti = w; ti < 4; ti += NW) {
+      // tiles of P: P^T, a lane has 4 neighbouring j of one i; a wave has one row of tiles or half of it
+      {
+        constexpr int NS = NW / 4;
+        const int ti = w & 3, i = 16 * ti + n;
         bf16x8 qf[NK];
 #pragma unroll
-        for (int t = 0; t < NK; ++t) qf[t] = *(const bf16x8*)(Qs + (16 * ti + n) * QLD + 32 * t + 8 * q);
-        const int i = 16 * ti + n;
-        for (int tj = 0; tj <= (ti | 1); ++tj) {
+        for (int t = 0; t < NK; ++t) qf[t] = *(const bf16x8*)(Qs + i * QLD + 32 * t + 8 * q);
+        for (int tj = w >> 2; tj <= (ti | 1); tj += NS) {
           f32x4 p{};
           if (tj <= ti) {
 #pragma unroll
@@ -284,59 +285,45 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void chunks(Args a) {
           *(uint2*)(Ps[1] + i * PLD + 16 * tj + 4 * q) = lo;
         }
       }
-      f32x4 acc[2][4];
+      f32x4 acc[4];
 #pragma unroll
-      for (int vt = 0; vt < 2; ++vt)
-#pragma unroll
-        for (int ti = 0; ti < 4; ++ti) acc[vt][ti] = f32x4{};
+      for (int ti = 0; ti < 4; ++ti) acc[ti] = f32x4{};
       if (live) {
 #pragma unroll
         for (int t = 0; t < NK; ++t) {
-          bf16x8 sh[2], sl[2], qf[4];
+          __builtin_amdgcn_sched_barrier(0);
+          bf16x8 sh, sl, qf[4];
 #pragma unroll
           for (int ti = 0; ti < 4; ++ti) qf[ti] = *(const bf16x8*)(Qs + (16 * ti + n) * QLD + 32 * t + 8 * q);
+          float x[8];
 #pragma unroll
-          for (int vt = 0; vt < 2; ++vt) {
-            float x[8];
+          for (int e = 0; e < 4; ++e) x[e] = S[2 * t][e], x[4 + e] = S[2 * t + 1][e];
+          split8(x, sh, sl);
 #pragma unroll
-            for (int e = 0; e < 4; ++e) x[e] = S[2 * t][vt][e], x[4 + e] = S[2 * t + 1][vt][e];
-            split8(x, sh[vt], sl[vt]);
-          }
+          for (int ti = 0; ti < 4; ++ti) acc[ti] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sl, qf[ti], acc[ti], 0, 0, 0);
 #pragma unroll
-          for (int ti = 0; ti < 4; ++ti)
-#pragma unroll
-            for (int vt = 0; vt < 2; ++vt) {
-              acc[vt][ti] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sl[vt], qf[ti], acc[vt][ti], 0, 0, 0);
-              acc[vt][ti] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sh[vt], qf[ti], acc[vt][ti], 0, 0, 0);
-            }
+          for (int ti = 0; ti < 4; ++ti) acc[ti] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sh, qf[ti], acc[ti], 0, 0, 0);
         }
 #pragma unroll
-        for (int ti = 0; ti < 4; ++ti) {
-          const float f = dec[16 * ti + n + 1];
-#pragma unroll
-          for (int vt = 0; vt < 2; ++vt) acc[vt][ti] *= f;
-        }
+        for (int ti = 0; ti < 4; ++ti) acc[ti] *= dec[16 * ti + n + 1];
       }
       __syncthreads();  // P is there
+      if (c0 + C < it.z) fetch(c0 + C);  // in flight from here on, where fewer registers are needed
+      __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
       for (int ti = 0; ti < 4; ++ti)
 #pragma unroll
         for (int ks = 0; ks <= ti / 2; ++ks) {
           const unsigned short* pp = Ps[0] + (16 * ti + n) * PLD + 32 * ks + 8 * q;
           const bf16x8 ph = *(const bf16x8*)pp, pl = *(const bf16x8*)(pp + (Ps[1] - Ps[0]));
-#pragma unroll
-          for (int vt = 0; vt < 2; ++vt) {
-            acc[vt][ti] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[ks][vt], pl, acc[vt][ti], 0, 0, 0);
-            acc[vt][ti] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[ks][vt], ph, acc[vt][ti], 0, 0, 0);
-          }
+          acc[ti] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[ks], pl, acc[ti], 0, 0, 0);
+          acc[ti] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[ks], ph, acc[ti], 0, 0, 0);
         }
 #pragma unroll
       for (int ti = 0; ti < 4; ++ti) {
         const int i = 16 * ti + n;
         if (i >= nc) continue;
-        float* op = a.o + ((row0 + c0 + i) * a.H + h) * a.VP + slab * VS + 32 * w + 4 * q;
-#pragma unroll
-        for (int vt = 0; vt < 2; ++vt) *(f32x4*)(op + 16 * vt) = acc[vt][ti];
+        *(f32x4*)(a.o + ((row0 + c0 + i) * a.H + h) * a.VP + slab * VS + 16 * w + 4 * q) = acc[ti];
       }
     }
 
@@ -344,31 +331,21 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void chunks(Args a) {
     {
       const float dn = dec[nc];
 #pragma unroll
-      for (int kt = 0; kt < 2 * NK; ++kt)
-#pragma unroll
-        for (int vt = 0; vt < 2; ++vt) S[kt][vt] *= dn;
+      for (int kt = 0; kt < 2 * NK; ++kt) S[kt] *= dn;
     }
 #pragma unroll
     for (int ks = 0; ks < 2; ++ks) {
-      bf16x8 vh[2], vl[2];
-      float f[8];
+      bf16x8 vh, vl;
+      float x[8];
 #pragma unroll
-      for (int e = 0; e < 8; ++e) f[e] = dec[max(nc - 1 - (32 * ks + 8 * q + e), 0)];  // rows past the end are zero
-#pragma unroll
-      for (int vt = 0; vt < 2; ++vt) {
-        float x[8];
-#pragma unroll
-        for (int e = 0; e < 8; ++e) x[e] = f[e] * bf2f((unsigned short)vf[ks][vt][e]);
-        split8(x, vh[vt], vl[vt]);
-      }
+      for (int e = 0; e < 8; ++e)  // rows past the end are zero
+        x[e] = dec[max(nc - 1 - (32 * ks + 8 * q + e), 0)] * bf2f((unsigned short)vf[ks][e]);
+      split8(x, vh, vl);
 #pragma unroll
       for (int kt = 0; kt < 2 * NK; ++kt) {
         const bf16x8 kf = column(Ks, QLD, ks, 16 * kt);
-#pragma unroll
-        for (int vt = 0; vt < 2; ++vt) {
-          S[kt][vt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, vl[vt], S[kt][vt], 0, 0, 0);
-          S[kt][vt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, vh[vt], S[kt][vt], 0, 0, 0);
-        }
+        S[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, vl, S[kt], 0, 0, 0);
+        S[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, vh, S[kt], 0, 0, 0);
       }
     }
     live = true;
@@ -379,9 +356,7 @@ __global__ __launch_bounds__(64 * NW, NW == 4 ? 2 : 1) void chunks(Args a) {
 #pragma unroll
   for (int kt = 0; kt < 2 * NK; ++kt)
 #pragma unroll
-    for (int vt = 0; vt < 2; ++vt)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) dst[(long)(16 * kt + 4 * q + r) * a.VP + vcol + 16 * vt] = S[kt][vt][r];
+    for (int r = 0; r < 4; ++r) dst[(long)(16 * kt + 4 * q + r) * a.VP + vcol] = S[kt][r];
 }
 
 // the segments' contributions -> the states they start from; grid: 1024 floats of a state, head, sequence
@@ -480,14 +455,14 @@ void run_step(const Args& a, int nseqs, hipStream_t s) {
 
 template <bool OUT>
 void run_chunks(const Args& a, int nitems, hipStream_t s) {
-  const int nw = a.VP == 64 ? 2 : 4;
-  const dim3 grid((unsigned)((long)nitems * a.H * (a.VP / (32 * nw)))), block(64 * nw);
+  const int nw = a.VP == 64 ? 4 : 8;
+  const dim3 grid((unsigned)((long)nitems * a.H * (a.VP / (16 * nw)))), block(64 * nw);
   if (a.KP == 64) {
-    if (nw == 2) hipLaunchKernelGGL((chunks<2, 2, OUT>), grid, block, 0, s, a);
-    else hipLaunchKernelGGL((chunks<2, 4, OUT>), grid, block, 0, s, a);
+    if (nw == 4) hipLaunchKernelGGL((chunks<2, 4, OUT>), grid, block, 0, s, a);
+    else hipLaunchKernelGGL((chunks<2, 8, OUT>), grid, block, 0, s, a);
   } else {
-    if (nw == 2) hipLaunchKernelGGL((chunks<4, 2, OUT>), grid, block, 0, s, a);
-    else hipLaunchKernelGGL((chunks<4, 4, OUT>), grid, block, 0, s, a);
+    if (nw == 4) hipLaunchKernelGGL((chunks<4, 4, OUT>), grid, block, 0, s, a);
+    else hipLaunchKernelGGL((chunks<4, 8, OUT>), grid, block, 0, s, a);
   }
 }
 

@@ -221,7 +221,7 @@ __device__ __forceinline__ void choose_softmax(const RouteArgs& a, float* z, flo
 // bf16: eight waves split the width, ET 16-expert MFMA tiles each, U steps' loads at a time
 template <int ET>
 __global__ __launch_bounds__(512) void route_mfma(RouteArgs a) {
-  constexpr int U = ET >= 8 ? 1 : ET >= 4 ? 2 : 4;
+  constexpr int U = ET >= 4 ? 2 : 8;
   extern __shared__ float lds[];
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, n = lane & 15, q = lane >> 4;
   const int t0 = blockIdx.x * RT, t = min(t0 + n, a.T - 1), kw = a.wp / 8;

@@ -186,17 +186,21 @@ __global__ __launch_bounds__(64) void merge(Args a) {
   const int row = blockIdx.x / a.H, h = blockIdx.x - row * a.H;
   const long brow = a.rows ? a.rows[row] : row;
   const long at = (long)row * a.nsplit * a.H + h;
-  float M = NEG;
-  for (int s = 0; s < a.nsplit; ++s) M = fmaxf(M, a.pml[2 * (at + (long)s * a.H)]);
-  for (int d = threadIdx.x; d < a.dvp; d += 64) {
-    float y = 0.f, L = 0.f;
-    for (int s = 0; s < a.nsplit; ++s) {
-      const long i = at + (long)s * a.H;
-      const float f = __builtin_amdgcn_exp2f(a.pml[2 * i] - M);
-      L = __builtin_fmaf(f, a.pml[2 * i + 1], L);
-      y = __builtin_fmaf(f, a.po[i * a.dvp + d], y);
-    }
-    ((unsigned short*)a.o)[brow * a.ldo + (long)h * a.dvp + d] = f2bf(y / L);
+  const int lane = threadIdx.x;
+  // one lane per split (at most 64): its factor, and the sum of all
+  const float* ml = a.pml + 2 * (at + (long)min(lane, a.nsplit - 1) * a.H);
+  const float m = lane < a.nsplit ? ml[0] : NEG, l = lane < a.nsplit ? ml[1] : 0.f;
+  float M = m;
+#pragma unroll
+  for (int x = 1; x < 64; x <<= 1) M = fmaxf(M, __shfl_xor(M, x));
+  const float f = __builtin_amdgcn_exp2f(m - M), inv = 1.0f / wave_sum(f * l);
+  for (int d0 = 0; d0 < a.dvp; d0 += 64) {
+    const int d = d0 + lane;
+    const float* p = a.po + at * a.dvp + min(d, a.dvp - 1);
+    float y = 0.f;
+#pragma unroll 8
+    for (int s = 0; s < a.nsplit; ++s) y = __builtin_fmaf(__shfl(f, s), p[(long)s * a.H * a.dvp], y);
+    if (d < a.dvp) ((unsigned short*)a.o)[brow * a.ldo + (long)h * a.dvp + d] = f2bf(y * inv);
   }
 }
 
@@ -438,7 +442,7 @@ bool mfma(const Args& a) { return (a.dkp == 64 || a.dkp == 128) && (a.dvp == 64 
 
 // nrows query tokens (batch row rows[i], or i), each over its sequence's pages up to its
 // position, from its chunk's first key on (chunk 0: from 0). bf16 with dkp, dvp 64 or 128,
-// split over the pages nsplit times (po, pml: partial results); plain != 0 (or fp32): any
+// split over the pages nsplit <= 64 times (po, pml: partial results); plain != 0 (or fp32): any
 // sizes, dvp up to 1024.
 KGS_EXPORT int kgs_paged_rows(const void* q, long ldq, const void* pages, void* o, long ldo, const void* bt, int W,
                               const void* tok_seq, const void* tok_pos, const void* rows, void* po, void* pml, float scale,
@@ -456,7 +460,7 @@ KGS_EXPORT int kgs_paged_rows(const void* q, long ldq, const void* pages, void* 
     return (int)hipGetLastError();
   }
   if (!mfma(a)) return KGS_ERR_ARG;
-  if (nsplit <= 0 || (nsplit > 1 && (!po || !pml)) || (long)nrows * H * nsplit > 0x7fffffff) return KGS_ERR_SHAPE;
+  if (nsplit <= 0 || nsplit > 64 || (nsplit > 1 && (!po || !pml)) || (long)nrows * H * nsplit > 0x7fffffff) return KGS_ERR_SHAPE;
   if (dkp == 64) dvp == 64 ? run_rows<2, 4>(a, nrows, s) : run_rows<2, 8>(a, nrows, s);
   else dvp == 64 ? run_rows<4, 4>(a, nrows, s) : run_rows<4, 8>(a, nrows, s);
   return (int)hipGetLastError();

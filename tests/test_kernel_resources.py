@@ -19,13 +19,13 @@ pytestmark = [pytest.mark.skipif(not Path(HIPCC).exists() and shutil.which("hipc
               pytest.mark.timeout(1800)]
 
 
-def _compile(src: str, odir: Path, save_temps: bool = False, subdir: str = "kernels") -> tuple[dict, str]:
+def _compile(src: str, odir: Path, save_temps: bool = False, subdir: str = "kernels", flags=()) -> tuple[dict, str]:
     """Resource remarks per kernel (and, with save_temps, the device assembly)."""
     cmd = [HIPCC if Path(HIPCC).exists() else "hipcc", "--offload-arch=gfx950", "-O3", "-std=c++17",
            "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-c",
            "-I", str(ROOT / "native" / "kernels"),
            str(ROOT / "native" / subdir / src), "-o", str(odir / (src + ".o")),
-           "-Rpass-analysis=kernel-resource-usage"]
+           "-Rpass-analysis=kernel-resource-usage", *flags]
     if save_temps:
         cmd.append("-save-temps=obj")
     out = subprocess.run(cmd, capture_output=True, text=True, timeout=1500, cwd=odir)
@@ -413,3 +413,13 @@ def test_p2p_allreduce_order_check_catches_weakened_builds(tmp_path, mutation):
     assert mutated != src
     bad = {n: e for n, e in _ar_build(tmp_path, mutated).items() if e}
     assert bad, "the weakened build passed the ordering check"
+
+
+def test_paged_and_lightning_kernels_do_not_spill(tmp_path):
+    """Attention over head pages and lightning attention: no spills, and the chunk kernel
+    (keys and values of 128) leaves room for a second workgroup of eight waves on a CU."""
+    for src in ("paged.hip", "lightning.hip"):
+        for name, r in _compile(src, tmp_path, flags=("-mllvm", "-amdgpu-mfma-vgpr-form=1"))[0].items():
+            assert r["VGPRs Spill"] == 0 and r["SGPRs Spill"] == 0, (name, r)
+            if "6chunksILi4ELi8ELb1EE" in name:
+                assert r["VGPRs"] <= 128 and 2 * r["LDS Size"] <= 160 * 1024, r
