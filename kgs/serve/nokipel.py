@@ -153,9 +153,6 @@ class ChunkedMixer:
         self.rotary = model.rotary(m.rot_dims, m.rot_base) if m.rot_dims else None
         self.o = w.proj(_output_matrix(w, p + "o", m.heads, m.vdim, h.dvp, wp, m.heads * h.dvp))
 
-    def cache(self, run: int) -> tuple[int, Heads]:
-        return run, self.heads
-
     def __call__(self, model, run: int, h: torch.Tensor, b: Batch) -> torch.Tensor:
         hd, m, plan = self.heads, self.m, b.plans[self.geo]
         z = self.win(h)

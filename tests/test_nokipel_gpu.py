@@ -362,3 +362,17 @@ def test_trace_run_program(tmp_path):
     check(read(0), wx[[0, 29]], "float32")
     check(read(2), torch.stack([wy[8], wx[39]]), "float32")
     assert not (tmp_path / "1.f32").exists()
+
+
+def test_serving_benchmark_on_a_model_folder(tmp_path, capsys):
+    """The command line, from a checkpoint to generated tokens."""
+    from kgs.serve.bench import main
+    from kgs.utils.safetensors import save_file
+
+    cfg, w = NM.model("first")
+    (tmp_path / "config.json").write_text(json.dumps(cfg.raw))
+    save_file(w, tmp_path / "model.safetensors")
+    assert main(["--model", str(tmp_path), "--requests", "5", "--input-len", "33", "--output-len", "6", "--max-batch", "4",
+                 "--max-model-len", "256", "--chunked-prefill", "48"]) == 0
+    out = json.loads(capsys.readouterr().out.strip().splitlines()[-1])
+    assert out["output_tok_per_s"] > 0 and out["stats"]["decode_tokens"] >= 5 * 5
