@@ -32,6 +32,7 @@ ARCHITECTURES = {a.name: a for a in (
     Architecture("Ruruzen", "kgs.models.ruruzen:RuruzenConfig", "kgs.serve.hybrid:HybridModel"),
     Architecture("Nufusun", "kgs.models.nufusun:NufusunConfig", "kgs.serve.nufusun:NufusunModel"),
     Architecture("Nokipel", "kgs.models.nokipel:NokipelConfig", "kgs.serve.nokipel:NokipelModel"),
+    Architecture("Vumalix", "kgs.models.vumalix:VumalixConfig", "kgs.serve.vumalix:VumalixModel"),
 )}
 
 

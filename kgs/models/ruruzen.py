@@ -42,6 +42,10 @@ class LatentSpec:
     kv_rank: int
     scale: float
     kv_from: int | None = None   # the layer whose cached latent this one reads (None: its own)
+    rot_dim: int = 0             # further query / key dimensions of a head that turn with the position
+    rot_base: float = 1.0
+    window: int = 0              # keys a token sees, itself among them; 0: all
+    gate_each: bool = False      # the output gate has a number per element, not per head
 
 
 @dataclass(frozen=True)

@@ -108,10 +108,16 @@ _SIGS = {
     "kgs_hyper_embed": ([_c_void_p] * 7 + [_c_int] * 3 + [_c_long] * 2 + [ctypes.c_float, _c_int, _c_void_p], _c_int),
     "kgs_act_mul": ([_c_void_p] * 2 + [_c_int] * 2 + [_c_long] * 2 + [_c_int, ctypes.c_float, _c_int, _c_void_p], _c_int),
     "kgs_softcap": ([_c_void_p] * 2 + [_c_int] * 2 + [_c_long, ctypes.c_float, _c_int, _c_void_p], _c_int),
-    "kgs_latent_norm": ([_c_void_p, _c_long] + [_c_int] * 6 + [_c_void_p] * 5 + [_c_int, ctypes.c_float, _c_int,
-                                                                                _c_void_p], _c_int),
-    "kgs_head_proj": ([_c_void_p] * 6 + [_c_long] * 5 + [_c_int] * 5 + [_c_void_p], _c_int),
-    "kgs_latent_attn": ([_c_void_p] * 10 + [_c_int] * 8 + [ctypes.c_float, _c_void_p], _c_int),
+    "kgs_poly_norm": ([_c_void_p, _c_long, _c_void_p, _c_void_p, _c_long] + [_c_int] * 3 + [ctypes.c_float, _c_int,
+                                                                                           _c_void_p], _c_int),
+    # post-normed residual with a convolution over time (postnorm.hip)
+    "kgs_postnorm": ([_c_void_p] * 4 + [_c_long, _c_void_p, _c_long] + [ctypes.c_float] * 2 + [_c_void_p] * 2 + [_c_int] * 2
+                     + [ctypes.c_float] + [_c_void_p] * 7 + [_c_long] + [_c_int] * 5 + [_c_void_p], _c_int),
+    "kgs_latent_norm": ([_c_void_p, _c_long] + [_c_int] * 8 + [_c_void_p] * 2 + [_c_int] * 2 + [_c_void_p] * 5
+                        + [_c_int, ctypes.c_float, _c_int, _c_void_p], _c_int),
+    "kgs_head_proj": ([_c_void_p] * 6 + [_c_long] * 5 + [_c_int] * 7 + [_c_void_p] * 2 + [_c_int] * 3 + [_c_void_p],
+                      _c_int),
+    "kgs_latent_attn": ([_c_void_p] * 10 + [_c_int] * 10 + [ctypes.c_float, _c_void_p], _c_int),
     # residual, talking-heads attention, mixture of experts (residual.hip, talking.hip, moe.hip)
     "kgs_residual_embed": ([_c_void_p] * 3 + [_c_long, ctypes.c_float] + [_c_void_p] * 2 + [_c_long, _c_void_p]
                            + [_c_int] * 5 + [ctypes.c_float] * 2 + [_c_int, _c_void_p], _c_int),
@@ -119,8 +125,8 @@ _SIGS = {
                          + [_c_void_p, _c_int] + [_c_void_p, _c_long, _c_void_p] * 2
                          + [_c_void_p] * 2 + [_c_long, ctypes.c_float] + [_c_void_p] * 2 + [_c_long, _c_void_p]
                          + [_c_int] * 5 + [ctypes.c_float] * 2 + [_c_int, _c_void_p], _c_int),
-    "kgs_talking_write": ([_c_void_p, _c_long] + [_c_void_p] * 3 + [_c_int] * 7 + [_c_void_p] * 2 + [_c_int] * 3
-                          + [_c_void_p], _c_int),
+    "kgs_talking_write": ([_c_void_p, _c_long] + [_c_void_p] * 3 + [_c_int] * 7 + [_c_void_p] * 2 + [_c_int] * 2
+                          + [_c_void_p] * 2 + [_c_int] * 2 + [ctypes.c_float] * 2 + [_c_int] * 2 + [_c_void_p], _c_int),
     "kgs_talking_rows": ([_c_void_p, _c_long, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_int] + [_c_void_p] * 8
                          + [_c_int] * 10 + [_c_void_p], _c_int),
     "kgs_talking_tiles": ([_c_void_p, _c_long, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_int, _c_void_p, _c_int,
@@ -133,16 +139,17 @@ _SIGS = {
                         + [ctypes.c_float] + [_c_int] * 3 + [_c_void_p], _c_int),
     # softmax attention over head pages, lightning attention (paged.hip, lightning.hip)
     "kgs_paged_rows": ([_c_void_p, _c_long, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_int] + [_c_void_p] * 5
-                       + [ctypes.c_float] + [_c_int] * 9 + [_c_void_p], _c_int),
+                       + [ctypes.c_float] + [_c_int] * 8 + [ctypes.c_float] * 3 + [_c_int] * 3 + [_c_void_p], _c_int),
     "kgs_paged_tiles": ([_c_void_p, _c_long, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_int, _c_void_p, _c_int,
-                         ctypes.c_float] + [_c_int] * 5 + [_c_void_p], _c_int),
+                         ctypes.c_float] + [_c_int] * 7 + [ctypes.c_float] * 3 + [_c_void_p], _c_int),
     "kgs_lightning_forward": ([_c_void_p, _c_long] + [_c_int] * 3 + [_c_void_p] * 5 + [_c_int, _c_void_p] * 2
                               + [_c_int, _c_void_p, _c_void_p, _c_int] + [_c_void_p] * 3 + [_c_int] * 4 + [_c_void_p], _c_int),
     "kgs_lightning_out": ([_c_void_p] * 3 + [_c_long, _c_void_p, _c_long] + [_c_int] * 3 + [ctypes.c_float, _c_int,
                                                                                              _c_void_p], _c_int),
-    "kgs_latent_attn_simple": ([_c_void_p] * 6 + [_c_int] * 4 + [ctypes.c_float, _c_int, _c_void_p], _c_int),
-    "kgs_attn_fwd_ragged_bf16": ([_c_void_p] * 5 + [_c_int] * 3 + [_c_long] * 4 + [ctypes.c_float, _c_void_p, _c_long,
-                                                                                  _c_void_p], _c_int),
+    "kgs_latent_attn_simple": ([_c_void_p] * 6 + [_c_int] * 6 + [ctypes.c_float, _c_int, _c_void_p], _c_int),
+    "kgs_attn_fwd_ragged_bf16": ([_c_void_p] * 5 + [_c_int] * 3 + [_c_long] * 4 + [ctypes.c_float, _c_void_p, _c_long]
+                                 + [_c_int] * 2 + [_c_void_p, _c_long, _c_int] + [_c_void_p] * 2 + [_c_int] * 3
+                                 + [_c_void_p], _c_int),
     "kgs_delta_forward": ([ctypes.POINTER(_c_void_p), ctypes.POINTER(_c_long), _c_void_p], _c_int),
     "kgs_delta_out": ([_c_void_p] * 4 + [_c_int] * 3 + [_c_long] * 2 + [ctypes.c_float, _c_int, _c_void_p], _c_int),
     # peer-to-peer all-reduce (native/kernels/allreduce_p2p.hip)

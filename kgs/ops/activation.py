@@ -1,5 +1,6 @@
 """Elementwise steps around the projections (``native/kernels/activation.hip``),
-bf16 or fp32: the gated feed-forward product and the logits' soft cap."""
+bf16 or fp32: the gated feed-forward product, the normed powers of a feed-forward row and
+the logits' soft cap."""
 from __future__ import annotations
 
 from dataclasses import dataclass
@@ -53,6 +54,20 @@ def act_mul(gu: torch.Tensor, act) -> torch.Tensor:
     rc = _lib.lib().kgs_act_mul(gu.data_ptr(), out.data_ptr(), rows, n, gu.stride(0), n, ACTS[gate.act], float(gate.limit),
                                 int(gu.dtype == torch.float32), _lib.stream_handle(gu.device))
     _lib.check(rc, f"act_mul[{rows}x{n}]")
+    return out
+
+
+def poly_norm(z: torch.Tensor, c: torch.Tensor, n: int, eps: float) -> torch.Tensor:
+    """``c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3`` row by row, N dividing by the root mean square
+    of the row's first ``n`` values (the others are zero padding); ``c`` fp32 ``[4]``."""
+    _mat(z, "z")
+    if c.dtype != torch.float32 or tuple(c.shape) != (4,) or not c.is_cuda:
+        raise ValueError("c must be four fp32 numbers on the GPU")
+    rows, cols = z.shape
+    out = torch.empty((rows, cols), dtype=z.dtype, device=z.device)
+    rc = _lib.lib().kgs_poly_norm(z.data_ptr(), z.stride(0), c.data_ptr(), out.data_ptr(), cols, rows, n, cols, float(eps),
+                                  int(z.dtype == torch.float32), _lib.stream_handle(z.device))
+    _lib.check(rc, f"poly_norm[{rows}x{n}]")
     return out
 
 

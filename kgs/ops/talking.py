@@ -41,6 +41,7 @@ class Heads:
     dkp: int             # padded query / key size
     dvp: int             # padded value size
     mfma: bool           # the MFMA kernels take it (bf16)
+    maps: int = 1        # 2: differential heads, dkp holds the keys of both maps
 
     @property
     def group(self) -> int:
@@ -233,23 +234,44 @@ class Rotary:
         self.table = t.float().to(device).contiguous()
 
 
-def write_kv(z: torch.Tensor, bias: torch.Tensor, pages: torch.Tensor, slots: torch.Tensor, h: Heads, ok: int,
-             ov: int, rotary: Rotary | None = None, pos: torch.Tensor | None = None) -> None:
+@dataclass
+class HeadNorm:
+    """RMS norm of every head's (and map's) q and k over its ``dim`` values, times ``wq`` /
+    ``wk`` (fp32, zero-padded to the head's columns)."""
+    wq: torch.Tensor
+    wk: torch.Tensor
+    dim: int
+    eps: float
+
+
+@dataclass(frozen=True)
+class Temperature:
+    """q at position p times ``1 + coef ln(floor((p + 1) / every) + 1)``."""
+    coef: float
+    every: int
+
+
+def write_kv(z: torch.Tensor, bias: torch.Tensor | None, pages: torch.Tensor, slots: torch.Tensor, h: Heads, ok: int,
+             ov: int, rotary: Rotary | None = None, pos: torch.Tensor | None = None, norm: HeadNorm | None = None,
+             temperature: Temperature | None = None) -> None:
     """``z [T, >=]`` holds q (columns 0 ..), k (``ok`` ..) and v (``ov`` ..), heads padded.
-    Adds the biases (``bias``: q, k, v one after another): q in place, k and v into
-    ``pages`` at ``slots`` (-1: dropped). ``rotary``: q and k turned by the rows' ``pos``
-    (int32 ``[T]``)."""
+    Adds the biases (``bias``: q, k, v one after another, or None): q in place, k and v into
+    ``pages`` at ``slots`` (-1: dropped). ``norm``: q and k normed per head and map; ``rotary``:
+    turned by the rows' ``pos`` (int32 ``[T]``); ``temperature``: q scaled by position."""
     T, nq, nk, nv = z.shape[0], h.heads * h.dkp, h.kv_heads * h.dkp, h.kv_heads * h.dvp
     if pages.dtype != z.dtype or not pages.is_contiguous() or pages.shape[1:] != (h.kv_heads, PAGE * (h.dkp + h.dvp)):
         raise ValueError(f"pages {tuple(pages.shape)} {pages.dtype} do not fit {h}")
-    turn = (0, 0, 0, 0)
-    if rotary is not None:
+    turn, seg = (0, 0, 0, 0), h.dkp // h.maps
+    if rotary is not None or temperature is not None:
         if pos is None or pos.dtype != torch.int32 or not pos.is_contiguous() or pos.shape[0] != T:
-            raise ValueError("rotary positions need contiguous int32 positions of the rows")
-        turn = (rotary.table.data_ptr(), pos.data_ptr(), *rotary.table.shape)
+            raise ValueError("positions of the rows must be contiguous int32")
+        turn = (0, pos.data_ptr(), 0, 0) if rotary is None else (rotary.table.data_ptr(), pos.data_ptr(), *rotary.table.shape)
+    normed = (0, 0, seg, seg, 0.0) if norm is None else (_f32(norm.wq, (seg,), "wq"), _f32(norm.wk, (seg,), "wk"), seg,
+                                                         norm.dim, float(norm.eps))
+    warm = (0.0, 0) if temperature is None else (float(temperature.coef), temperature.every)
     rc = _lib.lib().kgs_talking_write(_act(z, T, max(nq, ok + nk, ov + nv), z.dtype, "z"), z.stride(0),
-                                      _f32(bias, (nq + nk + nv,), "bias"), pages.data_ptr(), slots.data_ptr(), T, nq,
-                                      h.kv_heads, h.dkp, h.dvp, ok, ov, *turn, int(z.dtype == torch.float32),
+                                      0 if bias is None else _f32(bias, (nq + nk + nv,), "bias"), pages.data_ptr(), slots.data_ptr(), T, nq,
+                                      h.kv_heads, h.dkp, h.dvp, ok, ov, *turn, *normed, *warm, int(z.dtype == torch.float32),
                                       _lib.stream_handle(z.device))
     _lib.check(rc, f"talking_write[{T}]")
 

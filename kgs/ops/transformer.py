@@ -227,21 +227,38 @@ def attention_chunk(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, heads: in
 
 
 def attention_ragged(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, items: torch.Tensor, heads: int,
-                     head_dim: int, scale: float, out: torch.Tensor, gate: torch.Tensor | None = None) -> torch.Tensor:
+                     head_dim: int, scale: float, out: torch.Tensor, gate: torch.Tensor | None = None,
+                     each: bool = False, window: int = 0, kr: torch.Tensor | None = None, rotary=None,
+                     pos: torch.Tensor | None = None) -> torch.Tensor:
     """Causal flash attention of ragged prompt portions in one launch (head_dim 64
     or 128, as many key heads as query heads). ``items`` int32 ``[n, 4]``: a block
     of up to 128 query rows each -- its first row in ``q`` / ``out``, the row of
-    its sequence's key 0 in ``k`` / ``v``, the first row's position, the rows.
-    ``gate [rows, >= heads]``: head outputs times its sigmoid."""
+    its sequence's key 0 in ``k`` / ``v``, the number of the first row's own key, the rows.
+    ``gate [rows, >= heads]``: head outputs times its sigmoid (``each``: a column for every
+    output). ``window``: a row sees its own key and the ``window - 1`` before it (0: all).
+    ``kr [key rows, 32 or 64]``: a further part of every head's keys; ``q`` then has as many
+    columns after each head's ``head_dim``, turned by the rows' ``pos`` (``rotary``:
+    :class:`kgs.ops.talking.Rotary`, int32 positions)."""
+    hr = 0 if kr is None else kr.shape[1]
     for t, n in ((q, "q"), (k, "k"), (v, "v"), (out, "out")):
         _need(t, n)
     if items.dtype != torch.int32 or items.dim() != 2 or items.shape[1] != 4 or not items.is_contiguous():
         raise ValueError("items must be contiguous int32 [n, 4]")
+    turn = (0, 0, 0, 0)
+    if hr:
+        _need(kr, "kr")
+        if pos.dtype != torch.int32 or not pos.is_contiguous() or pos.shape[0] < q.shape[0]:
+            raise ValueError("rotary positions need contiguous int32 positions of the rows")
+        turn = (rotary.table.data_ptr(), pos.data_ptr(), *rotary.table.shape)
+    if gate is not None:
+        _need(gate, "gate")
     rc = _lib.lib().kgs_attn_fwd_ragged_bf16(q.data_ptr(), k.data_ptr(), v.data_ptr(), out.data_ptr(),
                                              items.data_ptr(), items.shape[0], heads, head_dim, q.stride(0),
                                              k.stride(0), v.stride(0), out.stride(0), float(scale),
                                              0 if gate is None else gate.data_ptr(),
-                                             0 if gate is None else gate.stride(0), _lib.stream_handle(q.device))
+                                             0 if gate is None else gate.stride(0), head_dim if each else 1, int(each),
+                                             0 if kr is None else kr.data_ptr(), 0 if kr is None else kr.stride(0), hr,
+                                             *turn, window, _lib.stream_handle(q.device))
     _lib.check(rc, "attention_ragged")
     return out
 

@@ -27,8 +27,8 @@ from kgs.ops import decode as D
 from kgs.ops.decode import PAGE
 from kgs.ops.delta import DeltaShape, DeltaState, delta_forward, delta_out
 from kgs.ops.hyper import MAX_STREAMS, hyper_embed, hyper_step
-from kgs.ops.latent import (KERNEL_SIZES, LatentCache, LatentRows, head_proj, latent_attention, latent_norm,
-                            padded_latent, split_count, waves_for)
+from kgs.ops.latent import (LatentCache, LatentRows, head_proj, latent_attention, latent_norm, mfma_sizes,
+                            padded_latent, padded_rot, split_count, waves_for, window_pages)
 from kgs.ops.linear import Projection
 from kgs.ops.transformer import attention_ragged
 
@@ -39,9 +39,14 @@ EXPAND_MIN = 16  # shorter portions are not worth the expansion's launches
 QBLOCK = 128  # query rows of one attention_ragged item
 
 
+def latent_row(m: LatentSpec) -> int:
+    """Columns of a cache row."""
+    return padded_latent(m.kv_rank) + padded_rot(m.rot_dim)
+
+
 def latent_sizes(cfg: RuruzenConfig) -> dict[int, int]:
-    """Padded latent size of every layer that caches one."""
-    return {i: padded_latent(x.mixer.kv_rank) for i, x in enumerate(cfg.layers)
+    """Columns of a cache row of every layer that caches a latent."""
+    return {i: latent_row(x.mixer) for i, x in enumerate(cfg.layers)
             if isinstance(x.mixer, LatentSpec) and x.mixer.kv_from is None}
 
 
@@ -69,14 +74,24 @@ class Geometry:
     heads: int
     rp: int
     hd: int                    # head size of the expanded form, 0: absorbed only
+    window: int = 0            # 0: every earlier key
+
+    def pages(self, pages: int, queries: int) -> int:
+        """Most of ``pages`` that a tile of ``queries`` tokens reads."""
+        return min(pages, window_pages(self.window, queries)) if self.window else pages
 
     def expand(self, n: int, pos0: int) -> bool:
         """Whether a portion of ``n`` tokens after ``pos0`` runs on expanded keys and
         values. Per head that expands every context token (``4 rp hd`` flops each)
         where the absorbed form maps every query token (as many), and pays ``4 hd``
         per (query, key) pair where the absorbed form pays ``4 rp``."""
-        pairs = n * (pos0 + 0.5 * n)
-        return self.hd > 0 and n >= EXPAND_MIN and pos0 * self.rp * self.hd < (self.rp - self.hd) * pairs
+        if self.window:
+            ctx = min(pos0, self.window - 1)
+            grow = min(n, max(0, self.window - pos0))  # tokens that see one key more than the last
+            pairs = grow * (pos0 + 0.5 * grow) + (n - grow) * self.window
+        else:
+            ctx, pairs = pos0, n * (pos0 + 0.5 * n)
+        return self.hd > 0 and n >= EXPAND_MIN and ctx * self.rp * self.hd < (self.rp - self.hd) * pairs
 
     def lay_out(self, pk: HostPack, row0, n, pos0, bt, row_seq, pos, refs):
         """Splits the sequences between the absorbed and the expanded form and adds
@@ -99,7 +114,7 @@ class Geometry:
             ident = len(sel) == len(n) and np.array_equal(q0, row0)
             order = None if ident else np.concatenate([np.arange(r, r + c) for r, c in zip(row0[sel], ns)])
             at = np.arange(len(row_seq)) if order is None else order
-            maxp = int((pos0[sel] + ns - 1).max()) // PAGE + 1
+            maxp = self.pages(int((pos0[sel] + ns - 1).max()) // PAGE + 1, 16 * waves // self.heads + 2)
             absorbed = ({"q0": pk.add(q0), "n": pk.add(ns), "pos0": pk.add(pos0[sel]),
                          "bt": refs[7] if ident else pk.add(bt[sel]),
                          "tok_seq": pk.add(np.repeat(np.arange(len(sel)), ns)), "tok_pos": pk.add(pos[at]),
@@ -110,12 +125,12 @@ class Geometry:
         if len(sel):
             items, ctx, base = [], [], 0
             for s in sel:
-                total = int(pos0[s] + n[s])
-                p = np.arange(total)
+                first = max(0, int(pos0[s]) - self.window + 1) if self.window else 0
+                p = np.arange(first, int(pos0[s] + n[s]))
                 ctx.append(bt[s][p // PAGE].astype(np.int64) * PAGE + p % PAGE)
                 for q in range(0, int(n[s]), QBLOCK):
-                    items.append((row0[s] + q, base, pos0[s] + q, min(QBLOCK, n[s] - q)))
-                base += total
+                    items.append((row0[s] + q, base, pos0[s] - first + q, min(QBLOCK, n[s] - q)))
+                base += len(p)
             items = np.array(items, np.int64)
             items = items[np.argsort(-(items[:, 2] + items[:, 3]), kind="stable")]
             expanded = (pk.add(items), pk.add(np.concatenate(ctx)))
@@ -142,37 +157,55 @@ class Geometry:
         return LatentPlan(LatentRows(
             nt=nb, q0=f["ar"], n=f["one"], pos0=positions, bt=block_tables, tok_seq=f["ar"], tok_pos=positions,
             rows=None, items=None, ntiles=nb * tiles, tiles=tiles, waves=waves,
-            nsplit=split_count(nb * tiles, block_tables.shape[1], self.rp)), None)
+            nsplit=split_count(nb * tiles, self.pages(block_tables.shape[1], 1), self.rp)), None)
 
 
 # -------------------------------------------------------------------- sublayers
+def neighbours(t: torch.Tensor, dim: int) -> torch.Tensor:
+    """Rows whose first half turns with the second one's, reordered to neighbouring pairs (a
+    score does not depend on the order that q and k share)."""
+    a, b = t.chunk(2, dim)
+    return torch.stack([a, b], dim + 1).flatten(dim, dim + 1)
+
+
 class LatentMixer:
+    """``pages`` of a call: the cache of the layer (default: the model's, by layer)."""
+
     def __init__(self, model, i: int, m: LatentSpec, w: Weights):
         p = f"l{i}.mix."
         cfg = model.cfg
         self.m, self.owner = m, i if m.kv_from is None else m.kv_from
         self.layer = i
         self.eps = cfg.eps
-        names = ["dq", "g"] + (["dkv"] if m.kv_from is None else [])
-        win, offs = w.stack([p + n for n in names], model.wp)
+        H, own = m.heads, m.kv_from is None
+        rp, hr = padded_latent(m.kv_rank), padded_rot(m.rot_dim)
+        both = max(m.dim, m.vdim)
+        hd = (64 if both <= 64 else 128 if both <= 128 else 0) if w.dtype == torch.bfloat16 and mfma_sizes(32, hr) else 0
+        self.hq, self.hv, self.hr = (hd, hd, hr) if hd else (pad64(m.dim), pad64(m.vdim), hr)
+        self.gate_cols = H * self.hv if m.gate_each else H
+        dkv = w.w[p + "dkv"] if own else None
+        parts = [w.w[p + "dq"], w.heads(w.w[p + "g"], H, m.vdim, self.hv) if m.gate_each else w.w[p + "g"]]
+        parts += [dkv[:m.kv_rank]] if own else []
+        parts += [neighbours(dkv[m.kv_rank:], 0)] if own and hr else []
+        win, offs = w.join(parts, model.wp)
         self.win = w.proj(win)
         self.oq, self.og = offs[0], offs[1]
-        self.oc = offs[2] if m.kv_from is None else 0
+        self.oc = offs[2] if own else 0
+        self.okr = offs[3] if own and hr else 0
+        self.rotary = model.rotary(m.rot_dim, m.rot_base) if hr else None
         self.wq = w.f32(p + "dq.norm")
-        self.wc = w.f32(p + "dkv.norm") if m.kv_from is None else None
+        self.wc = w.f32(p + "dkv.norm") if own else None
         self.qp = padk(m.q_rank)
-        rp = padded_latent(m.kv_rank)
-        both = max(m.dim, m.vdim)
-        hd = (64 if both <= 64 else 128 if both <= 128 else 0) if w.dtype == torch.bfloat16 else 0
-        self.hq, self.hv = (hd, hd) if hd else (pad64(m.dim), pad64(m.vdim))
-        self.geo = Geometry(m.heads, rp, hd)
-        H = m.heads
+        self.geo = Geometry(m.heads, rp, hd, m.window)
 
         def heads(name, d, dp, rank, rankp):
             t = w.w[p + name].to(w.device).to(w.dtype).reshape(H, d, rank)
             return _pad(t, dp, rankp)
 
-        self.uq = w.proj(heads("uq", m.dim, self.hq, m.q_rank, self.qp).reshape(H * self.hq, self.qp))
+        uq = w.w[p + "uq"].to(w.device).to(w.dtype).reshape(H, m.dim + m.rot_dim, m.q_rank)
+        uq = torch.cat([_pad(uq[:, :m.dim], self.hq, self.qp)]
+                       + ([_pad(neighbours(uq[:, m.dim:], 1), hr, self.qp)] if hr else []), 1)
+        self.uq = w.proj(uq.reshape(-1, self.qp))
         uk = heads("uk", m.dim, self.hq, m.kv_rank, rp)
         self.uv = heads("uv", m.vdim, self.hv, m.kv_rank, rp).contiguous()          # [H, HV, RP]
         self.ukt = uk.transpose(1, 2).contiguous()                                  # [H, RP, HQ]
@@ -180,30 +213,32 @@ class LatentMixer:
         o = w.w[p + "o"].to(w.device).to(w.dtype).reshape(cfg.width, H, m.vdim)
         self.o = w.proj(_pad(_pad(o, self.hv).reshape(cfg.width, H * self.hv), model.wp, H * self.hv))
 
-    def __call__(self, model, h: torch.Tensor, b: Batch) -> torch.Tensor:
-        m, geo = self.m, self.geo
+    def __call__(self, model, h: torch.Tensor, b: Batch, pages: torch.Tensor | None = None) -> torch.Tensor:
+        m, geo, hr = self.m, self.geo, self.hr
         z = self.win(h)
-        pages = model.cache.pages[self.owner]
+        if pages is None:
+            pages = model.cache.pages[self.owner]
         cq = latent_norm(z, self.oq, self.wq, self.qp, self.oc, self.wc, pages if self.wc is not None else None,
-                         b.slots, self.eps)
+                         b.slots, self.eps, geo.rp, self.okr, self.rotary, b.pos)
         q = self.uq(cq)
         T.op(f"L{self.layer} latent projections")
-        gate = z[:, self.og:self.og + m.heads]
+        gate = z[:, self.og:self.og + self.gate_cols]
         plan = b.plans[geo]
         a = torch.empty((h.shape[0], m.heads * self.hv), dtype=h.dtype, device=h.device)
         if plan.expanded is not None:
             e = plan.expanded
-            c = pages.view(-1, geo.rp).index_select(0, e.ctx_slots)
-            kv = self.ukv(c)
+            c = pages.view(-1, geo.rp + hr).index_select(0, e.ctx_slots)
+            kv = self.ukv(c[:, :geo.rp])
             n = m.heads * geo.hd
-            attention_ragged(q, kv[:, :n], kv[:, n:], e.items, m.heads, geo.hd, m.scale, a, gate=gate)
+            attention_ragged(q, kv[:, :n], kv[:, n:], e.items, m.heads, geo.hd, m.scale, a, gate=gate, each=m.gate_each,
+                             window=m.window, kr=c[:, geo.rp:] if hr else None, rotary=self.rotary, pos=b.pos)
             T.op(f"L{self.layer} expanded attention")
         if plan.absorbed is not None:
             r = plan.absorbed
-            ql = torch.empty((r.nt, m.heads * geo.rp), dtype=h.dtype, device=h.device)
-            head_proj(q, self.ukt, r.nt, ql, rows_in=r.rows)
-            ol = latent_attention(ql, pages, r, m.heads, m.scale)
-            head_proj(ol, self.uv, r.nt, a, rows_out=r.rows, gate=gate)
+            ql = torch.empty((r.nt, m.heads * (geo.rp + hr)), dtype=h.dtype, device=h.device)
+            head_proj(q, self.ukt, r.nt, ql, rows_in=r.rows, hr=hr, rotary=self.rotary, pos=r.tok_pos)
+            ol = latent_attention(ql, pages, r, m.heads, m.scale, hr, m.window)
+            head_proj(ol, self.uv, r.nt, a, rows_out=r.rows, gate=gate, each=m.gate_each)
             T.op(f"L{self.layer} latent attention")
         return self.o(a)
 

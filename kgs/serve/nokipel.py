@@ -29,7 +29,7 @@ from kgs.ops.lightning import (CHUNK_DIM, Decays, LightningShape, LightningState
 from kgs.ops.paged import (Portions, paged_heads, paged_rows, paged_tiles, portion_items, row_splits, tile_queries,
                            visible_pages)
 from kgs.ops.residual import MAX_WIDTH, Embedding, ExpertRows, Norm, Scaled, residual_add, residual_embed
-from kgs.ops.talking import HeadPages, Heads, QueryRows, Rotary, write_kv
+from kgs.ops.talking import HeadPages, Heads, QueryRows, write_kv
 
 from .ragged import DTYPES, Batch, HostPack, RaggedModel, Weights, _pad, pad64, pad128, pad256, padk
 from .trace import TRACE as T
@@ -70,7 +70,7 @@ class ChunkedGeometry:
             pages = max(visible_pages(int(p), self.chunk) for p in pos[at])
             rows = ({"tok_seq": refs[2] if whole else pk.add(row_seq[at]),
                      "tok_pos": refs[9] if whole else pk.add(pos[at]),
-                     "rows": None if whole else pk.add(at)}, len(at), row_splits(len(at), h.kv_heads, h.group, pages))
+                     "rows": None if whole else pk.add(at)}, len(at), row_splits(len(at), h.kv_heads, h.group, pages, h.maps))
         if tiled.any():
             sel = np.flatnonzero(tiled)
             items = pk.add(portion_items([(row0[s], s, pos0[s], n[s]) for s in sel], tile_queries(h), self.chunk))
@@ -89,7 +89,8 @@ class ChunkedGeometry:
         if self.chunk:
             pages = min(pages, (self.chunk - 1) // D.PAGE + 2)
         return ChunkedPlan(QueryRows(nb, block_tables, f["ar"], positions, None,
-                                     row_splits(nb, self.heads.kv_heads, self.heads.group, pages)), None)
+                                     row_splits(nb, self.heads.kv_heads, self.heads.group, pages,
+                                                self.heads.maps)), None)
 
 
 @dataclass(frozen=True)
@@ -120,21 +121,13 @@ def _head_rows(t: torch.Tensor, n: int, d: int, dp: int) -> torch.Tensor:
     return _pad(t.reshape(n, d, -1), dp, t.shape[-1]).reshape(n * dp, -1)
 
 
-def _input_matrix(w: Weights, p: str, parts, wp: int) -> tuple[torch.Tensor, list[int]]:
-    """Projections of one input (name, heads, size, padded size) as one matrix, each from
-    a multiple of 64 rows on; returns it and the first rows."""
-    mats, offs, at = [], [], 0
-    for name, n, d, dp in parts:
-        t = _head_rows(w.w[p + name].to(w.device).to(w.dtype), n, d, dp)
-        mats.append(_pad(t, pad64(n * dp), wp))
-        offs.append(at)
-        at += mats[-1].shape[0]
-    if at > 1024 and at % 256:  # whole 256-wide GEMM tiles
-        mats.append(torch.zeros((256 - at % 256, wp), dtype=w.dtype, device=w.device))
-    return torch.cat(mats).contiguous(), offs
+def input_matrix(w: Weights, p: str, parts, wp: int) -> tuple[torch.Tensor, list[int]]:
+    """Projections of one input (name, heads, size, padded size) as one matrix
+    (:meth:`Weights.join`)."""
+    return w.join([w.heads(w.w[p + name], n, d, dp) for name, n, d, dp in parts], wp)
 
 
-def _output_matrix(w: Weights, name: str, n: int, d: int, dp: int, wp: int, cols: int) -> torch.Tensor:
+def output_matrix(w: Weights, name: str, n: int, d: int, dp: int, wp: int, cols: int) -> torch.Tensor:
     o = w.w[name].to(w.device).to(w.dtype)
     return _pad(_pad(o.reshape(o.shape[0], n, d), dp).reshape(o.shape[0], n * dp), wp, cols)
 
@@ -146,12 +139,12 @@ class ChunkedMixer:
         h = self.heads
         self.geo = ChunkedGeometry(h, m.chunk)
         parts = (("q", m.heads, m.dim, h.dkp), ("k", m.kv_heads, m.dim, h.dkp), ("v", m.kv_heads, m.vdim, h.dvp))
-        win, self.offs = _input_matrix(w, p, parts, wp)
+        win, self.offs = input_matrix(w, p, parts, wp)
         self.win = w.proj(win)
         self.bias = torch.cat([_head_rows(w.f32(f"{p}{n}.b")[:, None], c, d, dp).reshape(-1)
                                for n, c, d, dp in parts]).contiguous()
         self.rotary = model.rotary(m.rot_dims, m.rot_base) if m.rot_dims else None
-        self.o = w.proj(_output_matrix(w, p + "o", m.heads, m.vdim, h.dvp, wp, m.heads * h.dvp))
+        self.o = w.proj(output_matrix(w, p + "o", m.heads, m.vdim, h.dvp, wp, m.heads * h.dvp))
 
     def __call__(self, model, run: int, h: torch.Tensor, b: Batch) -> torch.Tensor:
         hd, m, plan = self.heads, self.m, b.plans[self.geo]
@@ -175,14 +168,14 @@ class LightningMixer:
         s = self.shape
         self.geo = LightningGeometry(m.heads * s.slabs, w.dtype == torch.bfloat16 and m.dim <= CHUNK_DIM)
         parts = [(n, m.heads, m.dim, s.kp) for n in "qk"] + [(n, m.heads, m.vdim, s.vp) for n in "vg"]
-        win, offs = _input_matrix(w, p, parts, wp)
+        win, offs = input_matrix(w, p, parts, wp)
         self.win = w.proj(win)
         self.offs, self.og = tuple(offs[:3]), offs[3]
         self.decays = Decays(m.decay, w.device)
         self.count, n = m.heads * m.vdim, m.heads * s.vp
         self.norm = _head_rows(w.f32(p + "norm")[:, None], m.heads, m.vdim, s.vp).reshape(-1).contiguous()
         self.ld = padk(n)
-        self.o = w.proj(_output_matrix(w, p + "o", m.heads, m.vdim, s.vp, wp, self.ld))
+        self.o = w.proj(output_matrix(w, p + "o", m.heads, m.vdim, s.vp, wp, self.ld))
 
     def __call__(self, model, run: int, h: torch.Tensor, b: Batch) -> torch.Tensor:
         z = self.win(h)
@@ -247,7 +240,7 @@ class NokipelModel(RaggedModel):
                  packed_decode: bool = True):
         super().__init__()
         self.cfg, self.device, self.dtype = cfg, torch.device(device), DTYPES[dtype]
-        self.has_state, self.max_len, self._rotary = cfg.has_state, max_len, {}
+        self.has_state, self.max_len = cfg.has_state, max_len
         self.wp = pad256(cfg.width)
         if self.wp > MAX_WIDTH:
             raise ValueError(f"width {cfg.width} is above {MAX_WIDTH}")
@@ -288,11 +281,6 @@ class NokipelModel(RaggedModel):
     def _shapes(cfg: NokipelConfig) -> dict[int, LightningShape]:
         return {r: lightning_shape(cfg.layers[i].mixer) for r, (i, _) in enumerate(cfg.runs)
                 if isinstance(cfg.layers[i].mixer, LightningSpec)}
-
-    def rotary(self, dims: int, base: float) -> Rotary:
-        if (dims, base) not in self._rotary:
-            self._rotary[dims, base] = Rotary(dims, base, self.max_len, self.device)
-        return self._rotary[dims, base]
 
     @classmethod
     def for_engine(cls, cfg: NokipelConfig, ec, device, backend: str, num_pages: int) -> "NokipelModel":

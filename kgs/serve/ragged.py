@@ -20,6 +20,7 @@ import torch
 
 from kgs.ops.delta import RaggedSeqs, chunk_plan
 from kgs.ops.linear import Projection
+from kgs.ops.talking import Rotary
 
 DTYPES = {"bfloat16": torch.bfloat16, "float32": torch.float32}
 
@@ -100,12 +101,21 @@ class Weights:
     def mat(self, name: str, rows: int, cols: int) -> torch.Tensor:
         return _pad(self.w[name].to(self.device).to(self.dtype), rows, cols)
 
+    def heads(self, t: torch.Tensor, n: int, d: int, dp: int) -> torch.Tensor:
+        """``[n d, ..] -> [n dp, ..]`` on the device, every head padded."""
+        t = t.to(self.device).to(self.dtype)
+        return _pad(t.reshape(n, d, -1), dp, t.shape[-1]).reshape(n * dp, -1)
+
     def stack(self, names, cols: int) -> tuple[torch.Tensor, list[int]]:
         """Several projections of one input as one matrix, each from a multiple of
         64 rows on (a large one ends on whole GEMM tiles); returns it and the first rows."""
+        return self.join([self.w[name] for name in names], cols)
+
+    def join(self, tensors, cols: int) -> tuple[torch.Tensor, list[int]]:
+        """:meth:`stack` of tensors."""
         parts, offs, n = [], [], 0
-        for name in names:
-            p = self.mat(name, pad64(self.w[name].shape[0]), cols)
+        for t in tensors:
+            p = _pad(t.to(self.device).to(self.dtype), pad64(t.shape[0]), cols)
             offs.append(n)
             n += p.shape[0]
             parts.append(p)
@@ -130,7 +140,13 @@ class RaggedModel:
     def __init__(self):
         self._fixed: dict = {}
         self.geometries: set = set()
+        self.max_len, self._rotary = 0, {}  # positions of the rotary tables, and these
         self.on_layer = None  # tests: called with (layer, residual) after every layer
+
+    def rotary(self, dims: int, base: float) -> Rotary:
+        if (dims, base) not in self._rotary:
+            self._rotary[dims, base] = Rotary(dims, base, self.max_len, self.device)
+        return self._rotary[dims, base]
 
     @staticmethod
     def check_engine(ec, backend: str) -> None:

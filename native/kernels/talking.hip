@@ -66,7 +66,7 @@ typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
 struct WriteArgs {
   void* z;             // [T, ldz]: q | k | v from columns 0, ok, ov, heads padded to dkp / dvp
   long ldz;
-  const float* b;      // [nq + nk + nv] biases in that order
+  const float* b;      // [nq + nk + nv] biases in that order, or null
   void* pages;
   const int* slots;    // [T], -1: not cached
   int T, nq, G, dkp, dvp, ok, ov;
@@ -75,6 +75,13 @@ struct WriteArgs {
   const float* cs;
   const int* pos;      // [T]
   int npos, rot;
+  // RMS norm of q and k per `seg` columns (`dim` of them without the padding) times wq / wk [seg]
+  const float *wq, *wk;
+  int seg, dim;
+  float eps;
+  // q at position p times 1 + coef ln(floor((p + 1) / every) + 1); every 0: none
+  float coef;
+  int every;
 };
 
 template <typename T>
@@ -82,32 +89,80 @@ struct Vec8 {
   T v[8];
 };
 
-// One thread: 8 columns of 8 rows. q gets its bias (and rotation) in place; k and v get theirs and
-// go to the page, v as 8 tokens of a dim where the rows allow it.
-template <typename T>
+// One thread: 8 columns of 8 rows. q gets its bias (norm, rotation, temperature) in place; k and v
+// get theirs and go to the page, v as 8 tokens of a dim where the rows allow it. NORM: lanes of a
+// norm's columns: 0 no norm, 8 or 16, 1 any number (workgroups of whole norms, sums through LDS).
+template <typename T, int NORM>
 __global__ __launch_bounds__(256) void write_kv(WriteArgs a) {
   const int nk = a.G * a.dkp, nv = a.G * a.dvp;
-  const int col = (blockIdx.x * 256 + threadIdx.x) * 8, r0 = blockIdx.y * 8, nr = min(8, a.T - r0);
-  if (col >= a.nq + nk + nv) return;
-  const int kind = col < a.nq ? 0 : col < a.nq + nk ? 1 : 2;
-  const int c = kind == 0 ? col : kind == 1 ? col - a.nq : col - a.nq - nk;
+  const int per_wg = NORM == 1 ? 256 / (a.seg / 8) * (a.seg / 8) : 256;
+  const int col = (blockIdx.x * per_wg + threadIdx.x) * 8, r0 = blockIdx.y * 8, nr = min(8, a.T - r0);
+  const bool in = col < a.nq + nk + nv && (int)threadIdx.x < per_wg;
+  if (NORM != 1 && !in) return;
+  const int kind = !in || col >= a.nq + nk ? 2 : col < a.nq ? 0 : 1;
+  const int c = !in ? 0 : kind == 0 ? col : kind == 1 ? col - a.nq : col - a.nq - nk;
   const int zc = kind == 0 ? c : kind == 1 ? a.ok + c : a.ov + c;
-  const f32x4 b0 = *(const f32x4*)(a.b + col), b1 = *(const f32x4*)(a.b + col + 4);
-  const float b[8] = {b0[0], b0[1], b0[2], b0[3], b1[0], b1[1], b1[2], b1[3]};
-  const int dd = kind == 2 ? 0 : c % a.dkp;
+  float b[8] = {}, nw[8];
+  if (a.b && in) {
+    const f32x4 b0 = *(const f32x4*)(a.b + col), b1 = *(const f32x4*)(a.b + col + 4);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) b[i] = b0[i], b[4 + i] = b1[i];
+  }
+  const int dd = kind == 2 ? 0 : c % a.seg;
   const bool turn = a.cs && kind != 2 && dd < a.rot;
+  if (NORM && kind != 2) {
+    const float* wp = (kind ? a.wk : a.wq) + dd;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) nw[i] = wp[i];
+  }
   int sl[8];
 #pragma unroll
   for (int r = 0; r < 8; ++r) sl[r] = r < nr ? a.slots[r0 + r] : -1;
   Vec8<T> x[8];
-#pragma unroll
-  for (int r = 0; r < 8; ++r) {
-    x[r] = *(const Vec8<T>*)((const T*)a.z + (long)(r0 + min(r, nr - 1)) * a.ldz + zc);
-    float y[8];
+  auto biased = [&](int r, float (&y)[8]) {
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
       if constexpr (sizeof(T) == 2) y[i] = bf2f(x[r].v[i]) + b[i];
       else y[i] = x[r].v[i] + b[i];
+    }
+  };
+#pragma unroll
+  for (int r = 0; r < 8; ++r) x[r] = *(const Vec8<T>*)((const T*)a.z + (long)(r0 + min(r, nr - 1)) * a.ldz + zc);
+  float inv[8];
+  if constexpr (NORM != 0) {
+#pragma unroll
+    for (int r = 0; r < 8; ++r) {
+      float y[8], ss = 0.f;
+      biased(r, y);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) ss = __builtin_fmaf(y[i], y[i], ss);
+      if constexpr (NORM != 1) ss = sum8(ss);
+      if constexpr (NORM == 16) ss += dpp_move<0x140>(ss);
+      inv[r] = ss;
+    }
+    if constexpr (NORM == 1) {
+      __shared__ float part[8][256];
+#pragma unroll
+      for (int r = 0; r < 8; ++r) part[r][threadIdx.x] = inv[r];
+      __syncthreads();
+      if (!in) return;
+      const int t0 = threadIdx.x - threadIdx.x % (a.seg / 8);
+#pragma unroll
+      for (int r = 0; r < 8; ++r) {
+        inv[r] = 0.f;
+        for (int i = 0; i < a.seg / 8; ++i) inv[r] += part[r][t0 + i];
+      }
+    }
+#pragma unroll
+    for (int r = 0; r < 8; ++r) inv[r] = 1.0f / sqrtf(inv[r] / a.dim + a.eps);
+  }
+#pragma unroll
+  for (int r = 0; r < 8; ++r) {
+    float y[8];
+    biased(r, y);
+    if (NORM && kind != 2) {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) y[i] *= inv[r] * nw[i];
     }
     if (turn) {
       const float* p = a.cs + (long)min(max(a.pos[r0 + min(r, nr - 1)], 0), a.npos - 1) * a.rot + dd;
@@ -119,6 +174,11 @@ __global__ __launch_bounds__(256) void write_kv(WriteArgs a) {
         y[i] = rope_lo(u, v, cs[i], cs[i + 1]);
         y[i + 1] = rope_hi(u, v, cs[i], cs[i + 1]);
       }
+    }
+    if (a.every && kind == 0) {
+      const float f = __builtin_fmaf(a.coef, logf((float)((a.pos[r0 + min(r, nr - 1)] + 1) / a.every + 1)), 1.0f);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) y[i] *= f;
     }
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
@@ -1033,24 +1093,34 @@ int check(const Args& a, int n) {
 }  // namespace kgs
 
 // z [T, ldz] holds q from column 0, k from ok, v from ov (heads padded to dkp / dvp);
-// b their biases one after another (nq + G dkp + G dvp). q += b in place, k + b and
-// v + b go to their slots. cs not null: q and k rotated by the row's position, the
-// pairs (0, 1), (2, 3), .. of each head's first `rot` dims by cs [npos][rot / 2][cos, sin].
+// b their biases one after another (nq + G dkp + G dvp), or null. q += b in place, k + b and
+// v + b go to their slots. wq, wk not null: q and k normed per seg columns (dkp or a part of it;
+// dim without padding). cs not null: q and k rotated by the row's position, the
+// pairs (0, 1), (2, 3), .. of each seg's first `rot` dims by cs [npos][rot / 2][cos, sin].
+// every > 0: q times 1 + coef ln(floor((pos + 1) / every) + 1).
 KGS_EXPORT int kgs_talking_write(void* z, long ldz, const void* b, void* pages, const void* slots, int T, int nq, int G,
                                  int dkp, int dvp, int ok, int ov, const void* cs, const void* pos, int npos, int rot,
+                                 const void* wq, const void* wk, int seg, int dim, float eps, float coef, int every,
                                  int f32, hipStream_t s) {
   using namespace kgs::talking;
   if (T <= 0 || nq <= 0 || G <= 0 || dkp <= 0 || dvp <= 0 || dkp % 32 || dvp % 16 || nq % 8 || ok < nq ||
       ldz < ok + G * dkp || ldz < ov + G * dvp || T > 8 * 65535)
     return KGS_ERR_SHAPE;
+  if (seg <= 0 || seg % 8 || dkp % seg || dim <= 0 || dim > seg || every < 0 || (every && !pos) || !wq != !wk)
+    return KGS_ERR_SHAPE;
+  if (wq && (seg > 2048 || nq % dkp)) return KGS_ERR_SHAPE;
   if (ldz % 8 || ok % 8 || ov % 8 || (((uintptr_t)z | (uintptr_t)pages | (uintptr_t)b) & 15)) return KGS_ERR_ALIGN;
-  if (cs && (!pos || npos <= 0 || rot <= 0 || rot % 8 || rot > dkp || nq % dkp)) return KGS_ERR_SHAPE;
+  if (cs && (!pos || npos <= 0 || rot <= 0 || rot % 8 || rot > seg || nq % dkp)) return KGS_ERR_SHAPE;
   if ((uintptr_t)cs & 15) return KGS_ERR_ALIGN;
   WriteArgs a{z, ldz, (const float*)b, pages, (const int*)slots, T, nq, G, dkp, dvp, ok, ov,
-              (const float*)cs, (const int*)pos, npos, rot};
-  const dim3 grid(((nq + G * (dkp + dvp)) / 8 + 255) / 256, (T + 7) / 8);
-  if (f32) hipLaunchKernelGGL(write_kv<float>, grid, dim3(256), 0, s, a);
-  else hipLaunchKernelGGL(write_kv<unsigned short>, grid, dim3(256), 0, s, a);
+              (const float*)cs, (const int*)pos, npos, rot, (const float*)wq, (const float*)wk, seg, dim, eps, coef, every};
+  const int n = (nq + G * (dkp + dvp)) / 8;
+  const int norm = !wq ? 0 : seg == 64 ? 8 : seg == 128 ? 16 : 1, wg = norm == 1 ? 256 / (seg / 8) * (seg / 8) : 256;
+  const dim3 grid((n + wg - 1) / wg, (T + 7) / 8);
+  auto fn = f32 ? (norm == 0 ? write_kv<float, 0> : norm == 8 ? write_kv<float, 8> : norm == 16 ? write_kv<float, 16> : write_kv<float, 1>)
+                : (norm == 0 ? write_kv<unsigned short, 0> : norm == 8 ? write_kv<unsigned short, 8>
+                   : norm == 16 ? write_kv<unsigned short, 16> : write_kv<unsigned short, 1>);
+  hipLaunchKernelGGL(fn, grid, dim3(256), 0, s, a);
   return (int)hipGetLastError();
 }
 

@@ -77,11 +77,11 @@ def test_no_register_of_a_read_in_flight_is_touched(tmp_path):
     assert r.returncode == 0, r.stderr[-2000:]
     asm = (tmp_path / "l.s").read_text()
     seen = 0
-    for m in re.finditer(r"^(_ZN3kgs6latent4attnILi(\d+)E\S+):[^\n]*$", asm, re.M):
+    for m in re.finditer(r"^(_ZN3kgs6latent4attnILi(\d+)ELi(\d+)E\S+):[^\n]*$", asm, re.M):
         body = asm[m.end():asm.index(".Lfunc_end", m.end())].splitlines()
         bad, reads = outstanding_hazards(body)
         assert not bad, (m.group(1), bad[:5])
-        rt = int(m.group(2))
-        assert reads == 2 * rt + 4 * rt, (rt, reads)  # keys twice per step, four transposed reads per tile pair
+        rt, rk = int(m.group(2)), int(m.group(3))
+        assert reads == 2 * (rt + rk) + 4 * rt, (rt, rk, reads)  # keys twice per step, four transposed reads per tile pair
         seen += 1
-    assert seen == 8
+    assert seen == 3 * 8
