@@ -85,12 +85,12 @@ def parse(argv=None):
     ap.add_argument("--oversubscribe", action="store_true",
                     help="allow more ranks than GPUs (rank r on GPU r %% n): tests the multi-rank GPU path on a "
                          "1-GPU box, with --dist-backend gloo; not a benchmark configuration")
-    ap.add_argument("--workload", choices=("gemm", "ruruzen", "nufusun", "nokipel"), default="gemm",
-                    help="gemm = the benchmark; ruruzen, nufusun, nokipel = prefill and decode throughput of that design's "
+    ap.add_argument("--workload", choices=("gemm", "ruruzen", "nufusun", "nokipel", "vumalix"), default="gemm",
+                    help="gemm = the benchmark; ruruzen, nufusun, nokipel, vumalix = prefill and decode throughput of that design's "
                          "layer stack beside stacks of equal size, one GPU (kgs/serve/layer_bench.py)")
     ap.add_argument("--sizes", default="w2048,w4096", help="layer stacks: sizes, comma-separated")
     ap.add_argument("--layers", default=None, help="layer stacks: one letter per layer (ruruzen: L, S, D, default "
-                                                   "LDSD; nufusun: A, N, default AAAA; nokipel: L, M, C, A, default LAMC)")
+                                                   "LDSD; nufusun: A, N, default AAAA; nokipel: L, M, C, A, default LAMC; vumalix: L, S, A, default LASA)")
     ap.add_argument("--models", default=None, help="layer stacks: which models run, comma-separated (default: the design and the "
                                                    "closest others)")
     ap.add_argument("--cases", choices=("all", "prefill", "decode"), default="all", help="layer stacks: which steps")
@@ -162,7 +162,7 @@ def main(argv=None) -> int:
 
 
 def layer_workload(args) -> int:
-    """``--workload ruruzen|nufusun|nokipel``: one JSON line with every case of every model."""
+    """``--workload ruruzen|nufusun|nokipel|vumalix``: one JSON line with every case of every model."""
     import json
 
     from kgs.serve import layer_bench as lb

@@ -112,7 +112,7 @@ _SIGS = {
                                                                                            _c_void_p], _c_int),
     # post-normed residual with a convolution over time (postnorm.hip)
     "kgs_postnorm": ([_c_void_p] * 4 + [_c_long, _c_void_p, _c_long] + [ctypes.c_float] * 2 + [_c_void_p] * 2 + [_c_int] * 2
-                     + [ctypes.c_float] + [_c_void_p] * 7 + [_c_long] + [_c_int] * 5 + [_c_void_p], _c_int),
+                     + [ctypes.c_float] + [_c_void_p] * 7 + [_c_long] + [_c_int] * 4 + [_c_void_p], _c_int),
     "kgs_latent_norm": ([_c_void_p, _c_long] + [_c_int] * 8 + [_c_void_p] * 2 + [_c_int] * 2 + [_c_void_p] * 5
                         + [_c_int, ctypes.c_float, _c_int, _c_void_p], _c_int),
     "kgs_head_proj": ([_c_void_p] * 6 + [_c_long] * 5 + [_c_int] * 7 + [_c_void_p] * 2 + [_c_int] * 3 + [_c_void_p],

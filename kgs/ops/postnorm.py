@@ -19,7 +19,6 @@ from .hyper import _act, _f32
 from .residual import _tokens
 
 MAX_WIDTH = 16384
-BLOCK_ROWS = 2048  # rows from which a workgroup takes eight of them
 
 
 class ConvState:
@@ -87,7 +86,7 @@ class PostNorm:
             0 if conv is None else _f32(conv.w, (taps, self.wp), "conv"), state.rows.data_ptr() if moves else 0, taps,
             int(final is not None), float(final or 0.0), 0 if save is None else save.rows.data_ptr(),
             seqs.row_seq.data_ptr(), seqs.row0.data_ptr(), seqs.n.data_ptr(), seqs.pos0.data_ptr(), seqs.slot.data_ptr(),
-            h.data_ptr(), h.stride(0), T, self.width, self.wp, 8 if T >= BLOCK_ROWS else 1, int(f32),
+            h.data_ptr(), h.stride(0), T, self.width, self.wp, int(f32),
             _lib.stream_handle(h.device))
         _lib.check(rc, f"postnorm[{T}x{self.wp}]")
         return h

@@ -1,7 +1,7 @@
-"""Prefill and decode throughput of a Ruruzen, Nufusun or Nokipel layer stack at sizes
+"""Prefill and decode throughput of a Ruruzen, Nufusun, Nokipel or Vumalix layer stack at sizes
 that resemble a real model's layers (random weights), beside stacks of the closest other
 models of the same width, heads, feed-forward (where there are experts: those that a token
-uses) and depth: ``python bench.py --workload ruruzen|nufusun|nokipel``.
+uses) and depth: ``python bench.py --workload ruruzen|nufusun|nokipel|vumalix``.
 
 All run through :class:`LLMEngine`'s own step runners: prefill a whole prompt
 batch in one step, decode a hipGraph replay per step. Per case the median of
@@ -19,6 +19,7 @@ from kgs.models.llama import LlamaConfig
 from kgs.models.nokipel import NokipelConfig
 from kgs.models.nufusun import NufusunConfig
 from kgs.models.ruruzen import RuruzenConfig
+from kgs.models.vumalix import VumalixConfig
 from kgs.ops.decode import PAGE
 
 # name -> width, heads, q_rank, kv_rank, ff, Llama kv heads (head size 128 everywhere)
@@ -26,8 +27,9 @@ SIZES = {"w2048": (2048, 16, 768, 512, 8192, 4), "w4096": (4096, 32, 1536, 512, 
 EXPERTS, TOP = 16, 4     # experts of a layer and those a token uses, together as wide as ff
 IDENTITY = 2             # Nokipel: identity experts among them; one of the TOP is the shared expert
 ATTENTION_CHUNK = 5120   # Nokipel: positions of an attention chunk (3072 keys at the longest context below)
-LAYERS = {"ruruzen": "LDSD", "nufusun": "AAAA", "nokipel": "LAMC"}
-BESIDE = {"ruruzen": ("llama",), "nufusun": ("llama",), "nokipel": ("nufusun", "ruruzen")}
+WINDOW, ROT_DIM, TAPS = 2048, 64, 3  # Vumalix: of its latent attention, and of its convolutions
+LAYERS = {"ruruzen": "LDSD", "nufusun": "AAAA", "nokipel": "LAMC", "vumalix": "LASA"}
+BESIDE = {"ruruzen": ("llama",), "nufusun": ("llama",), "nokipel": ("nufusun", "ruruzen"), "vumalix": ("ruruzen", "nokipel")}
 VOCAB = 32000
 PREFILL = ((1, 8192), (8, 1024), (64, 128))              # sequences x tokens
 DECODE = ((1, 1024), (16, 1024), (64, 1024), (256, 1024), (16, 8192))  # batch x context
@@ -81,6 +83,25 @@ def nokipel(size: str, layers: str) -> NokipelConfig:
         "layers": [dict(zip(("type", "mixer", "mlp"), kinds[ch])) for ch in layers]})
 
 
+def vumalix(size: str, layers: str) -> VumalixConfig:
+    """``layers``: one letter per layer -- L latent attention, S latent attention with the
+    first L's weights, A differential attention (maps half as wide as a value, so that its
+    cache is as large as other designs'); all with a feed-forward."""
+    width, heads, qr, kr, ff, kv = SIZES[size]
+    latent = {"heads": heads, "dim": 128, "rot_dim": ROT_DIM, "vdim": 128, "q_rank": qr, "kv_rank": kr,
+              "scale": (128 + ROT_DIM) ** -0.5, "mask": {"size": WINDOW}, "rot": {"dims": ROT_DIM, "base": 1e4}}
+    attention = {"heads": heads, "kv_heads": kv, "dim": 64, "vdim": 128, "scale": 64 ** -0.5, "diff": 0.7,
+                 "q_temp": {"coef": 0.1, "every": 4096}}
+    out = []
+    for ch in layers:
+        e = {"type": "attention", "mixer": attention} if ch == "A" else {"type": "latent_attention", "mixer": latent}
+        if ch == "S":
+            e["weights_of"] = layers.index("L")
+        out.append({**e, "mlp": {"kind": "dense", "ff": ff}})
+    return VumalixConfig.from_dict({"architecture": "Vumalix", "vocab": VOCAB, "width": width, "norm": {"eps": 1e-5},
+                                    "canon": {"taps": TAPS}, "layers": out})
+
+
 def llama(size: str, layers: str) -> LlamaConfig:
     width, heads, _, _, ff, kv = SIZES[size]
     return LlamaConfig(hidden=width, intermediate=ff, heads=heads, kv_heads=kv, layers=len(layers), vocab=VOCAB)
@@ -126,7 +147,7 @@ def _time(run, steps: int) -> float:
 
 def run(sizes=("w2048", "w4096"), layers: str = "LDSD", rounds: int = 3, prefill=PREFILL, decode=DECODE,
         models=("ruruzen", "llama"), progress=lambda s: None) -> list[dict]:
-    """``models``: "ruruzen", "nufusun", "nokipel", "llama"; ``layers``: the first one's, a
+    """``models``: "ruruzen", "nufusun", "nokipel", "vumalix", "llama"; ``layers``: the first one's, a
     further design has its own."""
     from .engine import EngineConfig, LLMEngine
 
@@ -137,7 +158,7 @@ def run(sizes=("w2048", "w4096"), layers: str = "LDSD", rounds: int = 3, prefill
         ec = dict(num_pages=most // PAGE + 2 * nb + 2, max_batch=max(256, nb), max_model_len=16384)
         engines = {}
         for m in models:
-            make = {"ruruzen": ruruzen, "nufusun": nufusun, "nokipel": nokipel, "llama": llama}[m]
+            make = {"ruruzen": ruruzen, "nufusun": nufusun, "nokipel": nokipel, "vumalix": vumalix, "llama": llama}[m]
             cfg = make(size, layers if m in (models[0], "llama") else LAYERS[m])
             engines[m] = LLMEngine(cfg, EngineConfig(**ec))
             progress(f"{size} {m} ready")

@@ -10,20 +10,21 @@
 // A portion's first rows need rows of earlier steps: a sequence's state is a ring of its
 // last taps - 1 inputs, position p in entry p % (taps - 1). The launch that reads it never
 // writes it: entries are written by the next launch on the residual, from the x it reads
-// (`save`), so no row waits for another. Rows before the own ones of a workgroup are
-// computed again instead of read back, so the convolution needs x in two buffers (xi, xo).
+// (`save`), so no row waits for another.
 //
-// One workgroup takes B rows in a row of the batch; a thread the same columns of all. Long
-// convolutions and wide rows are a launch of their own (`conv`), which reads the rows back.
+// One workgroup per row. It computes the taps - 1 rows before its own again instead of waiting
+// for them, so the convolution needs x in two buffers (xi, xo); neighbouring rows run on one
+// XCD, whose L2 then has them (measured: as fast as two rows per workgroup, faster than four or
+// eight). Long convolutions and wide rows are a launch of their own (`conv`), which
+// reads the rows back.
 #include "kgs_common.h"
 
 namespace kgs {
 namespace postnorm {
 
 constexpr int MAX_NT = 512, MAX_NV = 4;  // 8-column pieces per thread
-constexpr int MAX_HALO = 3;              // rows before its own that `step` computes again
+constexpr int MAX_HALO = 3;              // rows that `step` computes again
 constexpr int HALO_NV = 2;               // pieces per thread up to which it does
-constexpr int BLOCK = 8;                 // rows of a workgroup in long batches
 
 struct Args {
   const float* xi;    // [T, wp]
@@ -95,19 +96,21 @@ __device__ __forceinline__ void block_sums(float (&s)[R], float (*part)[MAX_NT /
   }
 }
 
-template <typename T, int NV, int HALO, int B>
+template <typename T, int NV, int HALO>
 __global__ __launch_bounds__(MAX_NT) void step(Args a) {
-  constexpr int R = HALO + B;
+  constexpr int R = HALO + 1;
   __shared__ float part[R][MAX_NT / 64];
   const int tid = threadIdx.x, nt = blockDim.x, nc = a.wp / 8;
-  const int r0 = xcd_remap(blockIdx.x, gridDim.x) * B, nr = min(B, a.T - r0);
-  // rows computed again for the convolution: those of the first row's sequence
-  int again = 0;
-  if (HALO > 0) {
-    const int s = a.row_seq[r0];
-    again = min(HALO, r0 - a.row0[s]);
+  const int own = xcd_remap(blockIdx.x, gridDim.x);
+  // the row's sequence, its number in this batch, position and first ring entry
+  int sq = 0, i = 0, pos = 0, ring = 0;
+  if (HALO > 0 || a.save) {
+    sq = a.row_seq[own];
+    i = own - a.row0[sq];
+    pos = a.pos0[sq] + i;
+    ring = a.slot[sq] * (a.taps - 1);
   }
-  auto wanted = [&](int j) { return j < HALO ? j >= HALO - again : j - HALO < nr; };
+  const int first = HALO - min(HALO, i);  // rows from `first` on are computed, the last is the own one
 
   Raw<T> y[R][NV];
   float ss[R];
@@ -115,8 +118,8 @@ __global__ __launch_bounds__(MAX_NT) void step(Args a) {
 #pragma unroll
     for (int j = 0; j < R; ++j) {
       ss[j] = 0.f;
-      if (!wanted(j)) continue;
-      const T* yp = (const T*)a.y + (long)(r0 - HALO + j) * a.ldy;
+      if (j < first) continue;
+      const T* yp = (const T*)a.y + (long)(own - HALO + j) * a.ldy;
 #pragma unroll
       for (int k = 0; k < NV; ++k) {
         const int c = tid + k * nt;
@@ -135,8 +138,8 @@ __global__ __launch_bounds__(MAX_NT) void step(Args a) {
   float v[NV][8];
 #pragma unroll
   for (int j = 0; j < R; ++j) {
-    if (!wanted(j)) continue;
-    const int row = r0 - HALO + j;
+    if (j < first) continue;
+    const int row = own - HALO + j;
 #pragma unroll
     for (int k = 0; k < NV; ++k) {
       const int c = tid + k * nt;
@@ -144,19 +147,12 @@ __global__ __launch_bounds__(MAX_NT) void step(Args a) {
       if (a.tokens) load8((const T*)a.embed + (long)a.tokens[row] * a.lde + 8 * c, v[k]);
       else load8(a.xi + (long)row * a.wp + 8 * c, v[k]);
     }
-    int sq = 0, i = 0, pos = 0, ring = 0;
-    if (j >= HALO && (a.save || (HALO > 0 && a.cw))) {
-      sq = a.row_seq[row];
-      i = row - a.row0[sq];
-      pos = a.pos0[sq] + i;
-      ring = a.slot[sq] * (a.taps - 1);
-      if (a.save && a.n[sq] - i < a.taps) {
-        float* sp = a.save + (long)(ring + pos % (a.taps - 1)) * a.wp;
+    if (j == HALO && a.save && a.n[sq] - i < a.taps) {
+      float* sp = a.save + (long)(ring + pos % (a.taps - 1)) * a.wp;
 #pragma unroll
-        for (int k = 0; k < NV; ++k) {
-          const int c = tid + k * nt;
-          if (c < nc) store8(sp + 8 * c, v[k]);
-        }
+      for (int k = 0; k < NV; ++k) {
+        const int c = tid + k * nt;
+        if (c < nc) store8(sp + 8 * c, v[k]);
       }
     }
     if (!a.tokens) {
@@ -165,7 +161,7 @@ __global__ __launch_bounds__(MAX_NT) void step(Args a) {
 #pragma unroll
         for (int e = 0; e < 8; ++e) v[k][e] = __builtin_fmaf(ss[j], y[j][k].at(e), v[k][e]);
     }
-    if (j >= HALO) {
+    if (j == HALO) {
       float fin = 0.f;
       if (HALO == 0 && a.final) {
         float s[1] = {0.f};
@@ -207,17 +203,11 @@ __global__ __launch_bounds__(MAX_NT) void step(Args a) {
         store8((T*)a.h + (long)row * a.ldh + 8 * c, o);
       }
     }
-    if constexpr (HALO > 0) {
-#pragma unroll
-      for (int d = HALO - 1; d > 0; --d)
-#pragma unroll
-        for (int k = 0; k < NV; ++k)
-#pragma unroll
-          for (int e = 0; e < 8; ++e) prev[d][k][e] = prev[d - 1][k][e];
+    if (j < HALO) {
 #pragma unroll
       for (int k = 0; k < NV; ++k)
 #pragma unroll
-        for (int e = 0; e < 8; ++e) prev[0][k][e] = v[k][e];
+        for (int e = 0; e < 8; ++e) prev[HALO - 1 - j][k][e] = v[k][e];
     }
   }
 }
@@ -246,24 +236,15 @@ __global__ __launch_bounds__(256) void conv(Args a) {
 int threads(const Args& a) { return a.wp / 8 >= MAX_NT ? MAX_NT : (a.wp / 8 + 63) / 64 * 64; }
 int pieces(const Args& a) { return (a.wp / 8 + threads(a) - 1) / threads(a); }
 
-template <typename T, int NV, int HALO, int B>
-int launch_step(const Args& a, hipStream_t s) {
-  hipLaunchKernelGGL((step<T, NV, HALO, B>), dim3((a.T + B - 1) / B), dim3(threads(a)), 0, s, a);
-  return (int)hipGetLastError();
-}
-template <typename T, int HALO>
-int launch_halo(const Args& a, int block, hipStream_t s) {
-  if constexpr (sizeof(T) == 2)
-    if (block > 1) return pieces(a) <= 1 ? launch_step<T, 1, HALO, BLOCK>(a, s) : launch_step<T, 2, HALO, BLOCK>(a, s);
-  return pieces(a) <= 1 ? launch_step<T, 1, HALO, 1>(a, s) : launch_step<T, 2, HALO, 1>(a, s);
-}
 template <typename T>
-int launch(const Args& a, int halo, int block, hipStream_t s) {
-  if (halo == 1) return launch_halo<T, 1>(a, block, s);
-  if (halo == 2) return launch_halo<T, 2>(a, block, s);
-  if (halo == 3) return launch_halo<T, 3>(a, block, s);
-  const int nv = pieces(a);
-  return nv <= 1 ? launch_step<T, 1, 0, 1>(a, s) : nv <= 2 ? launch_step<T, 2, 0, 1>(a, s) : launch_step<T, 4, 0, 1>(a, s);
+int launch(const Args& a, int halo, hipStream_t s) {
+  static_assert(MAX_HALO == 3 && HALO_NV == 2 && MAX_NV == 4, "the instances below");
+  const bool one = pieces(a) <= 1;
+  auto fn = halo == 1 ? (one ? step<T, 1, 1> : step<T, 2, 1>) : halo == 2 ? (one ? step<T, 1, 2> : step<T, 2, 2>)
+            : halo == 3 ? (one ? step<T, 1, 3> : step<T, 2, 3>)
+                        : one ? step<T, 1, 0> : pieces(a) <= 2 ? step<T, 2, 0> : step<T, 4, 0>;
+  hipLaunchKernelGGL(fn, dim3(a.T), dim3(threads(a)), 0, s, a);
+  return (int)hipGetLastError();
 }
 
 }  // namespace postnorm
@@ -272,13 +253,12 @@ int launch(const Args& a, int halo, int block, hipStream_t s) {
 // x [T, wp] fp32: xo = xi + g y / rms(y) (tokens null), or embed[token]; then h [T, ldh]: xo,
 // its norm times gf (final), or xo plus its convolution (cw [taps][wp], row d the weight of
 // the row d before). A convolution of 2 to 4 taps and rows of up to 8192 columns in one launch
-// (xi and xo different buffers; block 8: eight rows per workgroup, bf16); others in two.
+// (xi and xo different buffers); others in two.
 // cstate, save: rings [slots][taps - 1][wp]; row_seq [T], row0 / n / pos0 / slot per sequence.
 KGS_EXPORT int kgs_postnorm(const void* xi, void* xo, const void* tokens, const void* embed, long lde, const void* y,
                             long ldy, float g, float eps, const void* cw, const void* cstate, int taps, int final,
                             float gf, void* save, const void* row_seq, const void* row0, const void* n, const void* pos0,
-                            const void* slot, void* h, long ldh, int T, int width, int wp, int block, int f32,
-                            hipStream_t s) {
+                            const void* slot, void* h, long ldh, int T, int width, int wp, int f32, hipStream_t s) {
   using namespace kgs::postnorm;
   if (T <= 0 || width <= 0 || wp < width || wp > MAX_NT * 8 * MAX_NV || ldh < wp || taps < 1) return KGS_ERR_SHAPE;
   if (tokens ? (!embed || lde < wp || save) : (!xi || !y || ldy < wp)) return KGS_ERR_SHAPE;
@@ -295,7 +275,7 @@ KGS_EXPORT int kgs_postnorm(const void* xi, void* xo, const void* tokens, const 
   const bool apart = cw && taps > 1 && (taps > MAX_HALO + 1 || pieces(a) > HALO_NV);
   if (apart) a.cw = nullptr;
   const int halo = a.cw ? taps - 1 : 0;
-  if (int rc = f32 ? launch<float>(a, halo, block, s) : launch<unsigned short>(a, halo, block, s)) return rc;
+  if (int rc = f32 ? launch<float>(a, halo, s) : launch<unsigned short>(a, halo, s)) return rc;
   if (!apart) return KGS_OK;
   a.cw = (const float*)cw, a.xi = a.xo;
   const dim3 grid(T, (wp / 8 + 255) / 256);

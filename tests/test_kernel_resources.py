@@ -417,9 +417,10 @@ def test_p2p_allreduce_order_check_catches_weakened_builds(tmp_path, mutation):
 
 
 def test_paged_and_lightning_kernels_do_not_spill(tmp_path):
-    """Attention over head pages and lightning attention: no spills, and the chunk kernel
-    (keys and values of 128) leaves room for a second workgroup of eight waves on a CU."""
-    for src in ("paged.hip", "lightning.hip"):
+    """Attention over head pages, latent and lightning attention, the post-normed residual: no
+    spills, and the chunk kernel (keys and values of 128) leaves room for a second workgroup of
+    eight waves on a CU."""
+    for src in ("paged.hip", "lightning.hip", "latent.hip", "postnorm.hip"):
         for name, r in _compile(src, tmp_path, flags=("-mllvm", "-amdgpu-mfma-vgpr-form=1"))[0].items():
             assert r["VGPRs Spill"] == 0 and r["SGPRs Spill"] == 0, (name, r)
             if "6chunksILi4ELi8ELb1EE" in name:
