@@ -57,7 +57,7 @@ def _mixer(where: str, kind: str, m) -> LatentSpec | DiffAttentionSpec:
         dims, base = _positive(where, m["rot"], "dims")[0], _number(where, m["rot"], "base")
         if dims != rot or rot % 2 or base <= 0:
             raise ValueError(f"{where}: rot.dims {dims} must be the even rot_dim {rot}, rot.base {base} positive")
-        window = _positive(where, m["mask"], "size")[0]
+        window = _positive(where, m["mask"], "size")[0] if m.get("mask") else 0
         return LatentSpec(heads, dim, vdim, qr, kr, scale, rot_dim=rot, rot_base=base, window=window, gate_each=True)
     if kind == ATTENTION:
         heads, kv, dim, vdim = _positive(where, m, "heads", "kv_heads", "dim", "vdim")
@@ -69,23 +69,33 @@ def _mixer(where: str, kind: str, m) -> LatentSpec | DiffAttentionSpec:
     raise ValueError(f"{where}: unknown mixer type {kind!r}")
 
 
+def _owner(entries, i: int) -> int:
+    """The layer whose weights layer ``i`` uses."""
+    j = i
+    for _ in entries:
+        k = entries[j].get("weights_of")
+        if k is None or k == j:
+            return j
+        if not isinstance(k, int) or isinstance(k, bool) or not 0 <= k < len(entries):
+            raise ValueError(f"layer {j}: weights_of {k!r} is no layer")
+        j = k
+    raise ValueError(f"layer {i}: no layer has the weights")
+
+
 def _layers(entries) -> tuple[LayerSpec, ...]:
     out = []
     for i, e in enumerate(entries):
         where, f = f"layer {i}", e.get("mlp")
         if f is not None and f.get("kind") != "dense":
             raise ValueError(f"{where}: unknown feed-forward kind {f.get('kind')!r}")
-        j = e.get("weights_of")
-        if j is not None and (not isinstance(j, int) or isinstance(j, bool) or not 0 <= j < len(entries)):
-            raise ValueError(f"{where}: weights_of {j!r} is no layer")
         out.append(LayerSpec(_mixer(where, e.get("type"), e.get("mixer")), None if f is None else _positive(where, f, "ff")[0],
-                             i if j is None else j))
+                             _owner(entries, i)))
     if not out:
         raise ValueError("a model needs at least one layer")
     for i, x in enumerate(out):
         o = out[x.owner]
-        if o.owner != x.owner or (o.mixer, o.ff) != (x.mixer, x.ff):
-            raise ValueError(f"layer {i} cannot use the weights of layer {x.owner}: that has none of its own or other sizes")
+        if (o.mixer, o.ff) != (x.mixer, x.ff):
+            raise ValueError(f"layer {i} cannot use the weights of layer {x.owner}, which has other sizes")
     return tuple(out)
 
 

@@ -36,6 +36,12 @@ def test_config_reads_every_size():
     assert [x.ff for x in c.layers] == [72, 100, 72, None, 100, 72]
     assert [x.owner for x in c.layers] == [0, 1, 0, 3, 1, 0] and c.owners == [0, 1, 3]
     assert VM.config("large").owners == [0, 2, 3]  # layer 1 uses a later one's
+    d = json.loads(json.dumps(c.raw))
+    d["layers"][5]["weights_of"] = 2  # which uses layer 0's
+    assert VumalixConfig.from_dict(d).layers == c.layers
+    d["layers"][5]["mixer"].pop("mask")
+    d["layers"][5].pop("weights_of")
+    assert VumalixConfig.from_dict(d).layers[5].mixer.window == 0
     assert c.has_state and not VM.config("stateless").has_state
 
 
@@ -57,7 +63,7 @@ def test_config_reads_every_size():
     lambda d: d["layers"][0]["mlp"].update(kind="gelu"),
     lambda d: d["layers"][0]["mlp"].update(ff=0),
     lambda d: d["layers"][2].update(weights_of=6), lambda d: d["layers"][2].update(weights_of=1),
-    lambda d: d["layers"][5].update(weights_of=2), lambda d: d["layers"][2].update(mlp=None),
+    lambda d: d["layers"][0].update(weights_of=2), lambda d: d["layers"][2].update(mlp=None),
     lambda d: d["canon"].update(taps=0), lambda d: d["norm"].pop("eps"),
     lambda d: d.update(width=0), lambda d: d.update(layers=[]),
 ])
