@@ -117,15 +117,16 @@ def latent_norm(z: torch.Tensor, oq: int, wq: torch.Tensor, qp: int, oc: int, wc
     ``pages`` at ``slots`` (-1: dropped). ``wc`` None: no latent of its own. ``rotary``: the
     columns from ``okr`` on, turned by the rows' ``pos``, follow the latent's ``rp``."""
     T = z.shape[0]
-    hr = pages.shape[2] - rp if rotary is not None else 0
+    hr = pages.shape[2] - rp if rotary is not None and wc is not None else 0
     nq, nc = wq.shape[0], 0 if wc is None else wc.shape[0]
     _act(z, T, max(oq + nq, oc + nc if nc else 0, okr + hr), z.dtype, "z")
     cq = torch.empty((T, qp), dtype=z.dtype, device=z.device)
     if nc and (pages.dtype != z.dtype or not pages.is_contiguous()):
         raise ValueError("pages must be contiguous and of z's dtype")
+    turn = _turns(rotary, pos, T) if hr else (0, 0, 0, 0)
     rc = _lib.lib().kgs_latent_norm(z.data_ptr(), z.stride(0), oq, nq, qp, oc, nc, pages.shape[2] - hr if nc else 0,
-                                    okr, hr, *(_turns(rotary, pos, T) if hr else (0, 0, 0, 0)), _f32(wq, (nq,), "wq"), _f32(wc, (nc,), "wc") if nc else 0, cq.data_ptr(),
-                                    pages.data_ptr() if nc else 0, slots.data_ptr(), T, float(eps),
+                                    okr, hr, *turn, _f32(wq, (nq,), "wq"), _f32(wc, (nc,), "wc") if nc else 0,
+                                    cq.data_ptr(), pages.data_ptr() if nc else 0, slots.data_ptr(), T, float(eps),
                                     int(z.dtype == torch.float32), _lib.stream_handle(z.device))
     _lib.check(rc, f"latent_norm[{T}]")
     return cq
